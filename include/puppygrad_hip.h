@@ -112,7 +112,10 @@ typedef struct pg_hip_options {
   uint32_t reserved;                /* must be 0 */
 } pg_hip_options;
 
-typedef struct pg_gpt2_model pg_gpt2_model;
+/* A model of any registered architecture (pg_model_create_from_dir); GPT-2 models are one of
+ * them and have a constructor from host weights besides. */
+typedef struct pg_model pg_model;
+typedef pg_model pg_gpt2_model;
 typedef struct pg_kv_cache pg_kv_cache;
 typedef struct pg_logits pg_logits;
 
@@ -139,7 +142,8 @@ uint64_t pg_kv_cache_seq_len(const pg_kv_cache* cache);
 uint64_t pg_kv_cache_max_seq_len(const pg_kv_cache* cache);
 uint32_t pg_kv_cache_batch(const pg_kv_cache* cache);
 /* The reference's `pub seq_len` field (src/models/gpt2/rust.rs:180); n must not
- * exceed max_seq_len.  Used to rewind a prefilled cache. */
+ * exceed max_seq_len.  Used to rewind a prefilled cache.  A stack model's recurrent state only
+ * goes back to 0. */
 pg_status pg_kv_cache_set_seq_len(pg_kv_cache* cache, uint64_t n);
 /* Copies one layer's K (which=0) or V (which=1) panel of sequence `b` to host:
  * [head][position][head_dim], the layout of Gpt2LayerKvCache
@@ -471,6 +475,63 @@ pg_status pg_hip_load_tuning(const char* path, pg_hip_options* options, int32_t*
  * present, supplies the tunables that `options` leaves at 0 (src/main.rs:2564-2586). */
 pg_status pg_gpt2_create_from_dir(const char* model_dir, const pg_hip_options* options,
                                   pg_gpt2_model** out);
+
+/* ---- models of any architecture ----
+ * The functions below take every model; their pg_gpt2_ namesakes above are the same functions
+ * under the names the GPT-2 adapter binds. */
+
+/* The model of a directory (config.json + model.safetensors).  The architecture is the one
+ * config.json names under `architecture`; a config.json without that key is a Hugging Face GPT-2's
+ * (pg_gpt2_create_from_dir).  An unknown name is PG_INVALID_CONFIG.
+ * "Tarepel" (a stack model): `layers` lists every layer with its mixers and their sizes; weights
+ * are BF16 or F32 tensors, kept as weight_storage says (PG_STORE_F32 or PG_STORE_BF16; activations
+ * and state are f32 either way).  A sequence's state has a fixed size, so its caches take
+ * sequences of any length. */
+pg_status pg_model_create_from_dir(const char* model_dir, const pg_hip_options* options, pg_model** out);
+void pg_model_destroy(pg_model* model);
+/* "gpt2" or the name config.json gives; owned by the model. */
+const char* pg_model_architecture(const pg_model* model);
+typedef struct pg_model_info {
+  uint64_t vocab_size;
+  uint64_t max_positions; /* n_positions; 2^30 where the architecture sets no limit */
+  uint64_t width;         /* of the residual stream */
+  uint64_t n_layer;
+} pg_model_info;
+pg_status pg_model_get_info(const pg_model* model, pg_model_info* out);
+pg_status pg_model_describe(const pg_model* model, char* dst, size_t cap);
+pg_status pg_model_prefill(const pg_model* model, pg_kv_cache* cache, const uint32_t* ids, size_t n,
+                           pg_logits** out);
+pg_status pg_model_prefill_batch(const pg_model* model, pg_kv_cache* cache, const uint32_t* ids,
+                                 size_t n, pg_logits** out);
+pg_status pg_model_prefill_profiled(const pg_model* model, pg_kv_cache* cache, const uint32_t* ids,
+                                    size_t n, pg_logits** out, pg_gpt2_operation_profile* profile);
+/* The next n tokens of a sequence, from the position and the state earlier calls left (a cleared
+ * cache: from position 0), in one portion; the cache must have batch 1.  `want` names n_want of
+ * them (increasing indices into ids); *out receives their logits, one row each in that order
+ * (null when n_want is 0).  With the last token among them decode_greedy may follow. */
+pg_status pg_model_extend(const pg_model* model, pg_kv_cache* cache, const uint32_t* ids, size_t n,
+                          const size_t* want, size_t n_want, pg_logits** out);
+pg_status pg_model_forward_one(const pg_model* model, pg_kv_cache* cache, uint32_t id, pg_logits** out);
+pg_status pg_model_forward_one_batch(const pg_model* model, pg_kv_cache* cache, const uint32_t* ids,
+                                     pg_logits** out);
+pg_status pg_model_forward(const pg_model* model, const uint32_t* ids, size_t n, float* dst, size_t dst_len);
+pg_status pg_model_decode_greedy(const pg_model* model, pg_kv_cache* cache, uint32_t max_new,
+                                 int64_t eos, uint32_t* out_ids, uint32_t* out_n,
+                                 pg_generation_stats* stats);
+pg_status pg_model_decode_greedy_batch(const pg_model* model, pg_kv_cache* cache, uint32_t steps,
+                                       uint32_t* out_ids, pg_generation_stats* stats);
+pg_status pg_model_stream_token_ids_with_stats(const pg_model* model, const uint32_t* ids, size_t n,
+                                               uint32_t max_new, int64_t eos, const pg_sampling* sampling,
+                                               uint64_t seed, pg_on_token on_token, void* user,
+                                               uint32_t* out_ids, size_t* out_n, pg_generation_stats* stats);
+/* (Stack models: the input projections count as qkv_projection, the mixers as attention, the
+ * products back to the residual as attention_projection and mlp_projection; the one-token step
+ * has both of these in one launch, counted as mlp_projection.) */
+pg_status pg_model_stream_token_ids_profiled(const pg_model* model, const uint32_t* ids, size_t n,
+                                             uint32_t max_new, int64_t eos, const pg_sampling* sampling,
+                                             uint64_t seed, pg_on_token on_token, void* user,
+                                             uint32_t* out_ids, size_t* out_n, pg_generation_stats* stats,
+                                             pg_gpt2_operation_profile* profile);
 
 /* Seeded synthetic inputs for benchmarks and tests (no reference counterpart;
  * the draw is the reference's splitmix64, src/models/generation.rs:244-267).

@@ -48,6 +48,11 @@ class pg_hip_options(C.Structure):
                 ("seq_gemm_min_tokens", C.c_uint32), ("reserved", C.c_uint32)]
 
 
+class pg_model_info(C.Structure):
+    _fields_ = [("vocab_size", C.c_uint64), ("max_positions", C.c_uint64), ("width", C.c_uint64),
+                ("n_layer", C.c_uint64)]
+
+
 class pg_sampling(C.Structure):
     _fields_ = [("temperature", C.c_float), ("has_top_p", C.c_int32), ("top_p", C.c_float),
                 ("has_top_k", C.c_int32), ("top_k", C.c_uint64), ("repeat_penalty", C.c_float),
@@ -177,6 +182,19 @@ SIGNATURES = {
     "pg_synth_token_ids": (None, [_u32p, C.c_uint64, C.c_uint64, C.c_uint64]),
     "pg_device_query": (C.c_int, [C.c_int32, C.POINTER(pg_device_info)]),
 }
+
+# the same functions under the names that take any architecture
+SIGNATURES.update({"pg_model_" + name: SIGNATURES["pg_gpt2_" + name] for name in (
+    "destroy", "describe", "prefill", "prefill_batch", "prefill_profiled", "forward_one",
+    "forward_one_batch", "forward", "decode_greedy", "decode_greedy_batch",
+    "stream_token_ids_with_stats", "stream_token_ids_profiled")})
+SIGNATURES.update({
+    "pg_model_create_from_dir": (C.c_int, [C.c_char_p, C.POINTER(pg_hip_options), C.POINTER(_vp)]),
+    "pg_model_architecture": (C.c_char_p, [_vp]),
+    "pg_model_get_info": (C.c_int, [_vp, C.POINTER(pg_model_info)]),
+    "pg_model_extend": (C.c_int, [_vp, _vp, _u32p, C.c_size_t, C.POINTER(C.c_size_t), C.c_size_t,
+                                  C.POINTER(_vp)]),
+})
 
 _lib = None
 

@@ -13,7 +13,7 @@ LIB_PATH = PKG_DIR / "libpuppygrad_hip.so"
 # (python -m puppygrad_amd.build --stamps; read by puppygrad_amd.decode_stamps).
 STAMPS_LIB_PATH = PKG_DIR / "libpuppygrad_hip_stamps.so"
 SOURCES = ["pg_kernels.hip", "pg_decode.hip", "pg_prefill.hip", "pg_ops_dev.hip", "pg_sample.hip",
-           "pg_host.cpp", "pg_assets.cpp"]
+           "pg_mixers.hip", "pg_host.cpp", "pg_stack.cpp", "pg_assets.cpp"]
 
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 # Packed-FP32 instruction selection is switched off for every device pass.
@@ -44,10 +44,12 @@ def build_library(verbose: bool = True, stamps: bool = False) -> Path:
             raise RuntimeError(f"hipcc failed on {src}:\n{text}")
         if verbose and text.strip():
             print(text, flush=True)
-    link = [HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", str(lib), *objs, "-lpthread"]
+    part = lib.with_suffix(".so.tmp")  # (a link that is cut short must not leave a library behind)
+    link = [HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", str(part), *objs, "-lpthread"]
     if verbose:
         print(" ".join(link), flush=True)
     subprocess.run(link, check=True)
+    os.replace(part, lib)
     return lib
 
 

@@ -23,266 +23,14 @@
 #include <vector>
 
 #include "pg_internal.h"
+#include "pg_json.h"
+#include "pg_stack.h"
 
 namespace {
 
 using pgh::fail;
-
-// ---------------------------------------------------------------------------
-// A small JSON reader (RFC 8259): enough for a safetensors header and config.json.
-// ---------------------------------------------------------------------------
-struct Json {
-  enum Kind { Null, Bool, Num, Str, Arr, Obj } kind = Null;
-  bool b = false;
-  double num = 0.0;
-  bool integral = false;  // written without fraction or exponent, and not negative
-  uint64_t u = 0;         // its value when integral
-  std::string str;
-  std::vector<Json> arr;
-  std::vector<std::pair<std::string, Json>> obj;  // file order; a later duplicate wins in find()
-
-  const Json* find(const std::string& key) const {
-    const Json* hit = nullptr;
-    for (const auto& kv : obj)
-      if (kv.first == key) hit = &kv.second;
-    return hit;
-  }
-};
-
-class JsonParser {
- public:
-  JsonParser(const char* b, const char* e) : begin_(b), p_(b), e_(e) {}
-
-  bool parse(Json& out, std::string& err) {
-    bool ok = value(out, 0);
-    if (ok) {
-      ws();
-      if (p_ != e_) ok = bad("trailing characters");
-    }
-    if (!ok) err = err_ + " at " + where();
-    return ok;
-  }
-
- private:
-  const char* begin_;
-  const char* p_;
-  const char* e_;
-  std::string err_;
-
-  std::string where() const {
-    size_t line = 1, col = 1;
-    for (const char* q = begin_; q < p_; ++q) {
-      if (*q == '\n') {
-        ++line;
-        col = 1;
-      } else {
-        ++col;
-      }
-    }
-    return "line " + std::to_string(line) + " column " + std::to_string(col);
-  }
-  void ws() {
-    while (p_ < e_ && (*p_ == ' ' || *p_ == '\t' || *p_ == '\n' || *p_ == '\r')) ++p_;
-  }
-  bool bad(const char* what) {
-    err_ = what;
-    return false;
-  }
-  bool literal(const char* word) {
-    const size_t n = std::strlen(word);
-    if ((size_t)(e_ - p_) < n || std::memcmp(p_, word, n) != 0) return bad("expected value");
-    p_ += n;
-    return true;
-  }
-  static void utf8(std::string& s, uint32_t cp) {
-    if (cp < 0x80) {
-      s += (char)cp;
-    } else if (cp < 0x800) {
-      s += (char)(0xC0 | (cp >> 6));
-      s += (char)(0x80 | (cp & 0x3F));
-    } else if (cp < 0x10000) {
-      s += (char)(0xE0 | (cp >> 12));
-      s += (char)(0x80 | ((cp >> 6) & 0x3F));
-      s += (char)(0x80 | (cp & 0x3F));
-    } else {
-      s += (char)(0xF0 | (cp >> 18));
-      s += (char)(0x80 | ((cp >> 12) & 0x3F));
-      s += (char)(0x80 | ((cp >> 6) & 0x3F));
-      s += (char)(0x80 | (cp & 0x3F));
-    }
-  }
-  bool hex4(uint32_t& v) {
-    if (e_ - p_ < 4) return bad("EOF while parsing a string");
-    v = 0;
-    for (int i = 0; i < 4; ++i) {
-      const char c = *p_++;
-      v <<= 4;
-      if (c >= '0' && c <= '9') v |= (uint32_t)(c - '0');
-      else if (c >= 'a' && c <= 'f') v |= (uint32_t)(c - 'a' + 10);
-      else if (c >= 'A' && c <= 'F') v |= (uint32_t)(c - 'A' + 10);
-      else return bad("invalid escape");
-    }
-    return true;
-  }
-  bool string(std::string& out) {
-    ++p_;  // opening quote
-    out.clear();
-    while (true) {
-      if (p_ == e_) return bad("EOF while parsing a string");
-      const unsigned char c = (unsigned char)*p_++;
-      if (c == '"') return true;
-      if (c < 0x20) return bad("control character found while parsing a string");
-      if (c != '\\') {
-        out += (char)c;
-        continue;
-      }
-      if (p_ == e_) return bad("EOF while parsing a string");
-      const char esc = *p_++;
-      switch (esc) {
-        case '"': out += '"'; break;
-        case '\\': out += '\\'; break;
-        case '/': out += '/'; break;
-        case 'b': out += '\b'; break;
-        case 'f': out += '\f'; break;
-        case 'n': out += '\n'; break;
-        case 'r': out += '\r'; break;
-        case 't': out += '\t'; break;
-        case 'u': {
-          uint32_t cp;
-          if (!hex4(cp)) return false;
-          if (cp >= 0xD800 && cp < 0xDC00) {
-            uint32_t lo;
-            if (e_ - p_ < 2 || p_[0] != '\\' || p_[1] != 'u') return bad("lone leading surrogate");
-            p_ += 2;
-            if (!hex4(lo)) return false;
-            if (lo < 0xDC00 || lo > 0xDFFF) return bad("lone leading surrogate");
-            cp = 0x10000 + ((cp - 0xD800) << 10) + (lo - 0xDC00);
-          } else if (cp >= 0xDC00 && cp <= 0xDFFF) {
-            return bad("lone trailing surrogate");
-          }
-          utf8(out, cp);
-          break;
-        }
-        default: return bad("invalid escape");
-      }
-    }
-  }
-  bool number(Json& out) {
-    const char* s = p_;
-    bool neg = false, frac = false;
-    if (p_ < e_ && *p_ == '-') {
-      neg = true;
-      ++p_;
-    }
-    if (p_ == e_ || *p_ < '0' || *p_ > '9') return bad("invalid number");
-    if (*p_ == '0') {
-      ++p_;
-    } else {
-      while (p_ < e_ && *p_ >= '0' && *p_ <= '9') ++p_;
-    }
-    if (p_ < e_ && *p_ == '.') {
-      frac = true;
-      ++p_;
-      if (p_ == e_ || *p_ < '0' || *p_ > '9') return bad("invalid number");
-      while (p_ < e_ && *p_ >= '0' && *p_ <= '9') ++p_;
-    }
-    if (p_ < e_ && (*p_ == 'e' || *p_ == 'E')) {
-      frac = true;
-      ++p_;
-      if (p_ < e_ && (*p_ == '+' || *p_ == '-')) ++p_;
-      if (p_ == e_ || *p_ < '0' || *p_ > '9') return bad("invalid number");
-      while (p_ < e_ && *p_ >= '0' && *p_ <= '9') ++p_;
-    }
-    const std::string text(s, p_);
-    out.kind = Json::Num;
-    out.num = std::strtod(text.c_str(), nullptr);
-    out.integral = false;
-    if (!neg && !frac && text.size() <= 19) {  // 19 digits always fit 64 bits
-      out.integral = true;
-      out.u = std::strtoull(text.c_str(), nullptr, 10);
-    }
-    return true;
-  }
-  bool value(Json& out, int depth) {
-    if (depth > 128) return bad("recursion limit exceeded");
-    ws();
-    if (p_ == e_) return bad("EOF while parsing a value");
-    switch (*p_) {
-      case '{': {
-        ++p_;
-        out.kind = Json::Obj;
-        ws();
-        if (p_ < e_ && *p_ == '}') {
-          ++p_;
-          return true;
-        }
-        while (true) {
-          ws();
-          if (p_ == e_ || *p_ != '"') return bad("key must be a string");
-          std::string key;
-          if (!string(key)) return false;
-          ws();
-          if (p_ == e_ || *p_ != ':') return bad("expected `:`");
-          ++p_;
-          Json v;
-          if (!value(v, depth + 1)) return false;
-          out.obj.emplace_back(std::move(key), std::move(v));
-          ws();
-          if (p_ < e_ && *p_ == ',') {
-            ++p_;
-            continue;
-          }
-          if (p_ < e_ && *p_ == '}') {
-            ++p_;
-            return true;
-          }
-          return bad("expected `,` or `}`");
-        }
-      }
-      case '[': {
-        ++p_;
-        out.kind = Json::Arr;
-        ws();
-        if (p_ < e_ && *p_ == ']') {
-          ++p_;
-          return true;
-        }
-        while (true) {
-          Json v;
-          if (!value(v, depth + 1)) return false;
-          out.arr.push_back(std::move(v));
-          ws();
-          if (p_ < e_ && *p_ == ',') {
-            ++p_;
-            continue;
-          }
-          if (p_ < e_ && *p_ == ']') {
-            ++p_;
-            return true;
-          }
-          return bad("expected `,` or `]`");
-        }
-      }
-      case '"':
-        out.kind = Json::Str;
-        return string(out.str);
-      case 't':
-        out.kind = Json::Bool;
-        out.b = true;
-        return literal("true");
-      case 'f':
-        out.kind = Json::Bool;
-        out.b = false;
-        return literal("false");
-      case 'n':
-        out.kind = Json::Null;
-        return literal("null");
-      default:
-        if (*p_ == '-' || (*p_ >= '0' && *p_ <= '9')) return number(out);
-        return bad("expected value");
-    }
-  }
-};
+using pgh::Json;
+using pgh::JsonParser;
 
 std::string shape_text(const std::vector<uint64_t>& shape) {  // Rust's {:?} of a Vec<usize>
   std::string s = "[";
@@ -508,12 +256,56 @@ pg_status config_uint(const std::string& path, const Json& root, const char* key
   return PG_OK;
 }
 
+pg_status read_text(const std::string& path, std::string* out, int* why) {
+  errno = 0;  // (an earlier call's value must not decide what a failed open means)
+  std::ifstream in(path, std::ios::binary);
+  if (!in) {
+    *why = errno ? errno : EIO;
+    return PG_ASSET;
+  }
+  std::stringstream buf;
+  buf << in.rdbuf();
+  *out = buf.str();
+  return PG_OK;
+}
+
 std::string join(const std::string& dir, const char* file) {
   if (dir.empty()) return file;
   return dir.back() == '/' ? dir + file : dir + "/" + file;
 }
 
 }  // namespace
+
+namespace pgh {
+
+pg_status read_json_file(const std::string& path, const char* what, Json* out) {
+  std::string text, err;
+  int why = 0;
+  if (read_text(path, &text, &why))  // ConfigLoadError::Read (src/models/config.rs:22-24)
+    return fail(PG_ASSET, std::string("failed to read ") + what + " " + path + ": " + std::strerror(why));
+  if (!JsonParser(text.data(), text.data() + text.size()).parse(*out, err))
+    return fail(PG_ASSET, std::string("failed to parse ") + what + " " + path + ": " + err);
+  if (out->kind != Json::Obj)
+    return fail(PG_ASSET, std::string("failed to parse ") + what + " " + path + ": invalid type, expected an object");
+  return PG_OK;
+}
+
+pg_status find_tensor(const pg_tensor_store& store, const std::string& name, TensorView* out) {
+  auto it = store.tensors.find(name);
+  if (it == store.tensors.end()) return not_found(name);
+  const TensorInfo& t = it->second;
+  if (t.dtype == "F32") out->dtype = TensorView::F32;
+  else if (t.dtype == "BF16") out->dtype = TensorView::BF16;
+  else if (t.dtype == "I32") out->dtype = TensorView::I32;
+  else return fail(PG_ASSET, "tensor " + name + " has dtype " + t.dtype + ", expected F32, BF16 or I32");
+  out->data = store.data + t.begin;
+  out->shape = t.shape;
+  out->count = 1;
+  for (uint64_t d : t.shape) out->count *= d;
+  return PG_OK;
+}
+
+}  // namespace pgh
 
 extern "C" {
 
@@ -557,20 +349,8 @@ pg_status pg_tensor_store_optional_f32(const pg_tensor_store* store, const char*
 
 pg_status pg_gpt2_load_config(const char* path, pg_gpt2_config* out) {
   if (!path || !out) return fail(PG_INVALID_INPUT, "null argument");
-  std::ifstream in(path, std::ios::binary);
-  if (!in)  // ConfigLoadError::Read (src/models/config.rs:22-24)
-    return fail(PG_ASSET, std::string("failed to read config ") + path + ": " +
-                              std::strerror(errno));
-  std::stringstream buf;
-  buf << in.rdbuf();
-  const std::string text = buf.str();
   Json root;
-  std::string err;
-  if (!JsonParser(text.data(), text.data() + text.size()).parse(root, err))
-    return fail(PG_ASSET, std::string("failed to parse config ") + path + ": " + err);
-  if (root.kind != Json::Obj)
-    return fail(PG_ASSET, std::string("failed to parse config ") + path +
-                              ": invalid type, expected struct HfGpt2Config");
+  if (pg_status s = pgh::read_json_file(path, "config", &root)) return s;
   pg_gpt2_config c{};
   bool have = false, have_pos = false, have_ctx = false, have_inner = false;
   uint64_t n_ctx = 0, n_inner = 0;
@@ -700,6 +480,46 @@ pg_status pg_gpt2_create_from_dir(const char* model_dir, const pg_hip_options* o
   w.n_blocks = blocks.size();
   // The upload reads each tensor once, straight from the mapping.
   return pg_gpt2_create(&cfg, &w, options, out);
+}
+
+// Architectures by what config.json says; the first that matches builds the model.
+namespace {
+struct Architecture {
+  bool (*matches)(const Json& config);
+  pg_status (*create)(const std::string& dir, const std::string& config_path, const Json& config,
+                      const pg_hip_options& opts, pg_model** out);
+};
+pg_status create_stack(const std::string& dir, const std::string& config_path, const Json& config,
+                       const pg_hip_options& opts, pg_model** out) {
+  pg_hip_options tuned = opts;
+  if (pg_status s = pg_hip_load_tuning(join(dir, "puppygrad-tune.json").c_str(), &tuned, nullptr)) return s;
+  std::unique_ptr<pg_tensor_store> st;
+  if (pg_status s = open_store(join(dir, "model.safetensors").c_str(), st)) return s;
+  return pgh::stack_create(config_path, config, *st, tuned, out);
+}
+pg_status create_gpt2(const std::string& dir, const std::string&, const Json&, const pg_hip_options& opts,
+                      pg_model** out) {
+  return pg_gpt2_create_from_dir(dir.c_str(), &opts, out);
+}
+const Architecture kArchitectures[] = {
+    {pgh::stack_config_matches, create_stack},
+    {[](const Json& c) { return c.find("architecture") == nullptr; }, create_gpt2},
+};
+}  // namespace
+
+pg_status pg_model_create_from_dir(const char* model_dir, const pg_hip_options* options, pg_model** out) {
+  if (!model_dir || !out) return fail(PG_INVALID_INPUT, "null argument");
+  *out = nullptr;
+  pg_hip_options opts{};
+  if (options) opts = *options;
+  const std::string config_path = join(model_dir, "config.json");
+  Json config;
+  if (pg_status s = pgh::read_json_file(config_path, "config", &config)) return s;
+  for (const Architecture& a : kArchitectures)
+    if (a.matches(config)) return a.create(model_dir, config_path, config, opts, out);
+  const Json* name = config.find("architecture");
+  return fail(PG_INVALID_CONFIG, "config " + config_path + ": unknown architecture" +
+                                     (name->kind == Json::Str ? " `" + name->str + "`" : ""));
 }
 
 }  // extern "C"

@@ -22,8 +22,16 @@
 
 #include "pg_internal.h"
 #include "pg_kernels.h"
+#include "pg_model.h"
+#include "pg_stack.h"
 
 namespace {
+
+using pgh::Cfg;
+using pgh::DevBuf;
+using pgh::ProfileMarks;
+using pgh::round_up;
+using pgh::select_device;
 
 thread_local std::string g_err;
 
@@ -37,136 +45,12 @@ pg_status fail(pg_status s, const std::string& msg) {
   return s;
 }
 
-#define PG_HIP(expr)                                                                  \
-  do {                                                                                \
-    hipError_t e__ = (expr);                                                          \
-    if (e__ != hipSuccess)                                                            \
-      return fail(PG_BACKEND, std::string("HIP error: ") + hipGetErrorString(e__) +   \
-                                  " at " #expr);                                      \
-  } while (0)
-
 using Clock = std::chrono::steady_clock;
 double since(Clock::time_point t0) {
   return std::chrono::duration<double>(Clock::now() - t0).count();
 }
 
-struct Cfg {
-  size_t V, P, C, L, H, I;
-  float eps;
-  size_t hd() const { return C / H; }
-};
-
 }  // namespace
-
-struct pg_gpt2_model {
-  Cfg cfg;
-  int device = 0;
-  int num_cus = 0;
-  pg_hip_options opts{};
-  float* arena = nullptr;  // one allocation holding every tensor
-  size_t arena_floats = 0;
-  float *wte = nullptr, *wpe = nullptr, *ln_f_g = nullptr, *ln_f_b = nullptr;
-  std::vector<pgk::LayerW> layers;
-  pgk::LayerW* d_layers = nullptr;  // the same table in device memory
-  bool persistent = false;          // batch-1 decode runs as one persistent launch
-  int persistent_grid = 0;          // workgroups of that launch (one per CU)
-  int attn_splits = 1;              // key splits per head in the persistent kernel
-  // tunables (pg_hip_options; defaults filled in at creation)
-  int item_keys = 128;              // keys per attention item of the persistent kernel
-  bool item_keys_auto = true;       // not set by the caller: 256-key items for launches that stay
-                                    // within 256 positions (one split per head: no merge hop)
-  bool item_keys_256_ok = false;    // the device holds the grid of the 256-key instance
-  int attn_blocks_per_cu = 4;       // per-operation / batched decode attention
-  int gemm_split_items = 3;         // tile GEMM split-K
-  int gemm_b9_min_rows = 1024;      // f32 rows on the bf16 matrix cores from this many input rows
-  size_t seq_gemm_min_tokens = 4;   // prompts at least this long take the GEMM prefill
-  int w_bf16 = 0;                   // wte and the block matrices are stored as bf16
-  // int8 storage (QuantizedRows, src/models/cpu.rs:26-56): the block matrices hold int8 rows
-  // with the scales in LayerW; wte stays f32 for the embedding (rust.rs:966-974 reads the f32
-  // table) and lm_w / lm_s are its quantised copy for the lm_head (rust.rs:1815-1849).
-  // Otherwise lm_w == wte and lm_s == nullptr.
-  int w_i8 = 0;
-  float* lm_w = nullptr;
-  float* lm_s = nullptr;
-  float* lm_f = nullptr;  // [2 V]: LN_f folded into the lm_head rows (pgk::launch_ln_fold)
-};
-
-struct pg_logits {
-  pg_kv_cache* owner;
-  float* data;  // device [rows][vocab]
-  uint32_t rows;
-  uint64_t vocab;
-};
-
-struct pg_kv_cache {
-  Cfg cfg;
-  int device = 0;
-  int num_cus = 0;
-  uint32_t B = 1;
-  size_t seq_len = 0;
-  float* kv = nullptr;  // [L][2][B][H][P][hd]
-  // per-sequence activation scratch, [B][...]
-  float* seq_scratch = nullptr;  // activations of the full-sequence (GEMM) forward, grown on demand
-  size_t seq_scratch_floats = 0;
-  float* gemm_ws = nullptr;      // split-K partial tiles of the batched decode step
-  size_t gemm_ws_floats = 0;
-  float *x = nullptr, *q = nullptr, *hbuf = nullptr, *part_acc = nullptr, *part_m = nullptr,
-        *part_l = nullptr, *logits_buf = nullptr;
-  float *qkv_b = nullptr, *xn_b = nullptr, *att_b = nullptr;  // batched step: [B][3C], [B][C], [B][C]
-  bool pack32 = false;  // batched step: xn_b, att_b and hbuf are packed (pgk::packed32_index)
-  // device-side candidate selection for sampling, allocated at first use: kept candidates
-  // (ids, then values, then [count]) and the recent ids of the repeat penalty, with pinned
-  // host mirrors
-  uint32_t* d_cand = nullptr;
-  uint32_t* h_cand = nullptr;
-  uint32_t* d_recent = nullptr;
-  uint32_t* h_recent = nullptr;
-  uint32_t* d_tok = nullptr;      // [B] token the next step embeds
-  uint32_t* d_out_ids = nullptr;  // [P][B] ids produced by greedy decode
-  uint32_t* h_ids = nullptr;      // pinned staging, [P][B]
-  // pinned staging of the prompts of full-sequence forwards, used in turn: the copy to the
-  // device is queued without waiting, and a buffer is reused once the copy of two calls ago
-  // has been made
-  uint32_t* h_prompt[2] = {nullptr, nullptr};
-  hipEvent_t ev_prompt[2] = {nullptr, nullptr};
-  unsigned prompt_turn = 0;
-  // streamed greedy generation: ids the persistent kernel writes straight into pinned host
-  // memory as it selects them ([P + 1], batch 1), and the device's address of that block
-  uint32_t* h_stream = nullptr;
-  uint32_t* h_stream_dev = nullptr;
-  hipStream_t stream = nullptr;
-  hipEvent_t ev0 = nullptr, ev1 = nullptr;
-  pg_logits logits{};
-  bool logits_valid = false;
-  // persistent decode: tagged activation words {epoch, f32} and the launch status
-  // One uncached block: the tagged argmax words, then the f32 exchange vectors (two buffers each)
-  unsigned long long* best_t = nullptr;
-  unsigned* xch = nullptr;
-  size_t best_words = 0;  // 64-bit words at best_t
-  size_t x_words = 0;     // 32-bit words at xch
-  // The exchange words are as a launch expects them: the last persistent launch on this cache
-  // ran to its end and the model has an even number of layers (the set a launch's first layer
-  // uses was then armed again during the last layer before it, and the other set is armed by
-  // the first layer before the second uses it, as between two forwards of one launch), so the
-  // next launch needs no k_arm_exchange in front of it.
-  bool xch_ready = false;
-  unsigned xch_set = 0;   // words from one set of exchange vectors to the other
-  // [grid][L + 1][16] time stamps of a profiled forward of the persistent kernel (allocated on
-  // first use; pg_gpt2_stream_token_ids_profiled)
-  unsigned long long* stamps = nullptr;
-  size_t tagged_bytes = 0;  // size of that allocation as the exchange pool counts it
-  unsigned* status = nullptr;
-  unsigned* h_status = nullptr;  // pinned
-  uint32_t* d_force = nullptr;   // [P] prompt ids for a one-launch prefill
-  unsigned epoch = 1;            // next unused epoch
-
-  float* k_panel(size_t l, size_t b) const {
-    return kv + (((l * 2 + 0) * B + b) * cfg.H) * cfg.P * cfg.hd();
-  }
-  float* v_panel(size_t l, size_t b) const {
-    return kv + (((l * 2 + 1) * B + b) * cfg.H) * cfg.P * cfg.hd();
-  }
-};
 
 namespace {
 
@@ -233,8 +117,6 @@ pg_status validate_weights(const Cfg& c, const pg_gpt2_weights_view& w) {
   return PG_OK;
 }
 
-size_t round_up(size_t n, size_t a) { return (n + a - 1) / a * a; }
-
 // Arena layout of an int8 matrix: rows * cols bytes, padded to a 256-byte boundary, then
 // the rows' f32 scales.  (Defined once here: model creation places tensors by it and the
 // GEMM drivers find a matrix's scales by it.)
@@ -242,29 +124,6 @@ constexpr size_t kArenaAlign = 64;  // floats
 size_t i8_matrix_floats(size_t rows, size_t cols) { return round_up((rows * cols + 3) / 4, kArenaAlign); }
 const float* i8_scales_of(const float* W, size_t rows, size_t cols) {
   return W + i8_matrix_floats(rows, cols);
-}
-
-struct DevBuf {
-  float* p = nullptr;
-  ~DevBuf() {
-    if (p) (void)hipFree(p);
-  }
-  pg_status alloc(size_t n) {
-    PG_HIP(hipMalloc(&p, std::max<size_t>(n, 1) * sizeof(float)));
-    return PG_OK;
-  }
-};
-
-pg_status select_device(int device) {
-  int n = 0;
-  hipError_t e = hipGetDeviceCount(&n);
-  if (e != hipSuccess || n == 0)
-    return fail(PG_BACKEND, "no HIP device available: the hip backend needs an AMD GPU");
-  if (device < 0 || device >= n)
-    return fail(PG_INVALID_CONFIG, "hip device " + std::to_string(device) +
-                                       " out of range for " + std::to_string(n) + " devices");
-  PG_HIP(hipSetDevice(device));
-  return PG_OK;
 }
 
 // validate_input (src/models/gpt2/rust.rs:1029-1051).
@@ -282,7 +141,11 @@ pg_status validate_input(const Cfg& c, const uint32_t* ids, size_t n) {
 }
 
 // Gpt2KvCache::check_compatible (src/models/gpt2/rust.rs:206-234).
-pg_status check_compatible(const pg_gpt2_model* m, const pg_kv_cache* c) {
+pg_status check_compatible(const pg_model* m, const pg_kv_cache* c) {
+  if (m->stack || c->stack) {  // the layers of a stack model differ in kind and size
+    if (c->stack_model != m) return fail(PG_INVALID_INPUT, "cache was made for another model");
+    return PG_OK;
+  }
   if (c->cfg.L != m->cfg.L)
     return fail(PG_INVALID_INPUT, "cache layer count " + std::to_string(c->cfg.L) +
                                       " does not match n_layer " + std::to_string(m->cfg.L));
@@ -306,56 +169,12 @@ pg_status check_compatible(const pg_gpt2_model* m, const pg_kv_cache* c) {
 // launches on the cache's stream.  The token comes from tok_ptr (device) when
 // it is non-null.  With want_logits false the final LayerNorm and lm_head are
 // skipped (prefill discards those logits, rust.rs:922-926).
-// Time stamps between the launches of one step, for the buckets of Gpt2OperationProfile
-// (src/models/gpt2/rust.rs:336-347): an event is recorded on the step's stream after each
-// operation; the span since the previous event belongs to that operation's bucket.
-struct ProfileMarks {
-  enum Bucket { kNone, kLayerNorm, kQkv, kAttention, kAttnProj, kMlpFc, kMlpProj, kLogits };
-  std::vector<hipEvent_t> events;
-  std::vector<Bucket> bucket;
-  size_t used = 0;
-  hipError_t mark(hipStream_t s, Bucket b) {
-    if (used == events.size()) {
-      hipEvent_t e = nullptr;
-      hipError_t r = hipEventCreate(&e);
-      if (r != hipSuccess) return r;
-      events.push_back(e);
-      bucket.push_back(kNone);
-    }
-    bucket[used] = b;
-    return hipEventRecord(events[used++], s);
-  }
-  // Adds the spans of the step just synchronised to `p` and rewinds.
-  hipError_t collect(pg_gpt2_operation_profile* p) {
-    for (size_t i = 1; i < used; ++i) {
-      float ms = 0.0f;
-      hipError_t r = hipEventElapsedTime(&ms, events[i - 1], events[i]);
-      if (r != hipSuccess) return r;
-      const double sec = (double)ms * 1e-3;
-      switch (bucket[i]) {
-        case kLayerNorm: p->layer_norm_s += sec; break;
-        case kQkv: p->qkv_projection_s += sec; break;
-        case kAttention: p->attention_s += sec; break;
-        case kAttnProj: p->attention_projection_s += sec; break;
-        case kMlpFc: p->mlp_fc_projection_s += sec; break;
-        case kMlpProj: p->mlp_projection_s += sec; break;
-        case kLogits: p->final_logits_s += sec; break;
-        case kNone: break;
-      }
-    }
-    used = 0;
-    return hipSuccess;
-  }
-  ~ProfileMarks() {
-    for (hipEvent_t e : events) (void)hipEventDestroy(e);
-  }
-};
 #define PG_MARK(b) \
   do {             \
     if (marks) PG_HIP(marks->mark(s, ProfileMarks::b)); \
   } while (0)
 
-pg_status enqueue_forward_one(const pg_gpt2_model* m, pg_kv_cache* c, size_t b,
+pg_status enqueue_forward_one(const pg_model* m, pg_kv_cache* c, size_t b,
                               const uint32_t* tok_ptr, uint32_t tok, size_t pos,
                               bool want_logits, ProfileMarks* marks = nullptr) {
   const Cfg& g = m->cfg;
@@ -483,7 +302,7 @@ constexpr unsigned kEpochWrap = 0xE0000000u;
 // could each hold part of the CUs while waiting for workgroups that cannot start.
 std::mutex g_persistent_mu;
 
-bool use_persistent(const pg_gpt2_model* m, const pg_kv_cache* c) {
+bool use_persistent(const pg_model* m, const pg_kv_cache* c) {
   return m->persistent && c->B == 1 && c->best_t != nullptr;
 }
 
@@ -519,7 +338,7 @@ struct PersistentRun {
 // force_ids[t] when force_ids is set (prefill), otherwise the first token comes from d_tok / tok
 // and later ones from the argmax of the previous step.  The epochs the launch will use are taken
 // off the cache's counter.
-pg_status persistent_params(const pg_gpt2_model* m, pg_kv_cache* c, const uint32_t* force_ids,
+pg_status persistent_params(const pg_model* m, pg_kv_cache* c, const uint32_t* force_ids,
                             bool lm_last_only, bool tok_from_ptr, uint32_t tok, size_t pos0,
                             size_t n_fwd, bool select_last, int64_t eos, uint32_t* out_ids_dev,
                             unsigned long long* stamps, pgk::DecodeParams* out) {
@@ -569,7 +388,7 @@ pg_status persistent_params(const pg_gpt2_model* m, pg_kv_cache* c, const uint32
   return PG_OK;
 }
 
-pg_status persistent_begin(const pg_gpt2_model* m, pg_kv_cache* c, const uint32_t* force_ids,
+pg_status persistent_begin(const pg_model* m, pg_kv_cache* c, const uint32_t* force_ids,
                            bool lm_last_only, bool tok_from_ptr, uint32_t tok, size_t pos0,
                            size_t n_fwd, bool select_last, int64_t eos, uint32_t* out_ids_dev,
                            bool timed, PersistentRun* run, unsigned long long* stamps = nullptr) {
@@ -648,7 +467,7 @@ pg_status persistent_end(pg_kv_cache* c, PersistentRun* run, size_t* done, bool*
 
 // The whole launch: begin, wait, end.  On return *done is the number of forwards executed and
 // *stopped says whether an EOS token ended the run early.
-pg_status run_persistent(const pg_gpt2_model* m, pg_kv_cache* c, const uint32_t* force_ids,
+pg_status run_persistent(const pg_model* m, pg_kv_cache* c, const uint32_t* force_ids,
                          bool lm_last_only, bool tok_from_ptr, uint32_t tok, size_t pos0,
                          size_t n_fwd, bool select_last, int64_t eos, uint32_t* out_ids_dev,
                          size_t* done, bool* stopped, bool timed,
@@ -665,7 +484,7 @@ constexpr size_t kGemmMinRows = 2;
 // Sequences of at least seq_gemm_min_tokens (a tunable, 4 by default) take the GEMM path in
 // prefill / forward; shorter ones run as that many single-token forwards (124M: 3 x 0.17 ms
 // against 0.6 ms for the launches of one GEMM pass; XL: 3 x 1.2 ms against 3.3 ms).
-bool gemm_path_ok(const pg_gpt2_model* m, size_t n) {
+bool gemm_path_ok(const pg_model* m, size_t n) {
   const Cfg& g = m->cfg;
   return n >= m->seq_gemm_min_tokens && n >= 2 && g.C % 16 == 0 && g.I % 16 == 0 &&
          (g.hd() == 64 || n * g.H * n * sizeof(float) <= (256u << 20));
@@ -677,7 +496,7 @@ bool gemm_path_ok(const pg_gpt2_model* m, size_t n) {
 // position land in the cache.  The last position's logits go to the cache's logits rows
 // b .. b + nb - 1; with all_logits set (nb = 1), the logits of every position are also copied
 // to dst ([n][V], host).
-pg_status run_sequence_gemm(const pg_gpt2_model* m, pg_kv_cache* c, size_t b, size_t nb,
+pg_status run_sequence_gemm(const pg_model* m, pg_kv_cache* c, size_t b, size_t nb,
                             const uint32_t* ids, size_t n_seq, float* all_logits_dst,
                             ProfileMarks* marks = nullptr) {
   const Cfg& g = m->cfg;
@@ -808,7 +627,7 @@ pg_status run_sequence_gemm(const pg_gpt2_model* m, pg_kv_cache* c, size_t b, si
 // every weight matrix is read once for the whole batch by the MFMA GEMM (M = B),
 // attention runs per (sequence, head, key split).  Token ids come from d_ids[B]
 // (device).  Needs n_embd and n_inner to be multiples of 16.
-pg_status enqueue_forward_batch(const pg_gpt2_model* m, pg_kv_cache* c, const uint32_t* d_ids,
+pg_status enqueue_forward_batch(const pg_model* m, pg_kv_cache* c, const uint32_t* d_ids,
                                 size_t pos) {
   const Cfg& g = m->cfg;
   const int B = (int)c->B, C = (int)g.C, I = (int)g.I, H = (int)g.H, hd = (int)g.hd(),
@@ -877,16 +696,66 @@ pg_status enqueue_forward_batch(const pg_gpt2_model* m, pg_kv_cache* c, const ui
   return PG_OK;
 }
 
-bool use_batched_step(const pg_gpt2_model* m, const pg_kv_cache* c) {
+bool use_batched_step(const pg_model* m, const pg_kv_cache* c) {
   return c->B > 1 && m->cfg.C % 16 == 0 && m->cfg.I % 16 == 0;
 }
 
-pg_status check_step(const pg_gpt2_model* m, const pg_kv_cache* c) {
+pg_status check_step(const pg_model* m, const pg_kv_cache* c) {
   // rust.rs:957-962
   if (c->seq_len >= c->cfg.P)
     return fail(PG_INVALID_INPUT, "cache is full at seq_len " + std::to_string(c->seq_len));
   (void)m;
   return PG_OK;
+}
+
+// The id buffers of a cache hold at least n ids from here on (GPT-2 caches: n_positions per
+// sequence from the start).
+pg_status ensure_ids(pg_kv_cache* c, size_t n) {
+  if (c->ids_cap >= n) return PG_OK;
+  n = round_up(n, 1024);
+  PG_HIP(hipStreamSynchronize(c->stream));
+  if (c->d_out_ids) (void)hipFree(c->d_out_ids);
+  if (c->h_ids) (void)hipHostFree(c->h_ids);
+  c->d_out_ids = nullptr;
+  c->h_ids = nullptr;
+  c->ids_cap = 0;
+  PG_HIP(hipMalloc(&c->d_out_ids, n * sizeof(uint32_t)));
+  PG_HIP(hipHostMalloc(&c->h_ids, n * sizeof(uint32_t), hipHostMallocDefault));
+  c->ids_cap = n;
+  return PG_OK;
+}
+
+// Stack models: n tokens of every sequence of the cache (ids[B][n], host) from the position they
+// stand at, logits of `rows` of the B * n rows to dst.
+pg_status stack_advance(const pg_model* m, pg_kv_cache* c, const uint32_t* ids, size_t n,
+                        const std::vector<int>& rows, float* dst, ProfileMarks* marks = nullptr) {
+  pg_status s;
+  if ((s = ensure_ids(c, c->B * std::min<size_t>(n, 8192)))) return s;
+  if ((s = pgh::stack_rows(m, c, ids, n, c->seq_len, rows, dst, marks))) return s;
+  PG_HIP(hipStreamSynchronize(c->stream));
+  c->seq_len += n;
+  return PG_OK;
+}
+// One token of every sequence (ids[B], host); logits to the cache's rows.
+pg_status stack_advance_one(const pg_model* m, pg_kv_cache* c, const uint32_t* ids, ProfileMarks* marks = nullptr) {
+  pg_status s;
+  if (c->seq_len == 0 && (s = pgh::stack_set_pos(c, 0))) return s;
+  if ((s = ensure_ids(c, c->B))) return s;
+  std::memcpy(c->h_ids, ids, c->B * sizeof(uint32_t));
+  PG_HIP(hipMemcpyAsync(c->d_tok, c->h_ids, c->B * sizeof(uint32_t), hipMemcpyHostToDevice, c->stream));
+  if ((s = pgh::stack_step(m, c, marks))) return s;
+  PG_HIP(hipStreamSynchronize(c->stream));
+  c->seq_len += 1;
+  return PG_OK;
+}
+// The whole prompts of all sequences, from position 0; logits of the last positions.
+pg_status stack_prefill(const pg_model* m, pg_kv_cache* c, const uint32_t* ids, size_t n,
+                        ProfileMarks* marks = nullptr) {
+  c->seq_len = 0;
+  if (n == 1) return stack_advance_one(m, c, ids, marks);
+  std::vector<int> rows;
+  for (size_t b = 0; b < c->B; ++b) rows.push_back((int)(b * n + n - 1));
+  return stack_advance(m, c, ids, n, rows, c->logits_buf, marks);
 }
 
 pg_status finish_logits(pg_kv_cache* c, pg_logits** out) {
@@ -895,6 +764,7 @@ pg_status finish_logits(pg_kv_cache* c, pg_logits** out) {
   c->logits.rows = c->B;
   c->logits.vocab = c->cfg.V;
   c->logits_valid = true;
+  c->next_valid = true;
   if (out) *out = &c->logits;
   return PG_OK;
 }
@@ -1047,7 +917,20 @@ pg_status sample_sorted(std::vector<Candidate>& cand, const pg_sampling& cfg, pg
 }  // namespace
 
 namespace pgh {
+pg_status select_device(int device) {
+  int n = 0;
+  hipError_t e = hipGetDeviceCount(&n);
+  if (e != hipSuccess || n == 0)
+    return fail(PG_BACKEND, "no HIP device available: the hip backend needs an AMD GPU");
+  if (device < 0 || device >= n)
+    return fail(PG_INVALID_CONFIG, "hip device " + std::to_string(device) +
+                                       " out of range for " + std::to_string(n) + " devices");
+  PG_HIP(hipSetDevice(device));
+  return PG_OK;
+}
+
 pg_status fail(pg_status s, const std::string& msg) { return ::fail(s, msg); }
+const char* architecture_of(const pg_model* m) { return m->stack ? m->stack->architecture.c_str() : "gpt2"; }
 pg_status validate_config(const pg_gpt2_config& c) { return ::validate_config(c); }
 }  // namespace pgh
 
@@ -1056,7 +939,7 @@ extern "C" {
 const char* pg_last_error_message(void) { return g_err.c_str(); }
 
 pg_status pg_gpt2_create(const pg_gpt2_config* config, const pg_gpt2_weights_view* weights,
-                         const pg_hip_options* options, pg_gpt2_model** out) {
+                         const pg_hip_options* options, pg_model** out) {
   if (!config || !weights || !out) return fail(PG_INVALID_INPUT, "null argument");
   *out = nullptr;
   pg_status s;
@@ -1084,7 +967,7 @@ pg_status pg_gpt2_create(const pg_gpt2_config* config, const pg_gpt2_weights_vie
   if (opts.reserved != 0) return fail(PG_INVALID_CONFIG, "hip backend options: reserved must be 0");
   if ((s = select_device(opts.device))) return s;
 
-  auto m = std::make_unique<pg_gpt2_model>();
+  auto m = std::make_unique<pg_model>();
   m->cfg = g;
   m->device = opts.device;
   m->opts = opts;
@@ -1125,7 +1008,7 @@ pg_status pg_gpt2_create(const pg_gpt2_config* config, const pg_gpt2_weights_vie
   PG_HIP(hipMalloc(&m->arena, total * sizeof(float)));
   m->arena_floats = total;
   struct Guard {
-    pg_gpt2_model* m;
+    pg_model* m;
     bool ok = false;
     ~Guard() {
       if (!ok && m->arena) (void)hipFree(m->arena);
@@ -1231,7 +1114,7 @@ pg_status pg_gpt2_create(const pg_gpt2_config* config, const pg_gpt2_weights_vie
   }
   PG_HIP(hipMalloc(&m->d_layers, g.L * sizeof(pgk::LayerW)));
   struct Guard2 {
-    pg_gpt2_model* m;
+    pg_model* m;
     bool ok = false;
     ~Guard2() {
       if (!ok && m->d_layers) (void)hipFree(m->d_layers);
@@ -1279,23 +1162,33 @@ pg_status pg_gpt2_create(const pg_gpt2_config* config, const pg_gpt2_weights_vie
   return PG_OK;
 }
 
-void pg_gpt2_destroy(pg_gpt2_model* m) {
+void pg_model_destroy(pg_model* m) {
   if (!m) return;
   if (hipSetDevice(m->device) == hipSuccess) {
     if (m->arena) (void)hipFree(m->arena);
     if (m->d_layers) (void)hipFree(m->d_layers);
+    m->stack.reset();
   }
   delete m;
 }
 
-pg_status pg_gpt2_get_config(const pg_gpt2_model* m, pg_gpt2_config* out) {
+pg_status pg_gpt2_get_config(const pg_model* m, pg_gpt2_config* out) {
   if (!m || !out) return fail(PG_INVALID_INPUT, "null argument");
+  if (m->stack) return fail(PG_INVALID_INPUT, "not a GPT-2 model");
   *out = pg_gpt2_config{m->cfg.V, m->cfg.P, m->cfg.C, m->cfg.L, m->cfg.H, m->cfg.I, m->cfg.eps};
   return PG_OK;
 }
 
-pg_status pg_gpt2_describe(const pg_gpt2_model* m, char* dst, size_t cap) {
+pg_status pg_model_describe(const pg_model* m, char* dst, size_t cap) {
   if (!m || !dst || cap == 0) return fail(PG_INVALID_INPUT, "null argument");
+  if (m->stack) {
+    std::snprintf(dst, cap, "hip (device=%d, compute_units=%d, weights=%s, architecture=%s, decode=%s, "
+                  "gemm_split_items_per_cu=%d, gemm_b9_min_rows=%d)",
+                  m->device, m->num_cus, m->w_bf16 ? "bf16" : "f32", pgh::architecture_of(m),
+                  m->opts.decode_path == PG_DECODE_KERNELS ? "kernels" : "graph", m->gemm_split_items,
+                  m->gemm_b9_min_rows);
+    return PG_OK;
+  }
   std::snprintf(dst, cap,
                 "hip (device=%d, compute_units=%d, weights=%s, decode=%s, attn_item_keys=%d, "
                 "attn_blocks_per_cu=%d, gemm_split_items_per_cu=%d, gemm_b9_min_rows=%d, "
@@ -1306,7 +1199,7 @@ pg_status pg_gpt2_describe(const pg_gpt2_model* m, char* dst, size_t cap) {
   return PG_OK;
 }
 
-pg_status pg_kv_cache_create(const pg_gpt2_model* m, uint32_t batch, pg_kv_cache** out) {
+pg_status pg_kv_cache_create(const pg_model* m, uint32_t batch, pg_kv_cache** out) {
   if (!m || !out) return fail(PG_INVALID_INPUT, "null argument");
   *out = nullptr;
   if (batch == 0) return fail(PG_INVALID_INPUT, "cache batch must be > 0");
@@ -1318,7 +1211,7 @@ pg_status pg_kv_cache_create(const pg_gpt2_model* m, uint32_t batch, pg_kv_cache
   c->device = m->device;
   c->num_cus = m->num_cus;
   c->B = batch;
-  const size_t B = batch, hd = g.hd();
+  const size_t B = batch, hd = m->stack ? 0 : g.hd();
   const size_t kv_floats = g.L * 2 * B * g.H * g.P * hd;
   const size_t parts = B * g.H * pgk::kMaxSplits;
   struct Guard {
@@ -1333,6 +1226,12 @@ pg_status pg_kv_cache_create(const pg_gpt2_model* m, uint32_t batch, pg_kv_cache
   PG_HIP(hipStreamCreateWithFlags(&raw->stream, hipStreamNonBlocking));
   PG_HIP(hipEventCreate(&raw->ev0));
   PG_HIP(hipEventCreate(&raw->ev1));
+  if (m->stack) {
+    if ((s = pgh::stack_cache_create(m, raw))) return s;
+    guard.ok = true;
+    *out = raw;
+    return PG_OK;
+  }
   PG_HIP(hipMalloc(&raw->kv, kv_floats * sizeof(float)));
   PG_HIP(hipMalloc(&raw->x, B * g.C * sizeof(float)));
   PG_HIP(hipMalloc(&raw->q, B * g.C * sizeof(float)));
@@ -1357,6 +1256,7 @@ pg_status pg_kv_cache_create(const pg_gpt2_model* m, uint32_t batch, pg_kv_cache
   PG_HIP(hipMalloc(&raw->d_tok, B * sizeof(uint32_t)));
   PG_HIP(hipMalloc(&raw->d_out_ids, g.P * B * sizeof(uint32_t)));
   PG_HIP(hipHostMalloc(&raw->h_ids, g.P * B * sizeof(uint32_t), hipHostMallocDefault));
+  raw->ids_cap = g.P * B;
   if (m->persistent && batch == 1) {
     // (every vector starts on a 64-byte line: the scalar probes read whole lines; n_embd is a
     // multiple of 64 here)
@@ -1390,6 +1290,8 @@ void pg_kv_cache_destroy(pg_kv_cache* c) {
   if (!c) return;
   if (hipSetDevice(c->device) == hipSuccess) {
     if (c->stream) (void)hipStreamSynchronize(c->stream);
+    c->stack.reset();
+    if (c->want_buf) (void)hipFree(c->want_buf);
     (void)hipFree(c->kv);
     (void)hipFree(c->x);
     (void)hipFree(c->q);
@@ -1429,8 +1331,10 @@ void pg_kv_cache_destroy(pg_kv_cache* c) {
 
 pg_status pg_kv_cache_clear(pg_kv_cache* c) {
   if (!c) return fail(PG_INVALID_INPUT, "null argument");
-  c->seq_len = 0;  // Gpt2KvCache::clear resets seq_len only (rust.rs:202-204)
-  c->logits_valid = false;
+  // Gpt2KvCache::clear resets seq_len only (rust.rs:202-204).  (The state of a stack model at
+  // position 0 is zero whatever its memory holds.)
+  c->seq_len = 0;
+  c->logits_valid = c->next_valid = false;
   return PG_OK;
 }
 uint64_t pg_kv_cache_seq_len(const pg_kv_cache* c) { return c ? c->seq_len : 0; }
@@ -1441,8 +1345,10 @@ pg_status pg_kv_cache_set_seq_len(pg_kv_cache* c, uint64_t n) {
   if (n > c->cfg.P)
     return fail(PG_INVALID_INPUT, "seq_len " + std::to_string(n) + " exceeds max_seq_len " +
                                       std::to_string(c->cfg.P));
+  if (c->stack && n != 0 && n != c->seq_len)
+    return fail(PG_INVALID_INPUT, "a recurrent state cannot be set back to position " + std::to_string(n));
   c->seq_len = n;
-  c->logits_valid = false;
+  c->logits_valid = c->next_valid = false;
   return PG_OK;
 }
 
@@ -1461,6 +1367,7 @@ pg_status pg_kv_cache_debug_set_epoch(pg_kv_cache* c, uint32_t epoch) {
 pg_status pg_kv_cache_read_layer(const pg_kv_cache* c, uint32_t b, uint32_t layer, uint32_t which,
                                  float* dst, size_t len) {
   if (!c || !dst) return fail(PG_INVALID_INPUT, "null argument");
+  if (c->stack) return fail(PG_INVALID_INPUT, "this architecture's cache has no K and V panels");
   const size_t panel = c->cfg.H * c->cfg.P * c->cfg.hd();
   if (b >= c->B || layer >= c->cfg.L || which > 1 || len != panel)
     return fail(PG_INVALID_INPUT, "cache panel index or length out of range");
@@ -1472,7 +1379,7 @@ pg_status pg_kv_cache_read_layer(const pg_kv_cache* c, uint32_t b, uint32_t laye
   return PG_OK;
 }
 
-pg_status pg_gpt2_prefill_batch(const pg_gpt2_model* m, pg_kv_cache* c, const uint32_t* ids,
+pg_status pg_model_prefill_batch(const pg_model* m, pg_kv_cache* c, const uint32_t* ids,
                                 size_t n, pg_logits** out) {
   if (!m || !c) return fail(PG_INVALID_INPUT, "null argument");
   pg_status s;
@@ -1481,7 +1388,11 @@ pg_status pg_gpt2_prefill_batch(const pg_gpt2_model* m, pg_kv_cache* c, const ui
   if ((s = check_compatible(m, c))) return s;
   if ((s = select_device(m->device))) return s;
   c->seq_len = 0;  // cache.clear() (rust.rs:918)
-  c->logits_valid = false;
+  c->logits_valid = c->next_valid = false;
+  if (m->stack) {
+    if ((s = stack_prefill(m, c, ids, n))) return s;
+    return finish_logits(c, out);
+  }
   if (gemm_path_ok(m, n) && m->opts.prefill_path == 0) {
     // all sequences in one pass over the weights, in groups of at most about 8192 rows
     const size_t group = std::max<size_t>(1, std::min<size_t>(c->B, 8192 / n));
@@ -1508,14 +1419,14 @@ pg_status pg_gpt2_prefill_batch(const pg_gpt2_model* m, pg_kv_cache* c, const ui
   return finish_logits(c, out);
 }
 
-pg_status pg_gpt2_prefill(const pg_gpt2_model* m, pg_kv_cache* c, const uint32_t* ids, size_t n,
+pg_status pg_model_prefill(const pg_model* m, pg_kv_cache* c, const uint32_t* ids, size_t n,
                           pg_logits** out) {
   if (!m || !c) return fail(PG_INVALID_INPUT, "null argument");
   if (c->B != 1) return fail(PG_INVALID_INPUT, "prefill needs a cache of batch 1");
-  return pg_gpt2_prefill_batch(m, c, ids, n, out);
+  return pg_model_prefill_batch(m, c, ids, n, out);
 }
 
-pg_status pg_gpt2_prefill_profiled(const pg_gpt2_model* m, pg_kv_cache* c, const uint32_t* ids,
+pg_status pg_model_prefill_profiled(const pg_model* m, pg_kv_cache* c, const uint32_t* ids,
                                    size_t n, pg_logits** out, pg_gpt2_operation_profile* profile) {
   if (!m || !c || !profile) return fail(PG_INVALID_INPUT, "null argument");
   if (c->B != 1) return fail(PG_INVALID_INPUT, "prefill needs a cache of batch 1");
@@ -1525,8 +1436,13 @@ pg_status pg_gpt2_prefill_profiled(const pg_gpt2_model* m, pg_kv_cache* c, const
   if ((s = check_compatible(m, c))) return s;
   if ((s = select_device(m->device))) return s;
   c->seq_len = 0;  // cache.clear() (rust.rs:918)
-  c->logits_valid = false;
+  c->logits_valid = c->next_valid = false;
   ProfileMarks marks;
+  if (m->stack) {
+    if ((s = stack_prefill(m, c, ids, n, &marks))) return s;
+    PG_HIP(marks.collect(profile));
+    return finish_logits(c, out);
+  }
   if (gemm_path_ok(m, n) && m->opts.prefill_path == 0) {
     if ((s = run_sequence_gemm(m, c, 0, 1, ids, n, nullptr, &marks))) return s;
     PG_HIP(marks.collect(profile));
@@ -1541,7 +1457,7 @@ pg_status pg_gpt2_prefill_profiled(const pg_gpt2_model* m, pg_kv_cache* c, const
   return finish_logits(c, out);
 }
 
-pg_status pg_gpt2_forward_one_batch(const pg_gpt2_model* m, pg_kv_cache* c, const uint32_t* ids,
+pg_status pg_model_forward_one_batch(const pg_model* m, pg_kv_cache* c, const uint32_t* ids,
                                     pg_logits** out) {
   if (!m || !c || !ids) return fail(PG_INVALID_INPUT, "null argument");
   pg_status s;
@@ -1552,6 +1468,11 @@ pg_status pg_gpt2_forward_one_batch(const pg_gpt2_model* m, pg_kv_cache* c, cons
                                         " exceeds vocab_size " + std::to_string(m->cfg.V));
   if ((s = check_step(m, c))) return s;
   if ((s = select_device(m->device))) return s;
+  if (m->stack) {
+    c->logits_valid = c->next_valid = false;
+    if ((s = stack_advance_one(m, c, ids))) return s;
+    return finish_logits(c, out);
+  }
   if (use_persistent(m, c)) {
     if ((s = run_persistent(m, c, nullptr, false, false, ids[0], c->seq_len, 1, false, -1,
                             nullptr, nullptr, nullptr, false)))
@@ -1573,14 +1494,14 @@ pg_status pg_gpt2_forward_one_batch(const pg_gpt2_model* m, pg_kv_cache* c, cons
   return finish_logits(c, out);
 }
 
-pg_status pg_gpt2_forward_one(const pg_gpt2_model* m, pg_kv_cache* c, uint32_t id,
+pg_status pg_model_forward_one(const pg_model* m, pg_kv_cache* c, uint32_t id,
                               pg_logits** out) {
   if (!m || !c) return fail(PG_INVALID_INPUT, "null argument");
   if (c->B != 1) return fail(PG_INVALID_INPUT, "forward_one needs a cache of batch 1");
-  return pg_gpt2_forward_one_batch(m, c, &id, out);
+  return pg_model_forward_one_batch(m, c, &id, out);
 }
 
-pg_status pg_gpt2_forward(const pg_gpt2_model* m, const uint32_t* ids, size_t n, float* dst,
+pg_status pg_model_forward(const pg_model* m, const uint32_t* ids, size_t n, float* dst,
                           size_t dst_len) {
   if (!m || !dst) return fail(PG_INVALID_INPUT, "null argument");
   pg_status s;
@@ -1592,6 +1513,21 @@ pg_status pg_gpt2_forward(const pg_gpt2_model* m, const uint32_t* ids, size_t n,
   pg_kv_cache* c = nullptr;
   if ((s = pg_kv_cache_create(m, 1, &c))) return s;
   std::unique_ptr<pg_kv_cache, void (*)(pg_kv_cache*)> holder(c, pg_kv_cache_destroy);
+  if (m->stack) {
+    // (in portions, so that the logits of a long sequence need not be on the device at once)
+    constexpr size_t kPart = 1024;
+    const size_t V = m->cfg.V;
+    DevBuf part;
+    if ((s = part.alloc(std::min(n, kPart) * V))) return s;
+    for (size_t t = 0; t < n; t += kPart) {
+      const size_t nt = std::min(kPart, n - t);
+      std::vector<int> rows(nt);
+      for (size_t i = 0; i < nt; ++i) rows[i] = (int)i;
+      if ((s = stack_advance(m, c, ids + t, nt, rows, part.p))) return s;
+      PG_HIP(hipMemcpy(dst + t * V, part.p, nt * V * sizeof(float), hipMemcpyDeviceToHost));
+    }
+    return PG_OK;
+  }
   if (gemm_path_ok(m, n) && m->opts.prefill_path == 0) return run_sequence_gemm(m, c, 0, 1, ids, n, dst);
   for (size_t i = 0; i < n; ++i) {
     if (use_persistent(m, c)) {
@@ -1608,6 +1544,73 @@ pg_status pg_gpt2_forward(const pg_gpt2_model* m, const uint32_t* ids, size_t n,
   return PG_OK;
 }
 
+// The next n tokens of the sequence.  Stack models run them as one portion from the state earlier
+// calls left; GPT-2's full-sequence kernels start at position 0, so that a portion runs through
+// them when it is a whole prompt and token by token otherwise.
+pg_status pg_model_extend(const pg_model* m, pg_kv_cache* c, const uint32_t* ids, size_t n,
+                          const size_t* want, size_t n_want, pg_logits** out) {
+  if (!m || !c || (n_want && (!want || !out))) return fail(PG_INVALID_INPUT, "null argument");
+  if (out) *out = nullptr;
+  if (c->B != 1) return fail(PG_INVALID_INPUT, "extend needs a cache of batch 1");
+  pg_status s;
+  if ((s = validate_input(m->cfg, ids, n))) return s;
+  for (size_t i = 0; i < n_want; ++i)
+    if (want[i] >= n || (i && want[i] <= want[i - 1]))
+      return fail(PG_INVALID_INPUT, "wanted places must increase and lie inside the portion");
+  if ((s = check_compatible(m, c))) return s;
+  if (n > c->cfg.P - std::min(c->seq_len, c->cfg.P))
+    return fail(PG_INVALID_INPUT, "cache is full at seq_len " + std::to_string(c->seq_len));
+  if ((s = select_device(m->device))) return s;
+  const size_t V = m->cfg.V;
+  c->logits_valid = c->next_valid = false;
+  const bool last = n_want && want[n_want - 1] == n - 1;
+  if (c->want_cap < n_want) {
+    PG_HIP(hipStreamSynchronize(c->stream));
+    if (c->want_buf) (void)hipFree(c->want_buf);
+    c->want_buf = nullptr;
+    c->want_cap = 0;
+    PG_HIP(hipMalloc(&c->want_buf, n_want * V * sizeof(float)));
+    c->want_cap = n_want;
+  }
+  if (m->stack && n > 1) {
+    std::vector<int> rows(want, want + n_want);
+    if ((s = stack_advance(m, c, ids, n, rows, c->want_buf))) return s;
+  } else if (!m->stack && c->seq_len == 0 && n_want == (size_t)last && n > 1) {
+    if ((s = pg_model_prefill(m, c, ids, n, nullptr))) return s;
+    if (last)
+      PG_HIP(hipMemcpyAsync(c->want_buf, c->logits_buf, V * sizeof(float), hipMemcpyDeviceToDevice, c->stream));
+  } else {
+    for (size_t i = 0, k = 0; i < n; ++i) {
+      if ((s = pg_model_forward_one(m, c, ids[i], nullptr))) return s;
+      if (k < n_want && want[k] == i) {
+        PG_HIP(hipMemcpyAsync(c->want_buf + k * V, c->logits_buf, V * sizeof(float), hipMemcpyDeviceToDevice, c->stream));
+        ++k;
+      }
+    }
+  }
+  // a wanted last position selects the next token
+  if (last)
+    PG_HIP(hipMemcpyAsync(c->logits_buf, c->want_buf + (n_want - 1) * V, V * sizeof(float), hipMemcpyDeviceToDevice, c->stream));
+  PG_HIP(hipStreamSynchronize(c->stream));
+  c->next_valid = last;
+  c->logits_valid = n_want > 0;
+  if (n_want) {
+    c->logits.owner = c;
+    c->logits.data = c->want_buf;
+    c->logits.rows = (uint32_t)n_want;
+    c->logits.vocab = V;
+    *out = &c->logits;
+  }
+  return PG_OK;
+}
+
+const char* pg_model_architecture(const pg_model* m) { return m ? pgh::architecture_of(m) : ""; }
+pg_status pg_model_get_info(const pg_model* m, pg_model_info* out) {
+  if (!m || !out) return fail(PG_INVALID_INPUT, "null argument");
+  *out = pg_model_info{m->cfg.V, m->cfg.P, m->cfg.C, m->cfg.L};
+  return PG_OK;
+}
+
 uint32_t pg_logits_rows(const pg_logits* l) { return l ? l->rows : 0; }
 uint64_t pg_logits_vocab(const pg_logits* l) { return l ? l->vocab : 0; }
 
@@ -1617,8 +1620,9 @@ pg_status pg_logits_argmax(pg_logits* l, uint32_t* out) {
   if (!c->logits_valid) return fail(PG_INVALID_INPUT, "logits handle is stale");
   pg_status s;
   if ((s = select_device(c->device))) return s;
-  PG_HIP(pgk::launch_argmax(l->data, (int)l->vocab, c->d_tok, c->stream, (int)l->rows));
-  PG_HIP(hipMemcpyAsync(c->h_ids, c->d_tok, l->rows * sizeof(uint32_t), hipMemcpyDeviceToHost,
+  if ((s = ensure_ids(c, l->rows))) return s;
+  PG_HIP(pgk::launch_argmax(l->data, (int)l->vocab, c->d_out_ids, c->stream, (int)l->rows));
+  PG_HIP(hipMemcpyAsync(c->h_ids, c->d_out_ids, l->rows * sizeof(uint32_t), hipMemcpyDeviceToHost,
                         c->stream));
   PG_HIP(hipStreamSynchronize(c->stream));
   std::memcpy(out, c->h_ids, l->rows * sizeof(uint32_t));
@@ -1692,9 +1696,10 @@ pg_status pg_logits_sample(pg_logits* l, uint32_t row, const uint32_t* history, 
   const bool penalised = !(sampling->repeat_penalty == 1.0f || sampling->repeat_last_n == 0);
   if (sampling->temperature <= 0.0f && !penalised) {
     // Pure greedy: argmax on the device, only the id crosses to the host.
-    PG_HIP(pgk::launch_argmax(l->data + (size_t)row * l->vocab, (int)l->vocab, c->d_tok + row,
+    if ((s = ensure_ids(c, 1))) return s;
+    PG_HIP(pgk::launch_argmax(l->data + (size_t)row * l->vocab, (int)l->vocab, c->d_out_ids,
                               c->stream));
-    PG_HIP(hipMemcpyAsync(c->h_ids, c->d_tok + row, sizeof(uint32_t), hipMemcpyDeviceToHost,
+    PG_HIP(hipMemcpyAsync(c->h_ids, c->d_out_ids, sizeof(uint32_t), hipMemcpyDeviceToHost,
                           c->stream));
     PG_HIP(hipStreamSynchronize(c->stream));
     *out = c->h_ids[0];
@@ -1791,11 +1796,11 @@ void pg_debug_sample_counts(uint64_t* device_draws, uint64_t* host_rows) {
 // prompt + generated reaches n_positions (rust.rs:496-498), so at most
 // P - seq_len tokens are selected.  With eos >= 0 the run may end early at the
 // first EOS; ids then still holds the EOS as its last entry and the caller drops it.
-static pg_status decode_core(const pg_gpt2_model* m, pg_kv_cache* c, size_t steps, int64_t eos,
+static pg_status decode_core(const pg_model* m, pg_kv_cache* c, size_t steps, int64_t eos,
                              uint32_t* ids, size_t* n_ids, pg_generation_stats* stats) {
   pg_status s;
   if ((s = check_compatible(m, c))) return s;
-  if (!c->logits_valid)
+  if (!c->next_valid)
     return fail(PG_INVALID_INPUT, "decode needs logits from prefill or forward_one");
   if ((s = select_device(m->device))) return s;
   const size_t B = c->B, V = m->cfg.V;
@@ -1827,13 +1832,25 @@ static pg_status decode_core(const pg_gpt2_model* m, pg_kv_cache* c, size_t step
                           c->stream));
     PG_HIP(hipStreamSynchronize(c->stream));
   } else {
+    if ((s = ensure_ids(c, n_steps * B))) return s;
     PG_HIP(hipEventRecord(c->ev0, c->stream));
     for (size_t i = 0; i < n_steps; ++i) {
       PG_HIP(pgk::launch_argmax(c->logits_buf, (int)V, c->d_tok, c->stream, (int)B));
       PG_HIP(hipMemcpyAsync(c->d_out_ids + i * B, c->d_tok, B * sizeof(uint32_t),
                             hipMemcpyDeviceToDevice, c->stream));
+      if (m->stack && eos >= 0) {
+        // a recurrent state cannot be set back: no forward may follow an EOS
+        PG_HIP(hipMemcpyAsync(c->h_ids, c->d_tok, sizeof(uint32_t), hipMemcpyDeviceToHost, c->stream));
+        PG_HIP(hipStreamSynchronize(c->stream));
+        if (c->h_ids[0] == (uint32_t)eos) {
+          n_out = i + 1;
+          break;
+        }
+      }
       if (i + 1 < n_steps) {
-        if (use_batched_step(m, c)) {
+        if (m->stack) {
+          if ((s = pgh::stack_step(m, c))) return s;
+        } else if (use_batched_step(m, c)) {
           if ((s = enqueue_forward_batch(m, c, c->d_tok, c->seq_len))) return s;
         } else {
           for (size_t b = 0; b < B; ++b)
@@ -1843,14 +1860,14 @@ static pg_status decode_core(const pg_gpt2_model* m, pg_kv_cache* c, size_t step
       }
     }
     PG_HIP(hipEventRecord(c->ev1, c->stream));
-    PG_HIP(hipMemcpyAsync(c->h_ids, c->d_out_ids, n_steps * B * sizeof(uint32_t),
+    PG_HIP(hipMemcpyAsync(c->h_ids, c->d_out_ids, n_out * B * sizeof(uint32_t),
                           hipMemcpyDeviceToHost, c->stream));
     PG_HIP(hipStreamSynchronize(c->stream));
     PG_HIP(hipEventElapsedTime(&ms, c->ev0, c->ev1));
   }
   std::memcpy(ids, c->h_ids, n_out * B * sizeof(uint32_t));
   *n_ids = n_out;
-  c->logits_valid = false;  // the logits the last selection used are consumed
+  c->logits_valid = c->next_valid = false;  // the logits the last selection used are consumed
   if (stats) {
     *stats = pg_generation_stats{};
     stats->generated_tokens = n_out;
@@ -1860,14 +1877,14 @@ static pg_status decode_core(const pg_gpt2_model* m, pg_kv_cache* c, size_t step
   return PG_OK;
 }
 
-pg_status pg_gpt2_decode_greedy_batch(const pg_gpt2_model* m, pg_kv_cache* c, uint32_t steps,
+pg_status pg_model_decode_greedy_batch(const pg_model* m, pg_kv_cache* c, uint32_t steps,
                                       uint32_t* out_ids, pg_generation_stats* stats) {
   if (!m || !c || !out_ids) return fail(PG_INVALID_INPUT, "null argument");
   size_t n = 0;
   return decode_core(m, c, steps, -1, out_ids, &n, stats);
 }
 
-pg_status pg_gpt2_decode_greedy(const pg_gpt2_model* m, pg_kv_cache* c, uint32_t max_new,
+pg_status pg_model_decode_greedy(const pg_model* m, pg_kv_cache* c, uint32_t max_new,
                                 int64_t eos, uint32_t* out_ids, uint32_t* out_n,
                                 pg_generation_stats* stats) {
   if (!m || !c || !out_ids || !out_n) return fail(PG_INVALID_INPUT, "null argument");
@@ -1889,7 +1906,7 @@ pg_status pg_gpt2_decode_greedy(const pg_gpt2_model* m, pg_kv_cache* c, uint32_t
     for (size_t i = 0; i < n; ++i)
       if (ids[i] == (uint32_t)eos) {
         n = i;
-        c->seq_len = start_len + i;
+        c->seq_len = start_len + i;  // (stack models: no forward ran past it)
         break;
       }
   }
@@ -1904,7 +1921,7 @@ pg_status pg_gpt2_decode_greedy(const pg_gpt2_model* m, pg_kv_cache* c, uint32_t
 
 // One forward of the per-operation path with its spans added to `profile`
 // (forward_one_profiled_with_scratch, src/models/gpt2/rust.rs:943-1006).
-static pg_status forward_one_profiled(const pg_gpt2_model* m, pg_kv_cache* c, uint32_t id,
+static pg_status forward_one_profiled(const pg_model* m, pg_kv_cache* c, uint32_t id,
                                       bool want_logits, ProfileMarks* marks,
                                       pg_gpt2_operation_profile* profile, pg_logits** out) {
   pg_status s;
@@ -1914,6 +1931,11 @@ static pg_status forward_one_profiled(const pg_gpt2_model* m, pg_kv_cache* c, ui
                                       std::to_string(m->cfg.V));
   if ((s = check_step(m, c))) return s;
   if ((s = select_device(m->device))) return s;
+  if (m->stack) {
+    if ((s = stack_advance_one(m, c, &id, marks))) return s;
+    PG_HIP(marks->collect(profile));
+    return finish_logits(c, out);
+  }
   if ((s = enqueue_forward_one(m, c, 0, nullptr, id, c->seq_len, want_logits, marks))) return s;
   PG_HIP(hipStreamSynchronize(c->stream));
   PG_HIP(marks->collect(profile));
@@ -1934,7 +1956,7 @@ static pg_status forward_one_profiled(const pg_gpt2_model* m, pg_kv_cache* c, ui
 //   last layer -> end of the launch (LN_f, lm_head, argmax)                final_logits
 // so the buckets of a forward add up to the launch's duration.  LayerNorm has no span of its
 // own here (it is folded into the rows that follow it): layer_norm_s stays 0.
-static pg_status forward_one_stamped(const pg_gpt2_model* m, pg_kv_cache* c, uint32_t id,
+static pg_status forward_one_stamped(const pg_model* m, pg_kv_cache* c, uint32_t id,
                                      pg_gpt2_operation_profile* profile, pg_logits** out) {
   pg_status s;
   if ((s = check_compatible(m, c))) return s;
@@ -1971,7 +1993,7 @@ static pg_status forward_one_stamped(const pg_gpt2_model* m, pg_kv_cache* c, uin
   return finish_logits(c, out);
 }
 
-static pg_status stream_core(const pg_gpt2_model* m, const uint32_t* ids, size_t n,
+static pg_status stream_core(const pg_model* m, const uint32_t* ids, size_t n,
                              uint32_t max_new, int64_t eos, const pg_sampling* sampling,
                              uint64_t seed, pg_on_token on_token, void* user, uint32_t* out_ids,
                              size_t* out_n, pg_generation_stats* stats,
@@ -1996,16 +2018,16 @@ static pg_status stream_core(const pg_gpt2_model* m, const uint32_t* ids, size_t
   // per-operation launches with events between them, the prompt token by token as
   // prefill_profiled does, rust.rs:906-927.)
   const bool stamped = profile && use_persistent(m, c) && m->cfg.L + 1 <= 64;
-  if (profile && stamped) {
+  if (profile && (stamped || m->stack)) {
     pg_gpt2_operation_profile pre{};
-    if ((s = pg_gpt2_prefill_profiled(m, c, ids, n, &logits, &pre))) return s;
+    if ((s = pg_model_prefill_profiled(m, c, ids, n, &logits, &pre))) return s;
     *profile = pre;
   } else if (profile) {
     if ((s = validate_input(m->cfg, ids, n))) return s;
     if ((s = pg_kv_cache_clear(c))) return s;
     for (size_t i = 0; i < n; ++i)
       if ((s = forward_one_profiled(m, c, ids[i], i + 1 == n, &marks, profile, &logits))) return s;
-  } else if ((s = pg_gpt2_prefill(m, c, ids, n, &logits))) {
+  } else if ((s = pg_model_prefill(m, c, ids, n, &logits))) {
     return s;
   }
   double prefill_s = since(prefill_start);
@@ -2089,7 +2111,7 @@ static pg_status stream_core(const pg_gpt2_model* m, const uint32_t* ids, size_t
       c->seq_len += stopped ? done : nf;
       base += nf;
     }
-    c->logits_valid = false;
+    c->logits_valid = c->next_valid = false;
   } else if (!profile && use_persistent(m, c) && m->cfg.V <= (uint64_t)pgk::kTopkMaxVocab &&
              m->cfg.P <= kMaxRecent && !g_no_sample_train &&
              (sampling->temperature <= 0.0f || !sampling->has_top_k || sampling->top_k <= kMaxCand)) {
@@ -2254,10 +2276,10 @@ static pg_status stream_core(const pg_gpt2_model* m, const uint32_t* ids, size_t
         if ((s = pg_logits_sample(logits, 0, output.data(), output.size(), sampling, &rng, &tok)))
           return s;
         if ((s = deliver(tok))) return s;
-        if (!ended && (s = pg_gpt2_forward_one(m, c, tok, &logits))) return s;
+        if (!ended && (s = pg_model_forward_one(m, c, tok, &logits))) return s;
       }
     }
-    c->logits_valid = false;
+    c->logits_valid = c->next_valid = false;
   } else {
   for (uint32_t it = 0; it < max_new; ++it) {
     if (output.size() >= m->cfg.P) break;
@@ -2277,7 +2299,7 @@ static pg_status stream_core(const pg_gpt2_model* m, const uint32_t* ids, size_t
       else if (profile)
         s = forward_one_profiled(m, c, tok, true, &marks, profile, &logits);
       else
-        s = pg_gpt2_forward_one(m, c, tok, &logits);
+        s = pg_model_forward_one(m, c, tok, &logits);
       if (s) return s;
     }
   }
@@ -2296,7 +2318,7 @@ static pg_status stream_core(const pg_gpt2_model* m, const uint32_t* ids, size_t
   return PG_OK;
 }
 
-pg_status pg_gpt2_stream_token_ids_with_stats(const pg_gpt2_model* m, const uint32_t* ids,
+pg_status pg_model_stream_token_ids_with_stats(const pg_model* m, const uint32_t* ids,
                                               size_t n, uint32_t max_new, int64_t eos,
                                               const pg_sampling* sampling, uint64_t seed,
                                               pg_on_token on_token, void* user, uint32_t* out_ids,
@@ -2305,7 +2327,7 @@ pg_status pg_gpt2_stream_token_ids_with_stats(const pg_gpt2_model* m, const uint
                      stats, nullptr);
 }
 
-pg_status pg_gpt2_stream_token_ids_profiled(const pg_gpt2_model* m, const uint32_t* ids,
+pg_status pg_model_stream_token_ids_profiled(const pg_model* m, const uint32_t* ids,
                                             size_t n, uint32_t max_new, int64_t eos,
                                             const pg_sampling* sampling, uint64_t seed,
                                             pg_on_token on_token, void* user, uint32_t* out_ids,
@@ -2314,6 +2336,53 @@ pg_status pg_gpt2_stream_token_ids_profiled(const pg_gpt2_model* m, const uint32
   if (!profile) return fail(PG_INVALID_INPUT, "null argument");
   return stream_core(m, ids, n, max_new, eos, sampling, seed, on_token, user, out_ids, out_n,
                      stats, profile);
+}
+
+// ---- the GPT-2 names of the entry points that take any model ---------------------------------
+void pg_gpt2_destroy(pg_gpt2_model* m) { pg_model_destroy(m); }
+pg_status pg_gpt2_describe(const pg_gpt2_model* m, char* dst, size_t cap) { return pg_model_describe(m, dst, cap); }
+pg_status pg_gpt2_prefill(const pg_gpt2_model* m, pg_kv_cache* c, const uint32_t* ids, size_t n, pg_logits** out) {
+  return pg_model_prefill(m, c, ids, n, out);
+}
+pg_status pg_gpt2_prefill_batch(const pg_gpt2_model* m, pg_kv_cache* c, const uint32_t* ids, size_t n,
+                                pg_logits** out) {
+  return pg_model_prefill_batch(m, c, ids, n, out);
+}
+pg_status pg_gpt2_prefill_profiled(const pg_gpt2_model* m, pg_kv_cache* c, const uint32_t* ids, size_t n,
+                                   pg_logits** out, pg_gpt2_operation_profile* profile) {
+  return pg_model_prefill_profiled(m, c, ids, n, out, profile);
+}
+pg_status pg_gpt2_forward_one(const pg_gpt2_model* m, pg_kv_cache* c, uint32_t id, pg_logits** out) {
+  return pg_model_forward_one(m, c, id, out);
+}
+pg_status pg_gpt2_forward_one_batch(const pg_gpt2_model* m, pg_kv_cache* c, const uint32_t* ids, pg_logits** out) {
+  return pg_model_forward_one_batch(m, c, ids, out);
+}
+pg_status pg_gpt2_forward(const pg_gpt2_model* m, const uint32_t* ids, size_t n, float* dst, size_t dst_len) {
+  return pg_model_forward(m, ids, n, dst, dst_len);
+}
+pg_status pg_gpt2_decode_greedy(const pg_gpt2_model* m, pg_kv_cache* c, uint32_t max_new, int64_t eos,
+                                uint32_t* out_ids, uint32_t* out_n, pg_generation_stats* stats) {
+  return pg_model_decode_greedy(m, c, max_new, eos, out_ids, out_n, stats);
+}
+pg_status pg_gpt2_decode_greedy_batch(const pg_gpt2_model* m, pg_kv_cache* c, uint32_t steps, uint32_t* out_ids,
+                                      pg_generation_stats* stats) {
+  return pg_model_decode_greedy_batch(m, c, steps, out_ids, stats);
+}
+pg_status pg_gpt2_stream_token_ids_with_stats(const pg_gpt2_model* m, const uint32_t* ids, size_t n,
+                                              uint32_t max_new, int64_t eos, const pg_sampling* sampling,
+                                              uint64_t seed, pg_on_token on_token, void* user, uint32_t* out_ids,
+                                              size_t* out_n, pg_generation_stats* stats) {
+  return pg_model_stream_token_ids_with_stats(m, ids, n, max_new, eos, sampling, seed, on_token, user, out_ids,
+                                              out_n, stats);
+}
+pg_status pg_gpt2_stream_token_ids_profiled(const pg_gpt2_model* m, const uint32_t* ids, size_t n,
+                                            uint32_t max_new, int64_t eos, const pg_sampling* sampling,
+                                            uint64_t seed, pg_on_token on_token, void* user, uint32_t* out_ids,
+                                            size_t* out_n, pg_generation_stats* stats,
+                                            pg_gpt2_operation_profile* profile) {
+  return pg_model_stream_token_ids_profiled(m, ids, n, max_new, eos, sampling, seed, on_token, user, out_ids,
+                                            out_n, stats, profile);
 }
 
 // ---- op-level entry points ---------------------------------------------------

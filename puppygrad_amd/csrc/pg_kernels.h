@@ -24,7 +24,9 @@ struct LayerW {
   const float *c_attn_f, *c_fc_f;
 };
 
-enum Prologue : int { PRO_NONE = 0, PRO_LN = 1, PRO_ATTN_COMBINE = 2 };
+// PRO_RMS: x / sqrt(mean(x^2) + eps) * ln_g[0], the mean over the first norm_n values (the
+// others are zeros)
+enum Prologue : int { PRO_NONE = 0, PRO_LN = 1, PRO_ATTN_COMBINE = 2, PRO_RMS = 3 };
 enum Epilogue : int { EPI_BIAS = 0, EPI_GELU = 1, EPI_RESID = 2, EPI_QKV = 3 };
 
 // y = epilogue(bias + W . prologue(x)) for one input vector.
@@ -43,6 +45,8 @@ struct GemvArgs {
   const float* ln_g;
   const float* ln_b;
   float eps;
+  int norm_n;  // PRO_RMS
+  float out_mul = 0.0f;  // EPI_BIAS: != 0 multiplies the result
   // PRO_ATTN_COMBINE: partial attention results per (head, split)
   const float* part_acc;  // [H][nsplit][hd]
   const float* part_m;    // [H][nsplit]
@@ -60,6 +64,21 @@ struct GemvArgs {
 };
 
 hipError_t launch_gemv(const GemvArgs& a, int prologue, int epilogue, hipStream_t s);
+
+// y[o] = resid[o] + s1[o] (W1[o] . x1) + s2[o] (W2[o] . x2) in one launch: the projections of the
+// two sublayers of a parallel layer back to the residual, with their layer scales.  K1 and K2
+// are multiples of 32 with K1 + K2 <= kPairMaxK; W2 may be null.
+struct GemvPair {
+  int w_bf16;
+  const float *W1, *W2;
+  const float *x1, *x2;
+  const float *s1, *s2;
+  const float* resid;
+  float* y;
+  int K1, K2, nout;
+};
+constexpr int kPairMaxK = 16320;
+hipError_t launch_gemv_pair(const GemvPair& a, hipStream_t s);
 
 // x = wte[tok] + wpe[pos]; tok comes from tok_ptr[0] when tok_ptr != nullptr.
 hipError_t launch_embed(float* x, const float* wte, const float* wpe, const uint32_t* tok_ptr,
@@ -145,7 +164,7 @@ struct SampleStep {
   size_t arm_words;
 };
 hipError_t launch_sample_step(const SampleStep& a, hipStream_t s);
-// x[b] = wte[ids[b]] + wpe[pos]
+// x[b] = wte[ids[b]] + wpe[pos] (wpe may be null)
 hipError_t launch_embed_batch(float* x, const float* wte, const float* wpe, const uint32_t* ids,
                               int batch, int pos, int C, hipStream_t s, int w_bf16 = 0);
 // Appends row b of qkv[B][3C] to position pos of sequence b's K and V panels.
@@ -188,6 +207,9 @@ struct GemmArgs {
   const float* W;
   const float* bias;
   const float* resid;
+  // Optional (GEMM_RESID): the product's column n is multiplied by col_scale[n] before it is
+  // added to the residual (layer scale).
+  const float* col_scale = nullptr;
   float* C;
   int M, N, K;
   int lda, ldc;
@@ -203,6 +225,9 @@ struct GemmArgs {
   const float* ln_g = nullptr;
   const float* ln_b = nullptr;
   float ln_eps = 0.0f;
+  // != 0: ln_out receives row / sqrt(mean(row^2) + ln_eps) * ln_g[0] instead, the mean over the
+  // first rms_cols columns (the others must hold zeros).
+  int rms_cols = 0;
   // Packed form of an activation matrix of at most 32 rows (see packed32_index): which of
   // A, C and ln_out are held that way.  Only the 32-row decode kernel reads a packed A, so
   // launch_gemm refuses the flags for any other form (gemm_takes_rows32 tells beforehand).
@@ -239,7 +264,7 @@ hipError_t launch_gemm(const GemmArgs& a, int epilogue, int num_cus, hipStream_t
 hipError_t launch_attn_prefill(const float* qkv, int T, int C, int H, int head_dim, int P,
                                float* kcache, float* vcache, float* out, float* scratch,
                                hipStream_t s, int nseq = 1, size_t kv_stride = 0);
-// rows rows; row t is position t % period of its sequence
+// rows rows; row t is position t % period of its sequence (wpe may be null)
 hipError_t launch_embed_rows(float* x, const float* wte, const float* wpe, const uint32_t* ids,
                              int rows, int C, hipStream_t s, int w_bf16 = 0, int period = 0);
 // (dst_packed: dst is a packed activation matrix, rows <= 32)

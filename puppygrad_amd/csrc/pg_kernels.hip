@@ -183,6 +183,14 @@ __global__ __launch_bounds__(kBlock) void k_gemv(GemvArgs a) {
   }
   __syncthreads();
   if (PRO == PRO_LN) ln_in_lds(sx, K, a.ln_g, a.ln_b, a.eps, red);
+  // RMS norm with one gain: a factor of the finished sums
+  float row_mul = 1.0f;
+  if (PRO == PRO_RMS) {
+    float ss = 0.0f;
+    for (int i = tid; i < K; i += kBlock) ss += sx[i] * sx[i];
+    row_mul = a.ln_g[0] / sqrtf(block_sum(ss, red) / (float)a.norm_n + a.eps);
+    if (a.out_mul != 0.0f) row_mul *= a.out_mul;
+  }
 
   if (row0 >= a.nout) return;
   float acc[RPW];
@@ -253,7 +261,7 @@ __global__ __launch_bounds__(kBlock) void k_gemv(GemvArgs a) {
     for (int r = 0; r < RPW; ++r) {
       int o = row0 + r;
       if (o >= a.nout) break;
-      float v = (a.bias ? a.bias[o] : 0.0f) + acc[r];
+      float v = (a.bias ? a.bias[o] : 0.0f) + (PRO == PRO_RMS ? row_mul * acc[r] : acc[r]);
       if (EPI == EPI_BIAS) {
         a.y[o] = v;
       } else if (EPI == EPI_GELU) {
@@ -271,6 +279,76 @@ __global__ __launch_bounds__(kBlock) void k_gemv(GemvArgs a) {
           dst[((size_t)h * a.P + a.pos) * a.head_dim + d] = v;
         }
       }
+    }
+  }
+}
+
+// launch_gemv_pair: one wavefront per row of both matrices, both inputs in LDS.
+template <int RPW, int WM>
+__global__ __launch_bounds__(kBlock) void k_gemv_pair(GemvPair a) {
+  extern __shared__ __attribute__((aligned(16))) float sx[];  // K1 + K2 floats
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int row0 = (blockIdx.x * kWaves + wave) * RPW;
+  constexpr int PER = WM == WM_F32X4 ? 4 : 8;  // weights per 16-byte chunk
+  constexpr int kPre = 4;
+  const int KV1 = a.K1 / PER, KV2 = a.K2 / PER, KV = KV1 + KV2;
+  const gv_u4* W1 = reinterpret_cast<const gv_u4*>(a.W1);
+  const gv_u4* W2 = reinterpret_cast<const gv_u4*>(a.W2);
+  // chunk j of row `row` of the two matrices side by side
+  auto chunk = [&](int row, int j) {
+    return __builtin_nontemporal_load(j < KV1 ? &W1[(size_t)row * KV1 + j] : &W2[(size_t)row * KV2 + (j - KV1)]);
+  };
+  gv_u4 pre[RPW][kPre];
+#pragma unroll
+  for (int r = 0; r < RPW; ++r)
+#pragma unroll
+    for (int i = 0; i < kPre; ++i) {
+      const int j = lane + 64 * i;
+      pre[r][i] = gv_u4{0u, 0u, 0u, 0u};
+      if (row0 + r < a.nout && j < KV) pre[r][i] = chunk(row0 + r, j);
+    }
+  for (int i = tid; i < a.K1; i += kBlock) sx[i] = a.x1[i];
+  for (int i = tid; i < a.K2; i += kBlock) sx[a.K1 + i] = a.x2[i];
+  __syncthreads();
+  if (row0 >= a.nout) return;
+  const float4* sx4 = reinterpret_cast<const float4*>(sx);
+  float acc1[RPW], acc2[RPW];
+#pragma unroll
+  for (int r = 0; r < RPW; ++r) acc1[r] = acc2[r] = 0.0f;
+#pragma unroll
+  for (int i = 0; i < kPre; ++i) {
+    const int j = lane + 64 * i;
+    if (j < KV) {
+#pragma unroll
+      for (int r = 0; r < RPW; ++r) {
+        const float d = chunk_dot<WM>(pre[r][i], sx4, j, 1.0f);
+        if (j < KV1) acc1[r] += d;
+        else acc2[r] += d;
+      }
+    }
+  }
+#pragma unroll 4
+  for (int j = lane + 64 * kPre; j < KV; j += 64) {
+#pragma unroll
+    for (int r = 0; r < RPW; ++r) {
+      const float d = chunk_dot<WM>(chunk(min(row0 + r, a.nout - 1), j), sx4, j, 1.0f);
+      if (j < KV1) acc1[r] += d;
+      else acc2[r] += d;
+    }
+  }
+#pragma unroll
+  for (int r = 0; r < RPW; ++r) {
+    acc1[r] = wave_sum(acc1[r]);
+    acc2[r] = wave_sum(acc2[r]);
+  }
+  if (lane == 0) {
+#pragma unroll
+    for (int r = 0; r < RPW; ++r) {
+      const int o = row0 + r;
+      if (o >= a.nout) break;
+      float v = a.resid[o] + a.s1[o] * acc1[r];
+      if (a.W2) v += a.s2[o] * acc2[r];
+      a.y[o] = v;
     }
   }
 }
@@ -936,7 +1014,7 @@ __global__ void k_embed_batch(float* x, const float* wte, const float* wpe, cons
   const int b = blockIdx.y;
   const int i = blockIdx.x * blockDim.x + threadIdx.x;
   if (i < C)
-    x[(size_t)b * C + i] = wte_at(wte, w_bf16, (size_t)ids[b] * C + i) + wpe[(size_t)pos * C + i];
+    x[(size_t)b * C + i] = wte_at(wte, w_bf16, (size_t)ids[b] * C + i) + (wpe ? wpe[(size_t)pos * C + i] : 0.0f);
 }
 
 // K/V append of cached_self_attention_into (rust.rs:1677-1683) for a batch: row b of
@@ -1127,11 +1205,24 @@ hipError_t launch_gemv(const GemvArgs& a, int prologue, int epilogue, hipStream_
   PG_CASE(PRO_NONE, EPI_RESID)
   PG_CASE(PRO_NONE, EPI_GELU)
   PG_CASE(PRO_LN, EPI_BIAS)
+  PG_CASE(PRO_RMS, EPI_BIAS)
   PG_CASE(PRO_LN, EPI_GELU)
   PG_CASE(PRO_LN, EPI_QKV)
   PG_CASE(PRO_ATTN_COMBINE, EPI_RESID)
 #undef PG_CASE
   return hipErrorInvalidValue;
+}
+
+hipError_t launch_gemv_pair(const GemvPair& a, hipStream_t s) {
+  if (a.K1 % 32 != 0 || a.K2 % 32 != 0 || a.K1 + a.K2 > kPairMaxK || (a.W2 == nullptr) != (a.K2 == 0))
+    return hipErrorInvalidValue;
+  const size_t lds = (size_t)(a.K1 + a.K2) * sizeof(float);
+  const dim3 grid((a.nout + kWaves - 1) / kWaves);
+  if (a.w_bf16)
+    hipLaunchKernelGGL((k_gemv_pair<1, WM_BF16X8>), grid, dim3(kBlock), lds, s, a);
+  else
+    hipLaunchKernelGGL((k_gemv_pair<1, WM_F32X4>), grid, dim3(kBlock), lds, s, a);
+  return hipGetLastError();
 }
 
 hipError_t launch_embed(float* x, const float* wte, const float* wpe, const uint32_t* tok_ptr,

@@ -8,6 +8,7 @@
 // the reference's token-by-token prefill (rust.rs:910-927), which the reference
 // itself checks against forward() at 1e-5 (rust.rs:1900-1913).
 #include "pg_kernels.h"
+#include "pg_mixers.h"
 
 #include <math.h>
 
@@ -24,6 +25,10 @@ typedef float f16v __attribute__((ext_vector_type(16)));
 
 __device__ __forceinline__ float gelu_tanh(float x) {
   return 0.5f * x * (1.0f + tanhf(0.7978846f * (x + 0.044715f * x * x * x)));
+}
+// What column n of a product adds to the residual (GemmArgs::col_scale).
+__device__ __forceinline__ float col_scaled(const GemmArgs& a, int n, float c) {
+  return a.col_scale ? a.col_scale[n] * c : c;
 }
 
 // ---------------------------------------------------------------------------
@@ -337,7 +342,7 @@ __global__ __launch_bounds__(256) void k_gemm(GemmArgs a) {
         if (m >= a.M) continue;
         float c = bias + acc[i][j][v];
         if (EPI == GEMM_GELU) c = gelu_tanh(c);
-        if (EPI == GEMM_RESID) c = a.resid[(size_t)m * a.ldc + n] + c;
+        if (EPI == GEMM_RESID) c = a.resid[(size_t)m * a.ldc + n] + col_scaled(a, n, c);
         a.C[(size_t)m * a.ldc + n] = c;
       }
     }
@@ -463,7 +468,7 @@ __device__ __forceinline__ void redo_tile(const GemmArgs& a, int mbase, int nbas
           }
           c = (a.bias ? a.bias[n] : 0.0f) + c;
           if (EPI == GEMM_GELU) c = gelu_tanh(c);
-          if (EPI == GEMM_RESID) c = a.resid[(size_t)m * a.ldc + n] + c;
+          if (EPI == GEMM_RESID) c = a.resid[(size_t)m * a.ldc + n] + col_scaled(a, n, c);
           a.C[(size_t)m * a.ldc + n] = c;
         }
     }
@@ -691,7 +696,7 @@ __global__ __launch_bounds__(256) void k_gemm_b3(GemmArgs a) {
         if (m >= a.M) continue;
         float c = bias + (WT == 2 ? wscale * acc[i][j][v] : acc[i][j][v]);
         if (EPI == GEMM_GELU) c = gelu_tanh(c);
-        if (EPI == GEMM_RESID) c = a.resid[(size_t)m * a.ldc + n] + c;
+        if (EPI == GEMM_RESID) c = a.resid[(size_t)m * a.ldc + n] + col_scaled(a, n, c);
         a.C[(size_t)m * a.ldc + n] = c;
       }
     }
@@ -899,7 +904,7 @@ __global__ __launch_bounds__(256) void k_gemm_b9(GemmArgs a) {
         if (m >= a.M) continue;
         float c = bias + acc[i][j][v];
         if (EPI == GEMM_GELU) c = gelu_tanh(c);
-        if (EPI == GEMM_RESID) c = a.resid[(size_t)m * a.ldc + n] + c;
+        if (EPI == GEMM_RESID) c = a.resid[(size_t)m * a.ldc + n] + col_scaled(a, n, c);
         a.C[(size_t)m * a.ldc + n] = c;
       }
     }
@@ -929,7 +934,7 @@ __global__ __launch_bounds__(256) void k_splitk_reduce(GemmArgs a, int parts) {
 #pragma unroll
   for (int k = 0; k < 4; ++k) {
     if (EPI == GEMM_GELU) c[k] = gelu_tanh(c[k]);
-    if (EPI == GEMM_RESID) c[k] = a.resid[m * a.ldc + n + k] + c[k];
+    if (EPI == GEMM_RESID) c[k] = a.resid[m * a.ldc + n + k] + col_scaled(a, (int)n + k, c[k]);
     dst[k] = c[k];
   }
 }
@@ -964,6 +969,7 @@ __global__ __launch_bounds__(256) void k_splitk_reduce_ln(GemmArgs a, int parts)
 #pragma unroll
     for (int p = 0; p < 8; ++p)
       v[q][p] = *reinterpret_cast<const f4*>(a.ws + (size_t)min(p, parts - 1) * stride + m * a.N + n);
+    if (a.rms_cols) return;
     lg[q] = *reinterpret_cast<const f4*>(a.ln_g + n);
     lb[q] = *reinterpret_cast<const f4*>(a.ln_b + n);
   };
@@ -988,11 +994,24 @@ __global__ __launch_bounds__(256) void k_splitk_reduce_ln(GemmArgs a, int parts)
 #pragma unroll
       for (int k = 0; k < 4; ++k) {
         if (EPI == GEMM_GELU) r[k] = gelu_tanh(r[k]);
-        if (EPI == GEMM_RESID) r[k] = a.resid[m * a.ldc + n + k] + r[k];
+        if (EPI == GEMM_RESID) r[k] = a.resid[m * a.ldc + n + k] + col_scaled(a, (int)n + k, r[k]);
       }
       c[q] = f4{r[0], r[1], r[2], r[3]};
       *reinterpret_cast<f4*>(a.C + m * a.ldc + n) = c[q];
     }
+  }
+  if (a.rms_cols) {  // RMS norm with one gain (columns past rms_cols hold zeros)
+    float ss = 0.0f;
+#pragma unroll
+    for (int q = 0; q < 4; ++q) ss += (c[q].x * c[q].x + c[q].y * c[q].y) + (c[q].z * c[q].z + c[q].w * c[q].w);
+    const float k = a.ln_g[0] / sqrtf(bsum(ss) / (float)a.rms_cols + a.ln_eps);
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      const int i = (int)threadIdx.x + 256 * q;
+      if (i < n4)
+        *reinterpret_cast<f4*>(a.ln_out + (a.ln_packed ? packed32_index(m, (size_t)i * 4) : m * a.N + (size_t)i * 4)) = c[q] * k;
+    }
+    return;
   }
   float sum = 0.0f;
 #pragma unroll
@@ -1118,7 +1137,7 @@ __global__ __launch_bounds__(256) void k_gemv_rows(GemmArgs a) {
   if (b >= a.M || n >= a.N) return;
   float c = (a.bias ? a.bias[n] : 0.0f) + acc[0];
   if (EPI == GEMM_GELU) c = gelu_tanh(c);
-  if (EPI == GEMM_RESID) c = a.resid[(size_t)b * a.ldc + n] + c;
+  if (EPI == GEMM_RESID) c = a.resid[(size_t)b * a.ldc + n] + col_scaled(a, n, c);
   a.C[(size_t)b * a.ldc + n] = c;
 }
 
@@ -1406,7 +1425,7 @@ __global__ __launch_bounds__(512) void k_gemm_rows32(GemmArgs a) {
     }
     float c = ebias[q] + sum;
     if (EPI == GEMM_GELU) c = gelu_tanh(c);
-    if (EPI == GEMM_RESID) c = eres[q] + c;
+    if (EPI == GEMM_RESID) c = eres[q] + col_scaled(a, n, c);
     a.C[a.c_packed ? packed32_index((size_t)b, (size_t)n) : (size_t)b * a.ldc + n] = c;
   }
 }
@@ -1433,7 +1452,7 @@ __global__ __launch_bounds__(256) void k_tail_reduce(GemmArgs a) {
 #pragma unroll
   for (int k = 0; k < 4; ++k) {
     if (EPI == GEMM_GELU) c[k] = gelu_tanh(c[k]);
-    if (EPI == GEMM_RESID) c[k] = a.resid[(size_t)m * a.ldc + n + k] + c[k];
+    if (EPI == GEMM_RESID) c[k] = a.resid[(size_t)m * a.ldc + n + k] + col_scaled(a, n + k, c[k]);
     dst[k] = c[k];
   }
 }
@@ -1724,7 +1743,7 @@ __global__ void k_embed_rows(float* x, const float* wte, const float* wpe, const
     const float e =
         w_bf16 ? __uint_as_float((unsigned)reinterpret_cast<const unsigned short*>(wte)[idx] << 16)
                : wte[idx];
-    x[(size_t)t * C + i] = e + wpe[(size_t)pos * C + i];
+    x[(size_t)t * C + i] = wpe ? e + wpe[(size_t)pos * C + i] : e;
   }
 }
 
@@ -2220,6 +2239,9 @@ hipError_t launch_gemm(const GemmArgs& a, int epi, int num_cus, hipStream_t s) {
   if (a.ln_out && a.ldc != a.N) return hipErrorInvalidValue;
   bool ln_done = false;
   hipError_t e = launch_gemm_form(a, epi, num_cus, s, &ln_done);
+  if (e == hipSuccess && a.ln_out && !ln_done && a.rms_cols)
+    return a.ln_packed ? hipErrorInvalidValue
+                       : launch_rms_rows(a.C, a.ln_out, a.M, a.rms_cols, a.N, a.ln_g, a.ln_eps, 1.0f, nullptr, s);
   if (e == hipSuccess && a.ln_out && !ln_done)
     e = launch_layer_norm_rows(a.C, a.ln_out, a.M, a.N, a.ln_g, a.ln_b, a.ln_eps, s, a.ln_packed);
   return e;

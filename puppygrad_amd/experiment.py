@@ -33,6 +33,7 @@ from typing import Iterable, List, Optional, Sequence
 from . import _lib, synth
 from .gpt2 import (GPT2_EOS_TOKEN_ID, GenerationStats, Gpt2Config, Gpt2HipConfig, Gpt2Model,
                    Gpt2OperationProfile, TextGenerationConfig)
+from .models import load_model
 from .runtime import Gpt2Runtime
 
 
@@ -331,7 +332,7 @@ def main(argv: Optional[Sequence[str]] = None) -> int:
     if text_prompts is not None:
         model = Gpt2Runtime.from_dir(args.model_dir, hip)
     elif args.model_dir:
-        model = Gpt2Model.from_dir(args.model_dir, hip)
+        model = load_model(args.model_dir, hip)
     else:
         kw = {"small": synth.GPT2_SMALL, "medium": synth.GPT2_MEDIUM, "large": synth.GPT2_LARGE,
               "xl": synth.GPT2_XL}[args.model]
@@ -339,8 +340,8 @@ def main(argv: Optional[Sequence[str]] = None) -> int:
         model = Gpt2Model.new(cfg, synth.random_weights(cfg, synth.WEIGHT_SEED_BASE + 1), hip)
     load_time = time.perf_counter() - t0
     core = model.model if text_prompts is not None else model
-    print(f"loaded GPT-2 with {core.describe()}", file=sys.stderr)
-    vocab = core.config.vocab_size
+    print(f"loaded {core.architecture} with {core.describe()}", file=sys.stderr)
+    vocab = core.vocab_size
     prompts = text_prompts if text_prompts is not None else [
         list(synth.token_ids(n, synth.TOKEN_SEED_BASE + 1, vocab))
         for n in _usize_list("prompt-tokens", args.prompt_tokens)]

@@ -16,8 +16,10 @@ import time
 import unicodedata
 from typing import Callable, List, Optional, Sequence, Tuple
 
-from .gpt2 import (GenerationStats, Gpt2Error, Gpt2GenerationConfig, Gpt2HipConfig, Gpt2Model,
-                   Gpt2OperationProfile, TextGenerationConfig)
+from .gpt2 import Gpt2GenerationConfig
+from .model import (GenerationStats, Gpt2Error, Gpt2HipConfig, Gpt2OperationProfile, Model,
+                    TextGenerationConfig)
+from .models import load_model
 
 REPLACEMENT_CHARACTER = "�"
 
@@ -126,7 +128,7 @@ class Gpt2Runtime:
     tokenizer.  Every generation below runs on the device through the C-ABI; the tokenizer and
     the streamer run on the host between token callbacks, as in the reference."""
 
-    def __init__(self, model: Gpt2Model, tokenizer: Gpt2Tokenizer):
+    def __init__(self, model: Model, tokenizer: Gpt2Tokenizer):
         self.model = model
         self.tokenizer = tokenizer
 
@@ -134,7 +136,7 @@ class Gpt2Runtime:
     def from_dir(cls, model_dir, hip_config: Optional[Gpt2HipConfig] = None) -> "Gpt2Runtime":
         """from_dir_with_backend (rust.rs:382-393): config.json, model.safetensors,
         tokenizer.json of one directory (src/models/gpt2/assets.rs:20-28)."""
-        model = Gpt2Model.from_dir(model_dir, hip_config)
+        model = load_model(model_dir, hip_config)
         tokenizer = Gpt2Tokenizer.from_file(os.path.join(os.fspath(model_dir), "tokenizer.json"))
         return cls(model, tokenizer)
 
@@ -166,9 +168,9 @@ class Gpt2Runtime:
     def _check_generation(self, generation: TextGenerationConfig) -> None:
         generation.validate()
         eos = generation.eos_token_id
-        if eos is not None and eos >= self.model.config.vocab_size:
+        if eos is not None and eos >= self.model.vocab_size:
             raise Gpt2Error("InvalidConfig",
-                            f"generation eos_token_id {eos} is outside vocab_size {self.model.config.vocab_size}")
+                            f"generation eos_token_id {eos} is outside vocab_size {self.model.vocab_size}")
 
     def stream_text_with_stats(self, prompt: str, generation: TextGenerationConfig,
                                on_text: Callable[[str], None], profiled: bool = False
