@@ -66,10 +66,15 @@ def main() -> int:
                     help="skip the other configurations (they run only beside the default workload)")
     ap.add_argument("--decode-path", default="auto", choices=["auto", "kernels", "persistent"])
     ap.add_argument("--workload", default="decode",
-                    choices=["decode", "prefill", "batch-decode", "sampled-stream"],
+                    choices=["decode", "prefill", "batch-decode", "sampled-stream", "tarepel"],
                     help="prefill: a step is one prefill of --prefill tokens (GEMM path, MFMA-bound); "
                          "batch-decode: a step is one greedy step of --batch sequences; "
-                         "sampled-stream: streamed generations of --steps tokens with sampled selection")
+                         "sampled-stream: streamed generations of --steps tokens with sampled selection; "
+                         "tarepel: prefill and decode of a Tarepel stack model at several widths beside "
+                         "GPT-2 models of the same width and parameters per layer")
+    ap.add_argument("--widths", default="768,1280,1600", help="widths of --workload tarepel")
+    ap.add_argument("--only", default="", help="--workload tarepel: stack or gpt2, and one of prefill, "
+                                               "decode, batch (profiling runs)")
     ap.add_argument("--batch", type=int, default=None,
                     help="sequences of a batched step (batch-decode: 16 by default; prefill: 1)")
     ap.add_argument("--bf16", action="store_true", help="store the weights as bf16 (fp32 arithmetic)")
@@ -87,6 +92,9 @@ def main() -> int:
         return 2
 
     from puppygrad_amd import Gpt2Config, Gpt2HipConfig, Gpt2Model, _lib, synth
+
+    if args.workload == "tarepel":
+        return bench_tarepel(args)
 
     model_kw = {"xl": synth.GPT2_XL, "large": synth.GPT2_LARGE, "medium": synth.GPT2_MEDIUM,
                 "small": synth.GPT2_SMALL}[args.model]
@@ -515,6 +523,99 @@ def bench_prefill(args, cfg, model, ids, n_prefill) -> int:
         result["roofline"] = hbm_roofline(gbs, "whole prefill (k_gemm_rows32, k_attn_prefill64, reduce + LayerNorm, lm_head)",
                                           algorithmic_bytes_per_step=int(wbytes))
     print(json.dumps(result), flush=True)
+    return 0
+
+
+def stack_layer_params(cfg) -> int:
+    """Parameters of a stack model's layers that a token meets (everything but embed and head)."""
+    from puppygrad_amd import synth
+    return sum(int(np.prod(s, dtype=np.int64)) for n, s in synth.stack_tensor_shapes(cfg).items()
+               if n not in ("embed", "head"))
+
+
+def bench_tarepel(args) -> int:
+    """Tarepel beside GPT-2 at the same width, layer count, vocabulary and (within 2 %) parameters
+    per layer, bf16-stored weights: prefill of 1024 tokens, batch-1 greedy decode from there and a
+    batch-32 step from 256 tokens.  `roofline` is that of the bound both share: the weights' bytes
+    at the HBM peak for decode, the products' flops at the bf16 matrix peak for prefill."""
+    import tempfile
+
+    from puppygrad_amd import Gpt2Config, Gpt2HipConfig, Gpt2Model, _lib, load_model, synth
+    hip = Gpt2HipConfig(weight_storage=_lib.PG_STORE_BF16)
+    layers, vocab, T, NB, TB = 8, 50257, 1024, 32, 256
+    only = [w for w in args.only.split(",") if w]
+    steps = min(args.steps, 127)
+
+    def want(*what):
+        return all(w in what for w in only) if only else True
+
+    def measure(model, params, name):
+        ids = synth.token_ids(T, synth.TOKEN_SEED_BASE + 7, vocab)
+        out = {"params_per_layer": params // layers}
+        wbytes = 2 * (params + vocab * model._info().width)
+        if want(name, "prefill"):
+            cache = model.new_kv_cache()
+            for _ in range(2):
+                model.prefill(ids, cache).argmax()
+            n, t0 = 8, time.time()
+            for _ in range(n):
+                logits = model.prefill(ids, cache)
+            logits.argmax()
+            sec = (time.time() - t0) / n
+            flops = 2.0 * params * T
+            out["prefill"] = {"tokens_per_s": round(T / sec, 1), "ms": round(sec * 1e3, 3),
+                              "product_tflops": round(flops / sec / 1e12, 1),
+                              "frac_bf16_mfma": round(flops / sec / 1e12 / BF16_MFMA_PEAK_TFLOPS, 4)}
+        if want(name, "decode"):
+            cache = model.new_kv_cache()
+            model.prefill(ids[:T - 160], cache)
+            model.decode_greedy(cache, 17)
+            model.prefill(ids[:T - 160], cache)
+            _, st = model.decode_greedy(cache, steps + 1)
+            sec = st.gpu_decode_time / steps
+            out["decode"] = {"tokens_per_s": round(1.0 / sec, 1), "us": round(sec * 1e6, 2),
+                             "frac_hbm": round(wbytes / sec / 1e9 / HBM_PEAK_GBS, 4)}
+        if want(name, "batch"):
+            cache = model.new_kv_cache(NB)
+            bids = np.stack([synth.token_ids(TB, synth.TOKEN_SEED_BASE + 100 + b, vocab) for b in range(NB)])
+            model.prefill_batch(bids, cache)
+            model.decode_greedy_batch(cache, 9)
+            model.prefill_batch(bids, cache)
+            _, st = model.decode_greedy_batch(cache, 65)
+            sec = st.gpu_decode_time / 64
+            out["batch_step"] = {"batch": NB, "tokens_per_s": round(NB / sec, 1), "us": round(sec * 1e6, 2),
+                                 "frac_hbm_weights": round(wbytes / sec / 1e9 / HBM_PEAK_GBS, 4)}
+        return out
+
+    rows = {}
+    for width in (int(w) for w in args.widths.split(",")):
+        entry = {}
+        if not only or "gpt2" not in only:
+            cfg = synth.tarepel_config(width, layers, vocab)
+            with tempfile.TemporaryDirectory() as tmp:
+                synth.write_model_dir(tmp, cfg, synth.stack_weights(cfg, synth.WEIGHT_SEED_BASE + 20))
+                model = load_model(tmp, hip)
+            entry["tarepel"] = measure(model, stack_layer_params(cfg), "stack")
+            log(f"[bench] width {width} tarepel: {entry['tarepel']}")
+            del model
+        if not only or "stack" not in only:
+            g = Gpt2Config(vocab_size=vocab, n_positions=T, n_embd=width, n_layer=layers, n_head=width // 64)
+            model = Gpt2Model.new(g, synth.random_weights(g, synth.WEIGHT_SEED_BASE + 21), hip)
+            entry["gpt2"] = measure(model, layers * 12 * width * width, "gpt2")
+            log(f"[bench] width {width} gpt2: {entry['gpt2']}")
+            del model
+        rows[str(width)] = entry
+    first = rows[str(max(int(w) for w in rows))]
+    value = first.get("tarepel", {}).get("decode", {}).get("tokens_per_s")
+    info = _devinfo()
+    print(json.dumps({
+        "metric": "decode tokens/sec, Tarepel 8 layers bf16-stored weights bs=1 (largest width)",
+        "value": value, "unit": "tokens/s", "n_gpus": 1, "steps": steps, "warmup": 16,
+        "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "f32", "data": "synthetic",
+        "config": {"workload": f"prefill of {T} tokens, batch-1 decode from {T - 160}, batch-{NB} step "
+                               f"from {TB}; {layers} layers, vocabulary {vocab}",
+                   "device": info.name.decode() or info.arch.decode(), "compute_units": info.compute_units},
+        "widths": rows}), flush=True)
     return 0
 
 

@@ -730,7 +730,7 @@ pg_status ensure_ids(pg_kv_cache* c, size_t n) {
 pg_status stack_advance(const pg_model* m, pg_kv_cache* c, const uint32_t* ids, size_t n,
                         const std::vector<int>& rows, float* dst, ProfileMarks* marks = nullptr) {
   pg_status s;
-  if ((s = ensure_ids(c, c->B * std::min<size_t>(n, 8192)))) return s;
+  if ((s = ensure_ids(c, c->B * std::min<size_t>(n, std::max<size_t>(32, 8192 / c->B))))) return s;
   if ((s = pgh::stack_rows(m, c, ids, n, c->seq_len, rows, dst, marks))) return s;
   PG_HIP(hipStreamSynchronize(c->stream));
   c->seq_len += n;

@@ -76,7 +76,11 @@ struct GemvPair {
   const float* resid;
   float* y;
   int K1, K2, nout;
+  // part_splits > 0: x1[part_col + i], i < part_n, is instead the sum over part[split][part_n][i]
+  const float* part = nullptr;
+  int part_splits = 0, part_n = 0, part_col = 0;
 };
+constexpr int kPairMaxSplits = 8;
 constexpr int kPairMaxK = 16320;
 hipError_t launch_gemv_pair(const GemvPair& a, hipStream_t s);
 

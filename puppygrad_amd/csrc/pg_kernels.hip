@@ -290,7 +290,7 @@ __global__ __launch_bounds__(kBlock) void k_gemv_pair(GemvPair a) {
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int row0 = (blockIdx.x * kWaves + wave) * RPW;
   constexpr int PER = WM == WM_F32X4 ? 4 : 8;  // weights per 16-byte chunk
-  constexpr int kPre = 4;
+  constexpr int kPre = 12;
   const int KV1 = a.K1 / PER, KV2 = a.K2 / PER, KV = KV1 + KV2;
   const gv_u4* W1 = reinterpret_cast<const gv_u4*>(a.W1);
   const gv_u4* W2 = reinterpret_cast<const gv_u4*>(a.W2);
@@ -307,8 +307,26 @@ __global__ __launch_bounds__(kBlock) void k_gemv_pair(GemvPair a) {
       pre[r][i] = gv_u4{0u, 0u, 0u, 0u};
       if (row0 + r < a.nout && j < KV) pre[r][i] = chunk(row0 + r, j);
     }
-  for (int i = tid; i < a.K1; i += kBlock) sx[i] = a.x1[i];
-  for (int i = tid; i < a.K2; i += kBlock) sx[a.K1 + i] = a.x2[i];
+  {
+    const float4* x1 = reinterpret_cast<const float4*>(a.x1);
+    const float4* x2 = reinterpret_cast<const float4*>(a.x2);
+    float4* d = reinterpret_cast<float4*>(sx);
+    const int n1 = a.K1 >> 2, n2 = a.K2 >> 2;
+    for (int i = tid; i < n1 + n2; i += kBlock) d[i] = i < n1 ? x1[i] : x2[i - n1];
+    if (a.part_splits > 0) {
+      // columns that are still partial sums
+      __syncthreads();
+      for (int i = tid; i < a.part_n; i += kBlock) {
+        float v[kPairMaxSplits];
+#pragma unroll
+        for (int k = 0; k < kPairMaxSplits; ++k) v[k] = a.part[(size_t)min(k, a.part_splits - 1) * a.part_n + i];
+        float s = 0.0f;
+#pragma unroll
+        for (int k = 0; k < kPairMaxSplits; ++k) s += k < a.part_splits ? v[k] : 0.0f;
+        sx[a.part_col + i] = s;
+      }
+    }
+  }
   __syncthreads();
   if (row0 >= a.nout) return;
   const float4* sx4 = reinterpret_cast<const float4*>(sx);

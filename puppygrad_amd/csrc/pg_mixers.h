@@ -14,7 +14,7 @@ namespace pgk {
 
 constexpr int kMixMaxDim = 256;   // key and value sizes per head
 constexpr int kMixMaxTaps = 16;   // short convolution
-constexpr int kSplitKeys = 128;   // keys per block of the attention's decode form
+constexpr int kSplitKeys = 64;   // keys per block of the attention's decode form
 
 // Rotary positions: the pair (i, i + half) of a head turns by position * freq[i], i < half; the
 // head's values from 2 * half on pass unchanged.
@@ -89,7 +89,8 @@ struct GatedMlp {
 // One decode step of a layer's mixers for all sequences, in one launch: attention, recurrence and
 // gated activation side by side (they read the same row of projections).  *d_pos is the
 // position.  With more than one key split (attn_splits > 1) the attention leaves partial sums in
-// part[b][split][heads][dim], which launch_attn_sum adds into the mixer outputs.
+// part[b][split][heads][dim] (zeros for splits without keys); they are added into the mixer
+// outputs by launch_attn_sum, or by the projection that reads them (GemvPair::part).
 struct MixDecode {
   int nseq;
   const int* d_pos;
@@ -120,14 +121,15 @@ struct MixRows {
   float* k_rot;       // [rows][kv_heads * dim]: rotated keys
   float* conv_out;    // [rows][channels]
   float* decay;       // gated linear attention: log alpha [rows][heads * dim]
-  float* o;           // recurrence read-outs [rows][heads * vdim]
+  float* work;        // chunk tiles of the recurrence (recurrence_work_floats)
+  size_t work_floats;
 };
 hipError_t launch_rotary_rows(const MixRows& r, const ChunkAttn& a, hipStream_t s);
 hipError_t launch_chunk_attn_rows(const MixRows& r, const ChunkAttn& a, hipStream_t s);
 hipError_t launch_short_conv_rows(const MixRows& r, const ShortConv& c, hipStream_t s);
+// The recurrence of all rows, normalised and gated, into the mixer output columns.
 hipError_t launch_recurrence_rows(const MixRows& r, const Recurrence& c, hipStream_t s);
-// o -> the mixer output columns (norm, gate, scale)
-hipError_t launch_gated_norm_rows(const MixRows& r, const Recurrence& c, hipStream_t s);
+size_t recurrence_work_floats(const Recurrence& c, int nseq, int n);
 hipError_t launch_gated_mlp_rows(const MixRows& r, const GatedMlp& m, hipStream_t s);
 // The rows that the caches keep: the last chunk's keys and values, the convolution's last inputs
 // (a or c may be null).

@@ -54,10 +54,14 @@ __device__ __forceinline__ float gla_log_decay(float z, float inv_tau) { return 
 // ---------------------------------------------------------------------------
 constexpr int kRG = 8;  // query heads of one key/value head that a block takes
 
-// LDS of a decode block, by role (floats).
+// LDS of a decode block (floats): the attention role's, the larger of the two.
 constexpr int kDecodeLds = kRG * kMixMaxDim + 2 * kMixMaxDim + kRG * kSplitKeys + 256 * kRG;
 
-// Keys [128 split, ...) of the current chunk against kRG query heads of key/value head g.
+// Keys [kSplitKeys split, ...) of the current chunk against kRG query heads of key/value head g.
+// NV: float4 per lane and key (sixteen lanes to a key).  Nothing that is loaded before the first
+// barrier depends on another load but the ring rows' bound, and all of a block's key rows are
+// requested together, then all of its value rows.
+template <int NV>
 __device__ void attn_role(const MixDecode& m, int b, int item, float* lds) {
   const ChunkAttn& a = m.attn;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -65,11 +69,33 @@ __device__ void attn_role(const MixDecode& m, int b, int item, float* lds) {
   const int split = item % m.attn_splits, rest = item / m.attn_splits;
   const int rg = rest % groups, g = rest / groups;
   const int r0 = rg * kRG, nr = min(kRG, R - r0);
-  const int pos = *m.d_pos, last = pos % a.chunk;  // ring row of the current token
-  const int j0 = split * kSplitKeys;
-  if (j0 > last) return;
-  const int nk = min(last + 1 - j0, kSplitKeys);
   const int dim = a.dim, dp = a.dim_pad, half = a.rot.half;
+  const int j0 = split * kSplitKeys;
+  const float* kring = a.kring + (size_t)b * a.ring_seq + (size_t)g * a.chunk * dp;
+  const float* vring = a.vring + (size_t)b * a.ring_seq + (size_t)g * a.chunk * dp;
+  const int pos = *m.d_pos, last = pos % a.chunk;  // ring row of the current token
+  if (j0 > last) {
+    // (every split's sums are added: the ones without keys are 0)
+    if (m.attn_splits > 1)
+      for (int i = tid; i < nr * dim; i += 256)
+        m.part[(((size_t)b * m.attn_splits + split) * a.heads + g * R + r0) * dim + i] = 0.0f;
+    return;
+  }
+  const int nk = min(last + 1 - j0, kSplitKeys);
+  const int own = last - j0;  // the current token's key in this split, if it is below nk
+  const int sub = lane >> 4, l16 = lane & 15;
+  // key rows: four to a wavefront and step
+  constexpr int KS = kSplitKeys / 16;
+  f4 kv[KS][NV];
+#pragma unroll
+  for (int q = 0; q < KS; ++q) {
+    const int j = min(16 * q + wave * 4 + sub, max(nk - 1, 0));
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int e = 4 * l16 + 64 * i;
+      kv[q][i] = *reinterpret_cast<const f4*>(kring + (size_t)(j0 + j) * dp + min(e, dp - 4));
+    }
+  }
   float* qs = lds;                       // [kRG][dp]
   float* kn = qs + kRG * dp;             // [dp] the current token's key, rotated
   float* vn = kn + dp;                   // [dp] ... as projected
@@ -78,88 +104,102 @@ __device__ void attn_role(const MixDecode& m, int b, int item, float* lds) {
   const float* y = m.y + (size_t)b * m.ld_y;
   const float* yk = y + a.k_col + g * dim;
   const float* yq = y + a.q_col + (size_t)(g * R + r0) * dim;
-  // rotate: one thread per value beyond the pairs' first halves
   for (int i = tid; i < dp; i += 256) {
     if (i < half) {
       float s, c;
-      turn(pos, a.rot.freq[i], &s, &c);
       const float u = yk[i], v = yk[i + half];
+      turn(pos, a.rot.freq[i], &s, &c);
       kn[i] = u * c - v * s;
       kn[i + half] = v * c + u * s;
       vn[i] = u;
       vn[i + half] = v;
-      for (int r = 0; r < nr; ++r) {
-        const float qu = yq[r * dim + i], qv = yq[r * dim + i + half];
-        qs[r * dp + i] = qu * c - qv * s;
-        qs[r * dp + i + half] = qv * c + qu * s;
-      }
     } else if (i >= 2 * half) {
       kn[i] = vn[i] = i < dim ? yk[i] : 0.0f;
-      for (int r = 0; r < nr; ++r) qs[r * dp + i] = i < dim ? yq[r * dim + i] : 0.0f;
+    }
+  }
+  // queries: a pair (or a value that passes) per thread
+  const int per = dp - half;
+  for (int i = tid; i < nr * per; i += 256) {
+    const int r = i / per, e = i - r * per;
+    if (e < half) {
+      float s, c;
+      const float u = yq[r * dim + e], v = yq[r * dim + e + half];
+      turn(pos, a.rot.freq[e], &s, &c);
+      qs[r * dp + e] = u * c - v * s;
+      qs[r * dp + e + half] = v * c + u * s;
+    } else {
+      qs[r * dp + e + half] = e + half < dim ? yq[r * dim + e + half] : 0.0f;
     }
   }
   __syncthreads();
-  float* kring = a.kring + (size_t)b * a.ring_seq + (size_t)g * a.chunk * dp;
-  float* vring = a.vring + (size_t)b * a.ring_seq + (size_t)g * a.chunk * dp;
-  const int own = last - j0;  // the current token's key in this split, if it is below nk
-  if (rg == 0 && own < kSplitKeys)
-    for (int i = tid; i < dp; i += 256) {
-      kring[(size_t)last * dp + i] = kn[i];
-      vring[(size_t)last * dp + i] = vn[i];
-    }
-  // scores: sixteen lanes to a key, four keys to a wavefront
-  const int sub = lane >> 4, l16 = lane & 15;
-#pragma unroll 2
-  for (int j = wave * 4 + sub; j < (nk + 15) / 16 * 16; j += 16) {
-    f4 kv[4];
-    const bool in = j < nk && j != own;
+  // value rows of this thread's column, requested ahead of the scores
+  int cols = 1;
+  while (cols < dim) cols <<= 1;
+  const int parts = 256 / cols, d = tid % cols, part = tid / cols;
+  constexpr int VB = 16;  // value rows in flight per thread
+  float vv[VB];
+  auto fetch_v = [&](int jb) {
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int e = 4 * l16 + 64 * i;
-      kv[i] = f4{0.f, 0.f, 0.f, 0.f};
-      if (e < dp) {
-        if (in) kv[i] = *reinterpret_cast<const f4*>(kring + (size_t)(j0 + j) * dp + e);
-        else if (j == own) kv[i] = *reinterpret_cast<const f4*>(kn + e);
-      }
+    for (int q = 0; q < VB; ++q) {
+      const int j = min(jb + part + parts * q, nk - 1);
+      vv[q] = vring[(size_t)(j0 + j) * dp + min(d, dp - 1)];
+    }
+  };
+  fetch_v(0);
+  if (rg == 0 && own < kSplitKeys) {
+    float* kw = a.kring + (size_t)b * a.ring_seq + ((size_t)g * a.chunk + last) * dp;
+    float* vw = a.vring + (size_t)b * a.ring_seq + ((size_t)g * a.chunk + last) * dp;
+    for (int i = tid; i < dp; i += 256) {
+      kw[i] = kn[i];
+      vw[i] = vn[i];
+    }
+  }
+#pragma unroll
+  for (int q = 0; q < KS; ++q) {
+    const int j = 16 * q + wave * 4 + sub;
+    if (16 * q >= nk) break;
+    if (j == own) {
+#pragma unroll
+      for (int i = 0; i < NV; ++i) kv[q][i] = *reinterpret_cast<const f4*>(kn + min(4 * l16 + 64 * i, dp - 4));
     }
 #pragma unroll
     for (int r = 0; r < kRG; ++r) {
       if (r >= nr) break;
       float s = 0.0f;
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
+      for (int i = 0; i < NV; ++i) {
         const int e = 4 * l16 + 64 * i;
         if (e < dp) {
-          const f4 q = *reinterpret_cast<const f4*>(qs + r * dp + e);
-          s += (kv[i].x * q.x + kv[i].y * q.y) + (kv[i].z * q.z + kv[i].w * q.w);
+          const f4 x = *reinterpret_cast<const f4*>(qs + r * dp + e);
+          s += (kv[q][i].x * x.x + kv[q][i].y * x.y) + (kv[q][i].z * x.z + kv[q][i].w * x.w);
         }
       }
       s += __shfl_xor(s, 8, 64);
       s += __shfl_xor(s, 4, 64);
       s += __shfl_xor(s, 2, 64);
       s += __shfl_xor(s, 1, 64);
-      if (l16 == 0 && j < nk) w[r * kSplitKeys + j] = sigmoid(s * a.scale + a.bias[g * R + r0 + r]);
+      if (l16 == 0) w[r * kSplitKeys + j] = j < nk ? sigmoid(s * a.scale + a.bias[g * R + r0 + r]) : 0.0f;
     }
   }
   __syncthreads();
-  // weighted values: a thread owns one value column and every kp-th key
-  int cols = 1;
-  while (cols < dim) cols <<= 1;
-  const int parts = 256 / cols, d = tid % cols, part = tid / cols;
   float acc[kRG];
 #pragma unroll
   for (int r = 0; r < kRG; ++r) acc[r] = 0.0f;
-  if (d < dim) {
-#pragma unroll 4
-    for (int j = part; j < nk; j += parts) {
-      const float v = j == own ? vn[d] : vring[(size_t)(j0 + j) * dp + d];
+  for (int jb = 0; jb < nk; jb += VB * parts) {
+    if (jb) fetch_v(jb);
+#pragma unroll
+    for (int q = 0; q < VB; ++q) {
+      const int j = jb + part + parts * q;
+      if (j >= nk) break;
+      const float v = j == own ? vn[min(d, dp - 1)] : vv[q];
 #pragma unroll
       for (int r = 0; r < kRG; ++r)
         if (r < nr) acc[r] += w[r * kSplitKeys + j] * v;
     }
   }
 #pragma unroll
-  for (int r = 0; r < kRG; ++r) red[(r * parts + part) * cols + d] = acc[r];
+  for (int r = 0; r < kRG; ++r)
+    if (r < nr) red[(r * parts + part) * cols + d] = acc[r];
   __syncthreads();
   for (int i = tid; i < nr * cols; i += 256) {
     const int r = i / cols, dd = i - r * cols;
@@ -168,14 +208,48 @@ __device__ void attn_role(const MixDecode& m, int b, int item, float* lds) {
     for (int p = 0; p < parts; ++p) s += red[(r * parts + p) * cols + dd];
     const int h = g * R + r0 + r;
     if (m.attn_splits > 1)
-      m.part[(((size_t)b * m.attn_splits + split) * a.heads + h) * dim + dd] = s;
+      m.part[(((size_t)b * m.attn_splits + split) * a.heads + h) * dim + dd] = s * a.out_scale;
     else
       m.out[(size_t)b * m.ld_out + a.out_col + h * dim + dd] = s * a.out_scale;
   }
 }
 
+// Channel ch of a short convolution at position pos (up to four taps: every load is issued at
+// once, whatever pos is), and the ring row of this position (no block reads it in this step).
+__device__ __forceinline__ float conv_channel(const ShortConv& c, const float* y, float* ring, int ch, int pos, bool keep) {
+  const float cur = y[c.col + ch];
+  float s = 0.0f;
+  if (c.taps <= 4) {
+    float x[4], w[4];
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      const int kk = min(k, c.taps - 1);
+      x[k] = ring[(size_t)kk * c.channels + ch];  // the input whose position is k modulo taps
+      w[k] = c.w[ch * c.taps + kk];
+    }
+    const int slot = pos % c.taps;
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      if (k >= c.taps) break;
+      int j = slot - k;  // tokens back
+      if (j < 0) j += c.taps;
+      const float in = j == 0 ? cur : pos >= j ? x[k] : 0.0f;
+      float wt = w[0];
+#pragma unroll
+      for (int i = 1; i < 4; ++i) wt = i == c.taps - 1 - j ? w[i] : wt;
+      s += wt * in;
+    }
+  } else {
+    s = c.w[ch * c.taps + c.taps - 1] * cur;
+    for (int j = 1; j < c.taps; ++j)
+      if (pos >= j) s += c.w[ch * c.taps + c.taps - 1 - j] * ring[(size_t)((pos - j) % c.taps) * c.channels + ch];
+  }
+  if (keep) ring[(size_t)(pos % c.taps) * c.channels + ch] = cur;
+  return silu(s);
+}
+
 // One head of the recurrence.  A thread owns column v of the state and every `parts`-th of its
-// rows, RPT of them, in registers.
+// rows, RPT of them, in registers (parts * RPT <= kMixMaxDim; q and k are 0 past dim).
 template <int RPT>
 __device__ void recurrence_role(const MixDecode& m, int b, int h, float* lds) {
   const Recurrence& c = m.rec;
@@ -189,47 +263,44 @@ __device__ void recurrence_role(const MixDecode& m, int b, int h, float* lds) {
   float* vs = ks + 256;            // [256]
   float* al = vs + 256;            // [256] decay per key channel
   float* red = al + 256;           // [256]
-  float* red4 = red + 256;         // [4]
-  const int pos = *m.d_pos;
+  float* red2 = red + 256;         // [256]
+  float* red4 = red2 + 256;        // [8]
   const float* y = m.y + (size_t)b * m.ld_y;
   float* S = c.state + (size_t)b * c.state_seq + (size_t)h * dim * vdim;
+  const int pos = *m.d_pos;
   float st[RPT];
-  // (at position 0 the state is zero whatever the memory holds)
 #pragma unroll
   for (int j = 0; j < RPT; ++j) {
-    const int i = part + parts * j;
-    st[j] = pos > 0 && v < vdim && i < dim ? S[(size_t)i * vdim + v] : 0.0f;
+    // (past the state's end: some value of it, which meets zeros of q and k and is not stored)
+    st[j] = S[(size_t)min(part + parts * j, dim - 1) * vdim + min(v, vdim - 1)];
   }
+  const int tv = min(tid, vdim - 1);
+  const float gate = y[c.g_col + h * vdim + tv], norm = c.norm[tv];
   const int kvh = h / (c.heads / c.kv_heads);
   float beta = 1.0f, g = 1.0f;
   if (c.delta) {
     const ShortConv& cv = c.conv;
     float* ring = cv.ring + (size_t)b * cv.ring_seq;
-    const int slot = pos % cv.taps;
-    // channel ch of the convolution; the row of this position goes to the ring (no block reads it
-    // in this step)
-    auto conv = [&](int ch, bool keep) {
-      const float cur = y[cv.col + ch];
-      float s = cv.w[ch * cv.taps + cv.taps - 1] * cur;
-      for (int j = 1; j < cv.taps; ++j)
-        if (pos >= j)
-          s += cv.w[ch * cv.taps + cv.taps - 1 - j] * ring[(size_t)((pos - j) % cv.taps) * cv.channels + ch];
-      if (keep) ring[(size_t)slot * cv.channels + ch] = cur;
-      return silu(s);
-    };
     const bool first = h % (c.heads / c.kv_heads) == 0;
-    float qv = 0.0f, kv = 0.0f;
-    if (tid < dim) {
-      qv = conv(c.q_col - cv.col + kvh * dim + tid, first);
-      kv = conv(c.k_col - cv.col + kvh * dim + tid, first);
+    const float yb = y[c.b_col + h], ya = y[c.a_col + h], al0 = c.a_log[h], dt = c.dt_bias[h];
+    const int td = min(tid, dim - 1);
+    float qv = conv_channel(cv, y, ring, c.q_col - cv.col + kvh * dim + td, pos, first && tid < dim);
+    float kv = conv_channel(cv, y, ring, c.k_col - cv.col + kvh * dim + td, pos, first && tid < dim);
+    const float x = conv_channel(cv, y, ring, c.v_col - cv.col + h * vdim + tv, pos, tid < vdim);
+    if (tid >= dim) qv = kv = 0.0f;
+    vs[tid] = x;
+    float qn = wave_sum(qv * qv), kn = wave_sum(kv * kv);
+    if ((tid & 63) == 0) {
+      red4[tid >> 6] = qn;
+      red4[4 + (tid >> 6)] = kn;
     }
-    if (tid < vdim) vs[tid] = conv(c.v_col - cv.col + h * vdim + tid, true);
-    const float qn = block_sum(qv * qv, red4), kn = block_sum(kv * kv, red4);
+    __syncthreads();
+    qn = (red4[0] + red4[1]) + (red4[2] + red4[3]);
+    kn = (red4[4] + red4[5]) + (red4[6] + red4[7]);
     qs[tid] = qv / sqrtf(qn + 1e-6f) * c.q_scale;
     ks[tid] = kv / sqrtf(kn + 1e-6f);
-    beta = sigmoid(y[c.b_col + h]);
-    g = expf(delta_log_decay(y[c.a_col + h], c.a_log[h], c.dt_bias[h]));
-    al[tid] = g;
+    beta = sigmoid(yb);
+    g = expf(delta_log_decay(ya, al0, dt));
   } else {
     float qv = 0.0f, kv = 0.0f, av = 1.0f;
     if (tid < dim) {
@@ -237,13 +308,29 @@ __device__ void recurrence_role(const MixDecode& m, int b, int h, float* lds) {
       kv = y[c.k_col + h * dim + tid];
       const float* a2 = c.a2 + (size_t)(h * dim + tid) * c.rank;
       float z = c.a2_bias[h * dim + tid];
-      for (int r = 0; r < c.rank; ++r) z += a2[r] * y[c.a_col + r];
+      int r = 0;
+      for (; r + 8 <= c.rank; r += 8) {
+        float w8[8], x8[8];
+#pragma unroll
+        for (int k = 0; k < 8; ++k) {
+          w8[k] = a2[r + k];
+          x8[k] = y[c.a_col + r + k];
+        }
+#pragma unroll
+        for (int k = 0; k < 8; ++k) z += w8[k] * x8[k];
+      }
+      for (; r < c.rank; ++r) z += a2[r] * y[c.a_col + r];
       av = expf(gla_log_decay(z, c.inv_tau));
     }
     qs[tid] = qv;
     ks[tid] = kv;
     al[tid] = av;
-    if (tid < vdim) vs[tid] = y[c.v_col + h * vdim + tid];
+    vs[tid] = y[c.v_col + h * vdim + tv];
+  }
+  // (at position 0 the state is zero whatever the memory holds)
+  if (pos == 0) {
+#pragma unroll
+    for (int j = 0; j < RPT; ++j) st[j] = 0.0f;
   }
   __syncthreads();
   float u = v < vdim ? vs[v] : 0.0f;
@@ -251,39 +338,48 @@ __device__ void recurrence_role(const MixDecode& m, int b, int h, float* lds) {
     float s = 0.0f;
 #pragma unroll
     for (int j = 0; j < RPT; ++j) {
-      const int i = part + parts * j;
       st[j] *= g;
-      if (i < dim) s += st[j] * ks[i];
+      s += st[j] * ks[part + parts * j];
     }
     red[tid] = s;
     __syncthreads();
     s = 0.0f;
     for (int p = 0; p < parts; ++p) s += red[p * cols + v];
     u = beta * (u - s);
-    __syncthreads();
+  } else {
+#pragma unroll
+    for (int j = 0; j < RPT; ++j) st[j] *= al[part + parts * j];
   }
   float o = 0.0f;
 #pragma unroll
   for (int j = 0; j < RPT; ++j) {
-    const int i = part + parts * j;
-    if (i < dim) {
-      st[j] = (c.delta ? st[j] : st[j] * al[i]) + ks[i] * u;
-      o += st[j] * qs[i];
-      if (v < vdim) S[(size_t)i * vdim + v] = st[j];
+    st[j] += ks[part + parts * j] * u;
+    o += st[j] * qs[part + parts * j];
+  }
+  if (v < vdim) {
+    float* dst = S + (size_t)part * vdim + v;
+    const int n = (dim - part + parts - 1) / parts;  // rows of this thread
+    if (n >= RPT) {
+#pragma unroll
+      for (int j = 0; j < RPT; ++j) dst[(size_t)j * parts * vdim] = st[j];
+    } else {
+#pragma unroll
+      for (int j = 0; j < RPT; ++j)
+        if (j < n) dst[(size_t)j * parts * vdim] = st[j];
     }
   }
-  red[tid] = o;
+  red2[tid] = o;
   __syncthreads();
   float out = 0.0f;
   if (tid < vdim)
-    for (int p = 0; p < parts; ++p) out += red[p * cols + tid];
+    for (int p = 0; p < parts; ++p) out += red2[p * cols + tid];
   const float ss = block_sum(out * out, red4);
   if (tid < vdim)
     m.out[(size_t)b * m.ld_out + c.out_col + h * vdim + tid] =
-        out / sqrtf(ss / (float)vdim + c.eps) * c.norm[tid] * silu(y[c.g_col + h * vdim + tid]) * c.out_scale;
+        out / sqrtf(ss / (float)vdim + c.eps) * norm * silu(gate) * c.out_scale;
 }
 
-template <int RPT>
+template <int RPT, int NV>
 __global__ __launch_bounds__(256) void k_mix_decode(MixDecode m, int attn_items, int rec_items) {
   __shared__ __attribute__((aligned(16))) float lds[kDecodeLds];
   const int b = blockIdx.y;
@@ -294,7 +390,7 @@ __global__ __launch_bounds__(256) void k_mix_decode(MixDecode m, int attn_items,
   }
   item -= rec_items;
   if (item < attn_items) {
-    attn_role(m, b, item, lds);
+    attn_role<NV>(m, b, item, lds);
     return;
   }
   item -= attn_items;
@@ -309,12 +405,11 @@ __global__ __launch_bounds__(256) void k_attn_sum(MixDecode m) {
   const ChunkAttn& a = m.attn;
   const int b = blockIdx.y, i = blockIdx.x * 256 + threadIdx.x, n = a.heads * a.dim;
   if (i >= n) return;
-  const int splits = (*m.d_pos % a.chunk) / kSplitKeys + 1;
   const float* p = m.part + (size_t)b * m.attn_splits * n + i;
   float s = 0.0f;
-#pragma unroll 4
-  for (int k = 0; k < splits; ++k) s += p[(size_t)k * n];
-  m.out[(size_t)b * m.ld_out + a.out_col + i] = s * a.out_scale;
+#pragma unroll 8
+  for (int k = 0; k < m.attn_splits; ++k) s += p[(size_t)k * n];
+  m.out[(size_t)b * m.ld_out + a.out_col + i] = s;
 }
 
 // ---------------------------------------------------------------------------
@@ -344,37 +439,55 @@ __global__ __launch_bounds__(256) void k_rotary_rows(MixRows r, ChunkAttn a) {
   }
 }
 
-// A block of four wavefronts owns 128 queries of one head, 32 to a wavefront, and walks the keys
-// from the first query's chunk start to the last query, 32 at a time, staged in LDS:
-//   S^T (keys x queries) = K . Q^T, Q in registers (lane (l, half) holds dims half DP/2 ..)
+// A block owns 32 queries of one head; its NW wavefronts take the key tiles (32 keys) from the
+// first query's chunk start to the last query in turn and add their results through LDS at the
+// end (the weights are not normalised: the sums simply add).  Per tile:
+//   S^T (keys x queries) = K . Q^T, Q in registers (lane (l, half) holds dims half DP/2 ..), K rows
+//     from a wavefront-private LDS tile
 //   weights sigmoid(S scale + bias), 0 outside the query's chunk and after the query
-//   O^T (dims x queries) += V^T . P^T, a lane's own weights are the operand
+//   O^T (dims x queries) += V^T . P^T, a lane's own weights are the operand, V rows from LDS
 // Keys before pos0 come from the ring, the others from this step's rows.
-template <int DP>
-__global__ __launch_bounds__(256) void k_chunk_attn_rows(MixRows r, ChunkAttn a) {
-  constexpr int KT = 32, LD = DP + 4, NB = DP / 32, NL = KT * DP / 4 / 256;
-  __shared__ __attribute__((aligned(16))) float Ks[KT][LD];
-  __shared__ __attribute__((aligned(16))) float Vs[KT][LD];
+// Grid: x = head, y = block of queries, z = sequence.
+template <int DP, int NW>
+__global__ __launch_bounds__(64 * NW, DP <= 64 ? 2 : 1) void k_chunk_attn_rows(MixRows r, ChunkAttn a) {
+  constexpr int KT = 32, LD = DP + 4, NB = DP / 32;
+  constexpr int NL = KT * DP / 4 / 64;   // float4 loads of K (and V) per lane and tile
+  constexpr bool PRE = DP <= 128;        // the next tile waits in registers
+  __shared__ __attribute__((aligned(16))) float Ks[NW][KT * LD];
+  __shared__ __attribute__((aligned(16))) float Vs[NW][KT * LD];
+  static_assert(KT * LD / 2 >= 32 * 33 - 32 || NB == 1, "two merge tiles fit the K tile");
+  static_assert(KT * LD >= 32 * 33, "a merge tile fits the K tile");
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int half = lane >> 5, l32 = lane & 31;
   const int h = blockIdx.x, b = blockIdx.z, g = h / (a.heads / a.kv_heads);
-  const int nqb = (r.n + 127) / 128;
-  const int t0 = (nqb - 1 - (int)blockIdx.y) * 128;  // first query of the block
-  const int tq = t0 + 32 * wave + l32;               // this lane's query
+  const int nqb = (r.n + 31) / 32;
+  const int t0 = (nqb - 1 - (int)blockIdx.y) * 32;  // first query of the block
+  const int tq = t0 + l32;                          // this lane's query
   const int dim = a.dim, dp = a.dim_pad;
   const size_t row0 = (size_t)b * r.n;
   const float* yb = r.y + row0 * r.ld_y;
   const float* krb = r.k_rot + row0 * a.kv_heads * dim + g * dim;
   const float* kring = a.kring + (size_t)b * a.ring_seq + (size_t)g * a.chunk * dp;
   const float* vring = a.vring + (size_t)b * a.ring_seq + (size_t)g * a.chunk * dp;
+  const bool vec = (dim & 3) == 0;
 
   float qr[DP / 2];
   {
     const float* q = yb + (size_t)min(tq, r.n - 1) * r.ld_y + a.q_col + h * dim;
+    if (vec) {
 #pragma unroll
-    for (int s = 0; s < DP / 2; ++s) {
-      const int d = half * (DP / 2) + s;
-      qr[s] = d < dim ? q[d] : 0.0f;
+      for (int s = 0; s < DP / 2; s += 4) {
+        const int d = half * (DP / 2) + s;
+        f4 x = f4{0.f, 0.f, 0.f, 0.f};
+        if (d < dim) x = *reinterpret_cast<const f4*>(q + d);
+        qr[s] = x.x; qr[s + 1] = x.y; qr[s + 2] = x.z; qr[s + 3] = x.w;
+      }
+    } else {
+#pragma unroll
+      for (int s = 0; s < DP / 2; ++s) {
+        const int d = half * (DP / 2) + s;
+        qr[s] = d < dim ? q[d] : 0.0f;
+      }
     }
   }
   f16v o[NB];
@@ -385,237 +498,613 @@ __global__ __launch_bounds__(256) void k_chunk_attn_rows(MixRows r, ChunkAttn a)
 
   const int pq = r.pos0 + tq;                 // positions
   const int lo = pq - pq % a.chunk;           // first key this lane's query sees
-  const int pb0 = r.pos0 + t0, pb1 = r.pos0 + min(t0 + 128, r.n) - 1;
-  const int kfirst = pb0 - pb0 % a.chunk;
+  const int pb0 = r.pos0 + t0, pb1 = r.pos0 + min(t0 + 32, r.n) - 1;
+  const int kfirst = pb0 - pb0 % a.chunk, lo1 = pb1 - pb1 % a.chunk;
   const int tiles = (pb1 - kfirst) / KT + 1;
-  // this wavefront's queries
-  const int w0 = t0 + 32 * wave, wp0 = r.pos0 + w0, wp1 = r.pos0 + min(w0 + 32, r.n) - 1;
-  const int wlo0 = wp0 - wp0 % a.chunk, wlo1 = wp1 - max(wp1, 0) % a.chunk;
   const float bias = a.bias[h];
-  const bool vec = (dim & 3) == 0;
+  float* ks = Ks[wave];
+  float* vs = Vs[wave];
 
-  f4 kreg[NL], vreg[NL];
-  auto fetch = [&](int tile) {
+  auto load_row = [&](int p, int d, f4& k, f4& v) __attribute__((always_inline)) {
+    k = v = f4{0.f, 0.f, 0.f, 0.f};
+    if (p > pb1 || d >= dp) return;
+    if (p < r.pos0) {
+      const size_t at = (size_t)(p % a.chunk) * dp + d;
+      k = *reinterpret_cast<const f4*>(kring + at);
+      v = *reinterpret_cast<const f4*>(vring + at);
+    } else {
+      const int t = p - r.pos0;
+      const float* kp = krb + (size_t)t * a.kv_heads * dim + d;
+      const float* vp = yb + (size_t)t * r.ld_y + a.k_col + g * dim + d;
+      if (vec) {
+        k = *reinterpret_cast<const f4*>(kp);
+        v = *reinterpret_cast<const f4*>(vp);
+      } else {
 #pragma unroll
-    for (int i = 0; i < NL; ++i) {
-      const int idx = tid + 256 * i, key = idx / (DP / 4), d = (idx % (DP / 4)) * 4;
-      const int p = kfirst + tile * KT + key;
-      f4 k = f4{0.f, 0.f, 0.f, 0.f}, v = k;
-      if (p <= pb1 && d < dp) {
-        if (p < r.pos0) {
-          const size_t at = (size_t)(p % a.chunk) * dp + d;
-          k = *reinterpret_cast<const f4*>(kring + at);
-          v = *reinterpret_cast<const f4*>(vring + at);
-        } else {
-          const int t = p - r.pos0;
-          const float* kp = krb + (size_t)t * a.kv_heads * dim + d;
-          const float* vp = yb + (size_t)t * r.ld_y + a.k_col + g * dim + d;
-          if (vec) {
-            k = *reinterpret_cast<const f4*>(kp);
-            v = *reinterpret_cast<const f4*>(vp);
-          } else {
-#pragma unroll
-            for (int e = 0; e < 4; ++e)
-              if (d + e < dim) {
-                k[e] = kp[e];
-                v[e] = vp[e];
-              }
+        for (int e = 0; e < 4; ++e)
+          if (d + e < dim) {
+            k[e] = kp[e];
+            v[e] = vp[e];
           }
-        }
       }
-      kreg[i] = k;
-      vreg[i] = v;
     }
   };
-  fetch(0);
-  for (int tile = 0; tile < tiles; ++tile) {
-    if (tile) __syncthreads();  // the last tile has been read
+  f4 kreg[PRE ? NL : 1], vreg[PRE ? NL : 1];
+  auto fetch = [&](int tile) __attribute__((always_inline)) {
+    if constexpr (PRE) {
+#pragma unroll
+      for (int i = 0; i < NL; ++i) {
+        const int idx = lane + 64 * i;
+        load_row(kfirst + tile * KT + idx / (DP / 4), (idx % (DP / 4)) * 4, kreg[i], vreg[i]);
+      }
+    }
+  };
+  if (wave < tiles) fetch(wave);
+  for (int tile = wave; tile < tiles; tile += NW) {
+    const int k0 = kfirst + tile * KT;
 #pragma unroll
     for (int i = 0; i < NL; ++i) {
-      const int idx = tid + 256 * i, key = idx / (DP / 4), d = (idx % (DP / 4)) * 4;
-      *reinterpret_cast<f4*>(&Ks[key][d]) = kreg[i];
-      *reinterpret_cast<f4*>(&Vs[key][d]) = vreg[i];
+      const int idx = lane + 64 * i, key = idx / (DP / 4), d = (idx % (DP / 4)) * 4;
+      f4 k, v;
+      if constexpr (PRE) {
+        k = kreg[i];
+        v = vreg[i];
+      } else {
+        load_row(k0 + key, d, k, v);
+      }
+      *reinterpret_cast<f4*>(&ks[key * LD + d]) = k;
+      *reinterpret_cast<f4*>(&vs[key * LD + d]) = v;
     }
-    __syncthreads();
-    if (tile + 1 < tiles) fetch(tile + 1);
-    const int k0 = kfirst + tile * KT;
-    if (w0 >= r.n || k0 > wp1 || k0 + KT - 1 < wlo0) continue;  // (wavefront-uniform)
+    // (each wavefront has its own tile and LDS executes a wavefront's accesses in order: only the
+    // compiler has to be kept from reordering)
+    __builtin_amdgcn_wave_barrier();
+    if (tile + NW < tiles) fetch(tile + NW);
     f16v s0, s1;
 #pragma unroll
     for (int v = 0; v < 16; ++v) s0[v] = s1[v] = 0.0f;
-    const f4* krow = reinterpret_cast<const f4*>(&Ks[l32][half * (DP / 2)]);
+    // V operands of the first 32 dims are read between the MFMAs of the first product
+    float vop[16];
+    const f4* krow = reinterpret_cast<const f4*>(&ks[l32 * LD + half * (DP / 2)]);
+    f4 k = krow[0];
 #pragma unroll
     for (int j = 0; j < DP / 8; ++j) {
-      const f4 k = krow[j];
-      s0 = __builtin_amdgcn_mfma_f32_32x32x2f32(k.x, qr[4 * j], s0, 0, 0, 0);
-      s1 = __builtin_amdgcn_mfma_f32_32x32x2f32(k.y, qr[4 * j + 1], s1, 0, 0, 0);
-      s0 = __builtin_amdgcn_mfma_f32_32x32x2f32(k.z, qr[4 * j + 2], s0, 0, 0, 0);
-      s1 = __builtin_amdgcn_mfma_f32_32x32x2f32(k.w, qr[4 * j + 3], s1, 0, 0, 0);
+      const f4 kc = k;
+      s0 = __builtin_amdgcn_mfma_f32_32x32x2f32(kc.x, qr[4 * j], s0, 0, 0, 0);
+      s1 = __builtin_amdgcn_mfma_f32_32x32x2f32(kc.y, qr[4 * j + 1], s1, 0, 0, 0);
+      if (j + 1 < DP / 8) k = krow[j + 1];
+      constexpr int PER = (16 + DP / 8 - 1) / (DP / 8);
+#pragma unroll
+      for (int v = j * PER; v < (j + 1) * PER && v < 16; ++v)
+        vop[v] = vs[(8 * (v >> 2) + 4 * half + (v & 3)) * LD + l32];
+      __builtin_amdgcn_sched_barrier(0);
+      s0 = __builtin_amdgcn_mfma_f32_32x32x2f32(kc.z, qr[4 * j + 2], s0, 0, 0, 0);
+      s1 = __builtin_amdgcn_mfma_f32_32x32x2f32(kc.w, qr[4 * j + 3], s1, 0, 0, 0);
+      __builtin_amdgcn_sched_barrier(0);
     }
     s0 += s1;
     // lane holds keys k0 + 8 (v / 4) + 4 half + v % 4 of its query
-    const bool edge = k0 + KT - 1 > wp0 || k0 < wlo1;
+    const bool edge = k0 + KT - 1 > pb0 || k0 < lo1;
+    const float zs = -1.44269504088896341f * a.scale, zb = -1.44269504088896341f * bias;
 #pragma unroll
-    for (int v = 0; v < 16; ++v) {
-      const int key = k0 + 8 * (v >> 2) + 4 * half + (v & 3);
-      const float z = s0[v] * a.scale + bias;
-      const float wgt = __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.44269504088896341f * z));
-      s0[v] = !edge || (key <= pq && key >= lo) ? wgt : 0.0f;
+    for (int v = 0; v < 16; ++v)
+      s0[v] = __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(fmaf(s0[v], zs, zb)));
+    if (edge) {
+#pragma unroll
+      for (int v = 0; v < 16; ++v) {
+        const int key = k0 + 8 * (v >> 2) + 4 * half + (v & 3);
+        if (!(key <= pq && key >= lo)) s0[v] = 0.0f;
+      }
     }
 #pragma unroll
-    for (int v = 0; v < 16; ++v) {
-      const int key = 8 * (v >> 2) + 4 * half + (v & 3);
+    for (int i = 0; i < NB; ++i) {
+      if (i > 0 && !PRE) {
 #pragma unroll
-      for (int i = 0; i < NB; ++i)
-        o[i] = __builtin_amdgcn_mfma_f32_32x32x2f32(Vs[key][32 * i + l32], s0[v], o[i], 0, 0, 0);
+        for (int v = 0; v < 16; ++v) vop[v] = vs[(8 * (v >> 2) + 4 * half + (v & 3)) * LD + 32 * i + l32];
+        __builtin_amdgcn_sched_barrier(0);
+      }
+      float nx[16];
+#pragma unroll
+      for (int v = 0; v < 16; ++v) {
+        o[i] = __builtin_amdgcn_mfma_f32_32x32x2f32(vop[v], s0[v], o[i], 0, 0, 0);
+        if (PRE && i + 1 < NB) nx[v] = vs[(8 * (v >> 2) + 4 * half + (v & 3)) * LD + 32 * (i + 1) + l32];
+      }
+      if (PRE && i + 1 < NB) {
+#pragma unroll
+        for (int v = 0; v < 16; ++v) vop[v] = nx[v];
+      }
+    }
+    __builtin_amdgcn_wave_barrier();
+  }
+  // the wavefronts' sums, in wavefront order: [dim][query] tiles, 32 dims at a time
+  float* dst = r.out + (row0 + min(tq, r.n - 1)) * r.ld_out + a.out_col + h * dim;
+  __syncthreads();
+#pragma unroll
+  for (int i = 0; i < NB; ++i) {
+    float* ob = ks + (i & 1) * (KT * LD / 2);
+#pragma unroll
+    for (int v = 0; v < 16; ++v) ob[(8 * (v >> 2) + 4 * half + (v & 3)) * 33 + l32] = o[i][v];
+    __syncthreads();
+    // lane (query l32, half) of wavefront w sums dims [32 / NW w, ..) of the tile
+    constexpr int ND = 32 / NW / 2;
+#pragma unroll
+    for (int e = 0; e < ND; ++e) {
+      const int d = (32 / NW) * wave + ND * half + e;
+      float sum = 0.0f;
+#pragma unroll
+      for (int w = 0; w < NW; ++w) sum += Ks[w][(i & 1) * (KT * LD / 2) + d * 33 + l32];
+      if (tq < r.n && 32 * i + d < dim) dst[32 * i + d] = sum * a.out_scale;
     }
   }
-  if (tq >= r.n) return;
-  float* dst = r.out + (row0 + tq) * r.ld_out + a.out_col + h * dim;
-#pragma unroll
-  for (int i = 0; i < NB; ++i)
-#pragma unroll
-    for (int v = 0; v < 16; ++v) {
-      const int d = 32 * i + 8 * (v >> 2) + 4 * half + (v & 3);
-      if (d < dim) dst[d] = o[i][v] * a.out_scale;
-    }
 }
 
+// A thread owns one channel of kConvRows consecutive tokens; up to TAPS - 1 inputs before them.
+constexpr int kConvRows = 16;
+template <int TAPS>
 __global__ __launch_bounds__(256) void k_short_conv_rows(MixRows r, ShortConv c) {
-  const int ch = blockIdx.x * 256 + threadIdx.x, row = blockIdx.y;
+  const int ch = blockIdx.x * 256 + threadIdx.x, b = blockIdx.z, t0 = blockIdx.y * kConvRows;
   if (ch >= c.channels) return;
-  const int b = row / r.n, t = row - b * r.n, pos = r.pos0 + t;
-  const float* w = c.w + ch * c.taps;
-  const float* ring = c.ring + (size_t)b * c.ring_seq;
-  float s = 0.0f;
-  for (int j = 0; j < c.taps; ++j) {
-    if (pos < j) break;
-    const float x = t >= j ? r.y[(size_t)(row - j) * r.ld_y + c.col + ch]
-                           : ring[(size_t)((pos - j) % c.taps) * c.channels + ch];
-    s += w[c.taps - 1 - j] * x;
+  const float* x = r.y + (size_t)b * r.n * r.ld_y + c.col + ch;
+  const float* ring = c.ring + (size_t)b * c.ring_seq + ch;
+  float w[TAPS], in[TAPS - 1 + kConvRows];
+#pragma unroll
+  for (int j = 0; j < TAPS; ++j) w[j] = j < c.taps ? c.w[ch * c.taps + c.taps - 1 - j] : 0.0f;  // j tokens back
+#pragma unroll
+  for (int i = 0; i < TAPS - 1 + kConvRows; ++i) {
+    const int t = t0 + i - (TAPS - 1), pos = r.pos0 + t;
+    in[i] = 0.0f;
+    if (t >= 0) {
+      in[i] = x[(size_t)min(t, r.n - 1) * r.ld_y];
+    } else if (pos >= 0 && -t < c.taps) {
+      in[i] = ring[(size_t)(pos % c.taps) * c.channels];
+    }
   }
-  r.conv_out[(size_t)row * c.channels + ch] = silu(s);
+#pragma unroll
+  for (int i = 0; i < kConvRows; ++i) {
+    if (t0 + i >= r.n) return;
+    float s = 0.0f;
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) s += w[j] * in[TAPS - 1 + i - j];
+    r.conv_out[((size_t)b * r.n + t0 + i) * c.channels + ch] = silu(s);
+  }
 }
 
-// log alpha of gated linear attention
-__global__ __launch_bounds__(256) void k_gla_decay_rows(MixRows r, Recurrence c) {
-  const int i = blockIdx.x * 256 + threadIdx.x, row = blockIdx.y, n = c.heads * c.dim;
+// log alpha of gated linear attention: a thread owns one channel of kDecayRows tokens
+constexpr int kDecayRows = 16, kDecayRank = 16;
+__global__ __launch_bounds__(256) void k_gla_decay_rows(MixRows r, Recurrence c, int rows) {
+  __shared__ float a1[kDecayRows][kDecayRank];
+  const int tid = threadIdx.x, i = blockIdx.x * 256 + tid, n = c.heads * c.dim, row0 = blockIdx.y * kDecayRows;
+  const int ii = min(i, n - 1);
+  float z[kDecayRows];
+#pragma unroll
+  for (int t = 0; t < kDecayRows; ++t) z[t] = c.a2_bias[ii];
+  for (int k0 = 0; k0 < c.rank; k0 += kDecayRank) {
+    float w[kDecayRank];
+#pragma unroll
+    for (int k = 0; k < kDecayRank; ++k) w[k] = k0 + k < c.rank ? c.a2[(size_t)ii * c.rank + k0 + k] : 0.0f;
+    __syncthreads();
+    {
+      const int t = tid / kDecayRank, k = tid % kDecayRank;
+      a1[t][k] = k0 + k < c.rank && row0 + t < rows ? r.y[(size_t)(row0 + t) * r.ld_y + c.a_col + k0 + k] : 0.0f;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int t = 0; t < kDecayRows; ++t)
+#pragma unroll
+      for (int k = 0; k < kDecayRank; ++k) z[t] += w[k] * a1[t][k];
+  }
   if (i >= n) return;
-  const float* a1 = r.y + (size_t)row * r.ld_y + c.a_col;
-  float z = c.a2_bias[i];
-  for (int k = 0; k < c.rank; ++k) z += c.a2[(size_t)i * c.rank + k] * a1[k];
-  r.decay[(size_t)row * n + i] = gla_log_decay(z, c.inv_tau);
+#pragma unroll
+  for (int t = 0; t < kDecayRows; ++t)
+    if (row0 + t < rows) r.decay[(size_t)(row0 + t) * n + i] = gla_log_decay(z[t], c.inv_tau);
 }
 
-// The recurrence token by token; a block owns one head of one sequence (layout of
-// recurrence_role).
-template <int RPT>
-__global__ __launch_bounds__(256) void k_recurrence_scan(MixRows r, Recurrence c) {
-  __shared__ float qs[256], ks[256], vs[256], al[256], red[256], red4[4];
-  const int tid = threadIdx.x, h = blockIdx.x, b = blockIdx.y;
-  const int dim = c.dim, vdim = c.vdim;
-  int cols = 1;
-  while (cols < vdim) cols <<= 1;
-  const int parts = 256 / cols, v = tid % cols, part = tid / cols;
-  float* S = c.state + (size_t)b * c.state_seq + (size_t)h * dim * vdim;
-  float st[RPT];
-#pragma unroll
-  for (int j = 0; j < RPT; ++j) {
-    const int i = part + parts * j;
-    st[j] = r.pos0 > 0 && v < vdim && i < dim ? S[(size_t)i * vdim + v] : 0.0f;
+// ---------------------------------------------------------------------------
+// The recurrences over many rows, kChunk tokens at a time.  With G_t the sum of the log decays of
+// a chunk's tokens up to t (per head, or per key channel), S0 the state before the chunk and
+//   Kd_t = exp(G_end - G_t) k_t,  Qd_t = exp(G_t) q_t,  P_tj = q_t . (exp(G_t - G_j) k_j), j <= t
+// the chunk's tokens write U into the state and read it out as
+//   S_end = exp(G_end) S0 + Kd^T U,   O = Qd S0 + P U,
+// where U = V for gated linear attention and, for the delta rule (whose k_t first reads the state),
+//   U = U0 - W S0,  (1 + A) [U0 | W] = [beta V | beta exp(G) K],  A_tj = beta_t exp(G_t - G_j) k_t . k_j, j < t.
+// All exponents are <= 0.  Three launches: the parts that need no state for every chunk at once,
+// the states from chunk to chunk (the only serial part), the read-outs for every chunk at once.
+// A chunk's tiles lie in the work area one after the other, 32 rows each, widths padded to
+// 32 (pads and rows past the end are zeros).
+// ---------------------------------------------------------------------------
+constexpr int kChunk = 32;
+
+struct ChunkWork {
+  int chunks;            // per sequence
+  int dp, ep;            // dim and vdim padded to 32
+  float *W, *U0, *Kd, *Qd, *P, *U, *S, *G;
+  // tile (sequence, chunk, head): W, Kd, Qd [32][dp]; U0, U [32][ep]; P [32][32]; S [dp][ep]; G [dp]
+  // (exp(G_end) per key channel)
+  __device__ __forceinline__ size_t tile(int b, int c, int h, int heads) const {
+    return ((size_t)b * chunks + c) * heads + h;
   }
+};
+
+// Floats of a sequence's work area per chunk and head.
+__host__ __device__ inline size_t chunk_floats(int dp, int ep, bool delta) {
+  return (size_t)32 * ((delta ? 3 : 2) * dp + (delta ? 2 : 1) * ep + 32) + (size_t)dp * ep + dp;
+}
+
+// One tile of 32 x 32 dot products over dp columns: rows x of X against rows of Y (LDS, LD apart),
+// columns [k0, k1); lane layout of v_mfma_f32_32x32x2_f32.
+__device__ __forceinline__ f16v dots32(const float* X, const float* Y, int LD, int k0, int k1, int lane) {
+  const int half = lane >> 5, l32 = lane & 31, n = (k1 - k0) / 2;
+  f16v s;
+#pragma unroll
+  for (int v = 0; v < 16; ++v) s[v] = 0.0f;
+  const float* x = X + l32 * LD + k0 + half * n;
+  const float* y = Y + l32 * LD + k0 + half * n;
+  for (int j = 0; j < n; j += 4) {
+    const f4 a = *reinterpret_cast<const f4*>(x + j), b = *reinterpret_cast<const f4*>(y + j);
+    s = __builtin_amdgcn_mfma_f32_32x32x2f32(a.x, b.x, s, 0, 0, 0);
+    s = __builtin_amdgcn_mfma_f32_32x32x2f32(a.y, b.y, s, 0, 0, 0);
+    s = __builtin_amdgcn_mfma_f32_32x32x2f32(a.z, b.z, s, 0, 0, 0);
+    s = __builtin_amdgcn_mfma_f32_32x32x2f32(a.w, b.w, s, 0, 0, 0);
+  }
+  return s;
+}
+
+// Delta rule, per (chunk, head, sequence): U0, W, Kd, Qd, P, G.
+__global__ __launch_bounds__(256) void k_delta_chunk(MixRows r, Recurrence c, ChunkWork w) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  __shared__ double Gs[kChunk];
+  __shared__ float beta[kChunk], eg[kChunk], ek[kChunk];
+  __shared__ float red[4][32 * 33];
+  __shared__ __attribute__((aligned(16))) float As[32][36];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int half = lane >> 5, l32 = lane & 31;
+  const int ci = blockIdx.x, h = blockIdx.y, b = blockIdx.z;
+  const int dim = c.dim, vdim = c.vdim, dp = w.dp, ep = w.ep, LD = dp + 4;
+  float* Ks = lds;            // [32][LD]
+  float* Qs = lds + 32 * LD;
+  const int t0 = ci * kChunk, nt = min(kChunk, r.n - t0);
+  const size_t row0 = (size_t)b * r.n + t0;
   const int kvh = h / (c.heads / c.kv_heads);
-  for (int t = 0; t < r.n; ++t) {
-    const size_t row = (size_t)b * r.n + t;
-    const float* y = r.y + row * r.ld_y;
-    float beta = 1.0f, g = 1.0f;
-    if (c.delta) {
-      const float* x = r.conv_out + row * c.conv.channels;
-      float qv = 0.0f, kv = 0.0f;
-      if (tid < dim) {
-        qv = x[c.q_col - c.conv.col + kvh * dim + tid];
-        kv = x[c.k_col - c.conv.col + kvh * dim + tid];
+  const int CH = c.conv.channels;
+  const float* xq = r.conv_out + row0 * CH + (c.q_col - c.conv.col) + kvh * dim;
+  const float* xk = r.conv_out + row0 * CH + (c.k_col - c.conv.col) + kvh * dim;
+  const float* xv = r.conv_out + row0 * CH + (c.v_col - c.conv.col) + h * vdim;
+  {
+    // eight threads to a row: q and k as unit vectors
+    const int t = tid >> 3, sub = tid & 7;
+    float qq = 0.0f, kk = 0.0f;
+#pragma unroll 4
+    for (int i = sub; i < dp; i += 8) {
+      float q = 0.0f, k = 0.0f;
+      if (t < nt && i < dim) {
+        q = xq[(size_t)t * CH + i];
+        k = xk[(size_t)t * CH + i];
       }
-      const float qn = block_sum(qv * qv, red4), kn = block_sum(kv * kv, red4);
-      qs[tid] = qv / sqrtf(qn + 1e-6f) * c.q_scale;
-      ks[tid] = kv / sqrtf(kn + 1e-6f);
-      if (tid < vdim) vs[tid] = x[c.v_col - c.conv.col + h * vdim + tid];
-      beta = sigmoid(y[c.b_col + h]);
-      g = expf(delta_log_decay(y[c.a_col + h], c.a_log[h], c.dt_bias[h]));
-    } else {
-      if (tid < dim) {
-        qs[tid] = y[c.q_col + h * dim + tid] * c.q_scale;
-        ks[tid] = y[c.k_col + h * dim + tid];
-        al[tid] = expf(r.decay[row * c.heads * dim + h * dim + tid]);
-      }
-      if (tid < vdim) vs[tid] = y[c.v_col + h * vdim + tid];
+      Qs[t * LD + i] = q;
+      Ks[t * LD + i] = k;
+      qq += q * q;
+      kk += k * k;
     }
-    __syncthreads();
-    float u = v < vdim ? vs[v] : 0.0f;
-    if (c.delta) {
-      float s = 0.0f;
 #pragma unroll
-      for (int j = 0; j < RPT; ++j) {
-        const int i = part + parts * j;
-        st[j] *= g;
-        if (i < dim) s += st[j] * ks[i];
-      }
-      red[tid] = s;
-      __syncthreads();
-      s = 0.0f;
-      for (int p = 0; p < parts; ++p) s += red[p * cols + v];
-      u = beta * (u - s);
-      __syncthreads();
+    for (int off = 4; off > 0; off >>= 1) {
+      qq += __shfl_xor(qq, off, 64);
+      kk += __shfl_xor(kk, off, 64);
     }
-    float o = 0.0f;
-#pragma unroll
-    for (int j = 0; j < RPT; ++j) {
-      const int i = part + parts * j;
-      if (i < dim) {
-        st[j] = (c.delta ? st[j] : st[j] * al[i]) + ks[i] * u;
-        o += st[j] * qs[i];
-      }
+    const float qm = c.q_scale / sqrtf(qq + 1e-6f), km = 1.0f / sqrtf(kk + 1e-6f);
+    for (int i = sub; i < dp; i += 8) {
+      Qs[t * LD + i] *= qm;
+      Ks[t * LD + i] *= km;
     }
-    red[tid] = o;
-    __syncthreads();
-    if (tid < vdim) {
-      float out = 0.0f;
-      for (int p = 0; p < parts; ++p) out += red[p * cols + tid];
-      r.o[row * c.heads * vdim + h * vdim + tid] = out;
-    }
-    __syncthreads();
   }
+  if (wave == 0) {
+    double g = 0.0;
+    float bt = 0.0f;
+    if (lane < nt) {
+      const float* y = r.y + (row0 + lane) * r.ld_y;
+      bt = sigmoid(y[c.b_col + h]);
+      g = (double)delta_log_decay(y[c.a_col + h], c.a_log[h], c.dt_bias[h]);
+    }
 #pragma unroll
-  for (int j = 0; j < RPT; ++j) {
-    const int i = part + parts * j;
-    if (v < vdim && i < dim) S[(size_t)i * vdim + v] = st[j];
+    for (int off = 1; off < 32; off <<= 1) {
+      const double up = __shfl_up(g, off, 64);
+      if (lane >= off) g += up;
+    }
+    const double end = __shfl(g, 31, 64);  // (tokens past the end decay by nothing)
+    if (lane < 32) {
+      Gs[lane] = g;
+      beta[lane] = bt;
+      eg[lane] = expf((float)g);
+      ek[lane] = expf((float)(end - g));
+    }
+  }
+  __syncthreads();
+  const size_t tile = w.tile(b, ci, h, c.heads);
+  {
+    // wavefronts 0, 1: k . k over half of the columns each; 2, 3: q . k
+    const int k0 = (wave & 1) * (dp / 2);
+    const f16v s = dots32(wave < 2 ? Ks : Qs, Ks, LD, k0, k0 + dp / 2, lane);
+#pragma unroll
+    for (int v = 0; v < 16; ++v) red[wave][(8 * (v >> 2) + 4 * half + (v & 3)) * 33 + l32] = s[v];
+  }
+  __syncthreads();
+  for (int i = tid; i < 1024; i += 256) {
+    const int t = i >> 5, j = i & 31, at = t * 33 + j;
+    const float e = j <= t ? expf((float)(Gs[t] - Gs[j])) : 0.0f;
+    As[t][j] = j < t ? beta[t] * e * (red[0][at] + red[1][at]) : 0.0f;
+    w.P[tile * 1024 + i] = e * (red[2][at] + red[3][at]);
+  }
+  __syncthreads();
+  // columns of [W | U0] by forward substitution, one per thread
+  for (int col = tid; col < dp + ep; col += 256) {
+    const bool isw = col < dp;
+    const int e = col - dp;
+    float x[kChunk];
+#pragma unroll
+    for (int t = 0; t < kChunk; ++t) {
+      float v = 0.0f;
+      if (isw) v = eg[t] * Ks[t * LD + col];
+      else if (t < nt && e < vdim) v = xv[(size_t)t * CH + e];
+      x[t] = beta[t] * v;
+    }
+#pragma unroll
+    for (int t = 1; t < kChunk; ++t) {
+      float s = x[t];
+#pragma unroll
+      for (int j = 0; j < t; j += 4) {
+        const f4 a4 = *reinterpret_cast<const f4*>(&As[t][j]);
+#pragma unroll
+        for (int k = 0; k < 4; ++k)
+          if (j + k < t) s -= a4[k] * x[j + k];
+      }
+      x[t] = s;
+      __builtin_amdgcn_sched_barrier(0);  // (row by row: all rows of A at once do not fit the registers)
+    }
+    float* dst = isw ? w.W + tile * 32 * dp + col : w.U0 + tile * 32 * ep + e;
+    const int ld = isw ? dp : ep;
+#pragma unroll
+    for (int t = 0; t < kChunk; ++t) dst[t * ld] = x[t];
+  }
+  for (int i = tid; i < 32 * dp; i += 256) {
+    const int t = i / dp, d = i - t * dp;
+    w.Kd[tile * 32 * dp + i] = ek[t] * Ks[t * LD + d];
+    w.Qd[tile * 32 * dp + i] = eg[t] * Qs[t * LD + d];
+  }
+  for (int i = tid; i < dp; i += 256) w.G[tile * dp + i] = eg[31];
+}
+
+// Gated linear attention, per (chunk, head, sequence): U (= V), Kd, Qd, P, G.
+__global__ __launch_bounds__(256) void k_gla_chunk(MixRows r, Recurrence c, ChunkWork w) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const int tid = threadIdx.x;
+  const int ci = blockIdx.x, h = blockIdx.y, b = blockIdx.z;
+  const int dim = c.dim, vdim = c.vdim, dp = w.dp, ep = w.ep, LD = dp + 1;
+  float* Ks = lds;  // [32][LD] each
+  float* Qs = lds + 32 * LD;
+  float* Gs = lds + 64 * LD;
+  const int t0 = ci * kChunk, nt = min(kChunk, r.n - t0);
+  const size_t row0 = (size_t)b * r.n + t0;
+  const size_t tile = w.tile(b, ci, h, c.heads);
+  for (int i = tid; i < 32 * dp; i += 256) {
+    const int t = i / dp, d = i - t * dp;
+    float q = 0.0f, k = 0.0f, g = 0.0f;
+    if (t < nt && d < dim) {
+      const float* y = r.y + (row0 + t) * r.ld_y + h * dim + d;
+      q = y[c.q_col] * c.q_scale;
+      k = y[c.k_col];
+      g = r.decay[(row0 + t) * c.heads * dim + h * dim + d];
+    }
+    Qs[t * LD + d] = q;
+    Ks[t * LD + d] = k;
+    Gs[t * LD + d] = g;
+  }
+  for (int i = tid; i < 32 * ep; i += 256) {
+    const int t = i / ep, e = i - t * ep;
+    w.U[tile * 32 * ep + i] = t < nt && e < vdim ? r.y[(row0 + t) * r.ld_y + c.v_col + h * vdim + e] : 0.0f;
+  }
+  __syncthreads();
+  for (int d = tid; d < dp; d += 256) {
+    float s = 0.0f;
+#pragma unroll
+    for (int t = 0; t < kChunk; ++t) {
+      s += Gs[t * LD + d];
+      Gs[t * LD + d] = s;
+    }
+    w.G[tile * dp + d] = expf(s);
+  }
+  __syncthreads();
+  for (int i = tid; i < 1024; i += 256) {
+    const int t = i >> 5, j = i & 31;
+    float s = 0.0f;
+    if (j <= t) {
+      const float *q = Qs + t * LD, *k = Ks + j * LD, *gt = Gs + t * LD, *gj = Gs + j * LD;
+#pragma unroll 8
+      for (int d = 0; d < dim; ++d) s += q[d] * k[d] * __builtin_amdgcn_exp2f(1.44269504088896341f * (gt[d] - gj[d]));
+    }
+    w.P[tile * 1024 + i] = s;
+  }
+  for (int i = tid; i < 32 * dp; i += 256) {
+    const int t = i / dp, d = i - t * dp;
+    const float g = Gs[t * LD + d];
+    w.Kd[tile * 32 * dp + i] = expf(Gs[31 * LD + d] - g) * Ks[t * LD + d];
+    w.Qd[tile * 32 * dp + i] = expf(g) * Qs[t * LD + d];
   }
 }
 
-// One wavefront per (row, head).
-__global__ __launch_bounds__(256) void k_gated_norm_rows(MixRows r, Recurrence c, int rows) {
-  const int lane = threadIdx.x & 63;
-  const int item = blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (item >= rows * c.heads) return;
-  const int row = item / c.heads, h = item - row * c.heads;
-  const float* o = r.o + (size_t)item * c.vdim;
-  float x[kMixMaxDim / 64], ss = 0.0f;
+// The states from chunk to chunk.  A block owns 32 value columns of one head; wavefront w keeps
+// the state's rows 32 w .. 32 w + 31 in the accumulator layout of the 32 x 32 MFMA, where register
+// v of lane (l, half) is row 8 (v / 4) + 4 half + v % 4 of column l.  In that layout the state is
+// an operand of W S as it is (step v multiplies the rows its two lane halves hold), and so is U
+// of Kd^T U.  The wavefronts' parts of W S meet in LDS, two buffers in turn.  The next chunk's
+// tiles are requested a chunk ahead.
+template <bool DELTA>
+__global__ __launch_bounds__(512) void k_chunk_states(MixRows r, Recurrence c, ChunkWork w) {
+  extern __shared__ float part[];  // [2][waves][16][64] (delta)
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, waves = blockDim.x >> 6;
+  const int half = lane >> 5, l32 = lane & 31;
+  const int ct = blockIdx.x, h = blockIdx.y, b = blockIdx.z;
+  const int dp = w.dp, ep = w.ep, dim = c.dim, vdim = c.vdim;
+  const int col = 32 * ct + l32;
+  float* state = c.state + (size_t)b * c.state_seq + (size_t)h * dim * vdim;
+  auto row_of = [&](int v) { return 8 * (v >> 2) + 4 * half + (v & 3); };
+  f16v S;
 #pragma unroll
-  for (int j = 0; j < kMixMaxDim / 64; ++j) {
-    const int e = lane + 64 * j;
-    x[j] = e < c.vdim ? o[e] : 0.0f;
-    ss += x[j] * x[j];
+  for (int v = 0; v < 16; ++v) {
+    const int i = 32 * wave + row_of(v);
+    S[v] = r.pos0 > 0 && i < dim && col < vdim ? state[(size_t)i * vdim + col] : 0.0f;
   }
-  const float inv = c.out_scale / sqrtf(wave_sum(ss) / (float)c.vdim + c.eps);
-  const float* gate = r.y + (size_t)row * r.ld_y + c.g_col + h * c.vdim;
-  float* dst = r.out + (size_t)row * r.ld_out + c.out_col + h * c.vdim;
+  f4 nw[4];
+  float nk[16], nu[16];
+  f4 ng[4];
+  auto fetch = [&](int ci) __attribute__((always_inline)) {
+    const size_t tile = w.tile(b, ci, h, c.heads);
+    const float* u = (DELTA ? w.U0 : w.U) + tile * 32 * ep + col;
+    const float* kd = w.Kd + tile * 32 * dp + 32 * wave + l32;
+    const float* g = w.G + tile * dp + 32 * wave + 4 * half;
+    if (DELTA) {
+      const float* wt = w.W + tile * 32 * dp + (size_t)l32 * dp + 32 * wave + 4 * half;
 #pragma unroll
-  for (int j = 0; j < kMixMaxDim / 64; ++j) {
-    const int e = lane + 64 * j;
-    if (e < c.vdim) dst[e] = x[j] * inv * c.norm[e] * silu(gate[e]);
+      for (int q = 0; q < 4; ++q) nw[q] = *reinterpret_cast<const f4*>(wt + 8 * q);
+    }
+#pragma unroll
+    for (int v = 0; v < 16; ++v) {
+      nu[v] = u[row_of(v) * ep];
+      nk[v] = kd[row_of(v) * dp];
+    }
+#pragma unroll
+    for (int q = 0; q < 4; ++q) ng[q] = *reinterpret_cast<const f4*>(g + 8 * q);
+  };
+  fetch(0);
+  for (int ci = 0; ci < w.chunks; ++ci) {
+    const size_t tile = w.tile(b, ci, h, c.heads);
+    f4 cw[4], cg[4];
+    float ck[16], u[16];
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      if (DELTA) cw[q] = nw[q];
+      cg[q] = ng[q];
+    }
+#pragma unroll
+    for (int v = 0; v < 16; ++v) {
+      ck[v] = nk[v];
+      u[v] = nu[v];
+    }
+    if (ci + 1 < w.chunks) fetch(ci + 1);
+    float* s0 = w.S + tile * dp * ep + (size_t)(32 * wave) * ep + col;
+#pragma unroll
+    for (int v = 0; v < 16; ++v) s0[row_of(v) * ep] = S[v];
+    if (DELTA) {
+      f16v p;
+#pragma unroll
+      for (int v = 0; v < 16; ++v) p[v] = 0.0f;
+#pragma unroll
+      for (int v = 0; v < 16; ++v) p = __builtin_amdgcn_mfma_f32_32x32x2f32(cw[v >> 2][v & 3], S[v], p, 0, 0, 0);
+      float* mine = part + (size_t)((ci & 1) * waves + wave) * 1024 + lane;
+#pragma unroll
+      for (int v = 0; v < 16; ++v) mine[64 * v] = p[v];
+      __syncthreads();
+      const float* all = part + (size_t)((ci & 1) * waves) * 1024 + lane;
+      for (int o = 0; o < waves; ++o)
+#pragma unroll
+        for (int v = 0; v < 16; ++v) u[v] -= all[(size_t)o * 1024 + 64 * v];
+      float* ud = w.U + tile * 32 * ep + col;
+#pragma unroll
+      for (int v = 0; v < 16; ++v)
+        if (v % waves == wave) ud[row_of(v) * ep] = u[v];
+    }
+#pragma unroll
+    for (int v = 0; v < 16; ++v) S[v] *= cg[v >> 2][v & 3];
+#pragma unroll
+    for (int v = 0; v < 16; ++v) S = __builtin_amdgcn_mfma_f32_32x32x2f32(ck[v], u[v], S, 0, 0, 0);
   }
-  if (h == 0)
-    for (int e = r.out_cols + lane; e < r.ld_out; e += 64) r.out[(size_t)row * r.ld_out + e] = 0.0f;
+#pragma unroll
+  for (int v = 0; v < 16; ++v) {
+    const int i = 32 * wave + row_of(v);
+    if (i < dim && col < vdim) state[(size_t)i * vdim + col] = S[v];
+  }
+}
+
+// The read-outs of one (chunk, head, sequence), normalised, gated and written to the mixer outputs.
+// A wavefront owns the 32-column tiles wave and wave + 4.
+__global__ __launch_bounds__(256) void k_chunk_out(MixRows r, Recurrence c, ChunkWork w) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  __shared__ __attribute__((aligned(16))) float Ps[32][36];
+  __shared__ float ss[4][32];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int half = lane >> 5, l32 = lane & 31;
+  const int ci = blockIdx.x, h = blockIdx.y, b = blockIdx.z;
+  const int dp = w.dp, ep = w.ep, vdim = c.vdim, LD = dp + 4;
+  const int t0 = ci * kChunk, nt = min(kChunk, r.n - t0);
+  const size_t row0 = (size_t)b * r.n + t0, tile = w.tile(b, ci, h, c.heads);
+  float* Qs = lds;
+  for (int i = tid; i < 8 * dp; i += 256) {
+    const int t = i / (dp / 4), d = (i - t * (dp / 4)) * 4;
+    *reinterpret_cast<f4*>(&Qs[t * LD + d]) = *reinterpret_cast<const f4*>(w.Qd + tile * 32 * dp + t * dp + d);
+  }
+  {
+    const int t = tid >> 3, d = (tid & 7) * 4;
+    *reinterpret_cast<f4*>(&Ps[t][d]) = *reinterpret_cast<const f4*>(w.P + tile * 1024 + t * 32 + d);
+  }
+  __syncthreads();
+  const int tiles = ep / 32;
+  f16v o[2];
+#pragma unroll
+  for (int v = 0; v < 16; ++v) o[0][v] = o[1][v] = 0.0f;
+#pragma unroll
+  for (int k = 0; k < 2; ++k) {
+    const int ct = wave + 4 * k;
+    if (ct >= tiles) break;
+    // rows half * dp / 2 + j of the state meet columns half * dp / 2 + j of Qd
+    const float* s = w.S + tile * dp * ep + (size_t)(half * (dp / 2)) * ep + 32 * ct + l32;
+    const float* q = Qs + l32 * LD + half * (dp / 2);
+    for (int j = 0; j < dp / 2; j += 16) {
+      float sv[16];
+#pragma unroll
+      for (int e = 0; e < 16; ++e) sv[e] = s[(size_t)(j + e) * ep];
+#pragma unroll
+      for (int e = 0; e < 16; e += 4) {
+        const f4 a4 = *reinterpret_cast<const f4*>(q + j + e);
+#pragma unroll
+        for (int k4 = 0; k4 < 4; ++k4) o[k] = __builtin_amdgcn_mfma_f32_32x32x2f32(a4[k4], sv[e + k4], o[k], 0, 0, 0);
+      }
+    }
+    const float* u = w.U + tile * 32 * ep + (size_t)(16 * half) * ep + 32 * ct + l32;
+    float uv[16];
+#pragma unroll
+    for (int e = 0; e < 16; ++e) uv[e] = u[e * ep];
+#pragma unroll
+    for (int e = 0; e < 16; e += 4) {
+      const f4 a4 = *reinterpret_cast<const f4*>(&Ps[l32][16 * half + e]);
+#pragma unroll
+      for (int k4 = 0; k4 < 4; ++k4) o[k] = __builtin_amdgcn_mfma_f32_32x32x2f32(a4[k4], uv[e + k4], o[k], 0, 0, 0);
+    }
+  }
+  // sums of squares per token: over the 32 lanes of a half, then over the wavefronts
+#pragma unroll
+  for (int v = 0; v < 16; ++v) {
+    float x = o[0][v] * o[0][v] + o[1][v] * o[1][v];
+#pragma unroll
+    for (int off = 16; off > 0; off >>= 1) x += __shfl_xor(x, off, 64);
+    if (l32 == 0) ss[wave][8 * (v >> 2) + 4 * half + (v & 3)] = x;
+  }
+  __syncthreads();
+#pragma unroll
+  for (int k = 0; k < 2; ++k) {
+    const int e = 32 * (wave + 4 * k) + l32;
+    if (e >= vdim) break;
+    const float norm = c.norm[e] * c.out_scale;
+#pragma unroll
+    for (int v = 0; v < 16; ++v) {
+      const int t = 8 * (v >> 2) + 4 * half + (v & 3);
+      if (t >= nt) continue;
+      const float sq = (ss[0][t] + ss[1][t]) + (ss[2][t] + ss[3][t]);
+      const size_t row = row0 + t;
+      r.out[row * r.ld_out + c.out_col + h * vdim + e] =
+          o[k][v] / sqrtf(sq / (float)vdim + c.eps) * norm * silu(r.y[row * r.ld_y + c.g_col + h * vdim + e]);
+    }
+  }
+  if (h == 0) {  // padding columns of the mixer outputs
+    const int pad = r.ld_out - r.out_cols;
+    for (int i = tid; i < nt * pad; i += 256) r.out[(row0 + i / pad) * r.ld_out + r.out_cols + i % pad] = 0.0f;
+  }
 }
 
 __global__ __launch_bounds__(256) void k_gated_mlp_rows(MixRows r, GatedMlp m) {
@@ -665,12 +1154,12 @@ __global__ __launch_bounds__(256) void k_rms_rows(const float* src, float* dst, 
 __global__ void k_set_int(int* p, int value) { *p = value; }
 __global__ void k_add_one(int* p) { *p += 1; }
 
-// Rows of a state column per thread (kernels with RPT): the next power of two.
+// Rows of a state column per thread (recurrence_role): the next power of two.
 int rows_per_thread(int dim, int vdim) {
   int cols = 1;
   while (cols < vdim) cols <<= 1;
   const int need = (dim + 256 / cols - 1) / (256 / cols);
-  int rpt = 4;
+  int rpt = 1;
   while (rpt < need) rpt <<= 1;
   return rpt;
 }
@@ -689,12 +1178,15 @@ hipError_t launch_mix_decode(const MixDecode& a, hipStream_t s) {
   const int mlp_items = a.has_mlp ? (a.mlp.ff_pad + 255) / 256 : 0;
   const dim3 grid((unsigned)(attn_items + rec_items + mlp_items), (unsigned)a.nseq);
   if (grid.x == 0) return hipSuccess;
-  switch (a.has_rec ? rows_per_thread(a.rec.dim, a.rec.vdim) : 4) {
-#define PG_RPT(N)                                                                        \
-  case N:                                                                                \
-    hipLaunchKernelGGL(k_mix_decode<N>, grid, dim3(256), 0, s, a, attn_items, rec_items); \
+  const int nv = !a.has_attn || a.attn.dim_pad <= 64 ? 1 : a.attn.dim_pad <= 128 ? 2 : 4;
+  switch (a.has_rec ? rows_per_thread(a.rec.dim, a.rec.vdim) : 1) {
+#define PG_RPT(N)                                                                                               \
+  case N:                                                                                                       \
+    if (nv == 1) hipLaunchKernelGGL((k_mix_decode<N, 1>), grid, dim3(256), 0, s, a, attn_items, rec_items);      \
+    else if (nv == 2) hipLaunchKernelGGL((k_mix_decode<N, 2>), grid, dim3(256), 0, s, a, attn_items, rec_items); \
+    else hipLaunchKernelGGL((k_mix_decode<N, 4>), grid, dim3(256), 0, s, a, attn_items, rec_items);              \
     break;
-    PG_RPT(4) PG_RPT(8) PG_RPT(16) PG_RPT(32) PG_RPT(64) PG_RPT(128) PG_RPT(256)
+    PG_RPT(1) PG_RPT(2) PG_RPT(4) PG_RPT(8) PG_RPT(16) PG_RPT(32) PG_RPT(64) PG_RPT(128) PG_RPT(256)
 #undef PG_RPT
     default: return hipErrorInvalidValue;
   }
@@ -713,14 +1205,16 @@ hipError_t launch_rotary_rows(const MixRows& r, const ChunkAttn& a, hipStream_t 
 }
 
 hipError_t launch_chunk_attn_rows(const MixRows& r, const ChunkAttn& a, hipStream_t s) {
-  const dim3 grid(a.heads, (r.n + 127) / 128, r.nseq);
-  const int dp = (a.dim + 31) / 32 * 32;
+  const dim3 grid(a.heads, (r.n + 31) / 32, r.nseq);
+  int dp = (a.dim + 31) / 32 * 32;
+  if (dp > 160) dp = 256;
+  // (as many wavefronts as the LDS of a CU holds tiles for)
   switch (dp) {
-#define PG_DP(N)                                                                   \
-  case N:                                                                          \
-    hipLaunchKernelGGL(k_chunk_attn_rows<N>, grid, dim3(256), 0, s, r, a);          \
+#define PG_DP(N, W)                                                                      \
+  case N:                                                                                \
+    hipLaunchKernelGGL((k_chunk_attn_rows<N, W>), grid, dim3(64 * W), 0, s, r, a);        \
     break;
-    PG_DP(32) PG_DP(64) PG_DP(96) PG_DP(128) PG_DP(160) PG_DP(192) PG_DP(224) PG_DP(256)
+    PG_DP(32, 4) PG_DP(64, 4) PG_DP(96, 4) PG_DP(128, 4) PG_DP(160, 2) PG_DP(256, 2)
 #undef PG_DP
     default: return hipErrorInvalidValue;
   }
@@ -728,29 +1222,71 @@ hipError_t launch_chunk_attn_rows(const MixRows& r, const ChunkAttn& a, hipStrea
 }
 
 hipError_t launch_short_conv_rows(const MixRows& r, const ShortConv& c, hipStream_t s) {
-  hipLaunchKernelGGL(k_short_conv_rows, dim3((c.channels + 255) / 256, r.nseq * r.n), dim3(256), 0, s, r, c);
+  const dim3 grid((c.channels + 255) / 256, (r.n + kConvRows - 1) / kConvRows, r.nseq);
+  if (c.taps <= 4)
+    hipLaunchKernelGGL(k_short_conv_rows<4>, grid, dim3(256), 0, s, r, c);
+  else
+    hipLaunchKernelGGL(k_short_conv_rows<kMixMaxTaps>, grid, dim3(256), 0, s, r, c);
   return hipGetLastError();
+}
+
+size_t recurrence_work_floats(const Recurrence& c, int nseq, int n) {
+  const int dp = (c.dim + 31) / 32 * 32, ep = (c.vdim + 31) / 32 * 32;
+  return chunk_floats(dp, ep, c.delta != 0) * (size_t)nseq * ((n + kChunk - 1) / kChunk) * c.heads;
 }
 
 hipError_t launch_recurrence_rows(const MixRows& r, const Recurrence& c, hipStream_t s) {
-  if (!c.delta)
-    hipLaunchKernelGGL(k_gla_decay_rows, dim3((c.heads * c.dim + 255) / 256, r.nseq * r.n), dim3(256), 0, s, r, c);
-  const dim3 grid(c.heads, r.nseq);
-  switch (rows_per_thread(c.dim, c.vdim)) {
-#define PG_RPT(N)                                                              \
-  case N:                                                                      \
-    hipLaunchKernelGGL(k_recurrence_scan<N>, grid, dim3(256), 0, s, r, c);      \
-    break;
-    PG_RPT(4) PG_RPT(8) PG_RPT(16) PG_RPT(32) PG_RPT(64) PG_RPT(128) PG_RPT(256)
-#undef PG_RPT
-    default: return hipErrorInvalidValue;
+  ChunkWork w{};
+  w.chunks = (r.n + kChunk - 1) / kChunk;
+  w.dp = (c.dim + 31) / 32 * 32;
+  w.ep = (c.vdim + 31) / 32 * 32;
+  const size_t tiles = (size_t)r.nseq * w.chunks * c.heads;
+  if (r.work_floats < recurrence_work_floats(c, r.nseq, r.n)) return hipErrorInvalidValue;
+  float* at = r.work;
+  auto take = [&](size_t per_tile) {
+    float* p = at;
+    at += per_tile * tiles;
+    return p;
+  };
+  w.S = take((size_t)w.dp * w.ep);
+  w.Kd = take((size_t)32 * w.dp);
+  w.Qd = take((size_t)32 * w.dp);
+  w.U = take((size_t)32 * w.ep);
+  w.P = take(1024);
+  w.G = take(w.dp);
+  if (c.delta) {
+    w.W = take((size_t)32 * w.dp);
+    w.U0 = take((size_t)32 * w.ep);
   }
-  return hipGetLastError();
-}
-
-hipError_t launch_gated_norm_rows(const MixRows& r, const Recurrence& c, hipStream_t s) {
-  const int rows = r.nseq * r.n;
-  hipLaunchKernelGGL(k_gated_norm_rows, dim3((rows * c.heads + 3) / 4), dim3(256), 0, s, r, c, rows);
+  const dim3 grid(w.chunks, c.heads, r.nseq);
+  const int waves = w.dp / 32;
+  // (large heads: more LDS than a launch gets by default)
+  if (w.dp > 128) {
+    const int most = 100 * 1024;
+    hipError_t e = hipFuncSetAttribute(c.delta ? reinterpret_cast<const void*>(&k_delta_chunk)
+                                               : reinterpret_cast<const void*>(&k_gla_chunk),
+                                       hipFuncAttributeMaxDynamicSharedMemorySize, most);
+    if (e != hipSuccess) return e;
+  }
+  if (c.delta) {
+    const size_t lds = 2 * 32 * (size_t)(w.dp + 4) * sizeof(float);
+    hipLaunchKernelGGL(k_delta_chunk, grid, dim3(256), lds, s, r, c, w);
+  } else {
+    const int rows = r.nseq * r.n;
+    hipLaunchKernelGGL(k_gla_decay_rows, dim3((c.heads * c.dim + 255) / 256, (rows + kDecayRows - 1) / kDecayRows),
+                       dim3(256), 0, s, r, c, rows);
+    const size_t lds = 3 * 32 * (size_t)(w.dp + 1) * sizeof(float);
+    hipLaunchKernelGGL(k_gla_chunk, grid, dim3(256), lds, s, r, c, w);
+  }
+  hipError_t e = hipGetLastError();
+  if (e != hipSuccess) return e;
+  const dim3 sgrid(w.ep / 32, c.heads, r.nseq);
+  if (c.delta)
+    hipLaunchKernelGGL(k_chunk_states<true>, sgrid, dim3(64 * waves), 2 * waves * 1024 * sizeof(float), s, r, c, w);
+  else
+    hipLaunchKernelGGL(k_chunk_states<false>, sgrid, dim3(64 * waves), 0, s, r, c, w);
+  if ((e = hipGetLastError()) != hipSuccess) return e;
+  hipLaunchKernelGGL(k_chunk_out, grid, dim3(256), 32 * (size_t)(w.dp + 4) * sizeof(float), s, r, c, w);
   return hipGetLastError();
 }
 

@@ -433,7 +433,6 @@ pg_status stack_create(const std::string& config_path, const Json& config, const
     if (l.has_rec) {
       if (l.rec.delta) m->max_conv = std::max(m->max_conv, l.rec.conv.channels);
       else m->max_decay = std::max(m->max_decay, up(l.rec.heads * l.rec.dim, 4));
-      m->max_values = std::max(m->max_values, up(l.rec.heads * l.rec.vdim, 4));
     }
   }
 
@@ -481,7 +480,7 @@ pg_status stack_cache_create(const pg_model* model, pg_kv_cache* c) {
   c->stack = st;  // (destroyed with the cache, also when what follows fails)
   c->stack_model = model;
   const size_t B = c->B;
-  if (B > 4096) return fail(PG_INVALID_INPUT, "cache batch must be at most 4096 for this architecture");
+  if (B > 1024) return fail(PG_INVALID_INPUT, "cache batch must be at most 1024 for this architecture");
   auto alloc = [&](size_t floats, float** p) -> pg_status {
     PG_HIP(hipMalloc(p, std::max<size_t>(floats, 4) * sizeof(float)));
     st->memory.push_back(*p);
@@ -618,27 +617,31 @@ pg_status step_launches(const pg_model* model, pg_kv_cache* c, ProfileMarks* mar
     d.attn_splits = l.has_attn ? pgk::attn_decode_splits(l.attn.chunk) : 1;
     d.part = st.part;
     PG_HIP(pgk::launch_mix_decode(d, s));
-    if (l.has_attn && d.attn_splits > 1) PG_HIP(pgk::launch_attn_sum(d, s));
+    // the attention's key splits are added by the projection of the one-sequence step, where
+    // they are few
+    const bool sum_in_pair = B == 1 && l.has_attn && d.attn_splits > 1 && d.attn_splits <= pgk::kPairMaxSplits;
+    if (l.has_attn && d.attn_splits > 1 && !sum_in_pair) PG_HIP(pgk::launch_attn_sum(d, s));
     PG_MARK(kAttention);
     const bool more = i + 1 < m.layers.size();
-    if (B == 1 && l.mix_pad + (l.has_mlp ? l.mlp.ff_pad : 0) <= pgk::kPairMaxK) {
+    if (B == 1) {
       pgk::GemvPair p{};
       p.w_bf16 = model->w_bf16;
       p.W1 = l.out_w; p.x1 = st.mix; p.s1 = l.ls1; p.K1 = l.mix_pad;
-      if (l.has_mlp) {
+      p.resid = st.x; p.y = st.x; p.nout = Cp;
+      if (sum_in_pair) {
+        p.part = st.part; p.part_splits = d.attn_splits; p.part_n = l.attn.heads * l.attn.dim;
+        p.part_col = l.attn.out_col;
+      }
+      const bool both = l.has_mlp && l.mix_pad + l.mlp.ff_pad <= pgk::kPairMaxK;
+      if (both) {
         p.W2 = l.down_w; p.x2 = st.act; p.s2 = l.ls2; p.K2 = l.mlp.ff_pad;
       }
-      p.resid = st.x; p.y = st.x; p.nout = Cp;
       PG_HIP(pgk::launch_gemv_pair(p, s));
-      PG_MARK(kMlpProj);
-    } else if (B == 1) {
-      pgk::GemvPair p{};
-      p.w_bf16 = model->w_bf16;
-      p.W1 = l.out_w; p.x1 = st.mix; p.s1 = l.ls1; p.K1 = l.mix_pad;
-      p.resid = st.x; p.y = st.x; p.nout = Cp;
-      PG_HIP(pgk::launch_gemv_pair(p, s));
-      p.W1 = l.down_w; p.x1 = st.act; p.s1 = l.ls2; p.K1 = l.mlp.ff_pad;
-      PG_HIP(pgk::launch_gemv_pair(p, s));
+      if (l.has_mlp && !both) {  // (too wide for one launch)
+        p.W1 = l.down_w; p.x1 = st.act; p.s1 = l.ls2; p.K1 = l.mlp.ff_pad;
+        p.part_splits = 0;
+        PG_HIP(pgk::launch_gemv_pair(p, s));
+      }
       PG_MARK(kMlpProj);
     } else {
       float* next_h = more ? st.h : nullptr;
@@ -701,10 +704,13 @@ pg_status rows_segment(const pg_model* model, pg_kv_cache* c, const uint32_t* d_
   auto r64 = [](size_t v) { return round_up(v, 64); };
   const size_t ws_floats = 8 * rows * Cp;
   struct Piece { float** p; size_t n; };
-  float *x, *h, *y, *mix, *act, *krot, *conv, *decay, *o, *ws;
+  float *x, *h, *y, *mix, *act, *krot, *conv, *decay, *work, *ws;
+  size_t work_floats = 0;
+  for (const StackLayer& l : m.layers)
+    if (l.has_rec) work_floats = std::max(work_floats, pgk::recurrence_work_floats(l.rec, (int)B, (int)n));
   const Piece pieces[] = {{&x, rows * Cp}, {&h, std::max(rows, want.size()) * Cp}, {&y, rows * m.max_in},
                           {&mix, rows * m.max_mix}, {&act, rows * m.max_ff}, {&krot, rows * m.max_keys},
-                          {&conv, rows * m.max_conv}, {&decay, rows * m.max_decay}, {&o, rows * m.max_values},
+                          {&conv, rows * m.max_conv}, {&decay, rows * m.max_decay}, {&work, work_floats},
                           {&ws, ws_floats}};
   size_t total = 0;
   for (const Piece& p : pieces) total += r64(p.n);
@@ -737,7 +743,8 @@ pg_status rows_segment(const pg_model* model, pg_kv_cache* c, const uint32_t* d_
     r.nseq = (int)B; r.n = (int)n; r.pos0 = (int)pos0;
     r.y = y; r.ld_y = l.n_in;
     r.out = mix; r.ld_out = l.mix_pad; r.out_cols = l.mix_cols;
-    r.act = act; r.k_rot = krot; r.conv_out = conv; r.decay = decay; r.o = o;
+    r.act = act; r.k_rot = krot; r.conv_out = conv; r.decay = decay;
+    r.work = work; r.work_floats = work_floats;
     if (l.has_attn) {
       PG_HIP(pgk::launch_rotary_rows(r, b.attn, s));
       PG_HIP(pgk::launch_chunk_attn_rows(r, b.attn, s));
@@ -745,7 +752,6 @@ pg_status rows_segment(const pg_model* model, pg_kv_cache* c, const uint32_t* d_
     if (l.has_rec) {
       if (l.rec.delta) PG_HIP(pgk::launch_short_conv_rows(r, b.rec.conv, s));
       PG_HIP(pgk::launch_recurrence_rows(r, b.rec, s));
-      PG_HIP(pgk::launch_gated_norm_rows(r, b.rec, s));
     }
     PG_HIP(pgk::launch_commit_rows(r, l.has_attn ? &b.attn : nullptr,
                                    l.has_rec && l.rec.delta ? &b.rec.conv : nullptr, s));
@@ -792,7 +798,7 @@ pg_status stack_rows(const pg_model* model, pg_kv_cache* c, const uint32_t* ids,
                      const std::vector<int>& rows, float* dst, ProfileMarks* marks) {
   constexpr size_t kSegmentRows = 8192;
   const size_t B = c->B, V = (size_t)model->stack->vocab;
-  const size_t seg = std::max<size_t>(1, kSegmentRows / B);
+  const size_t seg = std::max<size_t>(32, kSegmentRows / B);  // tokens (the recurrences' chunk at least)
   if (c->prompt_cap < B * std::min(n, seg)) {
     for (int i = 0; i < 2; ++i) {
       if (c->ev_prompt[i]) PG_HIP(hipEventSynchronize(c->ev_prompt[i]));

@@ -40,8 +40,7 @@ struct StackModel {
   std::vector<StackLayer> layers;
   float *embed = nullptr, *head = nullptr, *final_norm = nullptr;
   // largest of each over the layers
-  int max_in = 0, max_mix = 0, max_ff = 0, max_keys = 0, max_conv = 0, max_decay = 0, max_values = 0,
-      max_part = 0;
+  int max_in = 0, max_mix = 0, max_ff = 0, max_keys = 0, max_conv = 0, max_decay = 0, max_part = 0;
   std::vector<void*> memory;
   ~StackModel();
 };

@@ -125,3 +125,121 @@ def bf16_rounded(w: Gpt2Weights) -> Gpt2Weights:
         c_proj_mlp_b=b.c_proj_mlp_b) for b in w.blocks]
     return Gpt2Weights(wte=round_bf16(w.wte), wpe=w.wpe, blocks=blocks, ln_f_g=w.ln_f_g,
                        ln_f_b=w.ln_f_b)
+
+
+# ---- stack models (Tarepel) --------------------------------------------------------------------
+# Layers of a real model's proportions, by width: every layer has about the 12 width^2
+# parameters of a GPT-2 layer of that width.  attn: heads of 64, key/value heads, chunk; delta
+# and gla: heads with 128-value states; ff of either kind of layer.
+STACK_SIZES = {
+    768: dict(heads=12, kv_heads=4, chunk=512, delta=(8, 4, 128, 128), gla=(8, 64, 128), ff=(1088, 1696)),
+    1280: dict(heads=20, kv_heads=5, chunk=512, delta=(12, 6, 128, 128), gla=(12, 64, 128), ff=(2048, 3072)),
+    1600: dict(heads=25, kv_heads=5, chunk=512, delta=(16, 8, 128, 128), gla=(16, 64, 128), ff=(2560, 3712)),
+}
+STACK_GLA_RANK = 16
+
+
+def tarepel_config(width: int, n_layer: int, vocab: int = 50257) -> dict:
+    """A Tarepel config.json of STACK_SIZES[width]; every third layer is a gla layer."""
+    z = STACK_SIZES[width]
+    dh, dk, dd, dv = z["delta"]
+    gh, gd, gv = z["gla"]
+    parallel = {"type": "parallel", "mlp": {"kind": "dense", "ff": z["ff"][0]}, "mixer": {
+        "left": {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": 64, "vdim": 64, "scale": 0.125,
+                 "mask": {"size": z["chunk"]}, "rot": {"dims": 64, "base": 10000.0}},
+        "right": {"heads": dh, "kv_heads": dk, "dim": dd, "vdim": dv, "conv": 4},
+        "left_scale": 0.5, "right_scale": 1.0}}
+    gla = {"type": "gla", "mlp": {"kind": "dense", "ff": z["ff"][1]},
+           "mixer": {"heads": gh, "dim": gd, "vdim": gv, "tau": 8.0}}
+    return {"architecture": "Tarepel", "vocab": vocab, "width": width, "norm": {"eps": 1e-6},
+            "logit_scale": 1.0, "layers": [gla if i % 3 == 2 else parallel for i in range(n_layer)]}
+
+
+def stack_tensor_shapes(cfg: dict, rank: int = STACK_GLA_RANK) -> "dict[str, tuple]":
+    """Names and shapes of a Tarepel model's tensors."""
+    C, V = cfg["width"], cfg["vocab"]
+    out = {"embed": (V, C)}
+    for i, layer in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", layer["mixer"]
+        out[p + "norm1"] = ()
+        if layer["type"] == "parallel":
+            L, R = m["left"], m["right"]
+            hd, gd = L["heads"] * L["dim"], L["kv_heads"] * L["dim"]
+            q = p + "mix.left."
+            out.update({q + "q": (hd, C), q + "k": (gd, C), q + "pb": (L["heads"],), q + "o": (C, hd)})
+            qk, vv, H = R["kv_heads"] * R["dim"], R["heads"] * R["vdim"], R["heads"]
+            q = p + "mix.right."
+            out.update({q + "q": (qk, C), q + "q.conv": (qk, R["conv"]), q + "k": (qk, C),
+                        q + "k.conv": (qk, R["conv"]), q + "v": (vv, C), q + "v.conv": (vv, R["conv"]),
+                        q + "b": (H, C), q + "A_log": (H,), q + "norm": (R["vdim"],), q + "a": (H, C),
+                        q + "dt_bias": (H,), q + "g": (vv, C), q + "o": (C, vv)})
+        else:
+            qk, vv = m["heads"] * m["dim"], m["heads"] * m["vdim"]
+            q = p + "mix."
+            out.update({q + "q": (qk, C), q + "k": (qk, C), q + "v": (vv, C), q + "g": (vv, C),
+                        q + "o": (C, vv), q + "norm": (m["vdim"],), q + "a1": (rank, C),
+                        q + "a2": (qk, rank), q + "a2.b": (qk,)})
+        out[p + "ls1"] = (C,)
+        if layer.get("mlp"):
+            ff = layer["mlp"]["ff"]
+            out.update({p + "mlp.gate": (ff, C), p + "mlp.up": (ff, C), p + "mlp.down": (C, ff),
+                        p + "ls2": (C,)})
+    out.update({"final.norm": (), "head": (V, C)})
+    return out
+
+
+def bf16_bits(a: np.ndarray) -> np.ndarray:
+    """The bf16 bit patterns (uint16) of f32 values, nearest even."""
+    return (round_bf16(a).view(np.uint32) >> np.uint32(16)).astype(np.uint16)
+
+
+def write_model_dir(path, cfg: dict, tensors) -> None:
+    """config.json and a bf16 model.safetensors from an iterable of (name, f32 array)
+    (arrays are taken one at a time)."""
+    import json
+    import os
+    os.makedirs(path, exist_ok=True)
+    with open(os.path.join(path, "config.json"), "w", encoding="utf-8") as f:
+        json.dump(cfg, f)
+    header, at, body = {}, 0, os.path.join(path, "model.safetensors.body")
+    with open(body, "wb") as f:
+        for name, a in tensors:
+            bits = bf16_bits(np.asarray(a, np.float32).reshape(-1))
+            header[name] = {"dtype": "BF16", "shape": list(np.shape(a)), "data_offsets": [at, at + bits.nbytes]}
+            at += bits.nbytes
+            f.write(bits.tobytes())
+    text = json.dumps(header).encode()
+    text += b" " * (-len(text) % 8)
+    with open(os.path.join(path, "model.safetensors"), "wb") as f, open(body, "rb") as b:
+        f.write(len(text).to_bytes(8, "little") + text)
+        while True:
+            part = b.read(1 << 24)
+            if not part:
+                break
+            f.write(part)
+    os.remove(body)
+
+
+def stack_weights(cfg: dict, seed: int, std: float = 0.02):
+    """(name, array) of seeded random weights: N(0, std), with norm gains of 1, layer scales of
+    0.3, convolution taps around a mean filter and decays between a few and a few hundred
+    tokens."""
+    pos = 0
+    for name, shape in stack_tensor_shapes(cfg).items():
+        n = int(np.prod(shape, dtype=np.int64))
+        a = normal_f32(n, seed, pos, std)
+        pos += n
+        last = name.split(".")[-1]
+        if last.startswith("norm"):
+            a = a + np.float32(1.0)
+        elif last in ("ls1", "ls2"):
+            a = a + np.float32(0.3)
+        elif last == "conv":
+            a = a * np.float32(10.0) + np.float32(1.0 / shape[1])
+        elif last == "A_log":
+            a = a * np.float32(20.0)
+        elif last == "dt_bias":
+            a = a * np.float32(40.0) - np.float32(3.0)
+        elif name.endswith("a2.b"):
+            a = a * np.float32(40.0) + np.float32(2.0)
+        yield name, a.reshape(shape)
