@@ -739,7 +739,8 @@ pg_status stack_advance(const pg_model* m, pg_kv_cache* c, const uint32_t* ids, 
 // One token of every sequence (ids[B], host); logits to the cache's rows.
 pg_status stack_advance_one(const pg_model* m, pg_kv_cache* c, const uint32_t* ids, ProfileMarks* marks = nullptr) {
   pg_status s;
-  if (c->seq_len == 0 && (s = pgh::stack_set_pos(c, 0))) return s;
+  // (a generation that failed half-way may have left the list of ids set)
+  if ((c->seq_len == 0 || c->stack->lists_ids) && (s = pgh::stack_set_pos(c, c->seq_len))) return s;
   if ((s = ensure_ids(c, c->B))) return s;
   std::memcpy(c->h_ids, ids, c->B * sizeof(uint32_t));
   PG_HIP(hipMemcpyAsync(c->d_tok, c->h_ids, c->B * sizeof(uint32_t), hipMemcpyHostToDevice, c->stream));
@@ -1833,21 +1834,25 @@ static pg_status decode_core(const pg_model* m, pg_kv_cache* c, size_t steps, in
     PG_HIP(hipStreamSynchronize(c->stream));
   } else {
     if ((s = ensure_ids(c, n_steps * B))) return s;
+    if (m->stack && (s = pgh::stack_set_pos(c, c->seq_len, c->d_out_ids))) return s;
     PG_HIP(hipEventRecord(c->ev0, c->stream));
     for (size_t i = 0; i < n_steps; ++i) {
       PG_HIP(pgk::launch_argmax(c->logits_buf, (int)V, c->d_tok, c->stream, (int)B));
-      PG_HIP(hipMemcpyAsync(c->d_out_ids + i * B, c->d_tok, B * sizeof(uint32_t),
-                            hipMemcpyDeviceToDevice, c->stream));
+      bool end = i + 1 == n_steps;
       if (m->stack && eos >= 0) {
         // a recurrent state cannot be set back: no forward may follow an EOS
         PG_HIP(hipMemcpyAsync(c->h_ids, c->d_tok, sizeof(uint32_t), hipMemcpyDeviceToHost, c->stream));
         PG_HIP(hipStreamSynchronize(c->stream));
         if (c->h_ids[0] == (uint32_t)eos) {
           n_out = i + 1;
-          break;
+          end = true;
         }
       }
-      if (i + 1 < n_steps) {
+      if (!m->stack || end)  // (a stack model's steps list the ids they take)
+        PG_HIP(hipMemcpyAsync(c->d_out_ids + i * B, c->d_tok, B * sizeof(uint32_t),
+                              hipMemcpyDeviceToDevice, c->stream));
+      if (end) break;
+      {
         if (m->stack) {
           if ((s = pgh::stack_step(m, c))) return s;
         } else if (use_batched_step(m, c)) {
@@ -1860,6 +1865,7 @@ static pg_status decode_core(const pg_model* m, pg_kv_cache* c, size_t steps, in
       }
     }
     PG_HIP(hipEventRecord(c->ev1, c->stream));
+    if (m->stack && (s = pgh::stack_set_pos(c, c->seq_len))) return s;
     PG_HIP(hipMemcpyAsync(c->h_ids, c->d_out_ids, n_out * B * sizeof(uint32_t),
                           hipMemcpyDeviceToHost, c->stream));
     PG_HIP(hipStreamSynchronize(c->stream));

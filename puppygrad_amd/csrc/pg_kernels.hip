@@ -312,18 +312,24 @@ __global__ __launch_bounds__(kBlock) void k_gemv_pair(GemvPair a) {
     const float4* x2 = reinterpret_cast<const float4*>(a.x2);
     float4* d = reinterpret_cast<float4*>(sx);
     const int n1 = a.K1 >> 2, n2 = a.K2 >> 2;
-    for (int i = tid; i < n1 + n2; i += kBlock) d[i] = i < n1 ? x1[i] : x2[i - n1];
-    if (a.part_splits > 0) {
-      // columns that are still partial sums
-      __syncthreads();
-      for (int i = tid; i < a.part_n; i += kBlock) {
-        float v[kPairMaxSplits];
+    // columns that are still partial sums, then the others (whole float4 of the range are left out)
+    const int p0 = a.part_splits > 0 ? a.part_col : 0, p1 = a.part_splits > 0 ? p0 + a.part_n : 0;
+    for (int i = tid; i < p1 - p0; i += kBlock) {
+      float v[kPairMaxSplits];
 #pragma unroll
-        for (int k = 0; k < kPairMaxSplits; ++k) v[k] = a.part[(size_t)min(k, a.part_splits - 1) * a.part_n + i];
-        float s = 0.0f;
+      for (int k = 0; k < kPairMaxSplits; ++k) v[k] = a.part[(size_t)min(k, a.part_splits - 1) * a.part_n + i];
+      float s = 0.0f;
 #pragma unroll
-        for (int k = 0; k < kPairMaxSplits; ++k) s += k < a.part_splits ? v[k] : 0.0f;
-        sx[a.part_col + i] = s;
+      for (int k = 0; k < kPairMaxSplits; ++k) s += k < a.part_splits ? v[k] : 0.0f;
+      sx[p0 + i] = s;
+    }
+    for (int i = tid; i < n1 + n2; i += kBlock) {
+      const int e = 4 * i;
+      if (e >= p1 || e + 4 <= p0) {
+        d[i] = i < n1 ? x1[i] : x2[i - n1];
+      } else if (e < p0 || e + 4 > p1) {
+        for (int k = e; k < e + 4; ++k)
+          if (k < p0 || k >= p1) sx[k] = a.x1[k];
       }
     }
   }

@@ -140,9 +140,17 @@ hipError_t launch_commit_rows(const MixRows& r, const ChunkAttn* a, const ShortC
 // src is rows_at[r].
 hipError_t launch_rms_rows(const float* src, float* dst, int rows, int cols, int ld, const float* gain,
                            float eps, float scale, const int* rows_at, hipStream_t s);
-// *p = value
-hipError_t launch_set_int(int* p, int value, hipStream_t s);
-// *p += 1
-hipError_t launch_add_one(int* p, hipStream_t s);
+// What a one-token step keeps on the device: the position of the step that is running, that of the
+// next one, and, for generations that run ahead of the host, where the next ids are listed
+// (out[n_out][nseq], out may be null).
+struct StepWords {
+  int pos, next, n_out, unused;
+  uint32_t* out;
+};
+// The start of a step: x[b] = table[ids[b]] ([vocab][width], f32 or bf16), the ids are appended to
+// words->out, and the position advances.
+hipError_t launch_begin_step(float* x, const void* table, int table_bf16, const uint32_t* ids, int nseq, int width,
+                             StepWords* words, hipStream_t s);
+hipError_t launch_set_words(StepWords* words, int next, uint32_t* out, hipStream_t s);
 
 }  // namespace pgk

@@ -54,14 +54,15 @@ __device__ __forceinline__ float gla_log_decay(float z, float inv_tau) { return 
 // ---------------------------------------------------------------------------
 constexpr int kRG = 8;  // query heads of one key/value head that a block takes
 
-// LDS of a decode block (floats): the attention role's, the larger of the two.
-constexpr int kDecodeLds = kRG * kMixMaxDim + 2 * kMixMaxDim + kRG * kSplitKeys + 256 * kRG;
+// LDS of a decode block of NT threads (floats): the attention role's, the larger of the two.
+template <int NT>
+constexpr int kDecodeLds = kRG * kMixMaxDim + 2 * kMixMaxDim + kRG * kSplitKeys + NT * kRG;
 
 // Keys [kSplitKeys split, ...) of the current chunk against kRG query heads of key/value head g.
 // NV: float4 per lane and key (sixteen lanes to a key).  Nothing that is loaded before the first
 // barrier depends on another load but the ring rows' bound, and all of a block's key rows are
 // requested together, then all of its value rows.
-template <int NV>
+template <int NT, int NV>
 __device__ void attn_role(const MixDecode& m, int b, int item, float* lds) {
   const ChunkAttn& a = m.attn;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -77,7 +78,7 @@ __device__ void attn_role(const MixDecode& m, int b, int item, float* lds) {
   if (j0 > last) {
     // (every split's sums are added: the ones without keys are 0)
     if (m.attn_splits > 1)
-      for (int i = tid; i < nr * dim; i += 256)
+      for (int i = tid; i < nr * dim; i += NT)
         m.part[(((size_t)b * m.attn_splits + split) * a.heads + g * R + r0) * dim + i] = 0.0f;
     return;
   }
@@ -85,11 +86,11 @@ __device__ void attn_role(const MixDecode& m, int b, int item, float* lds) {
   const int own = last - j0;  // the current token's key in this split, if it is below nk
   const int sub = lane >> 4, l16 = lane & 15;
   // key rows: four to a wavefront and step
-  constexpr int KS = kSplitKeys / 16;
+  constexpr int KS = kSplitKeys * 16 / NT, KR = NT / 16;  // steps, keys per step
   f4 kv[KS][NV];
 #pragma unroll
   for (int q = 0; q < KS; ++q) {
-    const int j = min(16 * q + wave * 4 + sub, max(nk - 1, 0));
+    const int j = min(KR * q + wave * 4 + sub, max(nk - 1, 0));
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
       const int e = 4 * l16 + 64 * i;
@@ -100,11 +101,11 @@ __device__ void attn_role(const MixDecode& m, int b, int item, float* lds) {
   float* kn = qs + kRG * dp;             // [dp] the current token's key, rotated
   float* vn = kn + dp;                   // [dp] ... as projected
   float* w = vn + dp;                    // [kRG][kSplitKeys]
-  float* red = w + kRG * kSplitKeys;     // [256][kRG]
+  float* red = w + kRG * kSplitKeys;     // [NT][kRG]
   const float* y = m.y + (size_t)b * m.ld_y;
   const float* yk = y + a.k_col + g * dim;
   const float* yq = y + a.q_col + (size_t)(g * R + r0) * dim;
-  for (int i = tid; i < dp; i += 256) {
+  for (int i = tid; i < dp; i += NT) {
     if (i < half) {
       float s, c;
       const float u = yk[i], v = yk[i + half];
@@ -119,7 +120,7 @@ __device__ void attn_role(const MixDecode& m, int b, int item, float* lds) {
   }
   // queries: a pair (or a value that passes) per thread
   const int per = dp - half;
-  for (int i = tid; i < nr * per; i += 256) {
+  for (int i = tid; i < nr * per; i += NT) {
     const int r = i / per, e = i - r * per;
     if (e < half) {
       float s, c;
@@ -135,7 +136,7 @@ __device__ void attn_role(const MixDecode& m, int b, int item, float* lds) {
   // value rows of this thread's column, requested ahead of the scores
   int cols = 1;
   while (cols < dim) cols <<= 1;
-  const int parts = 256 / cols, d = tid % cols, part = tid / cols;
+  const int parts = NT / cols, d = tid % cols, part = tid / cols;
   constexpr int VB = 16;  // value rows in flight per thread
   float vv[VB];
   auto fetch_v = [&](int jb) {
@@ -149,15 +150,15 @@ __device__ void attn_role(const MixDecode& m, int b, int item, float* lds) {
   if (rg == 0 && own < kSplitKeys) {
     float* kw = a.kring + (size_t)b * a.ring_seq + ((size_t)g * a.chunk + last) * dp;
     float* vw = a.vring + (size_t)b * a.ring_seq + ((size_t)g * a.chunk + last) * dp;
-    for (int i = tid; i < dp; i += 256) {
+    for (int i = tid; i < dp; i += NT) {
       kw[i] = kn[i];
       vw[i] = vn[i];
     }
   }
 #pragma unroll
   for (int q = 0; q < KS; ++q) {
-    const int j = 16 * q + wave * 4 + sub;
-    if (16 * q >= nk) break;
+    const int j = KR * q + wave * 4 + sub;
+    if (KR * q >= nk) break;
     if (j == own) {
 #pragma unroll
       for (int i = 0; i < NV; ++i) kv[q][i] = *reinterpret_cast<const f4*>(kn + min(4 * l16 + 64 * i, dp - 4));
@@ -201,7 +202,7 @@ __device__ void attn_role(const MixDecode& m, int b, int item, float* lds) {
   for (int r = 0; r < kRG; ++r)
     if (r < nr) red[(r * parts + part) * cols + d] = acc[r];
   __syncthreads();
-  for (int i = tid; i < nr * cols; i += 256) {
+  for (int i = tid; i < nr * cols; i += NT) {
     const int r = i / cols, dd = i - r * cols;
     if (dd >= dim) continue;
     float s = 0.0f;
@@ -250,21 +251,21 @@ __device__ __forceinline__ float conv_channel(const ShortConv& c, const float* y
 
 // One head of the recurrence.  A thread owns column v of the state and every `parts`-th of its
 // rows, RPT of them, in registers (parts * RPT <= kMixMaxDim; q and k are 0 past dim).
-template <int RPT>
+template <int NT, int RPT>
 __device__ void recurrence_role(const MixDecode& m, int b, int h, float* lds) {
   const Recurrence& c = m.rec;
   const int tid = threadIdx.x;
   const int dim = c.dim, vdim = c.vdim;
   int cols = 1;
   while (cols < vdim) cols <<= 1;
-  const int parts = 256 / cols, v = tid % cols, part = tid / cols;
+  const int parts = NT / cols, v = tid % cols, part = tid / cols;
   float* qs = lds;                 // [256]
   float* ks = qs + 256;            // [256]
   float* vs = ks + 256;            // [256]
   float* al = vs + 256;            // [256] decay per key channel
-  float* red = al + 256;           // [256]
-  float* red2 = red + 256;         // [256]
-  float* red4 = red2 + 256;        // [8]
+  float* red = al + 256;           // [NT]
+  float* red2 = red + NT;          // [NT]
+  float* redw = red2 + NT;         // [2][NT / 64]
   const float* y = m.y + (size_t)b * m.ld_y;
   float* S = c.state + (size_t)b * c.state_seq + (size_t)h * dim * vdim;
   const int pos = *m.d_pos;
@@ -288,17 +289,19 @@ __device__ void recurrence_role(const MixDecode& m, int b, int h, float* lds) {
     float kv = conv_channel(cv, y, ring, c.k_col - cv.col + kvh * dim + td, pos, first && tid < dim);
     const float x = conv_channel(cv, y, ring, c.v_col - cv.col + h * vdim + tv, pos, tid < vdim);
     if (tid >= dim) qv = kv = 0.0f;
-    vs[tid] = x;
     float qn = wave_sum(qv * qv), kn = wave_sum(kv * kv);
-    if ((tid & 63) == 0) {
-      red4[tid >> 6] = qn;
-      red4[4 + (tid >> 6)] = kn;
+    if ((tid & 63) == 0 && tid < 256) {  // (nothing past kMixMaxDim = 256)
+      redw[tid >> 6] = qn;
+      redw[4 + (tid >> 6)] = kn;
     }
     __syncthreads();
-    qn = (red4[0] + red4[1]) + (red4[2] + red4[3]);
-    kn = (red4[4] + red4[5]) + (red4[6] + red4[7]);
-    qs[tid] = qv / sqrtf(qn + 1e-6f) * c.q_scale;
-    ks[tid] = kv / sqrtf(kn + 1e-6f);
+    qn = (redw[0] + redw[1]) + (redw[2] + redw[3]);
+    kn = (redw[4] + redw[5]) + (redw[6] + redw[7]);
+    if (tid < 256) {
+      vs[tid] = x;
+      qs[tid] = qv / sqrtf(qn + 1e-6f) * c.q_scale;
+      ks[tid] = kv / sqrtf(kn + 1e-6f);
+    }
     beta = sigmoid(yb);
     g = expf(delta_log_decay(ya, al0, dt));
   } else {
@@ -322,10 +325,12 @@ __device__ void recurrence_role(const MixDecode& m, int b, int h, float* lds) {
       for (; r < c.rank; ++r) z += a2[r] * y[c.a_col + r];
       av = expf(gla_log_decay(z, c.inv_tau));
     }
-    qs[tid] = qv;
-    ks[tid] = kv;
-    al[tid] = av;
-    vs[tid] = y[c.v_col + h * vdim + tv];
+    if (tid < 256) {
+      qs[tid] = qv;
+      ks[tid] = kv;
+      al[tid] = av;
+      vs[tid] = y[c.v_col + h * vdim + tv];
+    }
   }
   // (at position 0 the state is zero whatever the memory holds)
   if (pos == 0) {
@@ -373,28 +378,31 @@ __device__ void recurrence_role(const MixDecode& m, int b, int h, float* lds) {
   float out = 0.0f;
   if (tid < vdim)
     for (int p = 0; p < parts; ++p) out += red2[p * cols + tid];
-  const float ss = block_sum(out * out, red4);
+  float ss = wave_sum(out * out);
+  if ((tid & 63) == 0 && tid < 256) redw[tid >> 6] = ss;
+  __syncthreads();
+  ss = (redw[0] + redw[1]) + (redw[2] + redw[3]);
   if (tid < vdim)
     m.out[(size_t)b * m.ld_out + c.out_col + h * vdim + tid] =
         out / sqrtf(ss / (float)vdim + c.eps) * norm * silu(gate) * c.out_scale;
 }
 
-template <int RPT, int NV>
-__global__ __launch_bounds__(256) void k_mix_decode(MixDecode m, int attn_items, int rec_items) {
-  __shared__ __attribute__((aligned(16))) float lds[kDecodeLds];
+template <int NT, int RPT, int NV>
+__global__ __launch_bounds__(NT) void k_mix_decode(MixDecode m, int attn_items, int rec_items) {
+  __shared__ __attribute__((aligned(16))) float lds[kDecodeLds<NT>];
   const int b = blockIdx.y;
   int item = blockIdx.x;
   if (item < rec_items) {
-    recurrence_role<RPT>(m, b, item, lds);
+    recurrence_role<NT, RPT>(m, b, item, lds);
     return;
   }
   item -= rec_items;
   if (item < attn_items) {
-    attn_role<NV>(m, b, item, lds);
+    attn_role<NT, NV>(m, b, item, lds);
     return;
   }
   item -= attn_items;
-  const int j = item * 256 + threadIdx.x;
+  const int j = item * NT + threadIdx.x;
   if (j >= m.mlp.ff_pad) return;
   const float* y = m.y + (size_t)b * m.ld_y;
   m.act[(size_t)b * m.mlp.ff_pad + j] =
@@ -933,10 +941,10 @@ __global__ __launch_bounds__(256) void k_gla_chunk(MixRows r, Recurrence c, Chun
 // the state's rows 32 w .. 32 w + 31 in the accumulator layout of the 32 x 32 MFMA, where register
 // v of lane (l, half) is row 8 (v / 4) + 4 half + v % 4 of column l.  In that layout the state is
 // an operand of W S as it is (step v multiplies the rows its two lane halves hold), and so is U
-// of Kd^T U.  The wavefronts' parts of W S meet in LDS, two buffers in turn.  The next chunk's
-// tiles are requested a chunk ahead.
-template <bool DELTA>
-__global__ __launch_bounds__(512) void k_chunk_states(MixRows r, Recurrence c, ChunkWork w) {
+// of Kd^T U.  The wavefronts' parts of W S meet in LDS, two buffers in turn.  A chunk's tiles are
+// requested two chunks ahead (one with more than four wavefronts).  WAVES: the most of a block.
+template <bool DELTA, int WAVES>
+__global__ __launch_bounds__(64 * WAVES) void k_chunk_states(MixRows r, Recurrence c, ChunkWork w) {
   extern __shared__ float part[];  // [2][waves][16][64] (delta)
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, waves = blockDim.x >> 6;
   const int half = lane >> 5, l32 = lane & 31;
@@ -951,43 +959,29 @@ __global__ __launch_bounds__(512) void k_chunk_states(MixRows r, Recurrence c, C
     const int i = 32 * wave + row_of(v);
     S[v] = r.pos0 > 0 && i < dim && col < vdim ? state[(size_t)i * vdim + col] : 0.0f;
   }
-  f4 nw[4];
-  float nk[16], nu[16];
-  f4 ng[4];
-  auto fetch = [&](int ci) __attribute__((always_inline)) {
-    const size_t tile = w.tile(b, ci, h, c.heads);
+  struct Tiles {  // of one chunk
+    f4 w[4], g[4];
+    float k[16], u[16];
+  };
+  auto fetch = [&](int ci, Tiles& x) __attribute__((always_inline)) {
+    const size_t tile = w.tile(b, min(ci, w.chunks - 1), h, c.heads);
     const float* u = (DELTA ? w.U0 : w.U) + tile * 32 * ep + col;
     const float* kd = w.Kd + tile * 32 * dp + 32 * wave + l32;
     const float* g = w.G + tile * dp + 32 * wave + 4 * half;
     if (DELTA) {
       const float* wt = w.W + tile * 32 * dp + (size_t)l32 * dp + 32 * wave + 4 * half;
 #pragma unroll
-      for (int q = 0; q < 4; ++q) nw[q] = *reinterpret_cast<const f4*>(wt + 8 * q);
+      for (int q = 0; q < 4; ++q) x.w[q] = *reinterpret_cast<const f4*>(wt + 8 * q);
     }
 #pragma unroll
-    for (int v = 0; v < 16; ++v) {
-      nu[v] = u[row_of(v) * ep];
-      nk[v] = kd[row_of(v) * dp];
-    }
+    for (int v = 0; v < 16; ++v) x.u[v] = u[row_of(v) * ep];
 #pragma unroll
-    for (int q = 0; q < 4; ++q) ng[q] = *reinterpret_cast<const f4*>(g + 8 * q);
+    for (int v = 0; v < 16; ++v) x.k[v] = kd[row_of(v) * dp];
+#pragma unroll
+    for (int q = 0; q < 4; ++q) x.g[q] = *reinterpret_cast<const f4*>(g + 8 * q);
   };
-  fetch(0);
-  for (int ci = 0; ci < w.chunks; ++ci) {
+  auto chunk = [&](int ci, Tiles& x) __attribute__((always_inline)) {
     const size_t tile = w.tile(b, ci, h, c.heads);
-    f4 cw[4], cg[4];
-    float ck[16], u[16];
-#pragma unroll
-    for (int q = 0; q < 4; ++q) {
-      if (DELTA) cw[q] = nw[q];
-      cg[q] = ng[q];
-    }
-#pragma unroll
-    for (int v = 0; v < 16; ++v) {
-      ck[v] = nk[v];
-      u[v] = nu[v];
-    }
-    if (ci + 1 < w.chunks) fetch(ci + 1);
     float* s0 = w.S + tile * dp * ep + (size_t)(32 * wave) * ep + col;
 #pragma unroll
     for (int v = 0; v < 16; ++v) s0[row_of(v) * ep] = S[v];
@@ -996,7 +990,7 @@ __global__ __launch_bounds__(512) void k_chunk_states(MixRows r, Recurrence c, C
 #pragma unroll
       for (int v = 0; v < 16; ++v) p[v] = 0.0f;
 #pragma unroll
-      for (int v = 0; v < 16; ++v) p = __builtin_amdgcn_mfma_f32_32x32x2f32(cw[v >> 2][v & 3], S[v], p, 0, 0, 0);
+      for (int v = 0; v < 16; ++v) p = __builtin_amdgcn_mfma_f32_32x32x2f32(x.w[v >> 2][v & 3], S[v], p, 0, 0, 0);
       float* mine = part + (size_t)((ci & 1) * waves + wave) * 1024 + lane;
 #pragma unroll
       for (int v = 0; v < 16; ++v) mine[64 * v] = p[v];
@@ -1004,16 +998,42 @@ __global__ __launch_bounds__(512) void k_chunk_states(MixRows r, Recurrence c, C
       const float* all = part + (size_t)((ci & 1) * waves) * 1024 + lane;
       for (int o = 0; o < waves; ++o)
 #pragma unroll
-        for (int v = 0; v < 16; ++v) u[v] -= all[(size_t)o * 1024 + 64 * v];
+        for (int v = 0; v < 16; ++v) x.u[v] -= all[(size_t)o * 1024 + 64 * v];
       float* ud = w.U + tile * 32 * ep + col;
 #pragma unroll
       for (int v = 0; v < 16; ++v)
-        if (v % waves == wave) ud[row_of(v) * ep] = u[v];
+        if (v % waves == wave) ud[row_of(v) * ep] = x.u[v];
     }
 #pragma unroll
-    for (int v = 0; v < 16; ++v) S[v] *= cg[v >> 2][v & 3];
+    for (int v = 0; v < 16; ++v) S[v] *= x.g[v >> 2][v & 3];
 #pragma unroll
-    for (int v = 0; v < 16; ++v) S = __builtin_amdgcn_mfma_f32_32x32x2f32(ck[v], u[v], S, 0, 0, 0);
+    for (int v = 0; v < 16; ++v) S = __builtin_amdgcn_mfma_f32_32x32x2f32(x.k[v], x.u[v], S, 0, 0, 0);
+  };
+  // (past the end: the last chunk's tiles again, never used)
+  Tiles x0, x1;
+  int ci = 0;
+  fetch(0, x0);
+  if constexpr (WAVES <= 4) {
+    Tiles x2;
+    fetch(1, x1);
+    for (; ci + 3 <= w.chunks; ci += 3) {
+      fetch(ci + 2, x2);
+      chunk(ci, x0);
+      fetch(ci + 3, x0);
+      chunk(ci + 1, x1);
+      fetch(ci + 4, x1);
+      chunk(ci + 2, x2);
+    }
+    if (ci < w.chunks) chunk(ci, x0);
+    if (ci + 1 < w.chunks) chunk(ci + 1, x1);
+  } else {
+    for (; ci + 2 <= w.chunks; ci += 2) {
+      fetch(ci + 1, x1);
+      chunk(ci, x0);
+      fetch(ci + 2, x0);
+      chunk(ci + 1, x1);
+    }
+    if (ci < w.chunks) chunk(ci, x0);
   }
 #pragma unroll
   for (int v = 0; v < 16; ++v) {
@@ -1151,8 +1171,32 @@ __global__ __launch_bounds__(256) void k_rms_rows(const float* src, float* dst, 
   for (int i = threadIdx.x; i < ld; i += 256) y[i] = i < cols ? x[i] * k : 0.0f;
 }
 
-__global__ void k_set_int(int* p, int value) { *p = value; }
-__global__ void k_add_one(int* p) { *p += 1; }
+__global__ __launch_bounds__(256) void k_begin_step(float* x, const void* table, int table_bf16, const uint32_t* ids,
+                                                    int width, StepWords* words) {
+  const int b = blockIdx.y, i = blockIdx.x * 256 + threadIdx.x;
+  const size_t at = (size_t)ids[b] * width + i;
+  if (i < width)
+    x[(size_t)b * width + i] =
+        table_bf16 ? __uint_as_float((unsigned)static_cast<const unsigned short*>(table)[at] << 16)
+                   : static_cast<const float*>(table)[at];
+  if (blockIdx.x == 0 && b == 0) {  // (no other block touches the words)
+    const int n = words->n_out, p = words->next;
+    uint32_t* out = words->out;
+    if (out)
+      for (int k = threadIdx.x; k < (int)gridDim.y; k += 256) out[(size_t)n * gridDim.y + k] = ids[k];
+    __syncthreads();
+    if (threadIdx.x == 0) {
+      words->pos = p;
+      words->next = p + 1;
+      words->n_out = n + 1;
+    }
+  }
+}
+__global__ void k_set_words(StepWords* w, int next, uint32_t* out) {
+  w->next = next;
+  w->out = out;
+  w->n_out = 0;
+}
 
 // Rows of a state column per thread (recurrence_role): the next power of two.
 int rows_per_thread(int dim, int vdim) {
@@ -1175,18 +1219,22 @@ hipError_t launch_mix_decode(const MixDecode& a, hipStream_t s) {
     attn_items = a.attn.kv_heads * ((R + kRG - 1) / kRG) * a.attn_splits;
   }
   const int rec_items = a.has_rec ? a.rec.heads : 0;
-  const int mlp_items = a.has_mlp ? (a.mlp.ff_pad + 255) / 256 : 0;
+  // Rows of a state column per thread of a block of 256; blocks grow so that a thread holds few.
+  const int rows = a.has_rec ? rows_per_thread(a.rec.dim, a.rec.vdim) : 1;
+  const int nt = rows <= 8 ? 256 : rows == 16 ? 512 : 1024;
+  const int mlp_items = a.has_mlp ? (a.mlp.ff_pad + nt - 1) / nt : 0;
   const dim3 grid((unsigned)(attn_items + rec_items + mlp_items), (unsigned)a.nseq);
   if (grid.x == 0) return hipSuccess;
   const int nv = !a.has_attn || a.attn.dim_pad <= 64 ? 1 : a.attn.dim_pad <= 128 ? 2 : 4;
-  switch (a.has_rec ? rows_per_thread(a.rec.dim, a.rec.vdim) : 1) {
-#define PG_RPT(N)                                                                                               \
-  case N:                                                                                                       \
-    if (nv == 1) hipLaunchKernelGGL((k_mix_decode<N, 1>), grid, dim3(256), 0, s, a, attn_items, rec_items);      \
-    else if (nv == 2) hipLaunchKernelGGL((k_mix_decode<N, 2>), grid, dim3(256), 0, s, a, attn_items, rec_items); \
-    else hipLaunchKernelGGL((k_mix_decode<N, 4>), grid, dim3(256), 0, s, a, attn_items, rec_items);              \
+  switch (rows) {
+#define PG_RPT(R, NT, N)                                                                                             \
+  case R:                                                                                                            \
+    if (nv == 1) hipLaunchKernelGGL((k_mix_decode<NT, N, 1>), grid, dim3(NT), 0, s, a, attn_items, rec_items);        \
+    else if (nv == 2) hipLaunchKernelGGL((k_mix_decode<NT, N, 2>), grid, dim3(NT), 0, s, a, attn_items, rec_items);   \
+    else hipLaunchKernelGGL((k_mix_decode<NT, N, 4>), grid, dim3(NT), 0, s, a, attn_items, rec_items);                \
     break;
-    PG_RPT(1) PG_RPT(2) PG_RPT(4) PG_RPT(8) PG_RPT(16) PG_RPT(32) PG_RPT(64) PG_RPT(128) PG_RPT(256)
+    PG_RPT(1, 256, 1) PG_RPT(2, 256, 2) PG_RPT(4, 256, 4) PG_RPT(8, 256, 8) PG_RPT(16, 512, 8)
+    PG_RPT(32, 1024, 8) PG_RPT(64, 1024, 16) PG_RPT(128, 1024, 32) PG_RPT(256, 1024, 64)
 #undef PG_RPT
     default: return hipErrorInvalidValue;
   }
@@ -1281,10 +1329,15 @@ hipError_t launch_recurrence_rows(const MixRows& r, const Recurrence& c, hipStre
   hipError_t e = hipGetLastError();
   if (e != hipSuccess) return e;
   const dim3 sgrid(w.ep / 32, c.heads, r.nseq);
-  if (c.delta)
-    hipLaunchKernelGGL(k_chunk_states<true>, sgrid, dim3(64 * waves), 2 * waves * 1024 * sizeof(float), s, r, c, w);
+  const size_t slds = c.delta ? 2 * waves * 1024 * sizeof(float) : 0;
+  if (c.delta && waves <= 4)
+    hipLaunchKernelGGL((k_chunk_states<true, 4>), sgrid, dim3(64 * waves), slds, s, r, c, w);
+  else if (c.delta)
+    hipLaunchKernelGGL((k_chunk_states<true, 8>), sgrid, dim3(64 * waves), slds, s, r, c, w);
+  else if (waves <= 4)
+    hipLaunchKernelGGL((k_chunk_states<false, 4>), sgrid, dim3(64 * waves), slds, s, r, c, w);
   else
-    hipLaunchKernelGGL(k_chunk_states<false>, sgrid, dim3(64 * waves), 0, s, r, c, w);
+    hipLaunchKernelGGL((k_chunk_states<false, 8>), sgrid, dim3(64 * waves), slds, s, r, c, w);
   if ((e = hipGetLastError()) != hipSuccess) return e;
   hipLaunchKernelGGL(k_chunk_out, grid, dim3(256), 32 * (size_t)(w.dp + 4) * sizeof(float), s, r, c, w);
   return hipGetLastError();
@@ -1312,12 +1365,14 @@ hipError_t launch_rms_rows(const float* src, float* dst, int rows, int cols, int
   return hipGetLastError();
 }
 
-hipError_t launch_set_int(int* p, int value, hipStream_t s) {
-  hipLaunchKernelGGL(k_set_int, dim3(1), dim3(1), 0, s, p, value);
+hipError_t launch_begin_step(float* x, const void* table, int table_bf16, const uint32_t* ids, int nseq, int width,
+                             StepWords* words, hipStream_t s) {
+  hipLaunchKernelGGL(k_begin_step, dim3((width + 255) / 256, nseq), dim3(256), 0, s, x, table, table_bf16, ids, width,
+                     words);
   return hipGetLastError();
 }
-hipError_t launch_add_one(int* p, hipStream_t s) {
-  hipLaunchKernelGGL(k_add_one, dim3(1), dim3(1), 0, s, p);
+hipError_t launch_set_words(StepWords* words, int next, uint32_t* out, hipStream_t s) {
+  hipLaunchKernelGGL(k_set_words, dim3(1), dim3(1), 0, s, words, next, out);
   return hipGetLastError();
 }
 

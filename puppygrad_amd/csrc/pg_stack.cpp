@@ -502,9 +502,9 @@ pg_status stack_cache_create(const pg_model* model, pg_kv_cache* c) {
       if ((s = alloc(B * l.rec.heads * l.rec.dim * l.rec.vdim, &k.state))) return s;
     }
   }
-  float* pos = nullptr;
-  if ((s = alloc(1, &pos))) return s;
-  st->d_pos = reinterpret_cast<int*>(pos);
+  float* words = nullptr;
+  if ((s = alloc(sizeof(pgk::StepWords) / sizeof(float), &words))) return s;
+  st->words = reinterpret_cast<pgk::StepWords*>(words);
   if ((s = alloc(B * m.width_pad, &st->x)) || (s = alloc(B * m.width_pad, &st->h)) ||
       (s = alloc(B * m.max_in, &st->y)) || (s = alloc(B * m.max_mix, &st->mix)) ||
       (s = alloc(B * m.max_ff, &st->act)) || (s = alloc(B * m.max_part, &st->part)))
@@ -592,7 +592,7 @@ pg_status step_launches(const pg_model* model, pg_kv_cache* c, ProfileMarks* mar
   hipStream_t s = c->stream;
   const int B = (int)c->B, Cp = m.width_pad;
   const Gemm gemm{model, c->gemm_ws, c->gemm_ws_floats, B, s};
-  PG_HIP(pgk::launch_embed_batch(st.x, m.embed, nullptr, c->d_tok, B, 0, Cp, s, model->w_bf16));
+  PG_HIP(pgk::launch_begin_step(st.x, m.embed, model->w_bf16, c->d_tok, B, Cp, st.words, s));
   PG_MARK(kNone);
   for (size_t i = 0; i < m.layers.size(); ++i) {
     const StackLayer& l = m.layers[i];
@@ -608,7 +608,7 @@ pg_status step_launches(const pg_model* model, pg_kv_cache* c, ProfileMarks* mar
     }
     PG_MARK(kQkv);
     pgk::MixDecode d{};
-    d.nseq = B; d.d_pos = st.d_pos;
+    d.nseq = B; d.d_pos = &st.words->pos;
     d.y = st.y; d.ld_y = l.n_in;
     d.out = st.mix; d.ld_out = l.mix_pad;
     d.act = st.act;
@@ -656,14 +656,14 @@ pg_status step_launches(const pg_model* model, pg_kv_cache* c, ProfileMarks* mar
                        : head_rows(model, gemm, st.x, st.h, nullptr, c->logits_buf);
   if (r) return r;
   PG_MARK(kLogits);
-  PG_HIP(pgk::launch_add_one(st.d_pos, s));
   return PG_OK;
 }
 
 }  // namespace
 
-pg_status stack_set_pos(pg_kv_cache* c, size_t pos) {
-  PG_HIP(pgk::launch_set_int(c->stack->d_pos, (int)pos, c->stream));
+pg_status stack_set_pos(pg_kv_cache* c, size_t pos, uint32_t* out) {
+  c->stack->lists_ids = out != nullptr;
+  PG_HIP(pgk::launch_set_words(c->stack->words, (int)pos, out, c->stream));
   return PG_OK;
 }
 

@@ -51,7 +51,8 @@ struct StackCache {
     float *kring = nullptr, *vring = nullptr, *conv = nullptr, *state = nullptr;
   };
   std::vector<Layer> layers;
-  int* d_pos = nullptr;       // position of the next token, on the device
+  pgk::StepWords* words = nullptr;  // position of the next token, on the device
+  bool lists_ids = false;           // ... steps list their ids
   // one token of every sequence
   float *x = nullptr, *h = nullptr, *y = nullptr, *mix = nullptr, *act = nullptr, *part = nullptr;
   // many rows: one block, grown on demand
@@ -74,10 +75,11 @@ pg_status stack_cache_create(const pg_model* m, pg_kv_cache* c);
 // have their logits written to dst[n_rows][vocab] (device), in this order.
 pg_status stack_rows(const pg_model* m, pg_kv_cache* c, const uint32_t* ids, size_t n, size_t pos0,
                      const std::vector<int>& rows, float* dst, ProfileMarks* marks = nullptr);
-// Queues one token of every sequence: ids in c->d_tok, position in StackCache::d_pos (advanced);
+// Queues one token of every sequence: ids in c->d_tok, position in StackCache::words (advanced);
 // logits to c->logits_buf.
 pg_status stack_step(const pg_model* m, pg_kv_cache* c, ProfileMarks* marks = nullptr);
-// Sets the position on the device.
-pg_status stack_set_pos(pg_kv_cache* c, size_t pos);
+// Sets the position on the device, and where the steps from here on list their ids (device memory,
+// [step][B]; null: nowhere).
+pg_status stack_set_pos(pg_kv_cache* c, size_t pos, uint32_t* out = nullptr);
 
 }  // namespace pgh
