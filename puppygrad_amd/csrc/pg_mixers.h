@@ -14,7 +14,6 @@ namespace pgk {
 
 constexpr int kMixMaxDim = 256;   // key and value sizes per head
 constexpr int kMixMaxTaps = 16;   // short convolution
-constexpr int kSplitKeys = 64;   // keys per block of the attention's decode form
 
 // Rotary positions: the pair (i, i + half) of a head turns by position * freq[i], i < half; the
 // head's values from 2 * half on pass unchanged.
@@ -106,7 +105,8 @@ struct MixDecode {
   int attn_splits;
   float* part;
 };
-int attn_decode_splits(int chunk);
+// Key splits of a layer's attention (rec: the recurrence beside it, or null).
+int mix_decode_splits(const ChunkAttn& a, const Recurrence* rec);
 hipError_t launch_mix_decode(const MixDecode& a, hipStream_t s);
 hipError_t launch_attn_sum(const MixDecode& a, hipStream_t s);
 

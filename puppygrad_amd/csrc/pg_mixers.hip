@@ -56,22 +56,32 @@ constexpr int kRG = 8;  // query heads of one key/value head that a block takes
 
 // LDS of a decode block of NT threads (floats): the attention role's, the larger of the two.
 template <int NT>
-constexpr int kDecodeLds = kRG * kMixMaxDim + 2 * kMixMaxDim + kRG * kSplitKeys + NT * kRG;
+constexpr int kDecodeLds = 16 * (kMixMaxDim + 4) + 2 * kMixMaxDim + (NT / 64) * kRG * 64;
 
-// Keys [kSplitKeys split, ...) of the current chunk against kRG query heads of key/value head g.
-// NV: float4 per lane and key (sixteen lanes to a key).  Nothing that is loaded before the first
-// barrier depends on another load but the ring rows' bound, and all of a block's key rows are
-// requested together, then all of its value rows.
+// Keys [NT / 4 split, ...) of the current chunk against kRG query heads of key/value head g, sixteen
+// keys to a wavefront, on the f32 matrix cores (v_mfma_f32_16x16x4_f32: A operand lane l ->
+// A[l % 16][l / 16], B operand lane l -> B[l / 16][l % 16], D lane l, register v -> D[4 (l / 16) + v][l % 16]):
+//   S^T (keys x heads) = K . Q^T, lane (key, quarter) holding a quarter of the key's dims;
+//   O (heads x dims) += W . V: register v of a lane, the weight of key 4 (l / 16) + v, is the operand
+//   of step v as it is, against V's rows 4 (l / 16) + v.
+// The wavefronts' sums are added through LDS.  Nothing that is loaded before the first barrier
+// depends on another load but on the position.  NV: 64-dim parts of a head.
 template <int NT, int NV>
 __device__ void attn_role(const MixDecode& m, int b, int item, float* lds) {
+  constexpr int SK = NT / 4, NW = NT / 64;
+  constexpr int DQ = 16 * NV;           // dims of a lane's quarter, at most
+  constexpr bool PREV = NV <= 2;        // values requested together with the keys
+  typedef float f4v __attribute__((ext_vector_type(4)));
   const ChunkAttn& a = m.attn;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int l16 = lane & 15, quarter = lane >> 4;
   const int R = a.heads / a.kv_heads, groups = (R + kRG - 1) / kRG;
   const int split = item % m.attn_splits, rest = item / m.attn_splits;
   const int rg = rest % groups, g = rest / groups;
   const int r0 = rg * kRG, nr = min(kRG, R - r0);
   const int dim = a.dim, dp = a.dim_pad, half = a.rot.half;
-  const int j0 = split * kSplitKeys;
+  const int dq = (dim + 15) / 16 * 4;   // dims of a quarter
+  const int j0 = split * SK;
   const float* kring = a.kring + (size_t)b * a.ring_seq + (size_t)g * a.chunk * dp;
   const float* vring = a.vring + (size_t)b * a.ring_seq + (size_t)g * a.chunk * dp;
   const int pos = *m.d_pos, last = pos % a.chunk;  // ring row of the current token
@@ -82,72 +92,68 @@ __device__ void attn_role(const MixDecode& m, int b, int item, float* lds) {
         m.part[(((size_t)b * m.attn_splits + split) * a.heads + g * R + r0) * dim + i] = 0.0f;
     return;
   }
-  const int nk = min(last + 1 - j0, kSplitKeys);
-  const int own = last - j0;  // the current token's key in this split, if it is below nk
-  const int sub = lane >> 4, l16 = lane & 15;
-  // key rows: four to a wavefront and step
-  constexpr int KS = kSplitKeys * 16 / NT, KR = NT / 16;  // steps, keys per step
-  f4 kv[KS][NV];
+  const int nk = min(last + 1 - j0, SK);
+  const int own = last - j0;            // the current token's key in this split, if it is below nk
+  const int jk = 16 * wave + l16;       // this lane's key (scores)
+  const bool active = 16 * wave < nk;   // (wavefront-uniform)
+  f4 kv[4 * NV];
+  float vv[4 * NV][4];
+  auto fetch_v = [&]() __attribute__((always_inline)) {
 #pragma unroll
-  for (int q = 0; q < KS; ++q) {
-    const int j = min(KR * q + wave * 4 + sub, max(nk - 1, 0));
+    for (int v = 0; v < 4; ++v) {
+      const float* row = vring + (size_t)(j0 + min(16 * wave + 4 * quarter + v, nk - 1)) * dp;
 #pragma unroll
-    for (int i = 0; i < NV; ++i) {
-      const int e = 4 * l16 + 64 * i;
-      kv[q][i] = *reinterpret_cast<const f4*>(kring + (size_t)(j0 + j) * dp + min(e, dp - 4));
+      for (int t = 0; t < 4 * NV; ++t) vv[t][v] = row[min(16 * t + l16, dp - 1)];
     }
+  };
+  if (active) {
+    const float* row = kring + (size_t)(j0 + min(jk, nk - 1)) * dp;
+#pragma unroll
+    for (int i = 0; i < DQ / 4; ++i) kv[i] = *reinterpret_cast<const f4*>(row + min(quarter * dq + 4 * min(i, dq / 4 - 1), dp - 4));
+    if (PREV) fetch_v();
   }
-  float* qs = lds;                       // [kRG][dp]
-  float* kn = qs + kRG * dp;             // [dp] the current token's key, rotated
-  float* vn = kn + dp;                   // [dp] ... as projected
-  float* w = vn + dp;                    // [kRG][kSplitKeys]
-  float* red = w + kRG * kSplitKeys;     // [NT][kRG]
+  constexpr int QLD = 64 * NV + 4;
+  float* qs = lds;                      // [16][QLD], rows past nr and columns past dim are 0
+  float* kn = qs + 16 * QLD;            // [256] the current token's key, rotated
+  float* vn = kn + kMixMaxDim;          // [256] ... as projected
+  float* red = vn + kMixMaxDim;         // [NW][kRG][64]
   const float* y = m.y + (size_t)b * m.ld_y;
   const float* yk = y + a.k_col + g * dim;
   const float* yq = y + a.q_col + (size_t)(g * R + r0) * dim;
-  for (int i = tid; i < dp; i += NT) {
-    if (i < half) {
-      float s, c;
-      const float u = yk[i], v = yk[i + half];
-      turn(pos, a.rot.freq[i], &s, &c);
-      kn[i] = u * c - v * s;
-      kn[i + half] = v * c + u * s;
-      vn[i] = u;
-      vn[i + half] = v;
-    } else if (i >= 2 * half) {
-      kn[i] = vn[i] = i < dim ? yk[i] : 0.0f;
-    }
-  }
-  // queries: a pair (or a value that passes) per thread
-  const int per = dp - half;
-  for (int i = tid; i < nr * per; i += NT) {
+  // a pair (or values that pass, two apart) per thread; row nr is the key
+  const int per = 32 * NV;  // >= half, and 2 per >= dim
+  for (int i = tid; i < 17 * per; i += NT) {
     const int r = i / per, e = i - r * per;
+    const bool is_k = r == 16, live = r < nr || is_k;
+    const float* src = is_k ? yk : yq + r * dim;
+    float* dst = is_k ? kn : qs + r * QLD;
     if (e < half) {
-      float s, c;
-      const float u = yq[r * dim + e], v = yq[r * dim + e + half];
+      float u = 0.0f, v = 0.0f, s, c;
+      if (live) {
+        u = src[e];
+        v = src[e + half];
+      }
       turn(pos, a.rot.freq[e], &s, &c);
-      qs[r * dp + e] = u * c - v * s;
-      qs[r * dp + e + half] = v * c + u * s;
-    } else {
-      qs[r * dp + e + half] = e + half < dim ? yq[r * dim + e + half] : 0.0f;
+      dst[e] = u * c - v * s;
+      dst[e + half] = v * c + u * s;
+      if (is_k) {
+        vn[e] = u;
+        vn[e + half] = v;
+      }
+    }
+    // the values past the pairs: 2 half + (e, and e + per)
+#pragma unroll
+    for (int k = 0; k < 2; ++k) {
+      const int x = 2 * half + e + k * per;
+      if (x < 64 * NV) {
+        const float u = live && x < dim ? src[x] : 0.0f;
+        dst[x] = u;
+        if (is_k) vn[x] = u;
+      }
     }
   }
   __syncthreads();
-  // value rows of this thread's column, requested ahead of the scores
-  int cols = 1;
-  while (cols < dim) cols <<= 1;
-  const int parts = NT / cols, d = tid % cols, part = tid / cols;
-  constexpr int VB = 16;  // value rows in flight per thread
-  float vv[VB];
-  auto fetch_v = [&](int jb) {
-#pragma unroll
-    for (int q = 0; q < VB; ++q) {
-      const int j = min(jb + part + parts * q, nk - 1);
-      vv[q] = vring[(size_t)(j0 + j) * dp + min(d, dp - 1)];
-    }
-  };
-  fetch_v(0);
-  if (rg == 0 && own < kSplitKeys) {
+  if (rg == 0 && own < SK) {
     float* kw = a.kring + (size_t)b * a.ring_seq + ((size_t)g * a.chunk + last) * dp;
     float* vw = a.vring + (size_t)b * a.ring_seq + ((size_t)g * a.chunk + last) * dp;
     for (int i = tid; i < dp; i += NT) {
@@ -155,98 +161,114 @@ __device__ void attn_role(const MixDecode& m, int b, int item, float* lds) {
       vw[i] = vn[i];
     }
   }
+  f4v o[4 * NV];
 #pragma unroll
-  for (int q = 0; q < KS; ++q) {
-    const int j = KR * q + wave * 4 + sub;
-    if (KR * q >= nk) break;
-    if (j == own) {
+  for (int t = 0; t < 4 * NV; ++t) o[t] = f4v{0.f, 0.f, 0.f, 0.f};
+  if (active) {
+    f4v s = f4v{0.f, 0.f, 0.f, 0.f};
+    const float* q = qs + l16 * QLD + quarter * dq;
+    const float* ko = kn + quarter * dq;
 #pragma unroll
-      for (int i = 0; i < NV; ++i) kv[q][i] = *reinterpret_cast<const f4*>(kn + min(4 * l16 + 64 * i, dp - 4));
+    for (int i = 0; i < DQ / 4; ++i) {
+      if (4 * i >= dq) break;
+      f4 k4 = kv[i];
+      if (jk == own) k4 = *reinterpret_cast<const f4*>(ko + 4 * i);
+      const f4 q4 = *reinterpret_cast<const f4*>(q + 4 * i);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) s = __builtin_amdgcn_mfma_f32_16x16x4f32(k4[e], q4[e], s, 0, 0, 0);
+    }
+    if (!PREV) fetch_v();
+    const float bias = a.bias[g * R + r0 + min(l16, nr - 1)];
+    float w[4];
+#pragma unroll
+    for (int v = 0; v < 4; ++v) {
+      const int j = 16 * wave + 4 * quarter + v;
+      w[v] = j < nk ? sigmoid(s[v] * a.scale + bias) : 0.0f;
     }
 #pragma unroll
-    for (int r = 0; r < kRG; ++r) {
-      if (r >= nr) break;
-      float s = 0.0f;
+    for (int v = 0; v < 4; ++v) {
+      const bool mine = 16 * wave + 4 * quarter + v == own;
 #pragma unroll
-      for (int i = 0; i < NV; ++i) {
-        const int e = 4 * l16 + 64 * i;
-        if (e < dp) {
-          const f4 x = *reinterpret_cast<const f4*>(qs + r * dp + e);
-          s += (kv[q][i].x * x.x + kv[q][i].y * x.y) + (kv[q][i].z * x.z + kv[q][i].w * x.w);
-        }
+      for (int t = 0; t < 4 * NV; ++t) {
+        const float x = mine ? vn[16 * t + l16] : vv[t][v];
+        o[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(w[v], x, o[t], 0, 0, 0);
       }
-      s += __shfl_xor(s, 8, 64);
-      s += __shfl_xor(s, 4, 64);
-      s += __shfl_xor(s, 2, 64);
-      s += __shfl_xor(s, 1, 64);
-      if (l16 == 0) w[r * kSplitKeys + j] = j < nk ? sigmoid(s * a.scale + a.bias[g * R + r0 + r]) : 0.0f;
     }
   }
-  __syncthreads();
-  float acc[kRG];
+  // rows (heads) 4 quarter + v, dims 16 t + l16; 64 dims at a time
 #pragma unroll
-  for (int r = 0; r < kRG; ++r) acc[r] = 0.0f;
-  for (int jb = 0; jb < nk; jb += VB * parts) {
-    if (jb) fetch_v(jb);
+  for (int p = 0; p < NV; ++p) {
+    if (64 * p >= dim) break;
+    if (p) __syncthreads();
+    if (quarter < kRG / 4)
 #pragma unroll
-    for (int q = 0; q < VB; ++q) {
-      const int j = jb + part + parts * q;
-      if (j >= nk) break;
-      const float v = j == own ? vn[min(d, dp - 1)] : vv[q];
+      for (int t = 0; t < 4; ++t)
 #pragma unroll
-      for (int r = 0; r < kRG; ++r)
-        if (r < nr) acc[r] += w[r * kSplitKeys + j] * v;
+        for (int v = 0; v < 4; ++v) red[(wave * kRG + 4 * quarter + v) * 64 + 16 * t + l16] = o[4 * p + t][v];
+    __syncthreads();
+    for (int i = tid; i < nr * 64; i += NT) {
+      const int r = i >> 6, d = 64 * p + (i & 63);
+      if (d >= dim) continue;
+      float sum = 0.0f;
+#pragma unroll
+      for (int w = 0; w < NW; ++w) sum += red[w * kRG * 64 + i];
+      const int h = g * R + r0 + r;
+      if (m.attn_splits > 1)
+        m.part[(((size_t)b * m.attn_splits + split) * a.heads + h) * dim + d] = sum * a.out_scale;
+      else
+        m.out[(size_t)b * m.ld_out + a.out_col + h * dim + d] = sum * a.out_scale;
     }
-  }
-#pragma unroll
-  for (int r = 0; r < kRG; ++r)
-    if (r < nr) red[(r * parts + part) * cols + d] = acc[r];
-  __syncthreads();
-  for (int i = tid; i < nr * cols; i += NT) {
-    const int r = i / cols, dd = i - r * cols;
-    if (dd >= dim) continue;
-    float s = 0.0f;
-    for (int p = 0; p < parts; ++p) s += red[(r * parts + p) * cols + dd];
-    const int h = g * R + r0 + r;
-    if (m.attn_splits > 1)
-      m.part[(((size_t)b * m.attn_splits + split) * a.heads + h) * dim + dd] = s * a.out_scale;
-    else
-      m.out[(size_t)b * m.ld_out + a.out_col + h * dim + dd] = s * a.out_scale;
   }
 }
 
-// Channel ch of a short convolution at position pos (up to four taps: every load is issued at
-// once, whatever pos is), and the ring row of this position (no block reads it in this step).
-__device__ __forceinline__ float conv_channel(const ShortConv& c, const float* y, float* ring, int ch, int pos, bool keep) {
-  const float cur = y[c.col + ch];
-  float s = 0.0f;
+// N channels ch[] of a short convolution at position pos, and the ring rows of this position
+// (where keep[]; no block reads them in this step).  With up to four taps everything is loaded
+// before the first value is used.
+template <int N>
+__device__ __forceinline__ void conv_channels(const ShortConv& c, const float* y, float* ring, const int (&ch)[N],
+                                              const bool (&keep)[N], int pos, float (&out)[N]) {
+  float cur[N];
+#pragma unroll
+  for (int n = 0; n < N; ++n) cur[n] = y[c.col + ch[n]];
+  const int slot = pos % c.taps;
   if (c.taps <= 4) {
-    float x[4], w[4];
+    float x[N][4], w[N][4];
 #pragma unroll
-    for (int k = 0; k < 4; ++k) {
-      const int kk = min(k, c.taps - 1);
-      x[k] = ring[(size_t)kk * c.channels + ch];  // the input whose position is k modulo taps
-      w[k] = c.w[ch * c.taps + kk];
-    }
-    const int slot = pos % c.taps;
+    for (int n = 0; n < N; ++n)
 #pragma unroll
-    for (int k = 0; k < 4; ++k) {
-      if (k >= c.taps) break;
-      int j = slot - k;  // tokens back
-      if (j < 0) j += c.taps;
-      const float in = j == 0 ? cur : pos >= j ? x[k] : 0.0f;
-      float wt = w[0];
+      for (int k = 0; k < 4; ++k) {
+        const int kk = min(k, c.taps - 1);
+        x[n][k] = ring[(size_t)kk * c.channels + ch[n]];  // the input whose position is k modulo taps
+        w[n][k] = c.w[ch[n] * c.taps + kk];
+      }
 #pragma unroll
-      for (int i = 1; i < 4; ++i) wt = i == c.taps - 1 - j ? w[i] : wt;
-      s += wt * in;
+    for (int n = 0; n < N; ++n) {
+      float s = 0.0f;
+#pragma unroll
+      for (int k = 0; k < 4; ++k) {
+        int j = slot - k;  // tokens back
+        if (j < 0) j += c.taps;
+        const float in = k >= c.taps || pos < j ? 0.0f : j == 0 ? cur[n] : x[n][k];
+        float wt = w[n][0];
+#pragma unroll
+        for (int i = 1; i < 4; ++i) wt = i == c.taps - 1 - j ? w[n][i] : wt;
+        s += wt * in;
+      }
+      out[n] = silu(s);
     }
   } else {
-    s = c.w[ch * c.taps + c.taps - 1] * cur;
-    for (int j = 1; j < c.taps; ++j)
-      if (pos >= j) s += c.w[ch * c.taps + c.taps - 1 - j] * ring[(size_t)((pos - j) % c.taps) * c.channels + ch];
+#pragma unroll
+    for (int n = 0; n < N; ++n) {
+      float s = c.w[ch[n] * c.taps + c.taps - 1] * cur[n];
+      for (int j = 1; j < c.taps; ++j)
+        if (pos >= j)
+          s += c.w[ch[n] * c.taps + c.taps - 1 - j] * ring[(size_t)((pos - j) % c.taps) * c.channels + ch[n]];
+      out[n] = silu(s);
+    }
   }
-  if (keep) ring[(size_t)(pos % c.taps) * c.channels + ch] = cur;
-  return silu(s);
+#pragma unroll
+  for (int n = 0; n < N; ++n)
+    if (keep[n]) ring[(size_t)slot * c.channels + ch[n]] = cur[n];
 }
 
 // One head of the recurrence.  A thread owns column v of the state and every `parts`-th of its
@@ -285,9 +307,13 @@ __device__ void recurrence_role(const MixDecode& m, int b, int h, float* lds) {
     const bool first = h % (c.heads / c.kv_heads) == 0;
     const float yb = y[c.b_col + h], ya = y[c.a_col + h], al0 = c.a_log[h], dt = c.dt_bias[h];
     const int td = min(tid, dim - 1);
-    float qv = conv_channel(cv, y, ring, c.q_col - cv.col + kvh * dim + td, pos, first && tid < dim);
-    float kv = conv_channel(cv, y, ring, c.k_col - cv.col + kvh * dim + td, pos, first && tid < dim);
-    const float x = conv_channel(cv, y, ring, c.v_col - cv.col + h * vdim + tv, pos, tid < vdim);
+    const int ch[3] = {c.q_col - cv.col + kvh * dim + td, c.k_col - cv.col + kvh * dim + td,
+                       c.v_col - cv.col + h * vdim + tv};
+    const bool keep[3] = {first && tid < dim, first && tid < dim, tid < vdim};
+    float cq[3];
+    conv_channels<3>(cv, y, ring, ch, keep, pos, cq);
+    float qv = cq[0], kv = cq[1];
+    const float x = cq[2];
     if (tid >= dim) qv = kv = 0.0f;
     float qn = wave_sum(qv * qv), kn = wave_sum(kv * kv);
     if ((tid & 63) == 0 && tid < 256) {  // (nothing past kMixMaxDim = 256)
@@ -725,8 +751,8 @@ struct ChunkWork {
   int chunks;            // per sequence
   int dp, ep;            // dim and vdim padded to 32
   float *W, *U0, *Kd, *Qd, *P, *U, *S, *G;
-  // tile (sequence, chunk, head): W, Kd, Qd [32][dp]; U0, U [32][ep]; P [32][32]; S [dp][ep]; G [dp]
-  // (exp(G_end) per key channel)
+  // tile (sequence, chunk, head): W, Kd, Qd [32][dp]; U0, U [ep / 32][32][32]; P [32][32];
+  // S [ep / 32][dp][32]; G [dp] (exp(G_end) per key channel)
   __device__ __forceinline__ size_t tile(int b, int c, int h, int heads) const {
     return ((size_t)b * chunks + c) * heads + h;
   }
@@ -866,8 +892,8 @@ __global__ __launch_bounds__(256) void k_delta_chunk(MixRows r, Recurrence c, Ch
       x[t] = s;
       __builtin_amdgcn_sched_barrier(0);  // (row by row: all rows of A at once do not fit the registers)
     }
-    float* dst = isw ? w.W + tile * 32 * dp + col : w.U0 + tile * 32 * ep + e;
-    const int ld = isw ? dp : ep;
+    float* dst = isw ? w.W + tile * 32 * dp + col : w.U0 + tile * 32 * ep + (e >> 5) * 1024 + (e & 31);
+    const int ld = isw ? dp : 32;
 #pragma unroll
     for (int t = 0; t < kChunk; ++t) dst[t * ld] = x[t];
   }
@@ -905,7 +931,7 @@ __global__ __launch_bounds__(256) void k_gla_chunk(MixRows r, Recurrence c, Chun
     Gs[t * LD + d] = g;
   }
   for (int i = tid; i < 32 * ep; i += 256) {
-    const int t = i / ep, e = i - t * ep;
+    const int t = (i >> 5) & 31, e = (i >> 10) * 32 + (i & 31);
     w.U[tile * 32 * ep + i] = t < nt && e < vdim ? r.y[(row0 + t) * r.ld_y + c.v_col + h * vdim + e] : 0.0f;
   }
   __syncthreads();
@@ -942,14 +968,15 @@ __global__ __launch_bounds__(256) void k_gla_chunk(MixRows r, Recurrence c, Chun
 // v of lane (l, half) is row 8 (v / 4) + 4 half + v % 4 of column l.  In that layout the state is
 // an operand of W S as it is (step v multiplies the rows its two lane halves hold), and so is U
 // of Kd^T U.  The wavefronts' parts of W S meet in LDS, two buffers in turn.  A chunk's tiles are
-// requested two chunks ahead (one with more than four wavefronts).  WAVES: the most of a block.
+// requested two chunks ahead (one with more than four wavefronts).
 template <bool DELTA, int WAVES>
 __global__ __launch_bounds__(64 * WAVES) void k_chunk_states(MixRows r, Recurrence c, ChunkWork w) {
-  extern __shared__ float part[];  // [2][waves][16][64] (delta)
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, waves = blockDim.x >> 6;
+  extern __shared__ __attribute__((aligned(16))) float part[];  // [2][WAVES][4][64][4] (delta)
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int half = lane >> 5, l32 = lane & 31;
   const int ct = blockIdx.x, h = blockIdx.y, b = blockIdx.z;
-  const int dp = w.dp, ep = w.ep, dim = c.dim, vdim = c.vdim;
+  constexpr int dp = 32 * WAVES;
+  const int cts = w.ep / 32, dim = c.dim, vdim = c.vdim;
   const int col = 32 * ct + l32;
   float* state = c.state + (size_t)b * c.state_seq + (size_t)h * dim * vdim;
   auto row_of = [&](int v) { return 8 * (v >> 2) + 4 * half + (v & 3); };
@@ -965,49 +992,57 @@ __global__ __launch_bounds__(64 * WAVES) void k_chunk_states(MixRows r, Recurren
   };
   auto fetch = [&](int ci, Tiles& x) __attribute__((always_inline)) {
     const size_t tile = w.tile(b, min(ci, w.chunks - 1), h, c.heads);
-    const float* u = (DELTA ? w.U0 : w.U) + tile * 32 * ep + col;
-    const float* kd = w.Kd + tile * 32 * dp + 32 * wave + l32;
+    const float* u = (DELTA ? w.U0 : w.U) + (tile * cts + ct) * 1024 + 128 * half + l32;
+    const float* kd = w.Kd + tile * 32 * dp + 32 * wave + 4 * half * dp + l32;
     const float* g = w.G + tile * dp + 32 * wave + 4 * half;
     if (DELTA) {
-      const float* wt = w.W + tile * 32 * dp + (size_t)l32 * dp + 32 * wave + 4 * half;
+      const float* wt = w.W + tile * 32 * dp + 32 * wave + l32 * dp + 4 * half;
 #pragma unroll
       for (int q = 0; q < 4; ++q) x.w[q] = *reinterpret_cast<const f4*>(wt + 8 * q);
     }
 #pragma unroll
-    for (int v = 0; v < 16; ++v) x.u[v] = u[row_of(v) * ep];
+    for (int v = 0; v < 16; ++v) x.u[v] = u[(8 * (v >> 2) + (v & 3)) * 32];
 #pragma unroll
-    for (int v = 0; v < 16; ++v) x.k[v] = kd[row_of(v) * dp];
+    for (int v = 0; v < 16; ++v) x.k[v] = kd[(8 * (v >> 2) + (v & 3)) * dp];
 #pragma unroll
     for (int q = 0; q < 4; ++q) x.g[q] = *reinterpret_cast<const f4*>(g + 8 * q);
   };
   auto chunk = [&](int ci, Tiles& x) __attribute__((always_inline)) {
-    const size_t tile = w.tile(b, ci, h, c.heads);
-    float* s0 = w.S + tile * dp * ep + (size_t)(32 * wave) * ep + col;
+    __builtin_amdgcn_sched_barrier(0);
+    const size_t tile = w.tile(b, ci, h, c.heads) * cts + ct;
+    float* s0 = w.S + (tile * WAVES + wave) * 1024 + 128 * half + l32;
 #pragma unroll
-    for (int v = 0; v < 16; ++v) s0[row_of(v) * ep] = S[v];
+    for (int v = 0; v < 16; ++v) s0[(8 * (v >> 2) + (v & 3)) * 32] = S[v];
     if (DELTA) {
       f16v p;
 #pragma unroll
       for (int v = 0; v < 16; ++v) p[v] = 0.0f;
 #pragma unroll
       for (int v = 0; v < 16; ++v) p = __builtin_amdgcn_mfma_f32_32x32x2f32(x.w[v >> 2][v & 3], S[v], p, 0, 0, 0);
-      float* mine = part + (size_t)((ci & 1) * waves + wave) * 1024 + lane;
+      f4* mine = reinterpret_cast<f4*>(part) + (size_t)((ci & 1) * WAVES + wave) * 256 + lane;
 #pragma unroll
-      for (int v = 0; v < 16; ++v) mine[64 * v] = p[v];
+      for (int q = 0; q < 4; ++q) mine[64 * q] = f4{p[4 * q], p[4 * q + 1], p[4 * q + 2], p[4 * q + 3]};
       __syncthreads();
-      const float* all = part + (size_t)((ci & 1) * waves) * 1024 + lane;
-      for (int o = 0; o < waves; ++o)
+      const f4* all = reinterpret_cast<const f4*>(part) + (size_t)((ci & 1) * WAVES) * 256 + lane;
 #pragma unroll
-        for (int v = 0; v < 16; ++v) x.u[v] -= all[(size_t)o * 1024 + 64 * v];
-      float* ud = w.U + tile * 32 * ep + col;
+      for (int o = 0; o < WAVES; ++o)
 #pragma unroll
-      for (int v = 0; v < 16; ++v)
-        if (v % waves == wave) ud[row_of(v) * ep] = x.u[v];
+        for (int q = 0; q < 4; ++q) {
+          const f4 z = all[o * 256 + 64 * q];
+#pragma unroll
+          for (int e = 0; e < 4; ++e) x.u[4 * q + e] -= z[e];
+        }
+      if (wave == ci % WAVES) {
+        float* ud = w.U + tile * 1024 + 128 * half + l32;
+#pragma unroll
+        for (int v = 0; v < 16; ++v) ud[(8 * (v >> 2) + (v & 3)) * 32] = x.u[v];
+      }
     }
 #pragma unroll
     for (int v = 0; v < 16; ++v) S[v] *= x.g[v >> 2][v & 3];
 #pragma unroll
     for (int v = 0; v < 16; ++v) S = __builtin_amdgcn_mfma_f32_32x32x2f32(x.k[v], x.u[v], S, 0, 0, 0);
+    __builtin_amdgcn_sched_barrier(0);
   };
   // (past the end: the last chunk's tiles again, never used)
   Tiles x0, x1;
@@ -1073,12 +1108,12 @@ __global__ __launch_bounds__(256) void k_chunk_out(MixRows r, Recurrence c, Chun
     const int ct = wave + 4 * k;
     if (ct >= tiles) break;
     // rows half * dp / 2 + j of the state meet columns half * dp / 2 + j of Qd
-    const float* s = w.S + tile * dp * ep + (size_t)(half * (dp / 2)) * ep + 32 * ct + l32;
+    const float* s = w.S + tile * dp * ep + (size_t)ct * dp * 32 + half * (dp / 2) * 32 + l32;
     const float* q = Qs + l32 * LD + half * (dp / 2);
     for (int j = 0; j < dp / 2; j += 16) {
       float sv[16];
 #pragma unroll
-      for (int e = 0; e < 16; ++e) sv[e] = s[(size_t)(j + e) * ep];
+      for (int e = 0; e < 16; ++e) sv[e] = s[(j + e) * 32];
 #pragma unroll
       for (int e = 0; e < 16; e += 4) {
         const f4 a4 = *reinterpret_cast<const f4*>(q + j + e);
@@ -1086,10 +1121,10 @@ __global__ __launch_bounds__(256) void k_chunk_out(MixRows r, Recurrence c, Chun
         for (int k4 = 0; k4 < 4; ++k4) o[k] = __builtin_amdgcn_mfma_f32_32x32x2f32(a4[k4], sv[e + k4], o[k], 0, 0, 0);
       }
     }
-    const float* u = w.U + tile * 32 * ep + (size_t)(16 * half) * ep + 32 * ct + l32;
+    const float* u = w.U + tile * 32 * ep + ct * 1024 + 16 * half * 32 + l32;
     float uv[16];
 #pragma unroll
-    for (int e = 0; e < 16; ++e) uv[e] = u[e * ep];
+    for (int e = 0; e < 16; ++e) uv[e] = u[e * 32];
 #pragma unroll
     for (int e = 0; e < 16; e += 4) {
       const f4 a4 = *reinterpret_cast<const f4*>(&Ps[l32][16 * half + e]);
@@ -1210,18 +1245,24 @@ int rows_per_thread(int dim, int vdim) {
 
 }  // namespace
 
-int attn_decode_splits(int chunk) { return (chunk + kSplitKeys - 1) / kSplitKeys; }
+// Threads of a decode block: rows of a state column per thread of a block of 256; blocks grow so
+// that a thread holds few.
+static int decode_threads(int rows) { return rows <= 8 ? 256 : rows == 16 ? 512 : 1024; }
+
+int mix_decode_splits(const ChunkAttn& a, const Recurrence* rec) {
+  const int keys = decode_threads(rec ? rows_per_thread(rec->dim, rec->vdim) : 1) / 4;
+  return (a.chunk + keys - 1) / keys;
+}
 
 hipError_t launch_mix_decode(const MixDecode& a, hipStream_t s) {
   int attn_items = 0;
   if (a.has_attn) {
+    if (a.attn_splits != mix_decode_splits(a.attn, a.has_rec ? &a.rec : nullptr)) return hipErrorInvalidValue;
     const int R = a.attn.heads / a.attn.kv_heads;
     attn_items = a.attn.kv_heads * ((R + kRG - 1) / kRG) * a.attn_splits;
   }
   const int rec_items = a.has_rec ? a.rec.heads : 0;
-  // Rows of a state column per thread of a block of 256; blocks grow so that a thread holds few.
-  const int rows = a.has_rec ? rows_per_thread(a.rec.dim, a.rec.vdim) : 1;
-  const int nt = rows <= 8 ? 256 : rows == 16 ? 512 : 1024;
+  const int rows = a.has_rec ? rows_per_thread(a.rec.dim, a.rec.vdim) : 1, nt = decode_threads(rows);
   const int mlp_items = a.has_mlp ? (a.mlp.ff_pad + nt - 1) / nt : 0;
   const dim3 grid((unsigned)(attn_items + rec_items + mlp_items), (unsigned)a.nseq);
   if (grid.x == 0) return hipSuccess;
@@ -1278,15 +1319,22 @@ hipError_t launch_short_conv_rows(const MixRows& r, const ShortConv& c, hipStrea
   return hipGetLastError();
 }
 
+// Key size as the chunk kernels pad it: 32 rows of the state to a wavefront, and numbers of
+// wavefronts that k_chunk_states is instantiated for.
+static int chunk_dim(int dim) {
+  const int waves = (dim + 31) / 32;
+  return 32 * (waves == 5 ? 6 : waves == 7 ? 8 : waves);
+}
+
 size_t recurrence_work_floats(const Recurrence& c, int nseq, int n) {
-  const int dp = (c.dim + 31) / 32 * 32, ep = (c.vdim + 31) / 32 * 32;
+  const int dp = chunk_dim(c.dim), ep = (c.vdim + 31) / 32 * 32;
   return chunk_floats(dp, ep, c.delta != 0) * (size_t)nseq * ((n + kChunk - 1) / kChunk) * c.heads;
 }
 
 hipError_t launch_recurrence_rows(const MixRows& r, const Recurrence& c, hipStream_t s) {
   ChunkWork w{};
   w.chunks = (r.n + kChunk - 1) / kChunk;
-  w.dp = (c.dim + 31) / 32 * 32;
+  w.dp = chunk_dim(c.dim);
   w.ep = (c.vdim + 31) / 32 * 32;
   const size_t tiles = (size_t)r.nseq * w.chunks * c.heads;
   if (r.work_floats < recurrence_work_floats(c, r.nseq, r.n)) return hipErrorInvalidValue;
@@ -1330,14 +1378,16 @@ hipError_t launch_recurrence_rows(const MixRows& r, const Recurrence& c, hipStre
   if (e != hipSuccess) return e;
   const dim3 sgrid(w.ep / 32, c.heads, r.nseq);
   const size_t slds = c.delta ? 2 * waves * 1024 * sizeof(float) : 0;
-  if (c.delta && waves <= 4)
-    hipLaunchKernelGGL((k_chunk_states<true, 4>), sgrid, dim3(64 * waves), slds, s, r, c, w);
-  else if (c.delta)
-    hipLaunchKernelGGL((k_chunk_states<true, 8>), sgrid, dim3(64 * waves), slds, s, r, c, w);
-  else if (waves <= 4)
-    hipLaunchKernelGGL((k_chunk_states<false, 4>), sgrid, dim3(64 * waves), slds, s, r, c, w);
-  else
-    hipLaunchKernelGGL((k_chunk_states<false, 8>), sgrid, dim3(64 * waves), slds, s, r, c, w);
+  switch (waves) {
+#define PG_WAVES(N)                                                                                          \
+  case N:                                                                                                    \
+    if (c.delta) hipLaunchKernelGGL((k_chunk_states<true, N>), sgrid, dim3(64 * N), slds, s, r, c, w);        \
+    else hipLaunchKernelGGL((k_chunk_states<false, N>), sgrid, dim3(64 * N), slds, s, r, c, w);               \
+    break;
+    PG_WAVES(1) PG_WAVES(2) PG_WAVES(3) PG_WAVES(4) PG_WAVES(6) PG_WAVES(8)
+#undef PG_WAVES
+    default: return hipErrorInvalidValue;
+  }
   if ((e = hipGetLastError()) != hipSuccess) return e;
   hipLaunchKernelGGL(k_chunk_out, grid, dim3(256), 32 * (size_t)(w.dp + 4) * sizeof(float), s, r, c, w);
   return hipGetLastError();

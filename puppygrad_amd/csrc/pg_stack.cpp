@@ -428,7 +428,7 @@ pg_status stack_create(const std::string& config_path, const Json& config, const
     m->max_ff = std::max(m->max_ff, l.has_mlp ? l.mlp.ff_pad : 0);
     if (l.has_attn) {
       m->max_keys = std::max(m->max_keys, up(l.attn.kv_heads * l.attn.dim, 4));
-      m->max_part = std::max(m->max_part, pgk::attn_decode_splits(l.attn.chunk) * l.attn.heads * l.attn.dim);
+      m->max_part = std::max(m->max_part, pgk::mix_decode_splits(l.attn, l.has_rec ? &l.rec : nullptr) * l.attn.heads * l.attn.dim);
     }
     if (l.has_rec) {
       if (l.rec.delta) m->max_conv = std::max(m->max_conv, l.rec.conv.channels);
@@ -614,7 +614,7 @@ pg_status step_launches(const pg_model* model, pg_kv_cache* c, ProfileMarks* mar
     d.act = st.act;
     d.has_attn = l.has_attn; d.has_rec = l.has_rec; d.has_mlp = l.has_mlp;
     d.attn = b.attn; d.rec = b.rec; d.mlp = l.mlp;
-    d.attn_splits = l.has_attn ? pgk::attn_decode_splits(l.attn.chunk) : 1;
+    d.attn_splits = l.has_attn ? pgk::mix_decode_splits(l.attn, l.has_rec ? &l.rec : nullptr) : 1;
     d.part = st.part;
     PG_HIP(pgk::launch_mix_decode(d, s));
     // the attention's key splits are added by the projection of the one-sequence step, where
