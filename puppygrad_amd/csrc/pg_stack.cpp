@@ -353,6 +353,12 @@ StackModel::~StackModel() {
 }
 StackCache::~StackCache() {
   if (graph) (void)hipGraphExecDestroy(graph);
+  if (side) {
+    (void)hipStreamSynchronize(side);
+    (void)hipStreamDestroy(side);
+  }
+  if (forked) (void)hipEventDestroy(forked);
+  if (joined) (void)hipEventDestroy(joined);
   if (rows) (void)hipFree(rows);
   if (rows_at) (void)hipFree(rows_at);
   for (void* p : memory) (void)hipFree(p);
@@ -509,6 +515,9 @@ pg_status stack_cache_create(const pg_model* model, pg_kv_cache* c) {
       (s = alloc(B * m.max_in, &st->y)) || (s = alloc(B * m.max_mix, &st->mix)) ||
       (s = alloc(B * m.max_ff, &st->act)) || (s = alloc(B * m.max_part, &st->part)))
     return s;
+  PG_HIP(hipStreamCreateWithFlags(&st->side, hipStreamNonBlocking));
+  PG_HIP(hipEventCreateWithFlags(&st->forked, hipEventDisableTiming));
+  PG_HIP(hipEventCreateWithFlags(&st->joined, hipEventDisableTiming));
   c->gemm_ws_floats = 8 * B * (size_t)std::max(m.max_in, m.width_pad);
   PG_HIP(hipMalloc(&c->gemm_ws, c->gemm_ws_floats * sizeof(float)));
   PG_HIP(hipMalloc(&c->logits_buf, B * m.vocab * sizeof(float)));
@@ -704,14 +713,14 @@ pg_status rows_segment(const pg_model* model, pg_kv_cache* c, const uint32_t* d_
   auto r64 = [](size_t v) { return round_up(v, 64); };
   const size_t ws_floats = 8 * rows * Cp;
   struct Piece { float** p; size_t n; };
-  float *x, *h, *y, *mix, *act, *krot, *conv, *decay, *work, *ws;
+  float *x, *h, *y, *mix, *act, *krot, *conv, *decay, *work, *ws, *ws_side;
   size_t work_floats = 0;
   for (const StackLayer& l : m.layers)
     if (l.has_rec) work_floats = std::max(work_floats, pgk::recurrence_work_floats(l.rec, (int)B, (int)n));
   const Piece pieces[] = {{&x, rows * Cp}, {&h, std::max(rows, want.size()) * Cp}, {&y, rows * m.max_in},
                           {&mix, rows * m.max_mix}, {&act, rows * m.max_ff}, {&krot, rows * m.max_keys},
                           {&conv, rows * m.max_conv}, {&decay, rows * m.max_decay}, {&work, work_floats},
-                          {&ws, ws_floats}};
+                          {&ws, ws_floats}, {&ws_side, ws_floats}};
   size_t total = 0;
   for (const Piece& p : pieces) total += r64(p.n);
   if (st.rows_floats < total) {
@@ -745,30 +754,44 @@ pg_status rows_segment(const pg_model* model, pg_kv_cache* c, const uint32_t* d_
     r.out = mix; r.ld_out = l.mix_pad; r.out_cols = l.mix_cols;
     r.act = act; r.k_rot = krot; r.conv_out = conv; r.decay = decay;
     r.work = work; r.work_floats = work_floats;
+    const bool more = i + 1 < m.layers.size();
+    float* next_h = more ? h : nullptr;
+    const float* next_g = more ? m.layers[i + 1].norm : nullptr;
+    // The recurrence is a chain over the tokens that leaves most of the chip idle: with enough
+    // rows, the attention and the MLP (its result goes straight to the residual) run beside it.
+    const bool fork = !marks && rows >= 64 && l.has_rec && (l.has_attn || l.has_mlp);
+    hipStream_t side = fork ? st.side : s;
+    Gemm side_gemm = gemm;
+    side_gemm.s = side;
+    side_gemm.ws = fork ? ws_side : ws;
+    if (fork) {
+      PG_HIP(hipEventRecord(st.forked, s));
+      PG_HIP(hipStreamWaitEvent(side, st.forked, 0));
+    }
     if (l.has_attn) {
-      PG_HIP(pgk::launch_rotary_rows(r, b.attn, s));
-      PG_HIP(pgk::launch_chunk_attn_rows(r, b.attn, s));
+      PG_HIP(pgk::launch_rotary_rows(r, b.attn, side));
+      PG_HIP(pgk::launch_chunk_attn_rows(r, b.attn, side));
+      PG_HIP(pgk::launch_commit_rows(r, &b.attn, nullptr, side));
+    }
+    PG_MARK(kAttention);
+    if (l.has_mlp) {
+      PG_HIP(pgk::launch_gated_mlp_rows(r, l.mlp, side));
+      PG_MARK(kMlpFc);
+      PG_HIP(side_gemm(act, l.down_w, x, (int)Cp, l.mlp.ff_pad, l.ls2, nullptr, nullptr));
+      PG_MARK(kMlpProj);
     }
     if (l.has_rec) {
       if (l.rec.delta) PG_HIP(pgk::launch_short_conv_rows(r, b.rec.conv, s));
       PG_HIP(pgk::launch_recurrence_rows(r, b.rec, s));
+      if (l.rec.delta) PG_HIP(pgk::launch_commit_rows(r, nullptr, &b.rec.conv, s));
     }
-    PG_HIP(pgk::launch_commit_rows(r, l.has_attn ? &b.attn : nullptr,
-                                   l.has_rec && l.rec.delta ? &b.rec.conv : nullptr, s));
+    if (fork) {
+      PG_HIP(hipEventRecord(st.joined, side));
+      PG_HIP(hipStreamWaitEvent(s, st.joined, 0));
+    }
     PG_MARK(kAttention);
-    const bool more = i + 1 < m.layers.size();
-    float* next_h = more ? h : nullptr;
-    const float* next_g = more ? m.layers[i + 1].norm : nullptr;
-    if (l.has_mlp) {
-      PG_HIP(pgk::launch_gated_mlp_rows(r, l.mlp, s));
-      PG_MARK(kMlpFc);
-    }
-    PG_HIP(gemm(mix, l.out_w, x, (int)Cp, l.mix_pad, l.ls1, next_g, l.has_mlp ? nullptr : next_h));
+    PG_HIP(gemm(mix, l.out_w, x, (int)Cp, l.mix_pad, l.ls1, next_g, next_h));
     PG_MARK(kAttnProj);
-    if (l.has_mlp) {
-      PG_HIP(gemm(act, l.down_w, x, (int)Cp, l.mlp.ff_pad, l.ls2, next_g, next_h));
-      PG_MARK(kMlpProj);
-    }
   }
   if (want.size() == 1) {
     if (pg_status e = head_one(model, x + (size_t)want[0] * Cp, dst, s)) return e;

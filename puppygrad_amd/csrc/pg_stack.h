@@ -58,6 +58,10 @@ struct StackCache {
   // many rows: one block, grown on demand
   float* rows = nullptr;
   size_t rows_floats = 0;
+  // Steps of many rows run the recurrence of a layer on the cache's stream and everything that does
+  // not depend on it on this one (fork and join are events).
+  hipStream_t side = nullptr;
+  hipEvent_t forked = nullptr, joined = nullptr;
   int* rows_at = nullptr;     // rows whose logits are wanted
   size_t rows_at_cap = 0;
   hipGraphExec_t graph = nullptr;  // the one-token step
