@@ -963,118 +963,126 @@ __global__ __launch_bounds__(256) void k_gla_chunk(MixRows r, Recurrence c, Chun
   }
 }
 
-// The states from chunk to chunk.  A block owns 32 value columns of one head; wavefront w keeps
-// the state's rows 32 w .. 32 w + 31 in the accumulator layout of the 32 x 32 MFMA, where register
-// v of lane (l, half) is row 8 (v / 4) + 4 half + v % 4 of column l.  In that layout the state is
-// an operand of W S as it is (step v multiplies the rows its two lane halves hold), and so is U
-// of Kd^T U.  The wavefronts' parts of W S meet in LDS, two buffers in turn.  A chunk's tiles are
-// requested two chunks ahead (one with more than four wavefronts).
+// The states from chunk to chunk.  A block owns 16 value columns of one head; wavefront w keeps
+// the state's rows 32 w .. 32 w + 31 in the accumulator layout of v_mfma_f32_16x16x4_f32, where
+// register v of lane (l, quarter) of row tile a is row 16 a + 4 quarter + v of column l.  In that
+// layout the state is an operand of W S as it is (step (a, v) multiplies the rows its four lane
+// quarters hold), and so is U of Kd^T U.  The wavefronts' parts of W S meet in LDS, two buffers in
+// turn.  A chunk's tiles are requested two chunks ahead.
 template <bool DELTA, int WAVES>
 __global__ __launch_bounds__(64 * WAVES) void k_chunk_states(MixRows r, Recurrence c, ChunkWork w) {
-  extern __shared__ __attribute__((aligned(16))) float part[];  // [2][WAVES][4][64][4] (delta)
+  extern __shared__ __attribute__((aligned(16))) float part[];  // [2][WAVES][2][64][4] (delta)
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-  const int half = lane >> 5, l32 = lane & 31;
+  const int quarter = lane >> 4, l16 = lane & 15;
   const int ct = blockIdx.x, h = blockIdx.y, b = blockIdx.z;
   constexpr int dp = 32 * WAVES;
   const int cts = w.ep / 32, dim = c.dim, vdim = c.vdim;
-  const int col = 32 * ct + l32;
+  const int col = 16 * ct + l16;
+  const int at = (16 * (ct & 1)) + l16 + 4 * quarter * 32;  // of a [32][32] tile
   float* state = c.state + (size_t)b * c.state_seq + (size_t)h * dim * vdim;
-  auto row_of = [&](int v) { return 8 * (v >> 2) + 4 * half + (v & 3); };
-  f16v S;
+  f4 S[2];
 #pragma unroll
-  for (int v = 0; v < 16; ++v) {
-    const int i = 32 * wave + row_of(v);
-    S[v] = r.pos0 > 0 && i < dim && col < vdim ? state[(size_t)i * vdim + col] : 0.0f;
-  }
-  struct Tiles {  // of one chunk
-    f4 w[4], g[4];
-    float k[16], u[16];
+  for (int a = 0; a < 2; ++a)
+#pragma unroll
+    for (int v = 0; v < 4; ++v) {
+      const int i = 32 * wave + 16 * a + 4 * quarter + v;
+      S[a][v] = r.pos0 > 0 && i < dim && col < vdim ? state[(size_t)i * vdim + col] : 0.0f;
+    }
+  struct Tiles {  // of one chunk: W by (state row tile, token tile), the others by token tile
+    f4 w[2][2], g[2], u[2];
+    float k[2][2][4];
   };
   auto fetch = [&](int ci, Tiles& x) __attribute__((always_inline)) {
     const size_t tile = w.tile(b, min(ci, w.chunks - 1), h, c.heads);
-    const float* u = (DELTA ? w.U0 : w.U) + (tile * cts + ct) * 1024 + 128 * half + l32;
-    const float* kd = w.Kd + tile * 32 * dp + 32 * wave + 4 * half * dp + l32;
-    const float* g = w.G + tile * dp + 32 * wave + 4 * half;
+    const float* u = (DELTA ? w.U0 : w.U) + (tile * cts + (ct >> 1)) * 1024 + at;
+    const float* kd = w.Kd + tile * 32 * dp + 32 * wave + 4 * quarter * dp + l16;
+    const float* g = w.G + tile * dp + 32 * wave + 4 * quarter;
     if (DELTA) {
-      const float* wt = w.W + tile * 32 * dp + 32 * wave + l32 * dp + 4 * half;
+      const float* wt = w.W + tile * 32 * dp + 32 * wave + l16 * dp + 4 * quarter;
 #pragma unroll
-      for (int q = 0; q < 4; ++q) x.w[q] = *reinterpret_cast<const f4*>(wt + 8 * q);
+      for (int a = 0; a < 2; ++a)
+#pragma unroll
+        for (int t = 0; t < 2; ++t) x.w[a][t] = *reinterpret_cast<const f4*>(wt + 16 * a + 16 * t * dp);
     }
 #pragma unroll
-    for (int v = 0; v < 16; ++v) x.u[v] = u[(8 * (v >> 2) + (v & 3)) * 32];
+    for (int t = 0; t < 2; ++t)
 #pragma unroll
-    for (int v = 0; v < 16; ++v) x.k[v] = kd[(8 * (v >> 2) + (v & 3)) * dp];
+      for (int v = 0; v < 4; ++v) x.u[t][v] = u[(16 * t + v) * 32];
 #pragma unroll
-    for (int q = 0; q < 4; ++q) x.g[q] = *reinterpret_cast<const f4*>(g + 8 * q);
+    for (int t = 0; t < 2; ++t)
+#pragma unroll
+      for (int v = 0; v < 4; ++v)
+#pragma unroll
+        for (int a = 0; a < 2; ++a) x.k[a][t][v] = kd[(16 * t + v) * dp + 16 * a];
+#pragma unroll
+    for (int a = 0; a < 2; ++a) x.g[a] = *reinterpret_cast<const f4*>(g + 16 * a);
   };
   auto chunk = [&](int ci, Tiles& x) __attribute__((always_inline)) {
     __builtin_amdgcn_sched_barrier(0);
-    const size_t tile = w.tile(b, ci, h, c.heads) * cts + ct;
-    float* s0 = w.S + (tile * WAVES + wave) * 1024 + 128 * half + l32;
+    const size_t tile = w.tile(b, ci, h, c.heads) * cts + (ct >> 1);
+    float* s0 = w.S + (tile * WAVES + wave) * 1024 + at;
 #pragma unroll
-    for (int v = 0; v < 16; ++v) s0[(8 * (v >> 2) + (v & 3)) * 32] = S[v];
+    for (int a = 0; a < 2; ++a)
+#pragma unroll
+      for (int v = 0; v < 4; ++v) s0[(16 * a + v) * 32] = S[a][v];
     if (DELTA) {
-      f16v p;
+      f4 p[2] = {f4{0.f, 0.f, 0.f, 0.f}, f4{0.f, 0.f, 0.f, 0.f}};
 #pragma unroll
-      for (int v = 0; v < 16; ++v) p[v] = 0.0f;
+      for (int a = 0; a < 2; ++a)
 #pragma unroll
-      for (int v = 0; v < 16; ++v) p = __builtin_amdgcn_mfma_f32_32x32x2f32(x.w[v >> 2][v & 3], S[v], p, 0, 0, 0);
-      f4* mine = reinterpret_cast<f4*>(part) + (size_t)((ci & 1) * WAVES + wave) * 256 + lane;
+        for (int v = 0; v < 4; ++v)
 #pragma unroll
-      for (int q = 0; q < 4; ++q) mine[64 * q] = f4{p[4 * q], p[4 * q + 1], p[4 * q + 2], p[4 * q + 3]};
+          for (int t = 0; t < 2; ++t) p[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.w[a][t][v], S[a][v], p[t], 0, 0, 0);
+      f4* mine = reinterpret_cast<f4*>(part) + ((ci & 1) * WAVES + wave) * 128 + lane;
+      mine[0] = p[0];
+      mine[64] = p[1];
       __syncthreads();
-      const f4* all = reinterpret_cast<const f4*>(part) + (size_t)((ci & 1) * WAVES) * 256 + lane;
+      const f4* all = reinterpret_cast<const f4*>(part) + ((ci & 1) * WAVES) * 128 + lane;
 #pragma unroll
-      for (int o = 0; o < WAVES; ++o)
-#pragma unroll
-        for (int q = 0; q < 4; ++q) {
-          const f4 z = all[o * 256 + 64 * q];
-#pragma unroll
-          for (int e = 0; e < 4; ++e) x.u[4 * q + e] -= z[e];
-        }
+      for (int o = 0; o < WAVES; ++o) {
+        x.u[0] -= all[o * 128];
+        x.u[1] -= all[o * 128 + 64];
+      }
       if (wave == ci % WAVES) {
-        float* ud = w.U + tile * 1024 + 128 * half + l32;
+        float* ud = w.U + tile * 1024 + at;
 #pragma unroll
-        for (int v = 0; v < 16; ++v) ud[(8 * (v >> 2) + (v & 3)) * 32] = x.u[v];
+        for (int t = 0; t < 2; ++t)
+#pragma unroll
+          for (int v = 0; v < 4; ++v) ud[(16 * t + v) * 32] = x.u[t][v];
       }
     }
 #pragma unroll
-    for (int v = 0; v < 16; ++v) S[v] *= x.g[v >> 2][v & 3];
+    for (int a = 0; a < 2; ++a) S[a] *= x.g[a];
 #pragma unroll
-    for (int v = 0; v < 16; ++v) S = __builtin_amdgcn_mfma_f32_32x32x2f32(x.k[v], x.u[v], S, 0, 0, 0);
+    for (int t = 0; t < 2; ++t)
+#pragma unroll
+      for (int v = 0; v < 4; ++v)
+#pragma unroll
+        for (int a = 0; a < 2; ++a) S[a] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.k[a][t][v], x.u[t][v], S[a], 0, 0, 0);
     __builtin_amdgcn_sched_barrier(0);
   };
   // (past the end: the last chunk's tiles again, never used)
-  Tiles x0, x1;
+  Tiles x0, x1, x2;
   int ci = 0;
   fetch(0, x0);
-  if constexpr (WAVES <= 4) {
-    Tiles x2;
-    fetch(1, x1);
-    for (; ci + 3 <= w.chunks; ci += 3) {
-      fetch(ci + 2, x2);
-      chunk(ci, x0);
-      fetch(ci + 3, x0);
-      chunk(ci + 1, x1);
-      fetch(ci + 4, x1);
-      chunk(ci + 2, x2);
-    }
-    if (ci < w.chunks) chunk(ci, x0);
-    if (ci + 1 < w.chunks) chunk(ci + 1, x1);
-  } else {
-    for (; ci + 2 <= w.chunks; ci += 2) {
-      fetch(ci + 1, x1);
-      chunk(ci, x0);
-      fetch(ci + 2, x0);
-      chunk(ci + 1, x1);
-    }
-    if (ci < w.chunks) chunk(ci, x0);
+  fetch(1, x1);
+  for (; ci + 3 <= w.chunks; ci += 3) {
+    fetch(ci + 2, x2);
+    chunk(ci, x0);
+    fetch(ci + 3, x0);
+    chunk(ci + 1, x1);
+    fetch(ci + 4, x1);
+    chunk(ci + 2, x2);
   }
+  if (ci < w.chunks) chunk(ci, x0);
+  if (ci + 1 < w.chunks) chunk(ci + 1, x1);
 #pragma unroll
-  for (int v = 0; v < 16; ++v) {
-    const int i = 32 * wave + row_of(v);
-    if (i < dim && col < vdim) state[(size_t)i * vdim + col] = S[v];
-  }
+  for (int a = 0; a < 2; ++a)
+#pragma unroll
+    for (int v = 0; v < 4; ++v) {
+      const int i = 32 * wave + 16 * a + 4 * quarter + v;
+      if (i < dim && col < vdim) state[(size_t)i * vdim + col] = S[a][v];
+    }
 }
 
 // The read-outs of one (chunk, head, sequence), normalised, gated and written to the mixer outputs.
@@ -1245,9 +1253,10 @@ int rows_per_thread(int dim, int vdim) {
 
 }  // namespace
 
-// Threads of a decode block: rows of a state column per thread of a block of 256; blocks grow so
-// that a thread holds few.
-static int decode_threads(int rows) { return rows <= 8 ? 256 : rows == 16 ? 512 : 1024; }
+// Threads of a decode block.  rows: rows of a state column per thread of a block of 256; blocks grow
+// so that a thread holds at most 32 (128 x 128 states, 32 sequences: 36.6 us with 1024 threads,
+// 28.4 with 512, 31.4 with 256).
+static int decode_threads(int rows) { return rows <= 16 ? 256 : rows <= 64 ? 512 : 1024; }
 
 int mix_decode_splits(const ChunkAttn& a, const Recurrence* rec) {
   const int keys = decode_threads(rec ? rows_per_thread(rec->dim, rec->vdim) : 1) / 4;
@@ -1274,8 +1283,8 @@ hipError_t launch_mix_decode(const MixDecode& a, hipStream_t s) {
     else if (nv == 2) hipLaunchKernelGGL((k_mix_decode<NT, N, 2>), grid, dim3(NT), 0, s, a, attn_items, rec_items);   \
     else hipLaunchKernelGGL((k_mix_decode<NT, N, 4>), grid, dim3(NT), 0, s, a, attn_items, rec_items);                \
     break;
-    PG_RPT(1, 256, 1) PG_RPT(2, 256, 2) PG_RPT(4, 256, 4) PG_RPT(8, 256, 8) PG_RPT(16, 512, 8)
-    PG_RPT(32, 1024, 8) PG_RPT(64, 1024, 16) PG_RPT(128, 1024, 32) PG_RPT(256, 1024, 64)
+    PG_RPT(1, 256, 1) PG_RPT(2, 256, 2) PG_RPT(4, 256, 4) PG_RPT(8, 256, 8) PG_RPT(16, 256, 16)
+    PG_RPT(32, 512, 16) PG_RPT(64, 512, 32) PG_RPT(128, 1024, 32) PG_RPT(256, 1024, 64)
 #undef PG_RPT
     default: return hipErrorInvalidValue;
   }
@@ -1376,8 +1385,8 @@ hipError_t launch_recurrence_rows(const MixRows& r, const Recurrence& c, hipStre
   }
   hipError_t e = hipGetLastError();
   if (e != hipSuccess) return e;
-  const dim3 sgrid(w.ep / 32, c.heads, r.nseq);
-  const size_t slds = c.delta ? 2 * waves * 1024 * sizeof(float) : 0;
+  const dim3 sgrid(w.ep / 16, c.heads, r.nseq);
+  const size_t slds = c.delta ? 2 * waves * 512 * sizeof(float) : 0;
   switch (waves) {
 #define PG_WAVES(N)                                                                                          \
   case N:                                                                                                    \
