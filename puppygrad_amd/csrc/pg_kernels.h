@@ -201,7 +201,7 @@ hipError_t launch_quantize_rows(const float* src, void* q, float* scales, size_t
                                 hipStream_t s);
 
 // ---- full-sequence kernels (pg_prefill.hip) ----------------------------------------
-enum GemmEpilogue : int { GEMM_BIAS = 0, GEMM_GELU = 1, GEMM_RESID = 2 };
+enum GemmEpilogue : int { GEMM_BIAS = 0, GEMM_GELU = 1, GEMM_RESID = 2, GEMM_RESID_SCALED = 3 };
 // C[M,N] = epilogue(A[M,K] . W[N,K]^T + bias): A rows lda floats apart, C (and resid)
 // rows ldc apart, W dense [N][K]; bias may be nullptr.
 struct GemmArgs {
@@ -211,8 +211,8 @@ struct GemmArgs {
   const float* W;
   const float* bias;
   const float* resid;
-  // Optional (GEMM_RESID): the product's column n is multiplied by col_scale[n] before it is
-  // added to the residual (layer scale).
+  // GEMM_RESID_SCALED: the product's column n is multiplied by col_scale[n] before it is added to
+  // the residual (layer scale).
   const float* col_scale = nullptr;
   float* C;
   int M, N, K;
@@ -229,7 +229,7 @@ struct GemmArgs {
   const float* ln_g = nullptr;
   const float* ln_b = nullptr;
   float ln_eps = 0.0f;
-  // != 0: ln_out receives row / sqrt(mean(row^2) + ln_eps) * ln_g[0] instead, the mean over the
+  // (GEMM_RESID_SCALED) != 0: ln_out receives row / sqrt(mean(row^2) + ln_eps) * ln_g[0] instead, the mean over the
   // first rms_cols columns (the others must hold zeros).
   int rms_cols = 0;
   // Packed form of an activation matrix of at most 32 rows (see packed32_index): which of

@@ -26,9 +26,14 @@ typedef float f16v __attribute__((ext_vector_type(16)));
 __device__ __forceinline__ float gelu_tanh(float x) {
   return 0.5f * x * (1.0f + tanhf(0.7978846f * (x + 0.044715f * x * x * x)));
 }
-// What column n of a product adds to the residual (GemmArgs::col_scale).
+// Epilogues that add to the residual, and what column n of the product adds
+// (GEMM_RESID_SCALED: GemmArgs::col_scale).
+template <int EPI>
+constexpr bool kAddsResid = EPI == GEMM_RESID || EPI == GEMM_RESID_SCALED;
+template <int EPI>
 __device__ __forceinline__ float col_scaled(const GemmArgs& a, int n, float c) {
-  return a.col_scale ? a.col_scale[n] * c : c;
+  if constexpr (EPI == GEMM_RESID_SCALED) return a.col_scale[n] * c;
+  return c;
 }
 
 // ---------------------------------------------------------------------------
@@ -342,7 +347,7 @@ __global__ __launch_bounds__(256) void k_gemm(GemmArgs a) {
         if (m >= a.M) continue;
         float c = bias + acc[i][j][v];
         if (EPI == GEMM_GELU) c = gelu_tanh(c);
-        if (EPI == GEMM_RESID) c = a.resid[(size_t)m * a.ldc + n] + col_scaled(a, n, c);
+        if (kAddsResid<EPI>) c = a.resid[(size_t)m * a.ldc + n] + col_scaled<EPI>(a, n, c);
         a.C[(size_t)m * a.ldc + n] = c;
       }
     }
@@ -468,7 +473,7 @@ __device__ __forceinline__ void redo_tile(const GemmArgs& a, int mbase, int nbas
           }
           c = (a.bias ? a.bias[n] : 0.0f) + c;
           if (EPI == GEMM_GELU) c = gelu_tanh(c);
-          if (EPI == GEMM_RESID) c = a.resid[(size_t)m * a.ldc + n] + col_scaled(a, n, c);
+          if (kAddsResid<EPI>) c = a.resid[(size_t)m * a.ldc + n] + col_scaled<EPI>(a, n, c);
           a.C[(size_t)m * a.ldc + n] = c;
         }
     }
@@ -696,7 +701,7 @@ __global__ __launch_bounds__(256) void k_gemm_b3(GemmArgs a) {
         if (m >= a.M) continue;
         float c = bias + (WT == 2 ? wscale * acc[i][j][v] : acc[i][j][v]);
         if (EPI == GEMM_GELU) c = gelu_tanh(c);
-        if (EPI == GEMM_RESID) c = a.resid[(size_t)m * a.ldc + n] + col_scaled(a, n, c);
+        if (kAddsResid<EPI>) c = a.resid[(size_t)m * a.ldc + n] + col_scaled<EPI>(a, n, c);
         a.C[(size_t)m * a.ldc + n] = c;
       }
     }
@@ -904,7 +909,7 @@ __global__ __launch_bounds__(256) void k_gemm_b9(GemmArgs a) {
         if (m >= a.M) continue;
         float c = bias + acc[i][j][v];
         if (EPI == GEMM_GELU) c = gelu_tanh(c);
-        if (EPI == GEMM_RESID) c = a.resid[(size_t)m * a.ldc + n] + col_scaled(a, n, c);
+        if (kAddsResid<EPI>) c = a.resid[(size_t)m * a.ldc + n] + col_scaled<EPI>(a, n, c);
         a.C[(size_t)m * a.ldc + n] = c;
       }
     }
@@ -934,7 +939,7 @@ __global__ __launch_bounds__(256) void k_splitk_reduce(GemmArgs a, int parts) {
 #pragma unroll
   for (int k = 0; k < 4; ++k) {
     if (EPI == GEMM_GELU) c[k] = gelu_tanh(c[k]);
-    if (EPI == GEMM_RESID) c[k] = a.resid[m * a.ldc + n + k] + col_scaled(a, (int)n + k, c[k]);
+    if (kAddsResid<EPI>) c[k] = a.resid[m * a.ldc + n + k] + col_scaled<EPI>(a, (int)n + k, c[k]);
     dst[k] = c[k];
   }
 }
@@ -969,7 +974,7 @@ __global__ __launch_bounds__(256) void k_splitk_reduce_ln(GemmArgs a, int parts)
 #pragma unroll
     for (int p = 0; p < 8; ++p)
       v[q][p] = *reinterpret_cast<const f4*>(a.ws + (size_t)min(p, parts - 1) * stride + m * a.N + n);
-    if (a.rms_cols) return;
+    if (EPI == GEMM_RESID_SCALED && a.rms_cols) return;
     lg[q] = *reinterpret_cast<const f4*>(a.ln_g + n);
     lb[q] = *reinterpret_cast<const f4*>(a.ln_b + n);
   };
@@ -994,13 +999,13 @@ __global__ __launch_bounds__(256) void k_splitk_reduce_ln(GemmArgs a, int parts)
 #pragma unroll
       for (int k = 0; k < 4; ++k) {
         if (EPI == GEMM_GELU) r[k] = gelu_tanh(r[k]);
-        if (EPI == GEMM_RESID) r[k] = a.resid[m * a.ldc + n + k] + col_scaled(a, (int)n + k, r[k]);
+        if (kAddsResid<EPI>) r[k] = a.resid[m * a.ldc + n + k] + col_scaled<EPI>(a, (int)n + k, r[k]);
       }
       c[q] = f4{r[0], r[1], r[2], r[3]};
       *reinterpret_cast<f4*>(a.C + m * a.ldc + n) = c[q];
     }
   }
-  if (a.rms_cols) {  // RMS norm with one gain (columns past rms_cols hold zeros)
+  if (EPI == GEMM_RESID_SCALED && a.rms_cols) {  // RMS norm with one gain (columns past rms_cols hold zeros)
     float ss = 0.0f;
 #pragma unroll
     for (int q = 0; q < 4; ++q) ss += (c[q].x * c[q].x + c[q].y * c[q].y) + (c[q].z * c[q].z + c[q].w * c[q].w);
@@ -1137,7 +1142,7 @@ __global__ __launch_bounds__(256) void k_gemv_rows(GemmArgs a) {
   if (b >= a.M || n >= a.N) return;
   float c = (a.bias ? a.bias[n] : 0.0f) + acc[0];
   if (EPI == GEMM_GELU) c = gelu_tanh(c);
-  if (EPI == GEMM_RESID) c = a.resid[(size_t)b * a.ldc + n] + col_scaled(a, n, c);
+  if (kAddsResid<EPI>) c = a.resid[(size_t)b * a.ldc + n] + col_scaled<EPI>(a, n, c);
   a.C[(size_t)b * a.ldc + n] = c;
 }
 
@@ -1233,7 +1238,7 @@ __global__ __launch_bounds__(512) void k_gemm_rows32(GemmArgs a) {
     const int idx = tid + 512 * qq, b = idx / NR, n = n0 + idx % NR;
     const bool live = gridDim.y == 1 && idx < 32 * MT * NR && b < a.M && n < n1;
     ebias[qq] = live && a.bias ? a.bias[n] : 0.0f;
-    eres[qq] = live && EPI == GEMM_RESID ? a.resid[(size_t)b * a.ldc + n] : 0.0f;
+    eres[qq] = live && kAddsResid<EPI> ? a.resid[(size_t)b * a.ldc + n] : 0.0f;
     // int8 rows: the row's scale multiplies the row's sum (also a partial sum of a cut K)
     escale[qq] = WT == 2 && idx < 32 * MT * NR && b < a.M && n < n1 ? a.w_scale[n] : 1.0f;
   }
@@ -1425,7 +1430,7 @@ __global__ __launch_bounds__(512) void k_gemm_rows32(GemmArgs a) {
     }
     float c = ebias[q] + sum;
     if (EPI == GEMM_GELU) c = gelu_tanh(c);
-    if (EPI == GEMM_RESID) c = eres[q] + col_scaled(a, n, c);
+    if (kAddsResid<EPI>) c = eres[q] + col_scaled<EPI>(a, n, c);
     a.C[a.c_packed ? packed32_index((size_t)b, (size_t)n) : (size_t)b * a.ldc + n] = c;
   }
 }
@@ -1452,7 +1457,7 @@ __global__ __launch_bounds__(256) void k_tail_reduce(GemmArgs a) {
 #pragma unroll
   for (int k = 0; k < 4; ++k) {
     if (EPI == GEMM_GELU) c[k] = gelu_tanh(c[k]);
-    if (EPI == GEMM_RESID) c[k] = a.resid[(size_t)m * a.ldc + n + k] + col_scaled(a, n + k, c[k]);
+    if (kAddsResid<EPI>) c[k] = a.resid[(size_t)m * a.ldc + n + k] + col_scaled<EPI>(a, n + k, c[k]);
     dst[k] = c[k];
   }
 }
@@ -1818,6 +1823,8 @@ hipError_t launch_gemm_tile(const GemmArgs& a, int epi, hipStream_t s) {
     hipLaunchKernelGGL((k_gemm<BM, BN, GEMM_GELU, WBF, 0, BKT>), dim3(grid), dim3(256), 0, s, a);
   else if (epi == GEMM_RESID)
     hipLaunchKernelGGL((k_gemm<BM, BN, GEMM_RESID, WBF, 0, BKT>), dim3(grid), dim3(256), 0, s, a);
+  else if (epi == GEMM_RESID_SCALED)
+    hipLaunchKernelGGL((k_gemm<BM, BN, GEMM_RESID_SCALED, WBF, 0, BKT>), dim3(grid), dim3(256), 0, s, a);
   else
     return hipErrorInvalidValue;
   return hipGetLastError();
@@ -1840,6 +1847,8 @@ hipError_t launch_gemm_b3_shape(const GemmArgs& a0, int epi, hipStream_t s) {
     hipLaunchKernelGGL((k_gemm_b3<BM, BN, GEMM_GELU, 0, WT>), dim3(grid), dim3(256), 0, s, a);
   else if (epi == GEMM_RESID)
     hipLaunchKernelGGL((k_gemm_b3<BM, BN, GEMM_RESID, 0, WT>), dim3(grid), dim3(256), 0, s, a);
+  else if (epi == GEMM_RESID_SCALED)
+    hipLaunchKernelGGL((k_gemm_b3<BM, BN, GEMM_RESID_SCALED, 0, WT>), dim3(grid), dim3(256), 0, s, a);
   else
     return hipErrorInvalidValue;
   return hipGetLastError();
@@ -1873,6 +1882,8 @@ hipError_t launch_gemm_b9(const GemmArgs& a0, int epi, int parts, hipStream_t s,
     hipLaunchKernelGGL((k_gemm_b9<128, 128, GEMM_GELU>), dim3(grid), dim3(256), 0, s, a);
   else if (epi == GEMM_RESID)
     hipLaunchKernelGGL((k_gemm_b9<128, 128, GEMM_RESID>), dim3(grid), dim3(256), 0, s, a);
+  else if (epi == GEMM_RESID_SCALED)
+    hipLaunchKernelGGL((k_gemm_b9<128, 128, GEMM_RESID_SCALED>), dim3(grid), dim3(256), 0, s, a);
   else
     return hipErrorInvalidValue;
   return hipGetLastError();
@@ -1932,8 +1943,12 @@ hipError_t launch_splitk_reduce(const GemmArgs& a, int epi, int parts, hipStream
       hipLaunchKernelGGL((k_splitk_reduce_ln<GEMM_GELU, false>), dim3(a.M), dim3(256), 0, s, a, parts);
     else if (epi == GEMM_RESID && early)
       hipLaunchKernelGGL((k_splitk_reduce_ln<GEMM_RESID, true>), dim3(a.M), dim3(256), 0, s, a, parts);
+    else if (epi == GEMM_RESID_SCALED && early)
+      hipLaunchKernelGGL((k_splitk_reduce_ln<GEMM_RESID_SCALED, true>), dim3(a.M), dim3(256), 0, s, a, parts);
     else if (epi == GEMM_RESID)
       hipLaunchKernelGGL((k_splitk_reduce_ln<GEMM_RESID, false>), dim3(a.M), dim3(256), 0, s, a, parts);
+    else if (epi == GEMM_RESID_SCALED)
+      hipLaunchKernelGGL((k_splitk_reduce_ln<GEMM_RESID_SCALED, false>), dim3(a.M), dim3(256), 0, s, a, parts);
     else
       return hipErrorInvalidValue;
     *ln_done = true;
@@ -1946,6 +1961,8 @@ hipError_t launch_splitk_reduce(const GemmArgs& a, int epi, int parts, hipStream
     hipLaunchKernelGGL(k_splitk_reduce<GEMM_GELU>, dim3(rblocks), dim3(256), 0, s, a, parts);
   else if (epi == GEMM_RESID)
     hipLaunchKernelGGL(k_splitk_reduce<GEMM_RESID>, dim3(rblocks), dim3(256), 0, s, a, parts);
+  else if (epi == GEMM_RESID_SCALED)
+    hipLaunchKernelGGL(k_splitk_reduce<GEMM_RESID_SCALED>, dim3(rblocks), dim3(256), 0, s, a, parts);
   else
     return hipErrorInvalidValue;
   return hipGetLastError();
@@ -1967,6 +1984,8 @@ hipError_t launch_gemv_rows_r(const GemmArgs& a, int epi, hipStream_t s) {
     hipLaunchKernelGGL((k_gemv_rows<MB, R, GEMM_GELU, WBF>), grid, dim3(256), 0, s, a);
   else if (epi == GEMM_RESID)
     hipLaunchKernelGGL((k_gemv_rows<MB, R, GEMM_RESID, WBF>), grid, dim3(256), 0, s, a);
+  else if (epi == GEMM_RESID_SCALED)
+    hipLaunchKernelGGL((k_gemv_rows<MB, R, GEMM_RESID_SCALED, WBF>), grid, dim3(256), 0, s, a);
   else
     return hipErrorInvalidValue;
   return hipGetLastError();
@@ -2025,6 +2044,8 @@ hipError_t launch_gemm_rows32_m(const GemmArgs& a0, int epi, int parts, int rows
     hipLaunchKernelGGL((k_gemm_rows32<GEMM_GELU, WT, XP, M16, NR, MT>), grid, dim3(512), 0, s, a);
   else if (epi == GEMM_RESID)
     hipLaunchKernelGGL((k_gemm_rows32<GEMM_RESID, WT, XP, M16, NR, MT>), grid, dim3(512), 0, s, a);
+  else if (epi == GEMM_RESID_SCALED)
+    hipLaunchKernelGGL((k_gemm_rows32<GEMM_RESID_SCALED, WT, XP, M16, NR, MT>), grid, dim3(512), 0, s, a);
   else
     return hipErrorInvalidValue;
   return hipSuccess;
@@ -2078,6 +2099,9 @@ hipError_t launch_gemm_tail(const GemmArgs& a, int epi, hipStream_t s) {
   } else if (epi == GEMM_RESID) {
     hipLaunchKernelGGL((k_gemm<BM, BN, GEMM_RESID, WBF, 2, BKT>), dim3(grid), dim3(256), 0, s, a);
     hipLaunchKernelGGL((k_tail_reduce<BM, BN, GEMM_RESID>), rgrid, dim3(256), 0, s, a);
+  } else if (epi == GEMM_RESID_SCALED) {
+    hipLaunchKernelGGL((k_gemm<BM, BN, GEMM_RESID_SCALED, WBF, 2, BKT>), dim3(grid), dim3(256), 0, s, a);
+    hipLaunchKernelGGL((k_tail_reduce<BM, BN, GEMM_RESID_SCALED>), rgrid, dim3(256), 0, s, a);
   } else {
     return hipErrorInvalidValue;
   }
@@ -2237,6 +2261,8 @@ hipError_t launch_gemm_form(const GemmArgs& a, int epi, int num_cus, hipStream_t
 
 hipError_t launch_gemm(const GemmArgs& a, int epi, int num_cus, hipStream_t s) {
   if (a.ln_out && a.ldc != a.N) return hipErrorInvalidValue;
+  if ((epi == GEMM_RESID_SCALED) != (a.col_scale != nullptr) || (a.rms_cols && epi != GEMM_RESID_SCALED))
+    return hipErrorInvalidValue;
   bool ln_done = false;
   hipError_t e = launch_gemm_form(a, epi, num_cus, s, &ln_done);
   if (e == hipSuccess && a.ln_out && !ln_done && a.rms_cols)

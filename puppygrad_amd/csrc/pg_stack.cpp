@@ -567,7 +567,7 @@ struct Gemm {
     if (norm_out) {
       a.ln_out = norm_out; a.ln_g = norm_gain; a.ln_eps = m->stack->eps; a.rms_cols = m->stack->width;
     }
-    return pgk::launch_gemm(a, resid_scale ? pgk::GEMM_RESID : pgk::GEMM_BIAS, m->num_cus, s);
+    return pgk::launch_gemm(a, resid_scale ? pgk::GEMM_RESID_SCALED : pgk::GEMM_BIAS, m->num_cus, s);
   }
 };
 
