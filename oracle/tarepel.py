@@ -81,7 +81,7 @@ def short_conv(window, taps):
 
 
 def delta_step(S, q, k, v, g, beta):
-    """One head's gated delta rule: S [dim][vdim].  The read-out sees the current write."""
+    """One head's gated delta rule: S [dim][vdim]; decay, write, then read at q."""
     S = g * S
     u = beta * (v - S.T @ k)
     S = S + np.outer(k, u)

@@ -168,7 +168,7 @@ struct SampleStep {
   size_t arm_words;
 };
 hipError_t launch_sample_step(const SampleStep& a, hipStream_t s);
-// x[b] = wte[ids[b]] + wpe[pos] (wpe may be null)
+// x[b] = wte[ids[b]] + wpe[pos]
 hipError_t launch_embed_batch(float* x, const float* wte, const float* wpe, const uint32_t* ids,
                               int batch, int pos, int C, hipStream_t s, int w_bf16 = 0);
 // Appends row b of qkv[B][3C] to position pos of sequence b's K and V panels.

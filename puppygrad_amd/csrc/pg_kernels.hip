@@ -1038,7 +1038,7 @@ __global__ void k_embed_batch(float* x, const float* wte, const float* wpe, cons
   const int b = blockIdx.y;
   const int i = blockIdx.x * blockDim.x + threadIdx.x;
   if (i < C)
-    x[(size_t)b * C + i] = wte_at(wte, w_bf16, (size_t)ids[b] * C + i) + (wpe ? wpe[(size_t)pos * C + i] : 0.0f);
+    x[(size_t)b * C + i] = wte_at(wte, w_bf16, (size_t)ids[b] * C + i) + wpe[(size_t)pos * C + i];
 }
 
 // K/V append of cached_self_attention_into (rust.rs:1677-1683) for a batch: row b of
