@@ -13,7 +13,7 @@ LIB_PATH = PKG_DIR / "libpuppygrad_hip.so"
 # (python -m puppygrad_amd.build --stamps; read by puppygrad_amd.decode_stamps).
 STAMPS_LIB_PATH = PKG_DIR / "libpuppygrad_hip_stamps.so"
 SOURCES = ["pg_kernels.hip", "pg_decode.hip", "pg_prefill.hip", "pg_ops_dev.hip", "pg_sample.hip",
-           "pg_mixers.hip", "pg_host.cpp", "pg_stack.cpp", "pg_assets.cpp"]
+           "pg_mixers.hip", "pg_latent.hip", "pg_moe.hip", "pg_host.cpp", "pg_stack.cpp", "pg_assets.cpp"]
 
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 # Packed-FP32 instruction selection is switched off for every device pass.

@@ -25,9 +25,11 @@ struct LayerW {
 };
 
 // PRO_RMS: x / sqrt(mean(x^2) + eps) * ln_g[0], the mean over the first norm_n values (the
-// others are zeros)
-enum Prologue : int { PRO_NONE = 0, PRO_LN = 1, PRO_ATTN_COMBINE = 2, PRO_RMS = 3 };
-enum Epilogue : int { EPI_BIAS = 0, EPI_GELU = 1, EPI_RESID = 2, EPI_QKV = 3 };
+// others are zeros).  PRO_STACK: x, plus (add) the norm of a sublayer's output,
+// add / sqrt(mean(add^2) + eps) * add_gain, the sum also going to x_out; then (gain) an RMS norm
+// over each of `groups` equal parts of the first norm_n values.
+enum Prologue : int { PRO_NONE = 0, PRO_LN = 1, PRO_ATTN_COMBINE = 2, PRO_RMS = 3, PRO_STACK = 4 };
+enum Epilogue : int { EPI_BIAS = 0, EPI_GELU = 1, EPI_RESID = 2, EPI_QKV = 3, EPI_SQRELU = 4 };
 
 // y = epilogue(bias + W . prologue(x)) for one input vector.
 struct GemvArgs {
@@ -45,7 +47,11 @@ struct GemvArgs {
   const float* ln_g;
   const float* ln_b;
   float eps;
-  int norm_n;  // PRO_RMS
+  int norm_n;  // PRO_RMS, PRO_STACK
+  // PRO_STACK (add and gain may be null; vectors of at least K values, those past norm_n zeros)
+  const float *add = nullptr, *add_gain = nullptr, *gain = nullptr;
+  float* x_out = nullptr;  // not x itself: other blocks still read it
+  int add_n = 0, groups = 1;
   float out_mul = 0.0f;  // EPI_BIAS: != 0 multiplies the result
   // PRO_ATTN_COMBINE: partial attention results per (head, split)
   const float* part_acc;  // [H][nsplit][hd]
@@ -201,7 +207,11 @@ hipError_t launch_quantize_rows(const float* src, void* q, float* scales, size_t
                                 hipStream_t s);
 
 // ---- full-sequence kernels (pg_prefill.hip) ----------------------------------------
-enum GemmEpilogue : int { GEMM_BIAS = 0, GEMM_GELU = 1, GEMM_RESID = 2, GEMM_RESID_SCALED = 3 };
+// GEMM_SQRELU: max(v, 0)^2.  GEMM_SILU_PAIR (launch_gemm_grouped): columns 2 j and 2 j + 1 are a gate and
+// what it multiplies, C[.][j] = silu(gate) * up.
+enum GemmEpilogue : int {
+  GEMM_BIAS = 0, GEMM_GELU = 1, GEMM_RESID = 2, GEMM_RESID_SCALED = 3, GEMM_SQRELU = 4, GEMM_SILU_PAIR = 5
+};
 // C[M,N] = epilogue(A[M,K] . W[N,K]^T + bias): A rows lda floats apart, C (and resid)
 // rows ldc apart, W dense [N][K]; bias may be nullptr.
 struct GemmArgs {
@@ -247,6 +257,7 @@ struct GemmArgs {
   int plan_bm = 0, plan_bn = 0, plan_form = 0, plan_parts = 0;
   int plan_band = 0;  // band height of the tile numbering (0: chosen by the launcher)
   int plan_bk16 = 0;  // 1: k-tiles of 16 columns also where K would allow 32
+  const int *group_tile = nullptr, *group_rows = nullptr;  // launch_gemm_grouped
 };
 // Element (row b < 32, column k) of a packed activation matrix: the float4 of columns
 // 4j..4j+3 of all 32 rows lie next to each other, so that 32 lanes which each read four
@@ -261,6 +272,13 @@ bool gemm_supported(const GemmArgs& a);
 int gemm_split_parts(const GemmArgs& a, int num_cus, int bm = 64, int bn = 64);
 bool gemm_tail_plan(GemmArgs& a, int num_cus, int bm = 64, int bn = 64);
 hipError_t launch_gemm(const GemmArgs& a, int epilogue, int num_cus, hipStream_t s);
+// Many small products in one launch: rows are sorted by the matrix they meet.  Row m of the product
+// takes row group_rows[m] of A (any row where that is -1), and the rows of tile m / tile_rows meet
+// matrix group_tile[m / tile_rows] of W [groups][N][K] (-1: the tile is left out).  a.M counts the rows
+// with their padding, a multiple of tile_rows (64 or 128; 64 for f32 rows).  C has a row per m.
+// group_rows null: row m itself.  GEMM_BIAS (without bias) or GEMM_SILU_PAIR.
+hipError_t launch_gemm_grouped(const GemmArgs& a, int epilogue, int tile_rows, const int* group_tile,
+                               const int* group_rows, hipStream_t s);
 // Causal attention over qkv[T][3C] -> out[T][C]; also appends K, V to the cache panels.
 // scratch ([T*H][T] floats) is only used when head_dim != 64.
 // nseq sequences of T positions each, one after the other in qkv / out; sequence i's panels

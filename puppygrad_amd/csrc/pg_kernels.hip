@@ -182,6 +182,39 @@ __global__ __launch_bounds__(kBlock) void k_gemv(GemvArgs a) {
     for (int i = tid; i < K; i += kBlock) sx[i] = a.x[i];
   }
   __syncthreads();
+  if (PRO == PRO_STACK) {
+    if (a.add) {
+      float ss = 0.0f;
+      for (int i = tid; i < K; i += kBlock) {
+        const float v = a.add[i];
+        ss += v * v;
+      }
+      const float k = 1.0f / sqrtf(block_sum(ss, red) / (float)a.add_n + a.eps);
+      for (int i = tid; i < K; i += kBlock) {
+        sx[i] += a.add[i] * k * a.add_gain[i];
+        if (blockIdx.x == 0 && a.x_out) a.x_out[i] = sx[i];
+      }
+      __syncthreads();
+    }
+    if (a.gain) {
+      if (a.groups == 1) {
+        float ss = 0.0f;
+        for (int i = tid; i < a.norm_n; i += kBlock) ss += sx[i] * sx[i];
+        const float k = 1.0f / sqrtf(block_sum(ss, red) / (float)a.norm_n + a.eps);
+        for (int i = tid; i < a.norm_n; i += kBlock) sx[i] *= k * a.gain[i];
+      } else {  // one wavefront per part in turn
+        const int n = a.norm_n / a.groups;
+        for (int g = wave; g < a.groups; g += kWaves) {
+          float* v = sx + g * n;
+          float ss = 0.0f;
+          for (int i = lane; i < n; i += 64) ss += v[i] * v[i];
+          const float k = 1.0f / sqrtf(wave_sum(ss) / (float)n + a.eps);
+          for (int i = lane; i < n; i += 64) v[i] *= k * a.gain[g * n + i];
+        }
+      }
+      __syncthreads();
+    }
+  }
   if (PRO == PRO_LN) ln_in_lds(sx, K, a.ln_g, a.ln_b, a.eps, red);
   // RMS norm with one gain: a factor of the finished sums
   float row_mul = 1.0f;
@@ -266,6 +299,9 @@ __global__ __launch_bounds__(kBlock) void k_gemv(GemvArgs a) {
         a.y[o] = v;
       } else if (EPI == EPI_GELU) {
         a.y[o] = gelu_tanh(v);
+      } else if (EPI == EPI_SQRELU) {
+        const float p = fmaxf(v, 0.0f);
+        a.y[o] = p * p;
       } else if (EPI == EPI_RESID) {
         a.y[o] = a.resid[o] + v;  // add_in_place (cpu.rs:167-171)
       } else {  // EPI_QKV: K/V append of cached_self_attention_into (rust.rs:1677-1683)
@@ -1230,6 +1266,8 @@ hipError_t launch_gemv(const GemvArgs& a, int prologue, int epilogue, hipStream_
   PG_CASE(PRO_NONE, EPI_GELU)
   PG_CASE(PRO_LN, EPI_BIAS)
   PG_CASE(PRO_RMS, EPI_BIAS)
+  PG_CASE(PRO_STACK, EPI_BIAS)
+  PG_CASE(PRO_STACK, EPI_SQRELU)
   PG_CASE(PRO_LN, EPI_GELU)
   PG_CASE(PRO_LN, EPI_QKV)
   PG_CASE(PRO_ATTN_COMBINE, EPI_RESID)

@@ -23,6 +23,12 @@ __device__ __forceinline__ float sigmoid(float x) { return 1.0f / (1.0f + expf(-
 __device__ __forceinline__ float silu(float x) { return x / (1.0f + expf(-x)); }
 __device__ __forceinline__ float softplus(float x) { return fmaxf(x, 0.0f) + log1pf(expf(-fabsf(x))); }
 
+__device__ __forceinline__ f4 bf16x4(const unsigned short* p) {
+  const uint2 u = *reinterpret_cast<const uint2*>(p);
+  return f4{__uint_as_float(u.x << 16), __uint_as_float(u.x & 0xffff0000u), __uint_as_float(u.y << 16),
+            __uint_as_float(u.y & 0xffff0000u)};
+}
+
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll
   for (int off = 32; off > 0; off >>= 1) v += __shfl_xor(v, off, 64);
@@ -243,7 +249,7 @@ __device__ __forceinline__ void conv_channels(const ShortConv& c, const float* y
       }
 #pragma unroll
     for (int n = 0; n < N; ++n) {
-      float s = 0.0f;
+      float s = c.bias ? c.bias[ch[n]] : 0.0f;
 #pragma unroll
       for (int k = 0; k < 4; ++k) {
         int j = slot - k;  // tokens back
@@ -259,7 +265,7 @@ __device__ __forceinline__ void conv_channels(const ShortConv& c, const float* y
   } else {
 #pragma unroll
     for (int n = 0; n < N; ++n) {
-      float s = c.w[ch[n] * c.taps + c.taps - 1] * cur[n];
+      float s = (c.bias ? c.bias[ch[n]] : 0.0f) + c.w[ch[n] * c.taps + c.taps - 1] * cur[n];
       for (int j = 1; j < c.taps; ++j)
         if (pos >= j)
           s += c.w[ch[n] * c.taps + c.taps - 1 - j] * ring[(size_t)((pos - j) % c.taps) * c.channels + ch[n]];
@@ -271,11 +277,34 @@ __device__ __forceinline__ void conv_channels(const ShortConv& c, const float* y
     if (keep[n]) ring[(size_t)slot * c.channels + ch[n]] = cur[n];
 }
 
+// dst[i] = row row0 + i of a low-rank projection, i < n: eight lanes to a row.
+template <int NT>
+__device__ __forceinline__ void low_rank_rows(const LowRank& p, const float* y, int row0, int n, float* dst) {
+  const int sub = threadIdx.x & 7;
+  const float* x = y + p.col;
+  for (int i = threadIdx.x >> 3; i < n; i += NT / 8) {
+    const size_t at = (size_t)(row0 + i) * p.rank;
+    float s = 0.0f;
+    for (int k = 4 * sub; k < p.rank; k += 32) {
+      const f4 w = p.w_bf16 ? bf16x4(static_cast<const unsigned short*>(p.w) + at + k)
+                            : *reinterpret_cast<const f4*>(static_cast<const float*>(p.w) + at + k);
+      const f4 v = *reinterpret_cast<const f4*>(x + k);
+      s += (w.x * v.x + w.y * v.y) + (w.z * v.z + w.w * v.w);
+    }
+#pragma unroll
+    for (int off = 4; off > 0; off >>= 1) s += __shfl_xor(s, off, 64);
+    if (sub == 0) dst[i] = s;
+  }
+}
+
 // One head of the recurrence.  A thread owns column v of the state and every `parts`-th of its
 // rows, RPT of them, in registers (parts * RPT <= kMixMaxDim; q and k are 0 past dim).
-template <int NT, int RPT>
+// KIND: a RecurrenceKind, or -1 for REC_GLA or REC_DELTA as m.rec.kind says.
+template <int NT, int RPT, int KIND = -1>
 __device__ void recurrence_role(const MixDecode& m, int b, int h, float* lds) {
   const Recurrence& c = m.rec;
+  const bool delta = KIND < 0 ? c.kind == REC_DELTA : rec_reads_state(KIND);
+  constexpr bool kChannel = KIND == REC_CHANNEL_DELTA, kSsd = KIND == REC_SSD;
   const int tid = threadIdx.x;
   const int dim = c.dim, vdim = c.vdim;
   int cols = 1;
@@ -288,6 +317,7 @@ __device__ void recurrence_role(const MixDecode& m, int b, int h, float* lds) {
   float* red = al + 256;           // [NT]
   float* red2 = red + NT;          // [NT]
   float* redw = red2 + NT;         // [2][NT / 64]
+  float* gs = redw + 2 * (NT / 64);  // [256] REC_CHANNEL_DELTA: output gate
   const float* y = m.y + (size_t)b * m.ld_y;
   float* S = c.state + (size_t)b * c.state_seq + (size_t)h * dim * vdim;
   const int pos = *m.d_pos;
@@ -298,23 +328,37 @@ __device__ void recurrence_role(const MixDecode& m, int b, int h, float* lds) {
     st[j] = S[(size_t)min(part + parts * j, dim - 1) * vdim + min(v, vdim - 1)];
   }
   const int tv = min(tid, vdim - 1);
-  const float gate = y[c.g_col + h * vdim + tv], norm = c.norm[tv];
+  const float gate = kChannel ? 0.0f : y[c.g_col + h * vdim + tv], norm = kSsd ? 0.0f : c.norm[tv];
   const int kvh = h / (c.heads / c.kv_heads);
-  float beta = 1.0f, g = 1.0f;
-  if (c.delta) {
+  float beta = 1.0f, g = 1.0f, skip = 0.0f;
+  if (delta || kSsd) {
     const ShortConv& cv = c.conv;
     float* ring = cv.ring + (size_t)b * cv.ring_seq;
     const bool first = h % (c.heads / c.kv_heads) == 0;
-    const float yb = y[c.b_col + h], ya = y[c.a_col + h], al0 = c.a_log[h], dt = c.dt_bias[h];
+    const float yb = kSsd ? 0.0f : y[c.b_col + h], al0 = c.a_log[h];
+    const float ya = kChannel ? 0.0f : y[c.a_col + h], dt = kChannel ? 0.0f : c.dt_bias[h];
+    if (kChannel) {
+      low_rank_rows<NT>(c.low_a, y, h * dim, dim, al);
+      low_rank_rows<NT>(c.low_g, y, h * vdim, vdim, gs);
+    }
     const int td = min(tid, dim - 1);
     const int ch[3] = {c.q_col - cv.col + kvh * dim + td, c.k_col - cv.col + kvh * dim + td,
                        c.v_col - cv.col + h * vdim + tv};
     const bool keep[3] = {first && tid < dim, first && tid < dim, tid < vdim};
     float cq[3];
     conv_channels<3>(cv, y, ring, ch, keep, pos, cq);
-    float qv = cq[0], kv = cq[1];
-    const float x = cq[2];
+    float qv = cq[0], kv = cq[1], x = cq[2];
     if (tid >= dim) qv = kv = 0.0f;
+    if constexpr (kSsd) {
+      const float step = softplus(ya + dt);
+      g = expf(-expf(al0) * step);
+      skip = c.skip[h] * x;
+      if (tid < 256) {
+        vs[tid] = step * x;
+        qs[tid] = qv;
+        ks[tid] = kv;
+      }
+    } else {
     float qn = wave_sum(qv * qv), kn = wave_sum(kv * kv);
     if ((tid & 63) == 0 && tid < 256) {  // (nothing past kMixMaxDim = 256)
       redw[tid >> 6] = qn;
@@ -329,8 +373,13 @@ __device__ void recurrence_role(const MixDecode& m, int b, int h, float* lds) {
       ks[tid] = kv / sqrtf(kn + 1e-6f);
     }
     beta = sigmoid(yb);
-    g = expf(delta_log_decay(ya, al0, dt));
-  } else {
+    if constexpr (kChannel) {  // (al was written before the barrier above)
+      if (tid < dim) al[tid] = expf(delta_log_decay(al[tid], al0, c.dt_bias[h * dim + tid]));
+    } else {
+      g = expf(delta_log_decay(ya, al0, dt));
+    }
+    }
+  } else if constexpr (KIND < 0) {
     float qv = 0.0f, kv = 0.0f, av = 1.0f;
     if (tid < dim) {
       qv = y[c.q_col + h * dim + tid] * c.q_scale;
@@ -365,11 +414,11 @@ __device__ void recurrence_role(const MixDecode& m, int b, int h, float* lds) {
   }
   __syncthreads();
   float u = v < vdim ? vs[v] : 0.0f;
-  if (c.delta) {
+  if (delta) {
     float s = 0.0f;
 #pragma unroll
     for (int j = 0; j < RPT; ++j) {
-      st[j] *= g;
+      st[j] *= kChannel ? al[min(part + parts * j, dim - 1)] : g;
       s += st[j] * ks[part + parts * j];
     }
     red[tid] = s;
@@ -379,7 +428,7 @@ __device__ void recurrence_role(const MixDecode& m, int b, int h, float* lds) {
     u = beta * (u - s);
   } else {
 #pragma unroll
-    for (int j = 0; j < RPT; ++j) st[j] *= al[part + parts * j];
+    for (int j = 0; j < RPT; ++j) st[j] *= kSsd ? g : al[part + parts * j];
   }
   float o = 0.0f;
 #pragma unroll
@@ -404,13 +453,17 @@ __device__ void recurrence_role(const MixDecode& m, int b, int h, float* lds) {
   float out = 0.0f;
   if (tid < vdim)
     for (int p = 0; p < parts; ++p) out += red2[p * cols + tid];
+  if constexpr (kSsd) {
+    if (tid < vdim) m.out[(size_t)b * m.ld_out + c.out_col + h * vdim + tid] = (out + skip) * silu(gate);
+    return;
+  }
   float ss = wave_sum(out * out);
   if ((tid & 63) == 0 && tid < 256) redw[tid >> 6] = ss;
   __syncthreads();
   ss = (redw[0] + redw[1]) + (redw[2] + redw[3]);
   if (tid < vdim)
     m.out[(size_t)b * m.ld_out + c.out_col + h * vdim + tid] =
-        out / sqrtf(ss / (float)vdim + c.eps) * norm * silu(gate) * c.out_scale;
+        out / sqrtf(ss / (float)vdim + c.eps) * norm * (kChannel ? sigmoid(gs[tid]) : silu(gate)) * c.out_scale;
 }
 
 template <int NT, int RPT, int NV>
@@ -433,6 +486,12 @@ __global__ __launch_bounds__(NT) void k_mix_decode(MixDecode m, int attn_items, 
   const float* y = m.y + (size_t)b * m.ld_y;
   m.act[(size_t)b * m.mlp.ff_pad + j] =
       j < m.mlp.ff ? gelu_tanh(y[m.mlp.gate_col + j]) * y[m.mlp.up_col + j] : 0.0f;
+}
+
+template <int NT, int RPT, int KIND>
+__global__ __launch_bounds__(NT) void k_recurrence_decode(MixDecode m) {
+  __shared__ __attribute__((aligned(16))) float lds[kDecodeLds<NT>];
+  recurrence_role<NT, RPT, KIND>(m, blockIdx.y, blockIdx.x, lds);
 }
 
 __global__ __launch_bounds__(256) void k_attn_sum(MixDecode m) {
@@ -680,6 +739,7 @@ __global__ __launch_bounds__(256) void k_short_conv_rows(MixRows r, ShortConv c)
   const float* x = r.y + (size_t)b * r.n * r.ld_y + c.col + ch;
   const float* ring = c.ring + (size_t)b * c.ring_seq + ch;
   float w[TAPS], in[TAPS - 1 + kConvRows];
+  const float bias = c.bias ? c.bias[ch] : 0.0f;
 #pragma unroll
   for (int j = 0; j < TAPS; ++j) w[j] = j < c.taps ? c.w[ch * c.taps + c.taps - 1 - j] : 0.0f;  // j tokens back
 #pragma unroll
@@ -695,7 +755,7 @@ __global__ __launch_bounds__(256) void k_short_conv_rows(MixRows r, ShortConv c)
 #pragma unroll
   for (int i = 0; i < kConvRows; ++i) {
     if (t0 + i >= r.n) return;
-    float s = 0.0f;
+    float s = bias;
 #pragma unroll
     for (int j = 0; j < TAPS; ++j) s += w[j] * in[TAPS - 1 + i - j];
     r.conv_out[((size_t)b * r.n + t0 + i) * c.channels + ch] = silu(s);
@@ -739,7 +799,9 @@ __global__ __launch_bounds__(256) void k_gla_decay_rows(MixRows r, Recurrence c,
 // the chunk's tokens write U into the state and read it out as
 //   S_end = exp(G_end) S0 + Kd^T U,   O = Qd S0 + P U,
 // where U = V for gated linear attention and, for the delta rule (whose k_t first reads the state),
-//   U = U0 - W S0,  (1 + A) [U0 | W] = [beta V | beta exp(G) K],  A_tj = beta_t exp(G_t - G_j) k_t . k_j, j < t.
+//   U = U0 - W S0,  (1 + A) [U0 | W] = [beta V | beta exp(G) K],  A_tj = beta_t exp(G_t - G_j) k_t . k_j, j < t
+// (with decays per key channel the exponentials stand inside the dot products).  The state-space
+// recurrence is the form without reads, U = dt V.
 // All exponents are <= 0.  Three launches: the parts that need no state for every chunk at once,
 // the states from chunk to chunk (the only serial part), the read-outs for every chunk at once.
 // A chunk's tiles lie in the work area one after the other, 32 rows each, widths padded to
@@ -963,6 +1025,221 @@ __global__ __launch_bounds__(256) void k_gla_chunk(MixRows r, Recurrence c, Chun
   }
 }
 
+// State-space recurrence, per (chunk, head, sequence): U (= dt V), Kd, Qd, P, G.
+__global__ __launch_bounds__(256) void k_ssd_chunk(MixRows r, Recurrence c, ChunkWork w) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  __shared__ double Gs[kChunk];
+  __shared__ float step[kChunk], eg[kChunk], ek[kChunk];
+  __shared__ float red[4][32 * 33];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int half = lane >> 5, l32 = lane & 31;
+  const int ci = blockIdx.x, h = blockIdx.y, b = blockIdx.z;
+  const int dim = c.dim, vdim = c.vdim, dp = w.dp, ep = w.ep, LD = dp + 4;
+  float* Ks = lds;            // [32][LD]
+  float* Qs = lds + 32 * LD;
+  const int t0 = ci * kChunk, nt = min(kChunk, r.n - t0);
+  const size_t row0 = (size_t)b * r.n + t0;
+  const int kvh = h / (c.heads / c.kv_heads);
+  const int CH = c.conv.channels;
+  const float* xq = r.conv_out + row0 * CH + (c.q_col - c.conv.col) + kvh * dim;
+  const float* xk = r.conv_out + row0 * CH + (c.k_col - c.conv.col) + kvh * dim;
+  const float* xv = r.conv_out + row0 * CH + (c.v_col - c.conv.col) + h * vdim;
+  for (int i = tid; i < 32 * dp; i += 256) {
+    const int t = i / dp, d = i - t * dp;
+    const bool in = t < nt && d < dim;
+    Qs[t * LD + d] = in ? xq[(size_t)t * CH + d] : 0.0f;
+    Ks[t * LD + d] = in ? xk[(size_t)t * CH + d] : 0.0f;
+  }
+  if (wave == 0) {
+    double g = 0.0;
+    float dt = 0.0f;
+    if (lane < nt) {
+      dt = softplus(r.y[(row0 + lane) * r.ld_y + c.a_col + h] + c.dt_bias[h]);
+      g = (double)(-expf(c.a_log[h]) * dt);
+    }
+#pragma unroll
+    for (int off = 1; off < 32; off <<= 1) {
+      const double up = __shfl_up(g, off, 64);
+      if (lane >= off) g += up;
+    }
+    const double end = __shfl(g, 31, 64);
+    if (lane < 32) {
+      Gs[lane] = g;
+      step[lane] = dt;
+      eg[lane] = expf((float)g);
+      ek[lane] = expf((float)(end - g));
+    }
+  }
+  __syncthreads();
+  const size_t tile = w.tile(b, ci, h, c.heads);
+  {
+    const int k0 = wave * (dp / 4);  // q . k over a quarter of the columns each
+    const f16v s = dots32(Qs, Ks, LD, k0, k0 + dp / 4, lane);
+#pragma unroll
+    for (int v = 0; v < 16; ++v) red[wave][(8 * (v >> 2) + 4 * half + (v & 3)) * 33 + l32] = s[v];
+  }
+  for (int i = tid; i < 32 * ep; i += 256) {
+    const int t = (i >> 5) & 31, e = (i >> 10) * 32 + (i & 31);
+    w.U[tile * 32 * ep + i] = t < nt && e < vdim ? step[t] * xv[(size_t)t * CH + e] : 0.0f;
+  }
+  __syncthreads();
+  for (int i = tid; i < 1024; i += 256) {
+    const int t = i >> 5, j = i & 31, at = t * 33 + j;
+    const float e = j <= t ? expf((float)(Gs[t] - Gs[j])) : 0.0f;
+    w.P[tile * 1024 + i] = e * ((red[0][at] + red[1][at]) + (red[2][at] + red[3][at]));
+  }
+  for (int i = tid; i < 32 * dp; i += 256) {
+    const int t = i / dp, d = i - t * dp;
+    w.Kd[tile * 32 * dp + i] = ek[t] * Ks[t * LD + d];
+    w.Qd[tile * 32 * dp + i] = eg[t] * Qs[t * LD + d];
+  }
+  for (int i = tid; i < dp; i += 256) w.G[tile * dp + i] = eg[31];
+}
+
+// Delta rule with a decay per key channel, per (chunk, head, sequence): U0, W, Kd, Qd, P, G.  The
+// sums of the log decays (base 2) are kept as two floats each, so that their differences are as
+// exact as f32 however strongly the channel has decayed before.
+__global__ __launch_bounds__(256) void k_channel_delta_chunk(MixRows r, Recurrence c, ChunkWork w) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  __shared__ float beta[kChunk];
+  __shared__ __attribute__((aligned(16))) float As[32][36];
+  const int tid = threadIdx.x;
+  const int ci = blockIdx.x, h = blockIdx.y, b = blockIdx.z;
+  const int dim = c.dim, vdim = c.vdim, dp = w.dp, ep = w.ep, LD = dp + 1;
+  float* Ks = lds;  // [32][LD] each
+  float* Qs = lds + 32 * LD;
+  float* Gh = lds + 64 * LD;
+  float* Gl = lds + 96 * LD;
+  const int t0 = ci * kChunk, nt = min(kChunk, r.n - t0);
+  const size_t row0 = (size_t)b * r.n + t0;
+  const size_t tile = w.tile(b, ci, h, c.heads);
+  const int kvh = h / (c.heads / c.kv_heads);
+  const int CH = c.conv.channels;
+  const float* xq = r.conv_out + row0 * CH + (c.q_col - c.conv.col) + kvh * dim;
+  const float* xk = r.conv_out + row0 * CH + (c.k_col - c.conv.col) + kvh * dim;
+  const float* xv = r.conv_out + row0 * CH + (c.v_col - c.conv.col) + h * vdim;
+  {
+    // eight threads to a row: q and k as unit vectors
+    const int t = tid >> 3, sub = tid & 7;
+    float qq = 0.0f, kk = 0.0f;
+#pragma unroll 4
+    for (int i = sub; i < dp; i += 8) {
+      float q = 0.0f, k = 0.0f;
+      if (t < nt && i < dim) {
+        q = xq[(size_t)t * CH + i];
+        k = xk[(size_t)t * CH + i];
+      }
+      Qs[t * LD + i] = q;
+      Ks[t * LD + i] = k;
+      qq += q * q;
+      kk += k * k;
+    }
+#pragma unroll
+    for (int off = 4; off > 0; off >>= 1) {
+      qq += __shfl_xor(qq, off, 64);
+      kk += __shfl_xor(kk, off, 64);
+    }
+    const float qm = c.q_scale / sqrtf(qq + 1e-6f), km = 1.0f / sqrtf(kk + 1e-6f);
+    for (int i = sub; i < dp; i += 8) {
+      Qs[t * LD + i] *= qm;
+      Ks[t * LD + i] *= km;
+    }
+  }
+  if (tid < 32) beta[tid] = tid < nt ? sigmoid(r.y[(row0 + tid) * r.ld_y + c.b_col + h]) : 0.0f;
+  {
+    // log decays, then their sums down the chunk, a channel per thread
+    const float al = c.a_log[h];
+    for (int i = tid; i < 32 * dp; i += 256) {
+      const int t = i / dp, d = i - t * dp;
+      float g = 0.0f;
+      if (t < nt && d < dim)
+        g = delta_log_decay(r.decay[(row0 + t) * c.heads * dim + h * dim + d], al, c.dt_bias[h * dim + d]);
+      Gh[t * LD + d] = g;
+    }
+    __syncthreads();
+    for (int d = tid; d < dp; d += 256) {
+      double s = 0.0;
+#pragma unroll 8
+      for (int t = 0; t < kChunk; ++t) {
+        s += (double)Gh[t * LD + d];
+        const double s2 = s * 1.4426950408889634074;
+        const float hi = (float)s2;
+        Gh[t * LD + d] = hi;
+        Gl[t * LD + d] = (float)(s2 - (double)hi);
+      }
+    }
+  }
+  __syncthreads();
+  // the 496 pairs j < t: rows 31 - i and i together have 31 of them
+  for (int p = tid; p < 496; p += 256) {
+    const int i = p / 31, e = p - 31 * i;
+    const bool high = e < 31 - i;
+    const int t = high ? 31 - i : i, j = high ? e : e - (31 - i);
+    const float *q = Qs + t * LD, *kt = Ks + t * LD, *kj = Ks + j * LD;
+    const float *ht = Gh + t * LD, *hj = Gh + j * LD, *lt = Gl + t * LD, *lj = Gl + j * LD;
+    float sp = 0.0f, sa = 0.0f;
+#pragma unroll 4
+    for (int d = 0; d < dim; ++d) {
+      const float k = kj[d] * __builtin_amdgcn_exp2f((ht[d] - hj[d]) + (lt[d] - lj[d]));
+      sp = fmaf(q[d], k, sp);
+      sa = fmaf(kt[d], k, sa);
+    }
+    w.P[tile * 1024 + t * 32 + j] = sp;
+    w.P[tile * 1024 + j * 32 + t] = 0.0f;
+    As[t][j] = beta[t] * sa;
+    As[j][t] = 0.0f;
+  }
+  {
+    const int t = tid >> 3, sub = tid & 7;
+    float s = 0.0f;
+    for (int d = sub; d < dim; d += 8) s += Qs[t * LD + d] * Ks[t * LD + d];
+#pragma unroll
+    for (int off = 4; off > 0; off >>= 1) s += __shfl_xor(s, off, 64);
+    if (sub == 0) {
+      w.P[tile * 1024 + t * 33] = s;
+      As[t][t] = 0.0f;
+    }
+  }
+  __syncthreads();
+  // columns of [W | U0] by forward substitution, one per thread
+  for (int col = tid; col < dp + ep; col += 256) {
+    const bool isw = col < dp;
+    const int e = col - dp;
+    float x[kChunk];
+#pragma unroll
+    for (int t = 0; t < kChunk; ++t) {
+      float v = 0.0f;
+      if (isw) v = __builtin_amdgcn_exp2f(Gh[t * LD + col]) * Ks[t * LD + col];
+      else if (t < nt && e < vdim) v = xv[(size_t)t * CH + e];
+      x[t] = beta[t] * v;
+    }
+#pragma unroll
+    for (int t = 1; t < kChunk; ++t) {
+      float s = x[t];
+#pragma unroll
+      for (int j = 0; j < t; j += 4) {
+        const f4 a4 = *reinterpret_cast<const f4*>(&As[t][j]);
+#pragma unroll
+        for (int k = 0; k < 4; ++k)
+          if (j + k < t) s -= a4[k] * x[j + k];
+      }
+      x[t] = s;
+      __builtin_amdgcn_sched_barrier(0);  // (row by row: all rows of A at once do not fit the registers)
+    }
+    float* dst = isw ? w.W + tile * 32 * dp + col : w.U0 + tile * 32 * ep + (e >> 5) * 1024 + (e & 31);
+    const int ld = isw ? dp : 32;
+#pragma unroll
+    for (int t = 0; t < kChunk; ++t) dst[t * ld] = x[t];
+  }
+  for (int i = tid; i < 32 * dp; i += 256) {
+    const int t = i / dp, d = i - t * dp;
+    const float hi = Gh[t * LD + d], lo = Gl[t * LD + d];
+    w.Kd[tile * 32 * dp + i] = __builtin_amdgcn_exp2f((Gh[31 * LD + d] - hi) + (Gl[31 * LD + d] - lo)) * Ks[t * LD + d];
+    w.Qd[tile * 32 * dp + i] = __builtin_amdgcn_exp2f(hi) * Qs[t * LD + d];
+  }
+  for (int d = tid; d < dp; d += 256) w.G[tile * dp + d] = __builtin_amdgcn_exp2f(Gh[31 * LD + d]);
+}
+
 // The states from chunk to chunk.  A block owns 16 value columns of one head; wavefront w keeps
 // the state's rows 32 w .. 32 w + 31 in the accumulator layout of v_mfma_f32_16x16x4_f32, where
 // register v of lane (l, quarter) of row tile a is row 16 a + 4 quarter + v of column l.  In that
@@ -1086,7 +1363,8 @@ __global__ __launch_bounds__(64 * WAVES) void k_chunk_states(MixRows r, Recurren
 }
 
 // The read-outs of one (chunk, head, sequence), normalised, gated and written to the mixer outputs.
-// A wavefront owns the 32-column tiles wave and wave + 4.
+// KIND: REC_CHANNEL_DELTA, REC_SSD, or REC_GLA for the other two.  A wavefront owns the 32-column tiles wave and wave + 4.
+template <int KIND>
 __global__ __launch_bounds__(256) void k_chunk_out(MixRows r, Recurrence c, ChunkWork w) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   __shared__ __attribute__((aligned(16))) float Ps[32][36];
@@ -1153,13 +1431,25 @@ __global__ __launch_bounds__(256) void k_chunk_out(MixRows r, Recurrence c, Chun
   for (int k = 0; k < 2; ++k) {
     const int e = 32 * (wave + 4 * k) + l32;
     if (e >= vdim) break;
-    const float norm = c.norm[e] * c.out_scale;
+    const float norm = KIND == REC_SSD ? 0.0f : c.norm[e] * c.out_scale;
+    const float skip = KIND == REC_SSD ? c.skip[h] : 0.0f;
 #pragma unroll
     for (int v = 0; v < 16; ++v) {
       const int t = 8 * (v >> 2) + 4 * half + (v & 3);
       if (t >= nt) continue;
       const float sq = (ss[0][t] + ss[1][t]) + (ss[2][t] + ss[3][t]);
       const size_t row = row0 + t;
+      if constexpr (KIND == REC_SSD) {
+        const float x = r.conv_out[row * c.conv.channels + (c.v_col - c.conv.col) + h * vdim + e];
+        r.out[row * r.ld_out + c.out_col + h * vdim + e] =
+            (o[k][v] + skip * x) * silu(r.y[row * r.ld_y + c.g_col + h * vdim + e]);
+        continue;
+      }
+      if constexpr (KIND == REC_CHANNEL_DELTA) {
+        r.out[row * r.ld_out + c.out_col + h * vdim + e] =
+            o[k][v] / sqrtf(sq / (float)vdim + c.eps) * norm * sigmoid(r.gate[(row * c.heads + h) * vdim + e]);
+        continue;
+      }
       r.out[row * r.ld_out + c.out_col + h * vdim + e] =
           o[k][v] / sqrtf(sq / (float)vdim + c.eps) * norm * silu(r.y[row * r.ld_y + c.g_col + h * vdim + e]);
     }
@@ -1212,6 +1502,62 @@ __global__ __launch_bounds__(256) void k_rms_rows(const float* src, float* dst, 
   for (int i = threadIdx.x; i < cols; i += 256) ss += x[i] * x[i];
   const float k = gain[0] * scale / sqrtf(block_sum(ss, red) / (float)cols + eps);
   for (int i = threadIdx.x; i < ld; i += 256) y[i] = i < cols ? x[i] * k : 0.0f;
+}
+
+__global__ __launch_bounds__(256) void k_add_norm_rows(float* dst, const float* src, int cols, int ld, const float* gain,
+                                                       float eps, const int* slot, const float* weight, int top) {
+  __shared__ float red[4];
+  constexpr int PER = 8;  // columns a thread keeps; more are read again
+  const size_t row = blockIdx.x;
+  float* x = dst + row * ld;
+  auto value = [&](int i) -> float {
+    if (top == 0) return src[row * ld + i];
+    float s = 0.0f;
+    for (int k = 0; k < top; ++k) s += weight[row * top + k] * src[(size_t)slot[row * top + k] * ld + i];
+    return s;
+  };
+  float keep[PER], ss = 0.0f;
+#pragma unroll
+  for (int p = 0; p < PER; ++p) {
+    const int i = threadIdx.x + 256 * p;
+    keep[p] = i < cols ? value(i) : 0.0f;
+    ss += keep[p] * keep[p];
+  }
+  for (int i = threadIdx.x + 256 * PER; i < cols; i += 256) {
+    const float v = value(i);
+    ss += v * v;
+  }
+  const float k = 1.0f / sqrtf(block_sum(ss, red) / (float)cols + eps);
+#pragma unroll
+  for (int p = 0; p < PER; ++p) {
+    const int i = threadIdx.x + 256 * p;
+    if (i < cols) x[i] += keep[p] * k * gain[i];
+  }
+  for (int i = threadIdx.x + 256 * PER; i < cols; i += 256) x[i] += value(i) * k * gain[i];
+}
+
+// One wavefront per part of a row in turn.
+__global__ __launch_bounds__(256) void k_group_rms_rows(const float* src, int ld_src, float* dst, int ld_dst, int cols,
+                                                        int groups, const float* gain, float eps, const int* rows_at) {
+  const size_t row = rows_at ? rows_at[blockIdx.x] : blockIdx.x;
+  const float* x = src + row * ld_src;
+  float* y = dst + (size_t)blockIdx.x * ld_dst;
+  const int n = cols / groups, lane = threadIdx.x & 63;
+  if (groups == 1) {
+    __shared__ float red[4];
+    float ss = 0.0f;
+    for (int i = threadIdx.x; i < n; i += 256) ss += x[i] * x[i];
+    const float k = 1.0f / sqrtf(block_sum(ss, red) / (float)n + eps);
+    for (int i = threadIdx.x; i < n; i += 256) y[i] = x[i] * k * gain[i];
+  } else {
+    for (int g = threadIdx.x >> 6; g < groups; g += 4) {
+      float ss = 0.0f;
+      for (int i = lane; i < n; i += 64) ss += x[g * n + i] * x[g * n + i];
+      const float k = 1.0f / sqrtf(wave_sum(ss) / (float)n + eps);
+      for (int i = lane; i < n; i += 64) y[g * n + i] = x[g * n + i] * k * gain[g * n + i];
+    }
+  }
+  for (int i = cols + threadIdx.x; i < ld_dst; i += 256) y[i] = 0.0f;
 }
 
 __global__ __launch_bounds__(256) void k_begin_step(float* x, const void* table, int table_bf16, const uint32_t* ids,
@@ -1291,6 +1637,25 @@ hipError_t launch_mix_decode(const MixDecode& a, hipStream_t s) {
   return hipGetLastError();
 }
 
+hipError_t launch_recurrence_decode(const MixDecode& a, hipStream_t s) {
+  const dim3 grid((unsigned)a.rec.heads, (unsigned)a.nseq);
+  if (a.rec.kind != REC_CHANNEL_DELTA && a.rec.kind != REC_SSD) return launch_mix_decode(a, s);
+  switch (rows_per_thread(a.rec.dim, a.rec.vdim)) {
+#define PG_RPT(R, NT, N)                                                                                     \
+  case R:                                                                                                    \
+    if (a.rec.kind == REC_SSD)                                                                               \
+      hipLaunchKernelGGL((k_recurrence_decode<NT, N, REC_SSD>), grid, dim3(NT), 0, s, a);                     \
+    else                                                                                                     \
+      hipLaunchKernelGGL((k_recurrence_decode<NT, N, REC_CHANNEL_DELTA>), grid, dim3(NT), 0, s, a);           \
+    break;
+    PG_RPT(1, 256, 1) PG_RPT(2, 256, 2) PG_RPT(4, 256, 4) PG_RPT(8, 256, 8) PG_RPT(16, 256, 16)
+    PG_RPT(32, 512, 16) PG_RPT(64, 512, 32) PG_RPT(128, 1024, 32) PG_RPT(256, 1024, 64)
+#undef PG_RPT
+    default: return hipErrorInvalidValue;
+  }
+  return hipGetLastError();
+}
+
 hipError_t launch_attn_sum(const MixDecode& a, hipStream_t s) {
   const int n = a.attn.heads * a.attn.dim;
   hipLaunchKernelGGL(k_attn_sum, dim3((n + 255) / 256, a.nseq), dim3(256), 0, s, a);
@@ -1337,7 +1702,7 @@ static int chunk_dim(int dim) {
 
 size_t recurrence_work_floats(const Recurrence& c, int nseq, int n) {
   const int dp = chunk_dim(c.dim), ep = (c.vdim + 31) / 32 * 32;
-  return chunk_floats(dp, ep, c.delta != 0) * (size_t)nseq * ((n + kChunk - 1) / kChunk) * c.heads;
+  return chunk_floats(dp, ep, rec_reads_state(c.kind)) * (size_t)nseq * ((n + kChunk - 1) / kChunk) * c.heads;
 }
 
 hipError_t launch_recurrence_rows(const MixRows& r, const Recurrence& c, hipStream_t s) {
@@ -1359,7 +1724,8 @@ hipError_t launch_recurrence_rows(const MixRows& r, const Recurrence& c, hipStre
   w.U = take((size_t)32 * w.ep);
   w.P = take(1024);
   w.G = take(w.dp);
-  if (c.delta) {
+  const bool delta = rec_reads_state(c.kind);
+  if (delta) {
     w.W = take((size_t)32 * w.dp);
     w.U0 = take((size_t)32 * w.ep);
   }
@@ -1368,12 +1734,26 @@ hipError_t launch_recurrence_rows(const MixRows& r, const Recurrence& c, hipStre
   // (large heads: more LDS than a launch gets by default)
   if (w.dp > 128) {
     const int most = 100 * 1024;
-    hipError_t e = hipFuncSetAttribute(c.delta ? reinterpret_cast<const void*>(&k_delta_chunk)
-                                               : reinterpret_cast<const void*>(&k_gla_chunk),
-                                       hipFuncAttributeMaxDynamicSharedMemorySize, most);
-    if (e != hipSuccess) return e;
+    const void* kernel = c.kind == REC_DELTA ? reinterpret_cast<const void*>(&k_delta_chunk)
+                         : c.kind == REC_SSD ? reinterpret_cast<const void*>(&k_ssd_chunk)
+                                             : reinterpret_cast<const void*>(&k_gla_chunk);
+    if (c.kind != REC_CHANNEL_DELTA) {
+      hipError_t e = hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize, most);
+      if (e != hipSuccess) return e;
+    }
   }
-  if (c.delta) {
+  if (c.kind == REC_CHANNEL_DELTA) {
+    const size_t lds = 4 * 32 * (size_t)(w.dp + 1) * sizeof(float);
+    if (lds > 48 * 1024) {
+      hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&k_channel_delta_chunk),
+                                         hipFuncAttributeMaxDynamicSharedMemorySize, 140 * 1024);
+      if (e != hipSuccess) return e;
+    }
+    hipLaunchKernelGGL(k_channel_delta_chunk, grid, dim3(256), lds, s, r, c, w);
+  } else if (c.kind == REC_SSD) {
+    const size_t lds = 2 * 32 * (size_t)(w.dp + 4) * sizeof(float);
+    hipLaunchKernelGGL(k_ssd_chunk, grid, dim3(256), lds, s, r, c, w);
+  } else if (c.kind == REC_DELTA) {
     const size_t lds = 2 * 32 * (size_t)(w.dp + 4) * sizeof(float);
     hipLaunchKernelGGL(k_delta_chunk, grid, dim3(256), lds, s, r, c, w);
   } else {
@@ -1386,11 +1766,11 @@ hipError_t launch_recurrence_rows(const MixRows& r, const Recurrence& c, hipStre
   hipError_t e = hipGetLastError();
   if (e != hipSuccess) return e;
   const dim3 sgrid(w.ep / 16, c.heads, r.nseq);
-  const size_t slds = c.delta ? 2 * waves * 512 * sizeof(float) : 0;
+  const size_t slds = delta ? 2 * waves * 512 * sizeof(float) : 0;
   switch (waves) {
 #define PG_WAVES(N)                                                                                          \
   case N:                                                                                                    \
-    if (c.delta) hipLaunchKernelGGL((k_chunk_states<true, N>), sgrid, dim3(64 * N), slds, s, r, c, w);        \
+    if (delta) hipLaunchKernelGGL((k_chunk_states<true, N>), sgrid, dim3(64 * N), slds, s, r, c, w);        \
     else hipLaunchKernelGGL((k_chunk_states<false, N>), sgrid, dim3(64 * N), slds, s, r, c, w);               \
     break;
     PG_WAVES(1) PG_WAVES(2) PG_WAVES(3) PG_WAVES(4) PG_WAVES(6) PG_WAVES(8)
@@ -1398,7 +1778,10 @@ hipError_t launch_recurrence_rows(const MixRows& r, const Recurrence& c, hipStre
     default: return hipErrorInvalidValue;
   }
   if ((e = hipGetLastError()) != hipSuccess) return e;
-  hipLaunchKernelGGL(k_chunk_out, grid, dim3(256), 32 * (size_t)(w.dp + 4) * sizeof(float), s, r, c, w);
+  const size_t olds = 32 * (size_t)(w.dp + 4) * sizeof(float);
+  if (c.kind == REC_SSD) hipLaunchKernelGGL(k_chunk_out<REC_SSD>, grid, dim3(256), olds, s, r, c, w);
+  else if (c.kind == REC_CHANNEL_DELTA) hipLaunchKernelGGL(k_chunk_out<REC_CHANNEL_DELTA>, grid, dim3(256), olds, s, r, c, w);
+  else hipLaunchKernelGGL(k_chunk_out<REC_GLA>, grid, dim3(256), olds, s, r, c, w);
   return hipGetLastError();
 }
 
@@ -1421,6 +1804,20 @@ hipError_t launch_commit_rows(const MixRows& r, const ChunkAttn* a, const ShortC
 hipError_t launch_rms_rows(const float* src, float* dst, int rows, int cols, int ld, const float* gain,
                            float eps, float scale, const int* rows_at, hipStream_t s) {
   hipLaunchKernelGGL(k_rms_rows, dim3(rows), dim3(256), 0, s, src, dst, cols, ld, gain, eps, scale, rows_at);
+  return hipGetLastError();
+}
+
+hipError_t launch_add_norm_rows(float* dst, const float* src, int rows, int cols, int ld, const float* gain, float eps,
+                                const int* slot, const float* weight, int top, hipStream_t s) {
+  hipLaunchKernelGGL(k_add_norm_rows, dim3(rows), dim3(256), 0, s, dst, src, cols, ld, gain, eps, slot, weight, top);
+  return hipGetLastError();
+}
+
+hipError_t launch_group_rms_rows(const float* src, int ld_src, float* dst, int ld_dst, int rows, int cols, int groups,
+                                 const float* gain, float eps, const int* rows_at, hipStream_t s) {
+  if (groups < 1 || cols % groups != 0) return hipErrorInvalidValue;
+  hipLaunchKernelGGL(k_group_rms_rows, dim3(rows), dim3(256), 0, s, src, ld_src, dst, ld_dst, cols, groups, gain, eps,
+                     rows_at);
   return hipGetLastError();
 }
 

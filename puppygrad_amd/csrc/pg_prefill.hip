@@ -36,6 +36,21 @@ __device__ __forceinline__ float col_scaled(const GemmArgs& a, int n, float c) {
   return c;
 }
 
+__device__ __forceinline__ float sq_relu(float x) {
+  const float p = fmaxf(x, 0.0f);
+  return p * p;
+}
+// Grouped products: the row of A that row m takes.
+__device__ __forceinline__ int group_row(const GemmArgs& a, int m) {
+  return a.group_rows ? max(a.group_rows[m], 0) : m;
+}
+// GEMM_SILU_PAIR: column n of the product with its partner column in the neighbouring lane; even
+// columns write.
+__device__ __forceinline__ void store_silu_pair(const GemmArgs& a, int m, int n, float c) {
+  const float up = __shfl_xor(c, 1, 64);
+  if ((n & 1) == 0) a.C[(size_t)m * a.ldc + (n >> 1)] = c / (1.0f + expf(-c)) * up;
+}
+
 // ---------------------------------------------------------------------------
 // C[M,N] = epilogue(A[M,K] . W[N,K]^T + bias)   (transposed_dense_projection_into,
 // src/models/cpu.rs:58-75, for many rows at once)
@@ -140,7 +155,8 @@ __device__ __forceinline__ void tile_coords(int tile, int tiles_m, int tiles_n, 
 // a.ws[(tile - tail_first) * parts + part][BM][BN] and k_tail_reduce finishes them.
 // WT: how W is stored: 0 f32, 1 bf16, 2 int8 with a.w_scale[n] per row (a weight is
 // (float)q * scale, formed when the tile is loaded: QuantizedRows, cpu.rs:26-56).
-template <int BM, int BN, int EPI, int WT, int SPLIT = 0, int BKT = BK>
+// GROUPED: see launch_gemm_grouped.
+template <int BM, int BN, int EPI, int WT, int SPLIT = 0, int BKT = BK, bool GROUPED = false>
 __global__ __launch_bounds__(256) void k_gemm(GemmArgs a) {
   constexpr int WM = BM / 2, WN = BN / 2;  // per-wavefront tile
   constexpr int MB = WM / 32, NB = WN / 32;  // 32x32 blocks per wavefront
@@ -179,6 +195,8 @@ __global__ __launch_bounds__(256) void k_gemm(GemmArgs a) {
   int tm, tn;
   tile_coords(tile, (a.M + BM - 1) / BM, tiles_n, a.band_rows, &tm, &tn);
   const int m0 = tm * BM, n0 = tn * BN;
+  const int group = GROUPED ? a.group_tile[tm] : 0;
+  if (GROUPED && group < 0) return;
 
   // global load mapping: 4 lanes cover 16 consecutive k of one row
   const int lr = tid / LPR, lk = (tid % LPR) * 4;
@@ -186,12 +204,12 @@ __global__ __launch_bounds__(256) void k_gemm(GemmArgs a) {
   size_t Wg[BLD];  // element offsets into W
 #pragma unroll
   for (int i = 0; i < ALD; ++i)
-    Ag[i] = a.A + (size_t)min(m0 + lr + RPP * i, a.M - 1) * a.lda + lk;
+    Ag[i] = a.A + (size_t)(GROUPED ? group_row(a, m0 + lr + RPP * i) : min(m0 + lr + RPP * i, a.M - 1)) * a.lda + lk;
   float wsc[BLD];  // int8: the scale of each row this thread loads
 #pragma unroll
   for (int i = 0; i < BLD; ++i) {
     const int n = min(n0 + lr + RPP * i, a.N - 1);
-    Wg[i] = (size_t)n * a.K + lk;
+    Wg[i] = (size_t)n * a.K + lk + (GROUPED ? (size_t)group * a.N * a.K : 0);
     wsc[i] = WT == 2 ? a.w_scale[n] : 1.0f;
   }
 
@@ -346,7 +364,12 @@ __global__ __launch_bounds__(256) void k_gemm(GemmArgs a) {
         const int m = m0 + wm * WM + 32 * i + 8 * (v >> 2) + 4 * half + (v & 3);
         if (m >= a.M) continue;
         float c = bias + acc[i][j][v];
+        if constexpr (EPI == GEMM_SILU_PAIR) {
+          store_silu_pair(a, m, n, c);
+          continue;
+        }
         if (EPI == GEMM_GELU) c = gelu_tanh(c);
+        if (EPI == GEMM_SQRELU) c = sq_relu(c);
         if (kAddsResid<EPI>) c = a.resid[(size_t)m * a.ldc + n] + col_scaled<EPI>(a, n, c);
         a.C[(size_t)m * a.ldc + n] = c;
       }
@@ -473,6 +496,7 @@ __device__ __forceinline__ void redo_tile(const GemmArgs& a, int mbase, int nbas
           }
           c = (a.bias ? a.bias[n] : 0.0f) + c;
           if (EPI == GEMM_GELU) c = gelu_tanh(c);
+          if (EPI == GEMM_SQRELU) c = sq_relu(c);
           if (kAddsResid<EPI>) c = a.resid[(size_t)m * a.ldc + n] + col_scaled<EPI>(a, n, c);
           a.C[(size_t)m * a.ldc + n] = c;
         }
@@ -485,7 +509,7 @@ __device__ __forceinline__ void redo_tile(const GemmArgs& a, int mbase, int nbas
 // values are bf16 numbers as they are, so the same three products per value are exact; the
 // row's scale multiplies the row's sum at the end (the reference scales every weight,
 // cpu.rs:173-184: the two differ by rounding only).
-template <int BM, int BN, int EPI, int SPLIT = 0, int WT = 1>
+template <int BM, int BN, int EPI, int SPLIT = 0, int WT = 1, bool GROUPED = false>
 __global__ __launch_bounds__(256) void k_gemm_b3(GemmArgs a) {
   constexpr int KT = 32;                     // columns per k-tile
   constexpr int WM = BM / 2, WN = BN / 2;    // per-wavefront tile
@@ -512,6 +536,8 @@ __global__ __launch_bounds__(256) void k_gemm_b3(GemmArgs a) {
   int tm, tn;
   tile_coords(tile, (a.M + BM - 1) / BM, tiles_n, a.band_rows, &tm, &tn);
   const int m0 = tm * BM, n0 = tn * BN;
+  const int group = GROUPED ? a.group_tile[tm] : 0;
+  if (GROUPED && group < 0) return;
 
   // global loads: A eight lanes to a row (a float4 each), W four lanes to a row (8 bf16 each)
   const int ar = tid >> 3, ak = (tid & 7) * 4;
@@ -520,11 +546,12 @@ __global__ __launch_bounds__(256) void k_gemm_b3(GemmArgs a) {
   const float* Ag[ALD];
   const char* Wg[BLD];
 #pragma unroll
-  for (int i = 0; i < ALD; ++i) Ag[i] = a.A + (size_t)min(m0 + ar + 32 * i, a.M - 1) * a.lda + ak;
+  for (int i = 0; i < ALD; ++i)
+    Ag[i] = a.A + (size_t)(GROUPED ? group_row(a, m0 + ar + 32 * i) : min(m0 + ar + 32 * i, a.M - 1)) * a.lda + ak;
 #pragma unroll
   for (int i = 0; i < BLD; ++i) {
     constexpr int RP = WT == 2 ? 128 : 64;  // rows per pass
-    const size_t row = (size_t)min(n0 + br + RP * i, a.N - 1);
+    const size_t row = (size_t)min(n0 + br + RP * i, a.N - 1) + (GROUPED ? (size_t)group * a.N : 0);
     Wg[i] = reinterpret_cast<const char*>(a.W) + (WT == 2 ? row * a.K + (tid & 1) * 16 : (row * a.K + bp * 8) * 2);
   }
 
@@ -700,7 +727,12 @@ __global__ __launch_bounds__(256) void k_gemm_b3(GemmArgs a) {
         const int m = m0 + wm * WM + 32 * i + 8 * (v >> 2) + 4 * half + (v & 3);
         if (m >= a.M) continue;
         float c = bias + (WT == 2 ? wscale * acc[i][j][v] : acc[i][j][v]);
+        if constexpr (EPI == GEMM_SILU_PAIR) {
+          store_silu_pair(a, m, n, c);
+          continue;
+        }
         if (EPI == GEMM_GELU) c = gelu_tanh(c);
+        if (EPI == GEMM_SQRELU) c = sq_relu(c);
         if (kAddsResid<EPI>) c = a.resid[(size_t)m * a.ldc + n] + col_scaled<EPI>(a, n, c);
         a.C[(size_t)m * a.ldc + n] = c;
       }
@@ -909,6 +941,7 @@ __global__ __launch_bounds__(256) void k_gemm_b9(GemmArgs a) {
         if (m >= a.M) continue;
         float c = bias + acc[i][j][v];
         if (EPI == GEMM_GELU) c = gelu_tanh(c);
+        if (EPI == GEMM_SQRELU) c = sq_relu(c);
         if (kAddsResid<EPI>) c = a.resid[(size_t)m * a.ldc + n] + col_scaled<EPI>(a, n, c);
         a.C[(size_t)m * a.ldc + n] = c;
       }
@@ -939,6 +972,7 @@ __global__ __launch_bounds__(256) void k_splitk_reduce(GemmArgs a, int parts) {
 #pragma unroll
   for (int k = 0; k < 4; ++k) {
     if (EPI == GEMM_GELU) c[k] = gelu_tanh(c[k]);
+    if (EPI == GEMM_SQRELU) c[k] = sq_relu(c[k]);
     if (kAddsResid<EPI>) c[k] = a.resid[m * a.ldc + n + k] + col_scaled<EPI>(a, (int)n + k, c[k]);
     dst[k] = c[k];
   }
@@ -999,6 +1033,7 @@ __global__ __launch_bounds__(256) void k_splitk_reduce_ln(GemmArgs a, int parts)
 #pragma unroll
       for (int k = 0; k < 4; ++k) {
         if (EPI == GEMM_GELU) r[k] = gelu_tanh(r[k]);
+        if (EPI == GEMM_SQRELU) r[k] = sq_relu(r[k]);
         if (kAddsResid<EPI>) r[k] = a.resid[m * a.ldc + n + k] + col_scaled<EPI>(a, (int)n + k, r[k]);
       }
       c[q] = f4{r[0], r[1], r[2], r[3]};
@@ -1142,6 +1177,7 @@ __global__ __launch_bounds__(256) void k_gemv_rows(GemmArgs a) {
   if (b >= a.M || n >= a.N) return;
   float c = (a.bias ? a.bias[n] : 0.0f) + acc[0];
   if (EPI == GEMM_GELU) c = gelu_tanh(c);
+  if (EPI == GEMM_SQRELU) c = sq_relu(c);
   if (kAddsResid<EPI>) c = a.resid[(size_t)b * a.ldc + n] + col_scaled<EPI>(a, n, c);
   a.C[(size_t)b * a.ldc + n] = c;
 }
@@ -1430,6 +1466,7 @@ __global__ __launch_bounds__(512) void k_gemm_rows32(GemmArgs a) {
     }
     float c = ebias[q] + sum;
     if (EPI == GEMM_GELU) c = gelu_tanh(c);
+    if (EPI == GEMM_SQRELU) c = sq_relu(c);
     if (kAddsResid<EPI>) c = eres[q] + col_scaled<EPI>(a, n, c);
     a.C[a.c_packed ? packed32_index((size_t)b, (size_t)n) : (size_t)b * a.ldc + n] = c;
   }
@@ -1457,6 +1494,7 @@ __global__ __launch_bounds__(256) void k_tail_reduce(GemmArgs a) {
 #pragma unroll
   for (int k = 0; k < 4; ++k) {
     if (EPI == GEMM_GELU) c[k] = gelu_tanh(c[k]);
+    if (EPI == GEMM_SQRELU) c[k] = sq_relu(c[k]);
     if (kAddsResid<EPI>) c[k] = a.resid[(size_t)m * a.ldc + n + k] + col_scaled<EPI>(a, n + k, c[k]);
     dst[k] = c[k];
   }
@@ -1821,6 +1859,8 @@ hipError_t launch_gemm_tile(const GemmArgs& a, int epi, hipStream_t s) {
     hipLaunchKernelGGL((k_gemm<BM, BN, GEMM_BIAS, WBF, 0, BKT>), dim3(grid), dim3(256), 0, s, a);
   else if (epi == GEMM_GELU)
     hipLaunchKernelGGL((k_gemm<BM, BN, GEMM_GELU, WBF, 0, BKT>), dim3(grid), dim3(256), 0, s, a);
+  else if (epi == GEMM_SQRELU)
+    hipLaunchKernelGGL((k_gemm<BM, BN, GEMM_SQRELU, WBF, 0, BKT>), dim3(grid), dim3(256), 0, s, a);
   else if (epi == GEMM_RESID)
     hipLaunchKernelGGL((k_gemm<BM, BN, GEMM_RESID, WBF, 0, BKT>), dim3(grid), dim3(256), 0, s, a);
   else if (epi == GEMM_RESID_SCALED)
@@ -1845,6 +1885,8 @@ hipError_t launch_gemm_b3_shape(const GemmArgs& a0, int epi, hipStream_t s) {
     hipLaunchKernelGGL((k_gemm_b3<BM, BN, GEMM_BIAS, 0, WT>), dim3(grid), dim3(256), 0, s, a);
   else if (epi == GEMM_GELU)
     hipLaunchKernelGGL((k_gemm_b3<BM, BN, GEMM_GELU, 0, WT>), dim3(grid), dim3(256), 0, s, a);
+  else if (epi == GEMM_SQRELU)
+    hipLaunchKernelGGL((k_gemm_b3<BM, BN, GEMM_SQRELU, 0, WT>), dim3(grid), dim3(256), 0, s, a);
   else if (epi == GEMM_RESID)
     hipLaunchKernelGGL((k_gemm_b3<BM, BN, GEMM_RESID, 0, WT>), dim3(grid), dim3(256), 0, s, a);
   else if (epi == GEMM_RESID_SCALED)
@@ -1880,6 +1922,8 @@ hipError_t launch_gemm_b9(const GemmArgs& a0, int epi, int parts, hipStream_t s,
     hipLaunchKernelGGL((k_gemm_b9<128, 128, GEMM_BIAS>), dim3(grid), dim3(256), 0, s, a);
   else if (epi == GEMM_GELU)
     hipLaunchKernelGGL((k_gemm_b9<128, 128, GEMM_GELU>), dim3(grid), dim3(256), 0, s, a);
+  else if (epi == GEMM_SQRELU)
+    hipLaunchKernelGGL((k_gemm_b9<128, 128, GEMM_SQRELU>), dim3(grid), dim3(256), 0, s, a);
   else if (epi == GEMM_RESID)
     hipLaunchKernelGGL((k_gemm_b9<128, 128, GEMM_RESID>), dim3(grid), dim3(256), 0, s, a);
   else if (epi == GEMM_RESID_SCALED)
@@ -1941,6 +1985,10 @@ hipError_t launch_splitk_reduce(const GemmArgs& a, int epi, int parts, hipStream
       hipLaunchKernelGGL((k_splitk_reduce_ln<GEMM_GELU, true>), dim3(a.M), dim3(256), 0, s, a, parts);
     else if (epi == GEMM_GELU)
       hipLaunchKernelGGL((k_splitk_reduce_ln<GEMM_GELU, false>), dim3(a.M), dim3(256), 0, s, a, parts);
+    else if (epi == GEMM_SQRELU && early)
+      hipLaunchKernelGGL((k_splitk_reduce_ln<GEMM_SQRELU, true>), dim3(a.M), dim3(256), 0, s, a, parts);
+    else if (epi == GEMM_SQRELU)
+      hipLaunchKernelGGL((k_splitk_reduce_ln<GEMM_SQRELU, false>), dim3(a.M), dim3(256), 0, s, a, parts);
     else if (epi == GEMM_RESID && early)
       hipLaunchKernelGGL((k_splitk_reduce_ln<GEMM_RESID, true>), dim3(a.M), dim3(256), 0, s, a, parts);
     else if (epi == GEMM_RESID_SCALED && early)
@@ -1959,6 +2007,8 @@ hipError_t launch_splitk_reduce(const GemmArgs& a, int epi, int parts, hipStream
     hipLaunchKernelGGL(k_splitk_reduce<GEMM_BIAS>, dim3(rblocks), dim3(256), 0, s, a, parts);
   else if (epi == GEMM_GELU)
     hipLaunchKernelGGL(k_splitk_reduce<GEMM_GELU>, dim3(rblocks), dim3(256), 0, s, a, parts);
+  else if (epi == GEMM_SQRELU)
+    hipLaunchKernelGGL(k_splitk_reduce<GEMM_SQRELU>, dim3(rblocks), dim3(256), 0, s, a, parts);
   else if (epi == GEMM_RESID)
     hipLaunchKernelGGL(k_splitk_reduce<GEMM_RESID>, dim3(rblocks), dim3(256), 0, s, a, parts);
   else if (epi == GEMM_RESID_SCALED)
@@ -1982,6 +2032,8 @@ hipError_t launch_gemv_rows_r(const GemmArgs& a, int epi, hipStream_t s) {
     hipLaunchKernelGGL((k_gemv_rows<MB, R, GEMM_BIAS, WBF>), grid, dim3(256), 0, s, a);
   else if (epi == GEMM_GELU)
     hipLaunchKernelGGL((k_gemv_rows<MB, R, GEMM_GELU, WBF>), grid, dim3(256), 0, s, a);
+  else if (epi == GEMM_SQRELU)
+    hipLaunchKernelGGL((k_gemv_rows<MB, R, GEMM_SQRELU, WBF>), grid, dim3(256), 0, s, a);
   else if (epi == GEMM_RESID)
     hipLaunchKernelGGL((k_gemv_rows<MB, R, GEMM_RESID, WBF>), grid, dim3(256), 0, s, a);
   else if (epi == GEMM_RESID_SCALED)
@@ -2042,6 +2094,8 @@ hipError_t launch_gemm_rows32_m(const GemmArgs& a0, int epi, int parts, int rows
     hipLaunchKernelGGL((k_gemm_rows32<GEMM_BIAS, WT, XP, M16, NR, MT>), grid, dim3(512), 0, s, a);
   else if (epi == GEMM_GELU)
     hipLaunchKernelGGL((k_gemm_rows32<GEMM_GELU, WT, XP, M16, NR, MT>), grid, dim3(512), 0, s, a);
+  else if (epi == GEMM_SQRELU)
+    hipLaunchKernelGGL((k_gemm_rows32<GEMM_SQRELU, WT, XP, M16, NR, MT>), grid, dim3(512), 0, s, a);
   else if (epi == GEMM_RESID)
     hipLaunchKernelGGL((k_gemm_rows32<GEMM_RESID, WT, XP, M16, NR, MT>), grid, dim3(512), 0, s, a);
   else if (epi == GEMM_RESID_SCALED)
@@ -2096,6 +2150,9 @@ hipError_t launch_gemm_tail(const GemmArgs& a, int epi, hipStream_t s) {
   } else if (epi == GEMM_GELU) {
     hipLaunchKernelGGL((k_gemm<BM, BN, GEMM_GELU, WBF, 2, BKT>), dim3(grid), dim3(256), 0, s, a);
     hipLaunchKernelGGL((k_tail_reduce<BM, BN, GEMM_GELU>), rgrid, dim3(256), 0, s, a);
+  } else if (epi == GEMM_SQRELU) {
+    hipLaunchKernelGGL((k_gemm<BM, BN, GEMM_SQRELU, WBF, 2, BKT>), dim3(grid), dim3(256), 0, s, a);
+    hipLaunchKernelGGL((k_tail_reduce<BM, BN, GEMM_SQRELU>), rgrid, dim3(256), 0, s, a);
   } else if (epi == GEMM_RESID) {
     hipLaunchKernelGGL((k_gemm<BM, BN, GEMM_RESID, WBF, 2, BKT>), dim3(grid), dim3(256), 0, s, a);
     hipLaunchKernelGGL((k_tail_reduce<BM, BN, GEMM_RESID>), rgrid, dim3(256), 0, s, a);
@@ -2271,6 +2328,36 @@ hipError_t launch_gemm(const GemmArgs& a, int epi, int num_cus, hipStream_t s) {
   if (e == hipSuccess && a.ln_out && !ln_done)
     e = launch_layer_norm_rows(a.C, a.ln_out, a.M, a.N, a.ln_g, a.ln_b, a.ln_eps, s, a.ln_packed);
   return e;
+}
+
+hipError_t launch_gemm_grouped(const GemmArgs& a0, int epi, int tile_rows, const int* group_tile, const int* group_rows,
+                               hipStream_t s) {
+  GemmArgs a = a0;
+  a.group_tile = group_tile;
+  a.group_rows = group_rows;
+  if (!gemm_supported(a) || a.K % 32 != 0 || a.w_scale || a.bias || a.N % 2 != 0 || !group_tile || a.M % tile_rows != 0)
+    return hipErrorInvalidValue;
+  if (epi != GEMM_BIAS && epi != GEMM_SILU_PAIR) return hipErrorInvalidValue;
+  const int bn = a.w_bf16 ? 128 : 64;
+  const int tiles_m = a.M / tile_rows, tiles_n = (a.N + bn - 1) / bn, tiles = tiles_m * tiles_n;
+  a.band_rows = choose_band(tiles_m, std::max(1, (tiles + 7) / 8), tile_rows, bn);
+  const dim3 grid((tiles + 7) / 8 * 8);
+#define PG_GROUPED(KERNEL, BM, ...)                                                                          \
+  if (epi == GEMM_BIAS) hipLaunchKernelGGL((KERNEL<BM, GEMM_BIAS, __VA_ARGS__>), grid, dim3(256), 0, s, a);   \
+  else hipLaunchKernelGGL((KERNEL<BM, GEMM_SILU_PAIR, __VA_ARGS__>), grid, dim3(256), 0, s, a);
+#define PG_TILE(M, N) M, N
+  if (a.w_bf16 && tile_rows == 128) {
+    PG_GROUPED(k_gemm_b3, PG_TILE(128, 128), 0, 1, true)
+  } else if (a.w_bf16 && tile_rows == 64) {
+    PG_GROUPED(k_gemm_b3, PG_TILE(64, 128), 0, 1, true)
+  } else if (!a.w_bf16 && tile_rows == 64) {
+    PG_GROUPED(k_gemm, PG_TILE(64, 64), 0, 0, 32, true)
+  } else {
+    return hipErrorInvalidValue;
+  }
+#undef PG_TILE
+#undef PG_GROUPED
+  return hipGetLastError();
 }
 
 bool gemm_takes_rows32(int M, int K, int lda, int w_bf16) {

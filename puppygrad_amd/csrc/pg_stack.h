@@ -1,10 +1,13 @@
 // Stack models: decoders whose config.json lists their layers one by one, each with the kind and
-// the sizes of its sequence mixers.  A layer is x <- x + ls1 * mixers(h) + ls2 * mlp(h) with
-// h = RMS norm of x: its sublayers read one norm and are added together, so that a layer is one
-// product with all input projections side by side, the mixers, and the products back to x.
+// the sizes of its sequence mixers.  Two forms of layer:
+//  parallel (Tarepel): x <- x + ls1 * mixers(h) + ls2 * mlp(h) with h = RMS norm of x: the sublayers
+//    read one norm and are added together, so that a layer is one product with all input
+//    projections side by side, the mixers, and the products back to x;
+//  post-norm (Movudra): x <- x + norm1(mixer(x)), then x <- x + norm2(ff(x)): a sublayer's output is
+//    normed and added by whatever reads x next.
 //
-// The state of a sequence has a fixed size: one chunk of keys and values per attention, one
-// matrix per recurrent head, the last inputs of the short convolutions.
+// The state of a sequence has a fixed size: one chunk or window of keys and values (or latents) per
+// attention, one matrix per recurrent head, the last inputs of the short convolutions.
 #pragma once
 
 #include <memory>
@@ -18,8 +21,28 @@
 
 namespace pgh {
 
+// Feed-forward of a post-norm layer: max(W_up h + b, 0)^2 -> W_down + b, or a mixture of experts.
+struct PostFeedForward {
+  enum Kind { kNone, kDense, kMoe } kind = kNone;
+  int ff = 0, ff_pad = 0;                        // dense
+  float *up_w = nullptr, *up_b = nullptr;        // [ff_pad][width_pad]
+  float *down_w = nullptr, *down_b = nullptr;    // [width_pad][ff_pad]
+  pgk::Moe moe{};
+  float* router_w = nullptr;                     // [experts_pad][width_pad]
+};
+
 struct StackLayer {
   bool has_attn = false, has_rec = false, has_mlp = false;
+  // post-norm layers: exactly one of has_rec and has_latent
+  bool post_norm = false, has_latent = false;
+  pgk::LatentAttn latent{};
+  float* uq_w = nullptr;                         // [heads * (dim + rot_dim)][q_pad]
+  float* low_a_w = nullptr;                      // REC_CHANNEL_DELTA: as rec.low_a.w, low_g.w
+  float* low_g_w = nullptr;
+  int norm_groups = 0;                           // REC_SSD: norm of the mixer's output, and its gain
+  float* mix_norm = nullptr;
+  PostFeedForward ffn;
+  float *norm1 = nullptr, *norm2 = nullptr;      // gains [width_pad]
   // Cache pointers in these are null; the cache fills them in (StackCache::bind).
   pgk::ChunkAttn attn{};
   pgk::Recurrence rec{};
@@ -41,6 +64,9 @@ struct StackModel {
   float *embed = nullptr, *head = nullptr, *final_norm = nullptr;
   // largest of each over the layers
   int max_in = 0, max_mix = 0, max_ff = 0, max_keys = 0, max_conv = 0, max_decay = 0, max_part = 0;
+  // post-norm layers: final_norm has width_pad gains and logit_scale is 1
+  bool post_norm = false;
+  int max_q_rank = 0, max_q = 0, max_qa = 0, max_gate = 0;
   std::vector<void*> memory;
   ~StackModel();
 };
@@ -48,13 +74,26 @@ struct StackModel {
 // State and working memory of a pg_kv_cache of a stack model.
 struct StackCache {
   struct Layer {
-    float *kring = nullptr, *vring = nullptr, *conv = nullptr, *state = nullptr;
+    float *kring = nullptr, *vring = nullptr, *conv = nullptr, *state = nullptr, *latent = nullptr;
+  };
+  // Mixture of experts: router logits, activations, outputs by slot, and the route's lists.
+  struct MoeBuffers {
+    float *logits = nullptr, *act = nullptr, *slot_out = nullptr;
+    pgk::MoeRoute route{};
+    void bind(float* const (&p)[6]) {
+      int** at[6] = {&route.count, &route.rank, &route.expert, &route.slot, &route.slot_row, &route.tile};
+      for (int i = 0; i < 6; ++i) *at[i] = reinterpret_cast<int*>(p[i]);
+    }
   };
   std::vector<Layer> layers;
+  MoeBuffers moe;  // one token of every sequence
   pgk::StepWords* words = nullptr;  // position of the next token, on the device
   bool lists_ids = false;           // ... steps list their ids
   // one token of every sequence
   float *x = nullptr, *h = nullptr, *y = nullptr, *mix = nullptr, *act = nullptr, *part = nullptr;
+  // post-norm layers: the residual before and after a sublayer in turn (x, h), a sublayer's output,
+  // queries of latent attention (their latents normed, as projected, in the latent space)
+  float *sub = nullptr, *cq = nullptr, *q = nullptr, *qa = nullptr;
   // many rows: one block, grown on demand
   float* rows = nullptr;
   size_t rows_floats = 0;

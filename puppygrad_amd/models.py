@@ -13,7 +13,7 @@ from .model import Gpt2HipConfig, Model, _check
 
 
 class StackModel(Model):
-    """A model whose config.json lists its layers with their mixers (Tarepel).  `config` is that
+    """A model whose config.json lists its layers with their mixers (Tarepel, Movudra).  `config` is that
     file's object.  Weights are stored as `hip_config.weight_storage` says (f32 or bf16); a cache
     has a fixed size and takes sequences of any length."""
 
@@ -34,7 +34,8 @@ def _gpt2(handle, model_dir) -> Gpt2Model:
 
 
 # architecture (pg_model_architecture) -> what wraps its handle
-ARCHITECTURES: Dict[str, Callable[..., Model]] = {"gpt2": _gpt2, "Tarepel": StackModel.from_handle}
+ARCHITECTURES: Dict[str, Callable[..., Model]] = {"gpt2": _gpt2, "Tarepel": StackModel.from_handle,
+                                           "Movudra": StackModel.from_handle}
 
 
 def load_model(model_dir, hip_config: Optional[Gpt2HipConfig] = None) -> Model:
