@@ -66,15 +66,16 @@ def main() -> int:
                     help="skip the other configurations (they run only beside the default workload)")
     ap.add_argument("--decode-path", default="auto", choices=["auto", "kernels", "persistent"])
     ap.add_argument("--workload", default="decode",
-                    choices=["decode", "prefill", "batch-decode", "sampled-stream", "tarepel"],
+                    choices=["decode", "prefill", "batch-decode", "sampled-stream", "tarepel", "movudra"],
                     help="prefill: a step is one prefill of --prefill tokens (GEMM path, MFMA-bound); "
                          "batch-decode: a step is one greedy step of --batch sequences; "
                          "sampled-stream: streamed generations of --steps tokens with sampled selection; "
                          "tarepel: prefill and decode of a Tarepel stack model at several widths beside "
-                         "GPT-2 models of the same width and parameters per layer")
-    ap.add_argument("--widths", default="768,1280,1600", help="widths of --workload tarepel")
-    ap.add_argument("--only", default="", help="--workload tarepel: stack or gpt2, and one of prefill, "
-                                               "decode, batch (profiling runs)")
+                         "GPT-2 models of the same width and parameters per layer; "
+                         "movudra: the same for a Movudra model beside Tarepel")
+    ap.add_argument("--widths", default="768,1280,1600", help="widths of --workload tarepel and movudra")
+    ap.add_argument("--only", default="", help="--workload tarepel and movudra: a model's name (tarepel, movudra, "
+                                               "gpt2) and one of prefill, decode, batch (profiling runs)")
     ap.add_argument("--batch", type=int, default=None,
                     help="sequences of a batched step (batch-decode: 16 by default; prefill: 1)")
     ap.add_argument("--bf16", action="store_true", help="store the weights as bf16 (fp32 arithmetic)")
@@ -93,8 +94,8 @@ def main() -> int:
 
     from puppygrad_amd import Gpt2Config, Gpt2HipConfig, Gpt2Model, _lib, synth
 
-    if args.workload == "tarepel":
-        return bench_tarepel(args)
+    if args.workload in ("tarepel", "movudra"):
+        return bench_stack(args)
 
     model_kw = {"xl": synth.GPT2_XL, "large": synth.GPT2_LARGE, "medium": synth.GPT2_MEDIUM,
                 "small": synth.GPT2_SMALL}[args.model]
@@ -526,18 +527,29 @@ def bench_prefill(args, cfg, model, ids, n_prefill) -> int:
     return 0
 
 
-def stack_layer_params(cfg) -> int:
-    """Parameters of a stack model's layers that a token meets (everything but embed and head)."""
+def stack_layer_params(cfg, tokens: int = 1) -> int:
+    """Parameters of a stack model's layers that `tokens` tokens meet (everything but embed and head;
+    of a mixture of experts with its choices spread evenly)."""
     from puppygrad_amd import synth
-    return sum(int(np.prod(s, dtype=np.int64)) for n, s in synth.stack_tensor_shapes(cfg).items()
-               if n not in ("embed", "head"))
+    total = 0
+    for n, s in synth.stack_tensor_shapes(cfg).items():
+        if n in ("embed", "head"):
+            continue
+        share = 1.0
+        if ".mlp.e" in n:
+            r = cfg["layers"][int(n[1:n.index(".")])]["mlp"]["router"]
+            share = 1.0 - (1.0 - r["top"] / r["experts"]) ** tokens
+        total += share * int(np.prod(s, dtype=np.int64))
+    return int(total)
 
 
-def bench_tarepel(args) -> int:
-    """Tarepel beside GPT-2 at the same width, layer count, vocabulary and (within 2 %) parameters
-    per layer, bf16-stored weights: prefill of 1024 tokens, batch-1 greedy decode from there and a
-    batch-32 step from 256 tokens.  `roofline` is that of the bound both share: the weights' bytes
-    at the HBM peak for decode, the products' flops at the bf16 matrix peak for prefill."""
+def bench_stack(args) -> int:
+    """A stack model beside another model at the same width, layer count, vocabulary and (within 2 %)
+    parameters per layer that a token meets, bf16-stored weights: Tarepel beside GPT-2, Movudra
+    beside Tarepel.  Prefill of 1024 tokens, batch-1 greedy decode from there and a batch-32 step
+    from 256 tokens.  The fractions are of the bound the models share: the bytes of the weights
+    that the step meets at the HBM peak for decode, the products' flops at the bf16 matrix peak for
+    prefill."""
     import tempfile
 
     from puppygrad_amd import Gpt2Config, Gpt2HipConfig, Gpt2Model, _lib, load_model, synth
@@ -545,14 +557,16 @@ def bench_tarepel(args) -> int:
     layers, vocab, T, NB, TB = 8, 50257, 1024, 32, 256
     only = [w for w in args.only.split(",") if w]
     steps = min(args.steps, 127)
+    models = {"tarepel": ("tarepel", "gpt2"), "movudra": ("movudra", "tarepel")}[args.workload]
 
     def want(*what):
         return all(w in what for w in only) if only else True
 
-    def measure(model, params, name):
+    def measure(model, params, batch_params, name):
         ids = synth.token_ids(T, synth.TOKEN_SEED_BASE + 7, vocab)
         out = {"params_per_layer": params // layers}
-        wbytes = 2 * (params + vocab * model._info().width)
+        head = vocab * model._info().width
+        wbytes = 2 * (params + head)
         if want(name, "prefill"):
             cache = model.new_kv_cache()
             for _ in range(2):
@@ -584,32 +598,35 @@ def bench_tarepel(args) -> int:
             _, st = model.decode_greedy_batch(cache, 65)
             sec = st.gpu_decode_time / 64
             out["batch_step"] = {"batch": NB, "tokens_per_s": round(NB / sec, 1), "us": round(sec * 1e6, 2),
-                                 "frac_hbm_weights": round(wbytes / sec / 1e9 / HBM_PEAK_GBS, 4)}
+                                 "frac_hbm_weights": round(2 * (batch_params + head) / sec / 1e9 / HBM_PEAK_GBS, 4)}
         return out
 
     rows = {}
     for width in (int(w) for w in args.widths.split(",")):
         entry = {}
-        if not only or "gpt2" not in only:
-            cfg = synth.tarepel_config(width, layers, vocab)
-            with tempfile.TemporaryDirectory() as tmp:
-                synth.write_model_dir(tmp, cfg, synth.stack_weights(cfg, synth.WEIGHT_SEED_BASE + 20))
-                model = load_model(tmp, hip)
-            entry["tarepel"] = measure(model, stack_layer_params(cfg), "stack")
-            log(f"[bench] width {width} tarepel: {entry['tarepel']}")
-            del model
-        if not only or "stack" not in only:
-            g = Gpt2Config(vocab_size=vocab, n_positions=T, n_embd=width, n_layer=layers, n_head=width // 64)
-            model = Gpt2Model.new(g, synth.random_weights(g, synth.WEIGHT_SEED_BASE + 21), hip)
-            entry["gpt2"] = measure(model, layers * 12 * width * width, "gpt2")
-            log(f"[bench] width {width} gpt2: {entry['gpt2']}")
+        for name in models:
+            if only and any(m in only for m in models) and name not in only:
+                continue
+            if name == "gpt2":
+                g = Gpt2Config(vocab_size=vocab, n_positions=T, n_embd=width, n_layer=layers, n_head=width // 64)
+                model = Gpt2Model.new(g, synth.random_weights(g, synth.WEIGHT_SEED_BASE + 21), hip)
+                params = batch_params = layers * 12 * width * width
+            else:
+                make = {"tarepel": synth.tarepel_config, "movudra": synth.movudra_config}[name]
+                cfg = make(width, layers, vocab)
+                with tempfile.TemporaryDirectory() as tmp:
+                    synth.write_model_dir(tmp, cfg, synth.stack_weights(cfg, synth.WEIGHT_SEED_BASE + 20))
+                    model = load_model(tmp, hip)
+                params, batch_params = stack_layer_params(cfg), stack_layer_params(cfg, NB)
+            entry[name] = measure(model, params, batch_params, name)
+            log(f"[bench] width {width} {name}: {entry[name]}")
             del model
         rows[str(width)] = entry
     first = rows[str(max(int(w) for w in rows))]
-    value = first.get("tarepel", {}).get("decode", {}).get("tokens_per_s")
+    value = first.get(models[0], {}).get("decode", {}).get("tokens_per_s")
     info = _devinfo()
     print(json.dumps({
-        "metric": "decode tokens/sec, Tarepel 8 layers bf16-stored weights bs=1 (largest width)",
+        "metric": f"decode tokens/sec, {models[0].capitalize()} 8 layers bf16-stored weights bs=1 (largest width)",
         "value": value, "unit": "tokens/s", "n_gpus": 1, "steps": steps, "warmup": 16,
         "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "f32", "data": "synthetic",
         "config": {"workload": f"prefill of {T} tokens, batch-1 decode from {T - 160}, batch-{NB} step "

@@ -127,7 +127,7 @@ def bf16_rounded(w: Gpt2Weights) -> Gpt2Weights:
                        ln_f_b=w.ln_f_b)
 
 
-# ---- stack models (Tarepel) --------------------------------------------------------------------
+# ---- stack models (Tarepel, Movudra) --------------------------------------------------------------------
 # Layers of a real model's proportions, by width: every layer has about the 12 width^2
 # parameters of a GPT-2 layer of that width.  attn: heads of 64, key/value heads, chunk; delta
 # and gla: heads with 128-value states; ff of either kind of layer.
@@ -155,7 +155,94 @@ def tarepel_config(width: int, n_layer: int, vocab: int = 50257) -> dict:
             "logit_scale": 1.0, "layers": [gla if i % 3 == 2 else parallel for i in range(n_layer)]}
 
 
-def stack_tensor_shapes(cfg: dict, rank: int = STACK_GLA_RANK) -> "dict[str, tuple]":
+# Movudra: mamba2 (heads, groups, state, vdim), channel_delta (heads, kv_heads, dim, vdim, rank of decay
+# and gate), latent_attention (heads, dim, rot_dim, vdim, q_rank, kv_rank, window).
+MOVUDRA_SIZES = {
+    768: dict(mamba=(24, 1, 128, 64), delta=(6, 6, 128, 128, 128), latent=(8, 64, 32, 64, 384, 256, 512)),
+    1280: dict(mamba=(40, 2, 128, 64), delta=(10, 10, 128, 128, 128), latent=(10, 128, 64, 128, 512, 512, 512)),
+    1600: dict(mamba=(50, 2, 128, 64), delta=(16, 16, 128, 128, 128), latent=(16, 128, 64, 128, 768, 512, 512)),
+}
+MOVUDRA_EXPERTS, MOVUDRA_TOP = 8, 2
+
+
+def movudra_config(width: int, n_layer: int, vocab: int = 50257) -> dict:
+    """A Movudra config.json of MOVUDRA_SIZES[width]: the three mixers in turn, the first layer dense,
+    the others with experts; a token meets about 12 width^2 parameters in every layer."""
+    z = MOVUDRA_SIZES[width]
+    H, G, N, e = z["mamba"]
+    mamba = {"heads": H, "groups": G, "state": N, "vdim": e, "conv": 4, "norm_groups": G}
+    n_mamba = width * (2 * H * e + 2 * G * N + H) + width * H * e
+    H, G, d, e, r = z["delta"]
+    delta = {"heads": H, "kv_heads": G, "dim": d, "vdim": e, "conv": 4}
+    n_delta = width * (2 * G * d + 2 * H * e + H) + r * (2 * width + H * (d + e))
+    H, d, rot, e, q, kv, window = z["latent"]
+    latent = {"heads": H, "dim": d, "rot_dim": rot, "vdim": e, "q_rank": q, "kv_rank": kv, "scale": (d + rot) ** -0.5,
+              "mask": {"size": window}, "rot": {"dims": rot, "base": 10000.0, "scaling": {
+                  "factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+    n_latent = width * (q + kv + rot + H * e) + q * H * (d + rot) + kv * H * (d + e)
+    layers = []
+    for i in range(n_layer):
+        kind, mixer, n = (("mamba2", mamba, n_mamba), ("channel_delta", delta, n_delta),
+                          ("latent_attention", latent, n_latent))[i % 3]
+        rest = 12 * width * width - n
+        if i == 0:
+            mlp = {"kind": "dense", "ff": round(rest / (2 * width * 32)) * 32}
+        else:
+            mlp = {"kind": "moe", "router": {"experts": MOVUDRA_EXPERTS, "top": MOVUDRA_TOP},
+                   "expert": {"ff": round(rest / (3 * width * MOVUDRA_TOP * 32)) * 32}}
+        layers.append({"type": kind, "mixer": mixer, "mlp": mlp})
+    return {"architecture": "Movudra", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "layers": layers}
+
+
+def movudra_tensor_shapes(cfg: dict, ranks=(128, 128)) -> "dict[str, tuple]":
+    """Names and shapes of a Movudra model's tensors; ranks: of the decay and of the output gate."""
+    C, V = cfg["width"], cfg["vocab"]
+    out = {"embed": (V, C)}
+    for i, layer in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", layer["mixer"]
+        q = p + "mix."
+        out[p + "norm1"] = (C,)
+        if layer["type"] == "mamba2":
+            H, inner, gn = m["heads"], m["heads"] * m["vdim"], m["groups"] * m["state"]
+            ch = inner + 2 * gn
+            out.update({q + "in": (inner + ch + H, C), q + "conv": (ch, m["conv"]), q + "conv.b": (ch,), q + "dt_bias": (H,),
+                        q + "A_log": (H,), q + "D": (H,), q + "norm": (inner,), q + "o": (C, inner)})
+        elif layer["type"] == "channel_delta":
+            H, qk, vv, hd = m["heads"], m["kv_heads"] * m["dim"], m["heads"] * m["vdim"], m["heads"] * m["dim"]
+            for x, n in (("q", qk), ("k", qk), ("v", vv)):
+                out.update({q + x: (n, C), q + x + ".conv": (n, m["conv"])})
+            out.update({q + "b": (H, C), q + "A_log": (H,), q + "norm": (m["vdim"],), q + "a1": (ranks[0], C),
+                        q + "a2": (hd, ranks[0]), q + "dt_bias": (hd,), q + "g1": (ranks[1], C), q + "g2": (vv, ranks[1]),
+                        q + "o": (C, vv)})
+        else:
+            H, K = m["heads"], m["kv_rank"]
+            out.update({q + "dq": (m["q_rank"], C), q + "dq.norm": (m["q_rank"],),
+                        q + "uq": (H * (m["dim"] + m["rot_dim"]), m["q_rank"]), q + "dkv": (K + m["rot_dim"], C),
+                        q + "dkv.norm": (K,), q + "uk": (H * m["dim"], K), q + "uv": (H * m["vdim"], K), q + "sink": (H,),
+                        q + "o": (C, H * m["vdim"])})
+        f = layer.get("mlp")
+        if f:
+            out[p + "norm2"] = (C,)
+            q = p + "mlp."
+            if f["kind"] == "dense":
+                out.update({q + "up": (f["ff"], C), q + "up.b": (f["ff"],), q + "down": (C, f["ff"]), q + "down.b": (C,)})
+            else:
+                ff = f["expert"]["ff"]
+                for e in range(f["router"]["experts"]):
+                    out.update({f"{q}e{e}.gate": (ff, C), f"{q}e{e}.up": (ff, C), f"{q}e{e}.down": (C, ff)})
+                out[q + "router"] = (f["router"]["experts"], C)
+    out.update({"final.norm": (C,), "head": (V, C)})
+    return out
+
+
+def stack_tensor_shapes(cfg: dict, rank=None) -> "dict[str, tuple]":
+    """Names and shapes of a stack model's tensors (rank: what config.json leaves to the tensors)."""
+    if cfg["architecture"] == "Movudra":
+        return movudra_tensor_shapes(cfg, *([] if rank is None else [rank]))
+    return tarepel_tensor_shapes(cfg, *([] if rank is None else [rank]))
+
+
+def tarepel_tensor_shapes(cfg: dict, rank: int = STACK_GLA_RANK) -> "dict[str, tuple]":
     """Names and shapes of a Tarepel model's tensors."""
     C, V = cfg["width"], cfg["vocab"]
     out = {"embed": (V, C)}
@@ -190,7 +277,12 @@ def stack_tensor_shapes(cfg: dict, rank: int = STACK_GLA_RANK) -> "dict[str, tup
 
 def bf16_bits(a: np.ndarray) -> np.ndarray:
     """The bf16 bit patterns (uint16) of f32 values, nearest even."""
-    return (round_bf16(a).view(np.uint32) >> np.uint32(16)).astype(np.uint16)
+    a = np.ascontiguousarray(a, np.float32)
+    out = np.empty(a.shape, np.uint16)
+    flat, dst, step = a.reshape(-1), out.reshape(-1), 1 << 18  # (a piece that stays in the CPU's cache)
+    for i in range(0, flat.size, step):
+        dst[i:i + step] = round_bf16(flat[i:i + step]).view(np.uint32) >> np.uint32(16)
+    return out
 
 
 def write_model_dir(path, cfg: dict, tensors) -> None:
@@ -242,4 +334,6 @@ def stack_weights(cfg: dict, seed: int, std: float = 0.02):
             a = a * np.float32(40.0) - np.float32(3.0)
         elif name.endswith("a2.b"):
             a = a * np.float32(40.0) + np.float32(2.0)
+        elif last == "D":
+            a = a + np.float32(1.0)
         yield name, a.reshape(shape)

@@ -3,9 +3,6 @@ prompts, portions, decoding through the cache, batches, reused caches, chunk edg
 generation and the trace runner.  Configurations and weights are made here."""
 import json
 import os
-import subprocess
-import sys
-from pathlib import Path
 
 import numpy as np
 import pytest
@@ -13,11 +10,10 @@ import pytest
 import oracle.tarepel as orc
 from puppygrad_amd import (Gpt2Error, Gpt2HipConfig, LogitsSampler, StackModel, TextGenerationConfig, _lib,
                            argmax_logits, generate, load_model, synth)
+from stack_helpers import Pair as AnyPair, check, ref_greedy, run_trace, same_until_close
 
 pytestmark = pytest.mark.gpu
-ROOT = Path(__file__).resolve().parents[1]
 BF16, F32 = _lib.PG_STORE_BF16, _lib.PG_STORE_F32
-TOL = 2e-5  # root mean square difference over the vocabulary, in units of the logits' own
 
 
 def attn(heads=4, kv=2, dim=16, chunk=12, rot=None, base=1000.0, scale=None):
@@ -77,39 +73,9 @@ def weights(cfg, seed, rank=5, **fixed):
     return out
 
 
-class Pair:
-    """A model on the device and its oracle."""
-
-    def __init__(self, tmp_path, cfg, w, storage=BF16, **hip):
-        synth.write_model_dir(tmp_path, cfg, w.items())
-        self.dir = tmp_path
-        self.dev = load_model(tmp_path, Gpt2HipConfig(weight_storage=storage, **hip))
-        self.ref = orc.Model(cfg, w)
-        self.vocab = cfg["vocab"]
-
-    def ids(self, n, seed=1):
-        return [int(t) for t in synth.token_ids(n, 0xA11CE + seed, self.vocab)]
-
-    def portions(self, ids, sizes, cache=None):
-        """Logits of every position, the sequence cut into portions of the given sizes (the last
-        size repeats)."""
-        cache = cache or self.dev.new_kv_cache()
-        cache.clear()
-        rows, at, k = [], 0, 0
-        while at < len(ids):
-            n = min(sizes[min(k, len(sizes) - 1)], len(ids) - at)
-            lg = self.dev.extend(ids[at:at + n], cache, range(n)).to_host().reshape(n, -1)
-            rows.append(lg)
-            at, k = at + n, k + 1
-        assert cache.seq_len == len(ids)
-        return np.concatenate(rows)
-
-
-def check(got, want, tol=TOL, what="logits"):
-    got, want = np.atleast_2d(np.asarray(got, np.float64)), np.atleast_2d(want)
-    assert got.shape == want.shape
-    err = np.sqrt(np.mean((got - want) ** 2, axis=1)) / np.sqrt(np.mean(want ** 2))
-    assert np.isfinite(got).all() and err.max() <= tol, f"{what}: {err.max():.2e} at row {err.argmax()} of {len(err)}"
+class Pair(AnyPair):
+    def __init__(self, *args, **kw):
+        super().__init__(orc, *args, **kw)
 
 
 @pytest.fixture(scope="module")
@@ -444,26 +410,6 @@ def test_old_state_in_the_first_chunks(tmp_path):
 
 
 # ---- generation ------------------------------------------------------------------------------------
-def ref_greedy(p, ids, n):
-    """The oracle's greedy continuation and, per step, the gap between its two best logits."""
-    state, out, gaps = p.ref.new_state(), [], []
-    lg = p.ref.run(ids, state)[-1]
-    for _ in range(n):
-        top = np.sort(lg)[-2:]
-        gaps.append((top[1] - top[0]) / np.sqrt(np.mean(lg ** 2)))
-        out.append(int(np.argmax(lg)))
-        lg = p.ref.step(out[-1], state)
-    return out, gaps
-
-
-def same_until_close(got, want, gaps, tol=1e-4):
-    for i, (g, w) in enumerate(zip(got, want)):
-        if gaps[i] < tol:
-            return i
-        assert g == w, f"token {i}: {g} != {w}"
-    return len(want)
-
-
 @pytest.mark.parametrize("path", [_lib.PG_DECODE_AUTO, _lib.PG_DECODE_KERNELS], ids=["graph", "kernels"])
 def test_greedy_generation(tmp_path, path):
     p = Pair(tmp_path, MIXED, weights(MIXED, 11), decode_path=path)
@@ -540,14 +486,6 @@ def test_sampled_stream(mixed):
 
 
 # ---- trace runner, registry ------------------------------------------------------------------------
-def run_trace(model_dir, steps, out, dtype="bfloat16"):
-    text = "".join(json.dumps(s) + "\n" for s in steps)
-    r = subprocess.run([sys.executable, str(ROOT / "bin" / "trace_run"), "--model", str(model_dir), "--dtype", dtype,
-                        "--out", str(out), "--max-tokens", "64"], input=text, capture_output=True, text=True, timeout=100)
-    assert r.returncode == 0, r.stderr
-    assert [l for l in r.stdout.splitlines() if l.startswith("done")] == [f"done {s['step']}" for s in steps]
-
-
 def test_trace_runner(mixed, tmp_path):
     a, b, c = mixed.ids(30, seed=14), mixed.ids(8, seed=15), mixed.ids(9, seed=16)
     steps = [{"step": 0, "entries": [{"id": "a", "tokens": a[:20], "want": [0, 19, 7]}], "end": []},
