@@ -48,7 +48,8 @@ struct GemvArgs {
   const float* ln_b;
   float eps;
   int norm_n;  // PRO_RMS, PRO_STACK
-  // PRO_STACK (add and gain may be null; vectors of at least K values, those past norm_n zeros)
+  // PRO_STACK: K a multiple of 4; add and gain may be null; all vectors hold at least K values from a
+  // multiple of 16 bytes on, those past norm_n (add_n) zeros
   const float *add = nullptr, *add_gain = nullptr, *gain = nullptr;
   float* x_out = nullptr;  // not x itself: other blocks still read it
   int add_n = 0, groups = 1;
@@ -275,7 +276,7 @@ hipError_t launch_gemm(const GemmArgs& a, int epilogue, int num_cus, hipStream_t
 // Many small products in one launch: rows are sorted by the matrix they meet.  Row m of the product
 // takes row group_rows[m] of A (any row where that is -1), and the rows of tile m / tile_rows meet
 // matrix group_tile[m / tile_rows] of W [groups][N][K] (-1: the tile is left out).  a.M counts the rows
-// with their padding, a multiple of tile_rows (64 or 128; 64 for f32 rows).  C has a row per m.
+// with their padding, a multiple of tile_rows (32, 64 or, bf16 rows only, 128).  C has a row per m.
 // group_rows null: row m itself.  GEMM_BIAS (without bias) or GEMM_SILU_PAIR.
 hipError_t launch_gemm_grouped(const GemmArgs& a, int epilogue, int tile_rows, const int* group_tile,
                                const int* group_rows, hipStream_t s);

@@ -149,7 +149,7 @@ __device__ __forceinline__ float chunk_dot(gv_u4 w, const float4* sx4, int j, fl
 
 template <int PRO, int EPI, int RPW, int WM>
 __global__ __launch_bounds__(kBlock) void k_gemv(GemvArgs a) {
-  extern __shared__ float sx[];  // K floats
+  extern __shared__ __attribute__((aligned(16))) float sx[];  // K floats
   __shared__ float red[kWaves];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int K = a.K;
@@ -162,6 +162,29 @@ __global__ __launch_bounds__(kBlock) void k_gemv(GemvArgs a) {
   constexpr int kPre = 4;
   const int KV = WM == WM_F32X4 ? K >> 2 : WM == WM_BF16X8 ? K >> 3 : K >> 4;  // chunks per row
   const gv_u4* Wv = reinterpret_cast<const gv_u4*>(a.W);
+  // PRO_STACK: inputs of up to 4096 values and what they are normed with, in registers (asked for before
+  // the weights: loads return in order)
+  constexpr int kIn = 4;
+  const bool in_regs = PRO == PRO_STACK && K <= 4 * kIn * kBlock;
+  float4 vx[PRO == PRO_STACK ? kIn : 1], va[PRO == PRO_STACK ? kIn : 1], vg[PRO == PRO_STACK ? kIn : 1],
+      vn[PRO == PRO_STACK ? kIn : 1];
+  if constexpr (PRO == PRO_STACK) {
+    if (in_regs) {
+#pragma unroll
+      for (int p = 0; p < kIn; ++p) {
+        vx[p] = va[p] = vg[p] = vn[p] = float4{0.f, 0.f, 0.f, 0.f};
+        const int i = tid + kBlock * p;
+        if (4 * i < K) {
+          vx[p] = reinterpret_cast<const float4*>(a.x)[i];
+          if (a.add) {
+            va[p] = reinterpret_cast<const float4*>(a.add)[i];
+            vg[p] = reinterpret_cast<const float4*>(a.add_gain)[i];
+          }
+          if (a.gain) vn[p] = reinterpret_cast<const float4*>(a.gain)[i];
+        }
+      }
+    }
+  }
   gv_u4 pre[RPW][kPre];
   if (kVec) {
 #pragma unroll
@@ -175,7 +198,73 @@ __global__ __launch_bounds__(kBlock) void k_gemv(GemvArgs a) {
       }
   }
 
-  if (PRO == PRO_ATTN_COMBINE) {
+  if constexpr (PRO == PRO_STACK) {
+    if (in_regs) {
+      auto sq = [](const float4& v) { return (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w); };
+      if (a.add) {
+        float ss = 0.0f;
+#pragma unroll
+        for (int p = 0; p < kIn; ++p) ss += sq(va[p]);
+        const float k = 1.0f / sqrtf(block_sum(ss, red) / (float)a.add_n + a.eps);
+#pragma unroll
+        for (int p = 0; p < kIn; ++p) {
+          vx[p].x += va[p].x * k * vg[p].x;
+          vx[p].y += va[p].y * k * vg[p].y;
+          vx[p].z += va[p].z * k * vg[p].z;
+          vx[p].w += va[p].w * k * vg[p].w;
+          const int i = tid + kBlock * p;
+          if (blockIdx.x == 0 && a.x_out && 4 * i < K) reinterpret_cast<float4*>(a.x_out)[i] = vx[p];
+        }
+      }
+      if (a.gain && a.groups <= 4) {
+        // (values past norm_n are zeros)
+        float inv[4] = {0.f, 0.f, 0.f, 0.f};
+        const int n = a.norm_n / a.groups;
+        if (a.groups == 1) {
+          float ss = 0.0f;
+#pragma unroll
+          for (int p = 0; p < kIn; ++p) ss += sq(vx[p]);
+          inv[0] = 1.0f / sqrtf(block_sum(ss, red) / (float)n + a.eps);
+#pragma unroll
+          for (int p = 0; p < kIn; ++p) {
+            vx[p].x *= inv[0] * vn[p].x;
+            vx[p].y *= inv[0] * vn[p].y;
+            vx[p].z *= inv[0] * vn[p].z;
+            vx[p].w *= inv[0] * vn[p].w;
+          }
+        } else {
+          float ss[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+          for (int p = 0; p < kIn; ++p)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+              const int at = 4 * (tid + kBlock * p) + e;
+              const float v = (&vx[p].x)[e];
+#pragma unroll
+              for (int g = 0; g < 4; ++g) ss[g] += at >= g * n && at < (g + 1) * n ? v * v : 0.0f;
+            }
+#pragma unroll
+          for (int g = 0; g < 4; ++g)
+            if (g < a.groups) inv[g] = 1.0f / sqrtf(block_sum(ss[g], red) / (float)n + a.eps);
+#pragma unroll
+          for (int p = 0; p < kIn; ++p)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+              const int at = 4 * (tid + kBlock * p) + e;
+              const float k = at < n ? inv[0] : at < 2 * n ? inv[1] : at < 3 * n ? inv[2] : inv[3];
+              (&vx[p].x)[e] *= k * (&vn[p].x)[e];
+            }
+        }
+      }
+#pragma unroll
+      for (int p = 0; p < kIn; ++p) {
+        const int i = tid + kBlock * p;
+        if (4 * i < K) reinterpret_cast<float4*>(sx)[i] = vx[p];
+      }
+    }
+  }
+  if (in_regs) {
+  } else if (PRO == PRO_ATTN_COMBINE) {
     for (int i = tid; i < K; i += kBlock)
       sx[i] = attn_combine_elem(a.part_acc, a.part_m, a.part_l, a.nsplit, a.head_dim, i);
   } else {
@@ -183,7 +272,7 @@ __global__ __launch_bounds__(kBlock) void k_gemv(GemvArgs a) {
   }
   __syncthreads();
   if (PRO == PRO_STACK) {
-    if (a.add) {
+    if (a.add && !in_regs) {
       float ss = 0.0f;
       for (int i = tid; i < K; i += kBlock) {
         const float v = a.add[i];
@@ -196,7 +285,7 @@ __global__ __launch_bounds__(kBlock) void k_gemv(GemvArgs a) {
       }
       __syncthreads();
     }
-    if (a.gain) {
+    if (a.gain && !(in_regs && a.groups <= 4)) {
       if (a.groups == 1) {
         float ss = 0.0f;
         for (int i = tid; i < a.norm_n; i += kBlock) ss += sx[i] * sx[i];

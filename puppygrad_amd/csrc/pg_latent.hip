@@ -74,41 +74,66 @@ __device__ void latent_row(const LatentAttn& a, const float* src, int pos, float
 }
 
 // ---- one token per sequence ----
-// Queries in the latent space, times scale and log2(e): blocks (h < heads, part of 128 latent columns);
-// block (heads, 0) writes the token's row of the cache.
+// Queries in the latent space, times scale and log2(e): blocks (h < heads, part of 128 latent
+// columns) for NB sequences, which share what they read of W_uk; blocks (heads, 0) write the tokens'
+// rows of the caches.
+template <int NB>
 __global__ __launch_bounds__(256) void k_latent_query(LatentDecode m, LatentAttn a) {
-  __shared__ float qs[kMixMaxDim], red[4];
+  __shared__ float qs[NB][kMixMaxDim], red[4];
   __shared__ __attribute__((aligned(16))) float sums[8][128];
-  const int tid = threadIdx.x, h = blockIdx.x, b = blockIdx.z, pos = *m.d_pos;
+  constexpr int PRE = 16;
+  const int tid = threadIdx.x, h = blockIdx.x, b0 = blockIdx.z * NB, nb = min(NB, m.nseq - b0), pos = *m.d_pos;
   if (h == a.heads) {
     if (blockIdx.y == 0)
-      latent_row(a, m.y + (size_t)b * m.ld_y + a.c_col, pos, a.ring + (size_t)b * a.ring_seq + (size_t)(pos % a.window) * a.ld,
-                 red);
+      for (int b = b0; b < b0 + nb; ++b)
+        latent_row(a, m.y + (size_t)b * m.ld_y + a.c_col, pos, a.ring + (size_t)b * a.ring_seq + (size_t)(pos % a.window) * a.ld,
+                   red);
     return;
   }
-  const float* q = m.q + ((size_t)b * a.heads + h) * (a.dim + a.rot_dim);
-  float* qa = m.qa + ((size_t)b * a.heads + h) * a.ld;
+  const int dk = a.dim + a.rot_dim;
   const float mul = a.scale * kLog2e;
   // 32 threads to the 128 columns, four each; eight groups take every eighth row of W_uk
   const int col = blockIdx.y * 128 + (tid & 31) * 4, grp = tid >> 5;
-  f4 sum = f4{0.f, 0.f, 0.f, 0.f};
-  for (int i = tid; i < a.dim; i += 256) qs[i] = q[i];
-  __syncthreads();
-  if (col < a.kv_pad) {
-#pragma unroll 8
-    for (int d = grp; d < a.dim; d += 8) sum += load_w4(a.up_w, a.w_bf16, ((size_t)h * a.dim + d) * a.kv_pad + col) * qs[d];
-  }
-  *reinterpret_cast<f4*>(&sums[grp][(tid & 31) * 4]) = sum;
-  __syncthreads();
-  if (tid < 128 && blockIdx.y * 128 + tid < a.kv_pad) {
-    float s = 0.0f;
+  const size_t w0 = (size_t)h * a.dim * a.kv_pad + min(col, a.kv_pad - 4);
+  f4 w[PRE];
 #pragma unroll
-    for (int g = 0; g < 8; ++g) s += sums[g][tid];
-    qa[blockIdx.y * 128 + tid] = s * mul;
+  for (int i = 0; i < PRE; ++i) w[i] = load_w4(a.up_w, a.w_bf16, w0 + (size_t)min(grp + 8 * i, a.dim - 1) * a.kv_pad);
+#pragma unroll
+  for (int b = 0; b < NB; ++b)
+    if (tid < a.dim) qs[b][tid] = m.q[((size_t)(b0 + min(b, nb - 1)) * a.heads + h) * dk + tid];
+  __syncthreads();
+  f4 sum[NB];
+#pragma unroll
+  for (int b = 0; b < NB; ++b) sum[b] = f4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int i = 0; i < PRE; ++i)
+#pragma unroll
+    for (int b = 0; b < NB; ++b)
+      if (grp + 8 * i < a.dim) sum[b] += w[i] * qs[b][grp + 8 * i];
+#pragma unroll 8
+  for (int d = grp + 8 * PRE; d < a.dim; d += 8) {
+    const f4 x = load_w4(a.up_w, a.w_bf16, w0 + (size_t)d * a.kv_pad);
+#pragma unroll
+    for (int b = 0; b < NB; ++b) sum[b] += x * qs[b][d];
+  }
+#pragma unroll
+  for (int b = 0; b < NB; ++b) {
+    if (b) __syncthreads();
+    *reinterpret_cast<f4*>(&sums[grp][(tid & 31) * 4]) = sum[b];
+    __syncthreads();
+    if (b < nb && tid < 128 && blockIdx.y * 128 + tid < a.kv_pad) {
+      float s = 0.0f;
+#pragma unroll
+      for (int g = 0; g < 8; ++g) s += sums[g][tid];
+      m.qa[((size_t)(b0 + b) * a.heads + h) * a.ld + blockIdx.y * 128 + tid] = s * mul;
+    }
   }
   if (blockIdx.y == 0) {
-    const float* rq = q + a.dim;
-    for (int i = tid; i < (a.ld - a.kv_pad) / 2; i += 256) {
+    const int pairs = (a.ld - a.kv_pad) / 2;
+    for (int x = tid; x < nb * pairs; x += 256) {
+      const int b = x / pairs, i = x - b * pairs;
+      const float* rq = m.q + ((size_t)(b0 + b) * a.heads + h) * dk + a.dim;
+      float* qa = m.qa + ((size_t)(b0 + b) * a.heads + h) * a.ld + a.kv_pad;
       float u = 2 * i < a.rot_dim ? rq[2 * i] : 0.0f, v = 2 * i + 1 < a.rot_dim ? rq[2 * i + 1] : 0.0f;
       if (i < a.half) {
         float s, c;
@@ -119,30 +144,35 @@ __global__ __launch_bounds__(256) void k_latent_query(LatentDecode m, LatentAttn
         u = u0 * c - v * s;
         v = v * c + u0 * s;
       }
-      qa[a.kv_pad + 2 * i] = u * mul;
-      qa[a.kv_pad + 2 * i + 1] = v * mul;
+      qa[2 * i] = u * mul;
+      qa[2 * i + 1] = v * mul;
     }
   }
 }
 
-// Sixteen heads against a share of the cached rows, 64 rows at a time, on the f32 matrix cores
+// Sixteen heads against a share of the cached rows, 32 rows at a time, on the f32 matrix cores
 // (v_mfma_f32_16x16x4_f32: A operand lane l -> A[l % 16][l / 16], B operand lane l -> B[l / 16][l % 16],
 // D lane l, register v -> D[4 (l / 16) + v][l % 16]):
-//   S (rows x heads): wavefront w takes rows 16 w ..; four columns of a lane's quarter per step
+//   S (rows x heads): wavefront w takes rows 16 (w % 2) .. and every second 16 columns of them from
+//     16 (w / 2) on; four columns of a lane's quarter per step
 //   softmax over the rows in LDS, running maximum and sum per head
 //   O (heads x latent columns) += P . C: wavefront w owns the 16-column tiles w, w + 4, ...
-// Which position a row of the ring holds does not matter: the first min(position + 1, window) rows
-// are the ones that the token sees.  Grid: x = share, y = 16 heads, z = sequence.  NT: tiles of a wavefront.
+// Everything a tile needs is asked for before the first of it is used.  Which position a row of the
+// ring holds does not matter: the first min(position + 1, window) rows are the ones that the token
+// sees.  Grid: x = share, y = 16 heads, z = sequence.  NT: column tiles of a wavefront; a row has at most
+// 64 NT + 256 columns.
+constexpr int kShareRows = 32;
 template <int NT>
-__global__ __launch_bounds__(256) void k_latent_attn(LatentDecode m, LatentAttn a) {
+__global__ __launch_bounds__(256, 1) void k_latent_attn(LatentDecode m, LatentAttn a) {
+  constexpr int MAXLD = 64 * NT + kMixMaxDim, NS = MAXLD / 32, NQ = 16 * MAXLD / 1024;
   extern __shared__ __attribute__((aligned(16))) float qs[];  // [16][ld + 4]
-  __shared__ __attribute__((aligned(16))) float ps[16][68];
+  __shared__ __attribute__((aligned(16))) float ps[2][16][36];
   __shared__ float ms[16], ls[16], al[16];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, quarter = lane >> 4, l16 = lane & 15;
   const int split = blockIdx.x, h0 = blockIdx.y * 16, b = blockIdx.z;
   const int nh = min(16, a.heads - h0), ld = a.ld, LD = ld + 4;
   const int pos = *m.d_pos, n = min(pos + 1, a.window);
-  const int per = ((a.window + m.splits - 1) / m.splits + 63) / 64 * 64;
+  const int per = ((a.window + m.splits - 1) / m.splits + kShareRows - 1) / kShareRows * kShareRows;
   const int j0 = split * per, j1 = min(n, j0 + per);
   float* part = m.part + (((size_t)b * a.heads + h0) * m.splits + split) * (a.kv_pad + 2);
   const size_t part_h = (size_t)m.splits * (a.kv_pad + 2);
@@ -153,60 +183,85 @@ __global__ __launch_bounds__(256) void k_latent_attn(LatentDecode m, LatentAttn 
     }
     return;
   }
-  for (int i = tid; i < 4 * ld; i += 256) {
-    const int h = i / (ld / 4), d = (i - h * (ld / 4)) * 4;
-    f4 q = f4{0.f, 0.f, 0.f, 0.f};
-    if (h < nh) q = *reinterpret_cast<const f4*>(m.qa + ((size_t)b * a.heads + h0 + h) * ld + d);
-    *reinterpret_cast<f4*>(&qs[h * LD + d]) = q;
+  const float* ring = a.ring + (size_t)b * a.ring_seq;
+  const int tiles = a.kv_pad / 16, steps = ld / 16, rows16 = 16 * (wave & 1), first = wave >> 1;
+  f4 qr[NQ];
+  {
+    const f4* q = reinterpret_cast<const f4*>(m.qa + ((size_t)b * a.heads + h0) * ld);  // (16 rows, dense)
+#pragma unroll
+    for (int i = 0; i < NQ; ++i) {
+      const int x = tid + 256 * i;
+      qr[i] = f4{0.f, 0.f, 0.f, 0.f};
+      if (x < nh * (ld / 4)) qr[i] = q[x];
+    }
+  }
+  f4 kr[NS];
+  float cr[NT][8];
+  auto fetch = [&](int k0) __attribute__((always_inline)) {
+    const float* row = ring + (size_t)min(k0 + rows16 + l16, j1 - 1) * ld + 4 * quarter;
+#pragma unroll
+    for (int s = 0; s < NS; ++s)
+      if (first + 2 * s < steps) kr[s] = *reinterpret_cast<const f4*>(row + 16 * (first + 2 * s));
+#pragma unroll
+    for (int t = 0; t < NT; ++t)
+      if (wave + 4 * t < tiles) {
+#pragma unroll
+        for (int k = 0; k < 8; ++k)
+          cr[t][k] = ring[(size_t)min(k0 + 4 * k + quarter, j1 - 1) * ld + 16 * (wave + 4 * t) + l16];
+      }
+  };
+  fetch(j0);
+#pragma unroll
+  for (int i = 0; i < NQ; ++i) {
+    const int x = tid + 256 * i, h = x / (ld / 4);
+    if (h < 16) *reinterpret_cast<f4*>(&qs[h * LD + (x - h * (ld / 4)) * 4]) = qr[i];
   }
   if (tid < 16) {
     ms[tid] = kNone;
     ls[tid] = 0.0f;
   }
-  const float* ring = a.ring + (size_t)b * a.ring_seq;
   f4 o[NT];
 #pragma unroll
   for (int t = 0; t < NT; ++t) o[t] = f4{0.f, 0.f, 0.f, 0.f};
-  const int tiles = a.kv_pad / 16;
   __syncthreads();
-  for (int k0 = j0; k0 < j1; k0 += 64) {
+  for (int k0 = j0; k0 < j1; k0 += kShareRows) {
     {
-      const float* row = ring + (size_t)min(k0 + 16 * wave + l16, j1 - 1) * ld + 4 * quarter;
       const float* q = qs + l16 * LD + 4 * quarter;
       f4 s0 = f4{0.f, 0.f, 0.f, 0.f}, s1 = s0;
-#pragma unroll 8
-      for (int d = 0; d < ld; d += 16) {
-        const f4 k4 = *reinterpret_cast<const f4*>(row + d), q4 = *reinterpret_cast<const f4*>(q + d);
-        s0 = __builtin_amdgcn_mfma_f32_16x16x4f32(k4.x, q4.x, s0, 0, 0, 0);
-        s1 = __builtin_amdgcn_mfma_f32_16x16x4f32(k4.y, q4.y, s1, 0, 0, 0);
-        s0 = __builtin_amdgcn_mfma_f32_16x16x4f32(k4.z, q4.z, s0, 0, 0, 0);
-        s1 = __builtin_amdgcn_mfma_f32_16x16x4f32(k4.w, q4.w, s1, 0, 0, 0);
-      }
-      s0 += s1;
-      const int key = 16 * wave + 4 * quarter;
 #pragma unroll
-      for (int v = 0; v < 4; ++v)
-        if (k0 + key + v >= j1) s0[v] = -INFINITY;
-      *reinterpret_cast<f4*>(&ps[l16][key]) = s0;
+      for (int s = 0; s < NS; ++s)
+        if (first + 2 * s < steps) {
+          const f4 q4 = *reinterpret_cast<const f4*>(q + 16 * (first + 2 * s));
+          s0 = __builtin_amdgcn_mfma_f32_16x16x4f32(kr[s].x, q4.x, s0, 0, 0, 0);
+          s1 = __builtin_amdgcn_mfma_f32_16x16x4f32(kr[s].y, q4.y, s1, 0, 0, 0);
+          s0 = __builtin_amdgcn_mfma_f32_16x16x4f32(kr[s].z, q4.z, s0, 0, 0, 0);
+          s1 = __builtin_amdgcn_mfma_f32_16x16x4f32(kr[s].w, q4.w, s1, 0, 0, 0);
+        }
+      *reinterpret_cast<f4*>(&ps[first][l16][rows16 + 4 * quarter]) = s0 + s1;
     }
     __syncthreads();
     {
-      // sixteen lanes to a head, four rows each
-      const int h = 4 * wave + quarter;
-      f4 s = *reinterpret_cast<const f4*>(&ps[h][4 * l16]);
-      float mx = fmaxf(fmaxf(s.x, s.y), fmaxf(s.z, s.w));
+      // sixteen lanes to a head, two rows each
+      const int h = 4 * wave + quarter, key = 2 * l16;
+      float s[2], mx = -INFINITY;
+#pragma unroll
+      for (int v = 0; v < 2; ++v) {
+        s[v] = k0 + key + v < j1 ? ps[0][h][key + v] + ps[1][h][key + v] : -INFINITY;
+        mx = fmaxf(mx, s[v]);
+      }
 #pragma unroll
       for (int off = 8; off > 0; off >>= 1) mx = fmaxf(mx, __shfl_xor(mx, off, 64));
       const float old = ms[h], now = fmaxf(old, mx);
       float sum = 0.0f;
 #pragma unroll
-      for (int v = 0; v < 4; ++v) {
+      for (int v = 0; v < 2; ++v) {
         s[v] = exp2f(s[v] - now);
         sum += s[v];
       }
 #pragma unroll
       for (int off = 8; off > 0; off >>= 1) sum += __shfl_xor(sum, off, 64);
-      *reinterpret_cast<f4*>(&ps[h][4 * l16]) = s;
+      ps[0][h][key] = s[0];
+      ps[0][h][key + 1] = s[1];
       if (l16 == 0) {
         const float f = exp2f(old - now);
         al[h] = f;
@@ -217,25 +272,23 @@ __global__ __launch_bounds__(256) void k_latent_attn(LatentDecode m, LatentAttn 
     __syncthreads();
     {
       f4 f;
-      float p[16];
+      float p[8];
 #pragma unroll
       for (int v = 0; v < 4; ++v) f[v] = al[4 * quarter + v];
 #pragma unroll
-      for (int k = 0; k < 16; ++k) p[k] = ps[l16][4 * k + quarter];
+      for (int k = 0; k < 8; ++k) p[k] = ps[0][l16][4 * k + quarter];
 #pragma unroll
-      for (int t = 0; t < NT; ++t) {
-        const int tile = wave + 4 * t;
-        if (tile >= tiles) break;
-        o[t] *= f;
-        float c[16];
+      for (int t = 0; t < NT; ++t)
+        if (wave + 4 * t < tiles) {
+          o[t] *= f;
 #pragma unroll
-        for (int k = 0; k < 16; ++k)
-          c[k] = ring[(size_t)min(k0 + 4 * k + quarter, j1 - 1) * ld + 16 * tile + l16];
-#pragma unroll
-        for (int k = 0; k < 16; ++k) o[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(p[k], c[k], o[t], 0, 0, 0);
-      }
+          for (int k = 0; k < 8; ++k) o[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(p[k], cr[t][k], o[t], 0, 0, 0);
+        }
     }
-    __syncthreads();
+    if (k0 + kShareRows < j1) {
+      fetch(k0 + kShareRows);
+      __syncthreads();
+    }
   }
 #pragma unroll
   for (int t = 0; t < NT; ++t) {
@@ -253,43 +306,66 @@ __global__ __launch_bounds__(256) void k_latent_attn(LatentDecode m, LatentAttn 
   }
 }
 
-// The shares' sums brought together with the sink, and 32 rows of W_uv.  Grid: x = head, y = rows of
-// W_uv, z = sequence.
+// The shares' sums brought together with the sink, and 32 rows of W_uv, for NB sequences.  Grid: x =
+// head, y = rows of W_uv, z = sequences.  NC: 256-column pieces of a latent.
+constexpr int kMaxShares = 64;
+template <int NB, int NC>
 __global__ __launch_bounds__(256) void k_latent_out(LatentDecode m, LatentAttn a) {
-  extern __shared__ __attribute__((aligned(16))) float lds[];  // [kv_pad], [splits]
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, h = blockIdx.x, b = blockIdx.z;
-  float* os = lds;
-  float* ws = lds + a.kv_pad;
-  const float* part = m.part + ((size_t)b * a.heads + h) * m.splits * (a.kv_pad + 2);
-  const size_t ps = a.kv_pad + 2;
-  const float sink = a.sink[h] * kLog2e;
-  float mx = sink, sum = 0.0f;
-  for (int s = 0; s < m.splits; ++s) mx = fmaxf(mx, part[s * ps + a.kv_pad]);
-  for (int s = 0; s < m.splits; ++s) sum += part[s * ps + a.kv_pad + 1] * exp2f(part[s * ps + a.kv_pad] - mx);
-  const float inv = 1.0f / (sum + exp2f(sink - mx));
-  for (int s = tid; s < m.splits; s += 256)
-    ws[s] = part[s * ps + a.kv_pad + 1] > 0.0f ? exp2f(part[s * ps + a.kv_pad] - mx) * inv : 0.0f;
+  __shared__ __attribute__((aligned(16))) float os[NB][256 * NC];
+  __shared__ float ws[NB][kMaxShares];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, h = blockIdx.x;
+  const int b0 = blockIdx.z * NB, nb = min(NB, m.nseq - b0), e0 = blockIdx.y * 32 + wave;
+  const size_t ps = a.kv_pad + 2, seq = (size_t)a.heads * m.splits * ps;
+  const float* part = m.part + ((size_t)b0 * a.heads + h) * m.splits * ps;
+  // sequence `wave` (NB 1: every wavefront the same): a share per lane
+  if (wave < NB) {
+    const float* p = part + min(wave, nb - 1) * seq + min(lane, m.splits - 1) * ps + a.kv_pad;
+    const float sink = a.sink[h] * kLog2e;
+    const float mx = lane < m.splits ? p[0] : kNone, l = lane < m.splits ? p[1] : 0.0f;
+    float top = fmaxf(mx, sink);
+#pragma unroll
+    for (int off = 32; off > 0; off >>= 1) top = fmaxf(top, __shfl_xor(top, off, 64));
+    const float f = l > 0.0f ? exp2f(mx - top) : 0.0f;
+    const float sum = wave_sum(l * f) + exp2f(sink - top);
+    ws[wave][lane] = f / sum;
+  }
+  f4 w[8][NC];
+#pragma unroll
+  for (int r = 0; r < 8; ++r)
+#pragma unroll
+    for (int c = 0; c < NC; ++c)
+      w[r][c] = load_w4(a.up_w, a.w_bf16,
+                        ((size_t)a.v_row + h * a.vdim + min(e0 + 4 * r, a.vdim - 1)) * a.kv_pad + min(4 * lane + 256 * c, a.kv_pad - 4));
   __syncthreads();
-  for (int i = tid; i < a.kv_pad; i += 256) {
-    float o = 0.0f;
-    for (int s = 0; s < m.splits; ++s) {
-      const float w = ws[s];
-      if (w != 0.0f) o += w * part[s * ps + i];  // (a share without rows has left its sums unwritten)
+  for (int i = tid; i < 256 * NC; i += 256) {
+    const int at = min(i, a.kv_pad - 1);
+#pragma unroll
+    for (int b = 0; b < NB; ++b) {
+      const float* p = part + min(b, nb - 1) * seq + at;
+      float o = 0.0f;
+#pragma unroll 8
+      for (int s = 0; s < m.splits; ++s) {
+        const float f = ws[b][s], x = p[s * ps];
+        o += f != 0.0f ? f * x : 0.0f;  // (a share without rows has left its sums unwritten)
+      }
+      os[b][i] = i < a.kv_pad ? o : 0.0f;
     }
-    os[i] = o;
   }
   __syncthreads();
-  const int e1 = min(a.vdim, (int)blockIdx.y * 32 + 32);
-  for (int e = blockIdx.y * 32 + wave; e < e1; e += 4) {
-    const size_t at = ((size_t)a.v_row + h * a.vdim + e) * a.kv_pad;
-    float s = 0.0f;
-#pragma unroll 4
-    for (int i = 4 * lane; i < a.kv_pad; i += 256) {
-      const f4 w = load_w4(a.up_w, a.w_bf16, at + i), o = *reinterpret_cast<const f4*>(os + i);
-      s += (w.x * o.x + w.y * o.y) + (w.z * o.z + w.w * o.w);
+#pragma unroll
+  for (int b = 0; b < NB; ++b) {
+    if (b >= nb) break;
+    f4 o[NC];
+#pragma unroll
+    for (int c = 0; c < NC; ++c) o[c] = *reinterpret_cast<const f4*>(&os[b][4 * lane + 256 * c]);
+#pragma unroll
+    for (int r = 0; r < 8; ++r) {
+      float s = 0.0f;
+#pragma unroll
+      for (int c = 0; c < NC; ++c) s += (w[r][c].x * o[c].x + w[r][c].y * o[c].y) + (w[r][c].z * o[c].z + w[r][c].w * o[c].w);
+      s = wave_sum(s);
+      if (lane == 0 && e0 + 4 * r < a.vdim) m.out[(size_t)(b0 + b) * m.ld_out + a.out_col + h * a.vdim + e0 + 4 * r] = s;
     }
-    s = wave_sum(s);
-    if (lane == 0) m.out[(size_t)b * m.ld_out + a.out_col + h * a.vdim + e] = s;
   }
 }
 
@@ -549,14 +625,17 @@ hipError_t launch_attn_rows(const MixRows& r, const LatentAttn& a, const LatentR
 
 }  // namespace
 
-// Shares of the window: 64 rows each, 64 shares at most.
-int latent_decode_splits(const LatentAttn& a) { return std::min(64, (a.window + 63) / 64); }
+// Shares of the window: 32 rows each, 64 shares at most.
+int latent_decode_splits(const LatentAttn& a) { return std::min(kMaxShares, (a.window + kShareRows - 1) / kShareRows); }
 
 hipError_t launch_latent_decode(const LatentDecode& m, const LatentAttn& a, hipStream_t s) {
-  if (a.kv_pad > kLatentMaxRank || a.dim > kMixMaxDim || a.rot_dim > kMixMaxDim || a.vdim > kMixMaxDim || a.kv_pad % 32 != 0 ||
-      a.ld % 16 != 0 || m.splits != latent_decode_splits(a))
+  if (a.kv_pad > kLatentMaxRank || a.dim + a.rot_dim > kMixMaxDim || a.vdim > kMixMaxDim || a.kv_pad % 32 != 0 ||
+      a.ld % 16 != 0 || a.ld > a.kv_pad + kMixMaxDim || m.splits != latent_decode_splits(a))
     return hipErrorInvalidValue;
-  hipLaunchKernelGGL(k_latent_query, dim3(a.heads + 1, (a.kv_pad + 127) / 128, m.nseq), dim3(256), 0, s, m, a);
+  const int groups = (m.nseq + 3) / 4;  // batches: four sequences share what a block reads of the weights
+  const dim3 qgrid(a.heads + 1, (a.kv_pad + 127) / 128, m.nseq == 1 ? 1 : groups);
+  if (m.nseq == 1) hipLaunchKernelGGL(k_latent_query<1>, qgrid, dim3(256), 0, s, m, a);
+  else hipLaunchKernelGGL(k_latent_query<4>, qgrid, dim3(256), 0, s, m, a);
   const dim3 grid(m.splits, (a.heads + 15) / 16, m.nseq);
   const size_t lds = 16 * (size_t)(a.ld + 4) * sizeof(float);
   const void* kernel = a.kv_pad <= 256   ? reinterpret_cast<const void*>(&k_latent_attn<4>)
@@ -569,8 +648,18 @@ hipError_t launch_latent_decode(const LatentDecode& m, const LatentAttn& a, hipS
   if (a.kv_pad <= 256) hipLaunchKernelGGL(k_latent_attn<4>, grid, dim3(256), lds, s, m, a);
   else if (a.kv_pad <= 512) hipLaunchKernelGGL(k_latent_attn<8>, grid, dim3(256), lds, s, m, a);
   else hipLaunchKernelGGL(k_latent_attn<16>, grid, dim3(256), lds, s, m, a);
-  hipLaunchKernelGGL(k_latent_out, dim3(a.heads, (a.vdim + 31) / 32, m.nseq), dim3(256),
-                     (a.kv_pad + m.splits) * sizeof(float), s, m, a);
+  const dim3 ogrid(a.heads, (a.vdim + 31) / 32, m.nseq == 1 ? 1 : groups);
+#define PG_OUT(C)                                                                              \
+  if (m.nseq == 1) hipLaunchKernelGGL((k_latent_out<1, C>), ogrid, dim3(256), 0, s, m, a);     \
+  else hipLaunchKernelGGL((k_latent_out<4, C>), ogrid, dim3(256), 0, s, m, a);
+  if (a.kv_pad <= 256) {
+    PG_OUT(1)
+  } else if (a.kv_pad <= 512) {
+    PG_OUT(2)
+  } else {
+    PG_OUT(4)
+  }
+#undef PG_OUT
   return hipGetLastError();
 }
 

@@ -241,17 +241,32 @@ hipError_t launch_latent_attn_rows(const MixRows& r, const LatentAttn& a, const 
 // down[expert][width_pad][ff_pad].
 constexpr int kMoeMaxExperts = 1024;
 constexpr int kMoeMaxTop = 64;
+constexpr int kMoeMaxWidth = 16000;  // of the model and of an expert (rows staged in LDS)
 struct Moe {
   int experts, experts_pad, top;  // experts_pad: columns of a row of router logits
   int ff, ff_pad;
   const void *gate_up, *down;
   int w_bf16;
 };
-// A few rows: every (row, expert) pair reads its expert's weights.  x, out: [rows][width_pad]; logits:
-// [rows][experts_pad]; act: [rows * top][ff_pad].
-hipError_t launch_moe_few(const Moe& m, const float* x, const float* logits, float* act, float* out, int rows,
-                          int width_pad, hipStream_t s);
-// Many rows: pairs are sorted by expert into slots, each expert's padded to whole tiles of tile_rows.
+// One row.  x, out: [width_pad]; act: [top][ff_pad]; expert, weight: [top], filled by the launch.
+// logits: the router's, [experts_pad]; or null and router, [experts_pad][width_pad], and the row to be
+// brought up to date: x + add / rms(add) * add_gain (add may be null), written to x_out, which is
+// not x.
+struct MoeRow {
+  const float *x, *logits;
+  const void* router;
+  const float *add, *add_gain;
+  float* x_out;
+  int width, width_pad;
+  float eps;
+  float *act, *out;
+  int* expert;
+  float* weight;
+};
+// Whether a router is small enough to be multiplied by every block again.
+bool moe_router_fits(const Moe& m, int width_pad);
+hipError_t launch_moe_row(const Moe& m, const MoeRow& r, hipStream_t s);
+// Several rows: pairs are sorted by expert into slots, each expert's padded to whole tiles of tile_rows.
 struct MoeRoute {
   int tile_rows, max_slots;  // max_slots: moe_max_slots
   int* count;      // [experts]

@@ -277,23 +277,36 @@ __device__ __forceinline__ void conv_channels(const ShortConv& c, const float* y
     if (keep[n]) ring[(size_t)slot * c.channels + ch[n]] = cur[n];
 }
 
-// dst[i] = row row0 + i of a low-rank projection, i < n: eight lanes to a row.
+// dst[i] = row row0 + i of a low-rank projection, i < n: eight lanes to a row, four rows at a time.
 template <int NT>
 __device__ __forceinline__ void low_rank_rows(const LowRank& p, const float* y, int row0, int n, float* dst) {
+  constexpr int R = 4, STEP = NT / 8;
   const int sub = threadIdx.x & 7;
   const float* x = y + p.col;
-  for (int i = threadIdx.x >> 3; i < n; i += NT / 8) {
-    const size_t at = (size_t)(row0 + i) * p.rank;
-    float s = 0.0f;
+  for (int i0 = threadIdx.x >> 3; i0 - (int)(threadIdx.x >> 3) < n; i0 += R * STEP) {
+    float s[R];
+    size_t at[R];
+#pragma unroll
+    for (int q = 0; q < R; ++q) {
+      s[q] = 0.0f;
+      at[q] = (size_t)(row0 + min(i0 + q * STEP, n - 1)) * p.rank;
+    }
+#pragma unroll 4
     for (int k = 4 * sub; k < p.rank; k += 32) {
-      const f4 w = p.w_bf16 ? bf16x4(static_cast<const unsigned short*>(p.w) + at + k)
-                            : *reinterpret_cast<const f4*>(static_cast<const float*>(p.w) + at + k);
       const f4 v = *reinterpret_cast<const f4*>(x + k);
-      s += (w.x * v.x + w.y * v.y) + (w.z * v.z + w.w * v.w);
+#pragma unroll
+      for (int q = 0; q < R; ++q) {
+        const f4 w = p.w_bf16 ? bf16x4(static_cast<const unsigned short*>(p.w) + at[q] + k)
+                              : *reinterpret_cast<const f4*>(static_cast<const float*>(p.w) + at[q] + k);
+        s[q] += (w.x * v.x + w.y * v.y) + (w.z * v.z + w.w * v.w);
+      }
     }
 #pragma unroll
-    for (int off = 4; off > 0; off >>= 1) s += __shfl_xor(s, off, 64);
-    if (sub == 0) dst[i] = s;
+    for (int q = 0; q < R; ++q) {
+#pragma unroll
+      for (int off = 4; off > 0; off >>= 1) s[q] += __shfl_xor(s[q], off, 64);
+      if (sub == 0 && i0 + q * STEP < n) dst[i0 + q * STEP] = s[q];
+    }
   }
 }
 
@@ -1516,13 +1529,17 @@ __global__ __launch_bounds__(256) void k_add_norm_rows(float* dst, const float* 
     for (int k = 0; k < top; ++k) s += weight[row * top + k] * src[(size_t)slot[row * top + k] * ld + i];
     return s;
   };
-  float keep[PER], ss = 0.0f;
+  float keep[PER], old[PER], g[PER], ss = 0.0f;
 #pragma unroll
   for (int p = 0; p < PER; ++p) {
     const int i = threadIdx.x + 256 * p;
-    keep[p] = i < cols ? value(i) : 0.0f;
-    ss += keep[p] * keep[p];
+    const bool in = i < cols;
+    old[p] = in ? x[i] : 0.0f;
+    g[p] = in ? gain[i] : 0.0f;
+    keep[p] = in ? value(i) : 0.0f;
   }
+#pragma unroll
+  for (int p = 0; p < PER; ++p) ss += keep[p] * keep[p];
   for (int i = threadIdx.x + 256 * PER; i < cols; i += 256) {
     const float v = value(i);
     ss += v * v;
@@ -1531,33 +1548,59 @@ __global__ __launch_bounds__(256) void k_add_norm_rows(float* dst, const float* 
 #pragma unroll
   for (int p = 0; p < PER; ++p) {
     const int i = threadIdx.x + 256 * p;
-    if (i < cols) x[i] += keep[p] * k * gain[i];
+    if (i < cols) x[i] = old[p] + keep[p] * k * g[p];
   }
   for (int i = threadIdx.x + 256 * PER; i < cols; i += 256) x[i] += value(i) * k * gain[i];
 }
 
-// One wavefront per part of a row in turn.
+// Up to four parts of rows of up to 4096 columns: the row is kept in registers.  Otherwise a
+// wavefront takes a part at a time.
 __global__ __launch_bounds__(256) void k_group_rms_rows(const float* src, int ld_src, float* dst, int ld_dst, int cols,
                                                         int groups, const float* gain, float eps, const int* rows_at) {
+  __shared__ float red[4];
+  constexpr int PER = 16;
   const size_t row = rows_at ? rows_at[blockIdx.x] : blockIdx.x;
   const float* x = src + row * ld_src;
   float* y = dst + (size_t)blockIdx.x * ld_dst;
-  const int n = cols / groups, lane = threadIdx.x & 63;
-  if (groups == 1) {
-    __shared__ float red[4];
+  const int n = cols / groups, tid = threadIdx.x, lane = tid & 63;
+  if (groups <= 4 && cols <= 256 * PER) {
+    float v[PER], g[PER], ss[4] = {0.f, 0.f, 0.f, 0.f}, k[4];
+#pragma unroll
+    for (int p = 0; p < PER; ++p) {
+      const int i = tid + 256 * p;
+      v[p] = i < cols ? x[i] : 0.0f;
+      g[p] = i < cols ? gain[i] : 0.0f;
+    }
+#pragma unroll
+    for (int p = 0; p < PER; ++p) {
+      const int i = tid + 256 * p, part = (i >= n) + (i >= 2 * n) + (i >= 3 * n);
+#pragma unroll
+      for (int q = 0; q < 4; ++q) ss[q] += q == part ? v[p] * v[p] : 0.0f;
+    }
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      k[q] = 0.0f;
+      if (q < groups) k[q] = 1.0f / sqrtf(block_sum(ss[q], red) / (float)n + eps);
+    }
+#pragma unroll
+    for (int p = 0; p < PER; ++p) {
+      const int i = tid + 256 * p, part = (i >= n) + (i >= 2 * n) + (i >= 3 * n);
+      if (i < cols) y[i] = v[p] * (part == 0 ? k[0] : part == 1 ? k[1] : part == 2 ? k[2] : k[3]) * g[p];
+    }
+  } else if (groups == 1) {
     float ss = 0.0f;
-    for (int i = threadIdx.x; i < n; i += 256) ss += x[i] * x[i];
+    for (int i = tid; i < n; i += 256) ss += x[i] * x[i];
     const float k = 1.0f / sqrtf(block_sum(ss, red) / (float)n + eps);
-    for (int i = threadIdx.x; i < n; i += 256) y[i] = x[i] * k * gain[i];
+    for (int i = tid; i < n; i += 256) y[i] = x[i] * k * gain[i];
   } else {
-    for (int g = threadIdx.x >> 6; g < groups; g += 4) {
+    for (int g = tid >> 6; g < groups; g += 4) {
       float ss = 0.0f;
       for (int i = lane; i < n; i += 64) ss += x[g * n + i] * x[g * n + i];
       const float k = 1.0f / sqrtf(wave_sum(ss) / (float)n + eps);
       for (int i = lane; i < n; i += 64) y[g * n + i] = x[g * n + i] * k * gain[g * n + i];
     }
   }
-  for (int i = cols + threadIdx.x; i < ld_dst; i += 256) y[i] = 0.0f;
+  for (int i = cols + tid; i < ld_dst; i += 256) y[i] = 0.0f;
 }
 
 __global__ __launch_bounds__(256) void k_begin_step(float* x, const void* table, int table_bf16, const uint32_t* ids,

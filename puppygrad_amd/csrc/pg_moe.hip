@@ -79,90 +79,169 @@ __device__ __forceinline__ void choose_any(const float* z, int experts, int top,
   else choose_experts<kPerLane>(z, experts, top, each);
 }
 
-// A row of a matrix of f32 or bf16 against a vector in LDS, over the wavefront (n: a multiple of 32).
+// Sixteen bytes of a row of a matrix of f32 or bf16 against the values in LDS that they meet.
 template <bool BF16>
-__device__ __forceinline__ float row_dot(const void* w, size_t at, const float* x, int n) {
-  const int lane = threadIdx.x & 63;
-  float s = 0.0f;
-  if (BF16) {
-    const u4v* p = reinterpret_cast<const u4v*>(static_cast<const unsigned short*>(w) + at);
-#pragma unroll 4
-    for (int j = lane; j < n / 8; j += 64) {
-      const u4v u = __builtin_nontemporal_load(p + j);
-      const f4 a = *reinterpret_cast<const f4*>(x + 8 * j), b = *reinterpret_cast<const f4*>(x + 8 * j + 4);
-      s += __uint_as_float(u.x << 16) * a.x + __uint_as_float(u.x & 0xffff0000u) * a.y + __uint_as_float(u.y << 16) * a.z +
-           __uint_as_float(u.y & 0xffff0000u) * a.w + __uint_as_float(u.z << 16) * b.x +
-           __uint_as_float(u.z & 0xffff0000u) * b.y + __uint_as_float(u.w << 16) * b.z + __uint_as_float(u.w & 0xffff0000u) * b.w;
+__device__ __forceinline__ float chunk_dot(const u4v& u, const float* x) {
+  const f4 a = *reinterpret_cast<const f4*>(x);
+  if (!BF16)
+    return __uint_as_float(u.x) * a.x + __uint_as_float(u.y) * a.y + __uint_as_float(u.z) * a.z + __uint_as_float(u.w) * a.w;
+  const f4 b = *reinterpret_cast<const f4*>(x + 4);
+  return __uint_as_float(u.x << 16) * a.x + __uint_as_float(u.x & 0xffff0000u) * a.y + __uint_as_float(u.y << 16) * a.z +
+         __uint_as_float(u.y & 0xffff0000u) * a.w + __uint_as_float(u.z << 16) * b.x +
+         __uint_as_float(u.z & 0xffff0000u) * b.y + __uint_as_float(u.w << 16) * b.z + __uint_as_float(u.w & 0xffff0000u) * b.w;
+}
+
+constexpr int kRouterRows = 16;  // rows of a router that a wavefront multiplies at most
+
+// act[k][j] = silu(gate j . x) * (up j . x) of the row's k-th expert.  Every block brings x up to date
+// and routes the row for itself (a wavefront: every fourth row of the router); block (0, k) lists
+// the choice.  Grid: x = 4 RJ values of j, y = k.
+template <bool BF16, int RJ>
+__global__ __launch_bounds__(256) void k_moe_act(Moe m, MoeRow r) {
+  extern __shared__ __attribute__((aligned(16))) float xs[];
+  __shared__ float zs[4 * kRouterRows], red[4];
+  __shared__ int expert;
+  constexpr int PER = BF16 ? 8 : 4, IN = 4;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, k = blockIdx.y;
+  const int K = r.width_pad, n = K / PER, n4 = K / 4;
+  f4 vx[IN], va[IN], vg[IN];
+#pragma unroll
+  for (int p = 0; p < IN; ++p) {
+    vx[p] = va[p] = vg[p] = f4{0.f, 0.f, 0.f, 0.f};
+    const int i = tid + 256 * p;
+    if (i < n4) {
+      vx[p] = reinterpret_cast<const f4*>(r.x)[i];
+      if (r.add) {
+        va[p] = reinterpret_cast<const f4*>(r.add)[i];
+        vg[p] = reinterpret_cast<const f4*>(r.add_gain)[i];
+      }
+    }
+  }
+  if (r.add) {
+    float ss = 0.0f;
+#pragma unroll
+    for (int p = 0; p < IN; ++p) ss += (va[p].x * va[p].x + va[p].y * va[p].y) + (va[p].z * va[p].z + va[p].w * va[p].w);
+    for (int i = tid + 256 * IN; i < n4; i += 256) {
+      const f4 v = reinterpret_cast<const f4*>(r.add)[i];
+      ss += (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w);
+    }
+    ss = wave_sum(ss);
+    if (lane == 0) red[wave] = ss;
+    __syncthreads();
+    const float f = 1.0f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / (float)r.width + r.eps);
+#pragma unroll
+    for (int p = 0; p < IN; ++p) vx[p] += va[p] * f * vg[p];
+    for (int i = tid + 256 * IN; i < n4; i += 256) {
+      const f4 v = reinterpret_cast<const f4*>(r.x)[i] +
+                   reinterpret_cast<const f4*>(r.add)[i] * f * reinterpret_cast<const f4*>(r.add_gain)[i];
+      reinterpret_cast<f4*>(xs)[i] = v;
+      if (blockIdx.x == 0 && k == 0) reinterpret_cast<f4*>(r.x_out)[i] = v;
     }
   } else {
-    const f4* p = reinterpret_cast<const f4*>(static_cast<const float*>(w) + at);
-#pragma unroll 4
-    for (int j = lane; j < n / 4; j += 64) {
-      const f4 u = __builtin_nontemporal_load(p + j);
-      const f4 a = *reinterpret_cast<const f4*>(x + 4 * j);
-      s += u.x * a.x + u.y * a.y + u.z * a.z + u.w * a.w;
+    for (int i = tid + 256 * IN; i < n4; i += 256) reinterpret_cast<f4*>(xs)[i] = reinterpret_cast<const f4*>(r.x)[i];
+  }
+#pragma unroll
+  for (int p = 0; p < IN; ++p) {
+    const int i = tid + 256 * p;
+    if (i < n4) {
+      reinterpret_cast<f4*>(xs)[i] = vx[p];
+      if (r.add && blockIdx.x == 0 && k == 0) reinterpret_cast<f4*>(r.x_out)[i] = vx[p];
     }
   }
-  return s;
-}
-
-// act[row * top + k][j] = silu(gate j . x) * (up j . x) of the row's k-th expert.  Every block routes
-// its row again: the logits are few.  Grid: x = 4 values of j each, y = (row, k).
-template <bool BF16>
-__global__ __launch_bounds__(256) void k_moe_act(Moe m, const float* x, const float* logits, float* act, int width) {
-  extern __shared__ __attribute__((aligned(16))) float xs[];
-  __shared__ int expert;
-  const int tid = threadIdx.x, wave = tid >> 6;
-  const int row = blockIdx.y / m.top, k = blockIdx.y - row * m.top;
-  if (wave == 0)
-    choose_any(logits + (size_t)row * m.experts_pad, m.experts, k + 1, [&](int i, int e, float) {
-      if (i == k && tid == 0) expert = e;
-    });
-  for (int i = tid; i < width / 4; i += 256)
-    reinterpret_cast<f4*>(xs)[i] = reinterpret_cast<const f4*>(x + (size_t)row * width)[i];
   __syncthreads();
-  const int j = blockIdx.x * 4 + wave;
-  if (j >= m.ff_pad) return;
-  const size_t at = ((size_t)expert * 2 * m.ff_pad + 2 * j) * width;
-  float g = row_dot<BF16>(m.gate_up, at, xs, width), u = row_dot<BF16>(m.gate_up, at + width, xs, width);
-  g = wave_sum(g);
-  u = wave_sum(u);
-  if ((tid & 63) == 0) act[(size_t)blockIdx.y * m.ff_pad + j] = g / (1.0f + expf(-g)) * u;
-}
-
-// out[row][c] = sum over k of weight k * (down row c of expert k . act).  Grid: x = 4 values of c each,
-// y = row.  The activations of as many experts as fit lie in LDS at a time.
-template <bool BF16>
-__global__ __launch_bounds__(256) void k_moe_down(Moe m, const float* logits, const float* act, float* out, int width,
-                                                  int at_once) {
-  extern __shared__ __attribute__((aligned(16))) float as[];
-  __shared__ int expert[kMoeMaxTop];
-  __shared__ float weight[kMoeMaxTop];
-  const int tid = threadIdx.x, wave = tid >> 6, row = blockIdx.y, c = blockIdx.x * 4 + wave;
+  const float* z = r.logits;
+  if (r.router) {
+    const u4v* w = static_cast<const u4v*>(r.router);
+    float s[kRouterRows];
+#pragma unroll
+    for (int e = 0; e < kRouterRows; ++e) s[e] = 0.0f;
+    for (int j = lane; j < n; j += 64) {
+      u4v u[kRouterRows];
+#pragma unroll
+      for (int e = 0; e < kRouterRows; ++e)
+        if (wave + 4 * e < m.experts) u[e] = w[(size_t)(wave + 4 * e) * n + j];
+#pragma unroll
+      for (int e = 0; e < kRouterRows; ++e)
+        if (wave + 4 * e < m.experts) s[e] += chunk_dot<BF16>(u[e], xs + PER * j);
+    }
+#pragma unroll
+    for (int e = 0; e < kRouterRows; ++e)
+      if (wave + 4 * e < m.experts) {
+        s[e] = wave_sum(s[e]);
+        if (lane == 0) zs[wave + 4 * e] = s[e];
+      }
+    __syncthreads();
+    z = zs;
+  }
   if (wave == 0)
-    choose_any(logits + (size_t)row * m.experts_pad, m.experts, m.top, [&](int i, int e, float w) {
-      if (tid == 0) {
-        expert[i] = e;
-        weight[i] = w;
+    choose_any(z, m.experts, k + 1, [&](int i, int e, float w) {
+      if (i == k && tid == 0) {
+        expert = e;
+        if (blockIdx.x == 0) {
+          r.expert[k] = e;
+          r.weight[k] = w;
+        }
       }
     });
-  float s = 0.0f;
-  for (int k0 = 0; k0 < m.top; k0 += at_once) {
-    const int nk = min(at_once, m.top - k0);
-    __syncthreads();
-    const f4* src = reinterpret_cast<const f4*>(act + ((size_t)row * m.top + k0) * m.ff_pad);
-    for (int i = tid; i < nk * m.ff_pad / 4; i += 256) reinterpret_cast<f4*>(as)[i] = src[i];
-    __syncthreads();
-    if (c < width)
-      for (int k = 0; k < nk; ++k)
-        s += weight[k0 + k] *
-             row_dot<BF16>(m.down, ((size_t)expert[k0 + k] * width + c) * m.ff_pad, as + k * m.ff_pad, m.ff_pad);
+  __syncthreads();
+  const int j0 = (blockIdx.x * 4 + wave) * RJ;
+  if (j0 >= m.ff_pad) return;
+  // rows 2 j and 2 j + 1, RJ values of j (ff_pad is a multiple of 32)
+  const u4v* w = static_cast<const u4v*>(m.gate_up) + ((size_t)expert * 2 * m.ff_pad + 2 * j0) * n;
+  float s[2 * RJ];
+#pragma unroll
+  for (int q = 0; q < 2 * RJ; ++q) s[q] = 0.0f;
+#pragma unroll 2
+  for (int i = lane; i < n; i += 64) {
+    u4v u[2 * RJ];
+#pragma unroll
+    for (int q = 0; q < 2 * RJ; ++q) u[q] = __builtin_nontemporal_load(w + (size_t)q * n + i);
+#pragma unroll
+    for (int q = 0; q < 2 * RJ; ++q) s[q] += chunk_dot<BF16>(u[q], xs + PER * i);
   }
-  s = wave_sum(s);
-  if (c < width && (tid & 63) == 0) out[(size_t)row * width + c] = s;
+#pragma unroll
+  for (int q = 0; q < 2 * RJ; ++q) s[q] = wave_sum(s[q]);
+  if (lane == 0)
+#pragma unroll
+    for (int q = 0; q < RJ; ++q)
+      r.act[(size_t)k * m.ff_pad + j0 + q] = s[2 * q] / (1.0f + expf(-s[2 * q])) * s[2 * q + 1];
 }
 
-// ---- many rows: pairs sorted by expert ----
+// out[c] = sum over k of weight k * (down row c of expert k . act): one dot product over the experts'
+// rows one after the other, against the weighted activations in LDS (as many experts as fit at a
+// time).  Grid: x = 4 values of c.
+template <bool BF16>
+__global__ __launch_bounds__(256) void k_moe_down(Moe m, MoeRow r, int at_once) {
+  extern __shared__ __attribute__((aligned(16))) float as[];
+  constexpr int PER = BF16 ? 8 : 4, PRE = 8;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c = min((int)blockIdx.x * 4 + wave, r.width_pad - 1);
+  const int n = m.ff_pad / PER, n4 = m.ff_pad / 4;
+  const u4v* down = static_cast<const u4v*>(m.down);
+  float s = 0.0f;
+  for (int k0 = 0; k0 < m.top; k0 += at_once) {
+    const int nk = min(at_once, m.top - k0), chunks = nk * n;
+    auto load = [&](int j) {
+      const int k = j / n;
+      return __builtin_nontemporal_load(down + ((size_t)r.expert[k0 + k] * r.width_pad + c) * n + (j - k * n));
+    };
+    u4v pre[PRE];  // the weights' first chunks are on their way while the activations are staged
+#pragma unroll
+    for (int p = 0; p < PRE; ++p) pre[p] = load(min(lane + 64 * p, chunks - 1));
+    __syncthreads();
+    const f4* src = reinterpret_cast<const f4*>(r.act + (size_t)k0 * m.ff_pad);
+    for (int i = tid; i < nk * n4; i += 256) reinterpret_cast<f4*>(as)[i] = src[i] * r.weight[k0 + i / n4];
+    __syncthreads();
+#pragma unroll
+    for (int p = 0; p < PRE; ++p)
+      if (lane + 64 * p < chunks) s += chunk_dot<BF16>(pre[p], as + PER * (lane + 64 * p));
+#pragma unroll 4
+    for (int j = lane + 64 * PRE; j < chunks; j += 64) s += chunk_dot<BF16>(load(j), as + PER * j);
+  }
+  s = wave_sum(s);
+  if (lane == 0) r.out[c] = s;
+}
+
+// ---- several rows: pairs sorted by expert ----
 constexpr int kRouteRows = 16;  // rows of a block
 
 __global__ __launch_bounds__(256) void k_moe_clear(MoeRoute r, int experts, int slots) {
@@ -200,26 +279,30 @@ __global__ __launch_bounds__(256) void k_moe_choose(Moe m, MoeRoute r, const flo
   }
 }
 
+// One wavefront: running sums of the padded counts.
+__device__ void first_slots(const Moe& m, int tile_rows, const int* count, int* first) {
+  const int lane = threadIdx.x & 63;
+  int at = 0;
+  for (int e0 = 0; e0 < m.experts; e0 += 64) {
+    const int e = e0 + lane;
+    const int n = e < m.experts ? (count[e] + tile_rows - 1) / tile_rows * tile_rows : 0;
+    int s = n;
+#pragma unroll
+    for (int off = 1; off < 64; off <<= 1) {
+      const int up = __shfl_up(s, off, 64);
+      if (lane >= off) s += up;
+    }
+    if (e < m.experts) first[e] = at + s - n;
+    at += __shfl(s, 63, 64);
+  }
+  if (lane == 0) first[m.experts] = at;
+}
+
 // First slot of every expert, the experts of the tiles, the slots of this block's pairs.
 __global__ __launch_bounds__(256) void k_moe_place(Moe m, MoeRoute r, int pairs) {
   __shared__ int first[kMoeMaxExperts + 1];
   const int tid = threadIdx.x;
-  if (tid < 64) {  // one wavefront: running sums of the padded counts
-    int at = 0;
-    for (int e0 = 0; e0 < m.experts; e0 += 64) {
-      const int e = e0 + tid;
-      const int n = e < m.experts ? (r.count[e] + r.tile_rows - 1) / r.tile_rows * r.tile_rows : 0;
-      int s = n;
-#pragma unroll
-      for (int off = 1; off < 64; off <<= 1) {
-        const int up = __shfl_up(s, off, 64);
-        if (tid >= off) s += up;
-      }
-      if (e < m.experts) first[e] = at + s - n;
-      at += __shfl(s, 63, 64);
-    }
-    if (tid == 0) first[m.experts] = at;
-  }
+  if (tid < 64) first_slots(m, r.tile_rows, r.count, first);
   __syncthreads();
   if (blockIdx.x == 0)
     for (int e = tid; e < m.experts; e += 256)
@@ -231,23 +314,57 @@ __global__ __launch_bounds__(256) void k_moe_place(Moe m, MoeRoute r, int pairs)
   r.slot_row[s] = p / m.top;
 }
 
+// All of it in one block, for a few rows.
+constexpr int kRouteSmallRows = 128;
+__global__ __launch_bounds__(1024) void k_moe_route_small(Moe m, MoeRoute r, const float* logits, int rows) {
+  __shared__ int count[kMoeMaxExperts], first[kMoeMaxExperts + 1];
+  const int tid = threadIdx.x, wave = tid >> 6;
+  for (int i = tid; i < m.experts; i += 1024) count[i] = 0;
+  for (int i = tid; i < r.max_slots; i += 1024) r.slot_row[i] = -1;
+  for (int i = tid; i < r.max_slots / r.tile_rows; i += 1024) r.tile[i] = -1;
+  __syncthreads();
+  for (int row = wave; row < rows; row += 16)
+    choose_any(logits + (size_t)row * m.experts_pad, m.experts, m.top, [&](int k, int e, float w) {
+      if ((tid & 63) == 0) {
+        const size_t p = (size_t)row * m.top + k;
+        r.expert[p] = e;
+        r.weight[p] = w;
+        r.rank[p] = atomicAdd(&count[e], 1);
+      }
+    });
+  __syncthreads();
+  if (tid < 64) first_slots(m, r.tile_rows, count, first);
+  __syncthreads();
+  for (int e = tid; e < m.experts; e += 1024)
+    for (int t = first[e] / r.tile_rows; t < first[e + 1] / r.tile_rows; ++t) r.tile[t] = e;
+  for (int p = tid; p < rows * m.top; p += 1024) {
+    const int s = first[r.expert[p]] + r.rank[p];
+    r.slot[p] = s;
+    r.slot_row[s] = p / m.top;
+  }
+}
+
 }  // namespace
 
-hipError_t launch_moe_few(const Moe& m, const float* x, const float* logits, float* act, float* out, int rows,
-                          int width_pad, hipStream_t s) {
-  constexpr int kLds = 16000;  // floats of activations at once
-  if (m.experts > kMoeMaxExperts || m.top > kMoeMaxTop || m.top > m.experts || m.ff_pad > kLds || width_pad > 16320 ||
-      m.ff_pad % 32 != 0 || width_pad % 32 != 0 || rows < 1 || (long)rows * m.top > 65535)
+bool moe_router_fits(const Moe& m, int width_pad) { return m.experts <= 4 * kRouterRows && (long)m.experts * width_pad <= 65536; }
+
+hipError_t launch_moe_row(const Moe& m, const MoeRow& r, hipStream_t s) {
+  if (m.experts > kMoeMaxExperts || m.top > kMoeMaxTop || m.top > m.experts || m.ff_pad > kMoeMaxWidth || r.width_pad > kMoeMaxWidth ||
+      m.ff_pad % 32 != 0 || r.width_pad % 32 != 0 || (r.logits == nullptr) == (r.router == nullptr) ||
+      (r.router && !moe_router_fits(m, r.width_pad)))
     return hipErrorInvalidValue;
-  const dim3 up((m.ff_pad + 3) / 4, rows * m.top), down((width_pad + 3) / 4, rows);
-  const int at_once = std::min(m.top, kLds / m.ff_pad);
-  const size_t xl = (size_t)width_pad * sizeof(float), al = (size_t)at_once * m.ff_pad * sizeof(float);
+  const int rj = (long)m.ff_pad * m.top >= 2048 ? 2 : 1;
+  const dim3 up(m.ff_pad / (4 * rj), m.top), down((r.width_pad + 3) / 4);
+  const int at_once = std::min(m.top, kMoeMaxWidth / m.ff_pad);
+  const size_t xl = (size_t)r.width_pad * sizeof(float), al = (size_t)at_once * m.ff_pad * sizeof(float);
   if (m.w_bf16) {
-    hipLaunchKernelGGL(k_moe_act<true>, up, dim3(256), xl, s, m, x, logits, act, width_pad);
-    hipLaunchKernelGGL(k_moe_down<true>, down, dim3(256), al, s, m, logits, act, out, width_pad, at_once);
+    if (rj == 2) hipLaunchKernelGGL((k_moe_act<true, 2>), up, dim3(256), xl, s, m, r);
+    else hipLaunchKernelGGL((k_moe_act<true, 1>), up, dim3(256), xl, s, m, r);
+    hipLaunchKernelGGL(k_moe_down<true>, down, dim3(256), al, s, m, r, at_once);
   } else {
-    hipLaunchKernelGGL(k_moe_act<false>, up, dim3(256), xl, s, m, x, logits, act, width_pad);
-    hipLaunchKernelGGL(k_moe_down<false>, down, dim3(256), al, s, m, logits, act, out, width_pad, at_once);
+    if (rj == 2) hipLaunchKernelGGL((k_moe_act<false, 2>), up, dim3(256), xl, s, m, r);
+    else hipLaunchKernelGGL((k_moe_act<false, 1>), up, dim3(256), xl, s, m, r);
+    hipLaunchKernelGGL(k_moe_down<false>, down, dim3(256), al, s, m, r, at_once);
   }
   return hipGetLastError();
 }
@@ -262,6 +379,10 @@ hipError_t launch_moe_route(const Moe& m, const MoeRoute& r, const float* logits
   if (m.experts > kMoeMaxExperts || m.top > kMoeMaxTop || m.top > m.experts || r.max_slots != moe_max_slots(m, rows, r.tile_rows))
     return hipErrorInvalidValue;
   const int pairs = rows * m.top;
+  if (rows <= kRouteSmallRows) {
+    hipLaunchKernelGGL(k_moe_route_small, dim3(1), dim3(1024), 0, s, m, r, logits, rows);
+    return hipGetLastError();
+  }
   hipLaunchKernelGGL(k_moe_clear, dim3((std::max(m.experts, r.max_slots) + 255) / 256), dim3(256), 0, s, r, m.experts,
                      r.max_slots);
   hipLaunchKernelGGL(k_moe_choose, dim3((rows + kRouteRows - 1) / kRouteRows), dim3(256), 0, s, m, r, logits, rows);

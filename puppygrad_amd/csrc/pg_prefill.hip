@@ -1207,11 +1207,13 @@ __global__ __launch_bounds__(256) void k_gemv_rows(GemmArgs a) {
 // are used twice).
 // WT: W holds f32 (0), bf16 (1) or int8 rows with a.w_scale (2; a weight is (float)q * scale,
 // formed when its piece is read back; row-major input of up to 32 rows only).
-template <int EPI, int WT, bool XP, bool M16, int NR, int MT>
+// GROUPED: see launch_gemm_grouped; blockIdx.z is the tile of 32 rows.
+template <int EPI, int WT, bool XP, bool M16, int NR, int MT, bool GROUPED = false>
 __global__ __launch_bounds__(512) void k_gemm_rows32(GemmArgs a) {
   static_assert(NR == 32 || (NR == 16 && M16), "rows per block");
   static_assert(MT == 1 || (MT == 2 && !M16 && !XP && WT != 2), "input rows");
   static_assert(WT != 2 || !XP, "int8 rows: row-major input");
+  static_assert(!GROUPED || (!XP && !M16 && MT == 1 && WT != 2), "grouped rows");
   constexpr int CPP = WT == 2 ? 16 : WT == 1 ? 8 : 4;  // columns in a 16-byte piece of a W row
   constexpr int XF = CPP / 4;            // float4 of input that meet one piece
   constexpr int KS = 4 * CPP;            // columns per step: 64 bytes of a row of W
@@ -1224,6 +1226,9 @@ __global__ __launch_bounds__(512) void k_gemm_rows32(GemmArgs a) {
   constexpr int PD = 2;                  // steps requested ahead (3, 4, 6 measured slower)
   __shared__ __attribute__((aligned(16))) float slab[8][SLAB];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int row0 = GROUPED ? 32 * (int)blockIdx.z : 0, M = GROUPED ? 32 : a.M;
+  const int group = GROUPED ? a.group_tile[blockIdx.z] : 0;
+  if (GROUPED && group < 0) return;
   // operand position of the lane: row orow, 16-byte piece opc of the row's 64 bytes
   const int orow = M16 ? (lane & 15) : (lane & 31);
   const int opc = M16 ? (lane >> 4) : (lane >> 5);
@@ -1242,8 +1247,9 @@ __global__ __launch_bounds__(512) void k_gemm_rows32(GemmArgs a) {
   // loads: four lanes to a row of W (q, t); rows q and 16 + q
   const int q = lane >> 2, t = lane & 3;
   const size_t rowbytes = (size_t)a.K * (WT == 2 ? 1 : WT == 1 ? 2 : 4);
-  const char* wpa = reinterpret_cast<const char*>(a.W) + (size_t)min(n0 + q, n1 - 1) * rowbytes + 16 * t;
-  const char* wpb = reinterpret_cast<const char*>(a.W) + (size_t)min(n0 + 16 + q, n1 - 1) * rowbytes + 16 * t;
+  const char* wg = reinterpret_cast<const char*>(a.W) + (GROUPED ? (size_t)group * a.N * rowbytes : 0);
+  const char* wpa = wg + (size_t)min(n0 + q, n1 - 1) * rowbytes + 16 * t;
+  const char* wpb = wg + (size_t)min(n0 + 16 + q, n1 - 1) * rowbytes + 16 * t;
   // input: packed, straight into operand form (k-block kb of row r at (kb * 32 + r) * 4);
   // row-major, KS / 4 lanes to a row
   constexpr int XL = KS / 4;             // lanes to an input row
@@ -1260,7 +1266,7 @@ __global__ __launch_bounds__(512) void k_gemm_rows32(GemmArgs a) {
       xw[j] = 0;
     } else {
       const int r = xq + (64 / XL) * j;
-      xp[j] = a.A + (size_t)min(r, a.M - 1) * a.lda + 4 * xc;
+      xp[j] = a.A + (size_t)(GROUPED ? group_row(a, row0 + r) : min(r, M - 1)) * a.lda + 4 * xc;
       xw[j] = r * XSTR + 4 * xc;
     }
   }
@@ -1272,11 +1278,11 @@ __global__ __launch_bounds__(512) void k_gemm_rows32(GemmArgs a) {
 #pragma unroll
   for (int qq = 0; qq < 2 * MT; ++qq) {
     const int idx = tid + 512 * qq, b = idx / NR, n = n0 + idx % NR;
-    const bool live = gridDim.y == 1 && idx < 32 * MT * NR && b < a.M && n < n1;
+    const bool live = gridDim.y == 1 && idx < 32 * MT * NR && b < M && n < n1;
     ebias[qq] = live && a.bias ? a.bias[n] : 0.0f;
     eres[qq] = live && kAddsResid<EPI> ? a.resid[(size_t)b * a.ldc + n] : 0.0f;
     // int8 rows: the row's scale multiplies the row's sum (also a partial sum of a cut K)
-    escale[qq] = WT == 2 && idx < 32 * MT * NR && b < a.M && n < n1 ? a.w_scale[n] : 1.0f;
+    escale[qq] = WT == 2 && idx < 32 * MT * NR && b < M && n < n1 ? a.w_scale[n] : 1.0f;
   }
 
   f16v acc[MT];   // 32-row form
@@ -1455,7 +1461,7 @@ __global__ __launch_bounds__(512) void k_gemm_rows32(GemmArgs a) {
 #pragma unroll
   for (int q = 0; q < 2 * MT; ++q) {
     const int idx = tid + 512 * q, b = idx / NR, nl = idx % NR, n = n0 + nl;
-    if (idx >= 32 * MT * NR || b >= a.M || n >= n1) continue;
+    if (idx >= 32 * MT * NR || b >= M || n >= n1) continue;
     float sum = red_at(0, b, nl);
 #pragma unroll
     for (int w = 1; w < 8; ++w) sum += red_at(w, b, nl);
@@ -1465,10 +1471,14 @@ __global__ __launch_bounds__(512) void k_gemm_rows32(GemmArgs a) {
       continue;
     }
     float c = ebias[q] + sum;
+    if constexpr (EPI == GEMM_SILU_PAIR) {
+      store_silu_pair(a, row0 + b, n, c);
+      continue;
+    }
     if (EPI == GEMM_GELU) c = gelu_tanh(c);
     if (EPI == GEMM_SQRELU) c = sq_relu(c);
     if (kAddsResid<EPI>) c = eres[q] + col_scaled<EPI>(a, n, c);
-    a.C[a.c_packed ? packed32_index((size_t)b, (size_t)n) : (size_t)b * a.ldc + n] = c;
+    a.C[a.c_packed ? packed32_index((size_t)b, (size_t)n) : (size_t)(row0 + b) * a.ldc + n] = c;
   }
 }
 
@@ -2338,6 +2348,19 @@ hipError_t launch_gemm_grouped(const GemmArgs& a0, int epi, int tile_rows, const
   if (!gemm_supported(a) || a.K % 32 != 0 || a.w_scale || a.bias || a.N % 2 != 0 || !group_tile || a.M % tile_rows != 0)
     return hipErrorInvalidValue;
   if (epi != GEMM_BIAS && epi != GEMM_SILU_PAIR) return hipErrorInvalidValue;
+  if (tile_rows == 32) {  // few rows: blocks own rows of W, as many as leave two blocks to a CU
+    const int tiles = a.M / 32;
+    a.rows_per_block = std::max(8, std::min(32, (int)((long)a.N * std::min(tiles, 16) / 512) / 2 * 2));
+    const dim3 grid((a.N + a.rows_per_block - 1) / a.rows_per_block, 1, tiles);
+    if (tiles > 65535) return hipErrorInvalidValue;
+#define PG_ROWS(EPI, WT) hipLaunchKernelGGL((k_gemm_rows32<EPI, WT, false, false, 32, 1, true>), grid, dim3(512), 0, s, a)
+    if (epi == GEMM_BIAS && a.w_bf16) PG_ROWS(GEMM_BIAS, 1);
+    else if (epi == GEMM_BIAS) PG_ROWS(GEMM_BIAS, 0);
+    else if (a.w_bf16) PG_ROWS(GEMM_SILU_PAIR, 1);
+    else PG_ROWS(GEMM_SILU_PAIR, 0);
+#undef PG_ROWS
+    return hipGetLastError();
+  }
   const int bn = a.w_bf16 ? 128 : 64;
   const int tiles_m = a.M / tile_rows, tiles_n = (a.N + bn - 1) / bn, tiles = tiles_m * tiles_n;
   a.band_rows = choose_band(tiles_m, std::max(1, (tiles + 7) / 8), tile_rows, bn);

@@ -355,7 +355,7 @@ pg_status read_post_ff(const Node& n, LayerPlan* p) {
   Node expert, router;
   f.kind = PostFeedForward::kMoe;
   if ((s = n.object("expert", &expert)) || (s = n.object("router", &router))) return s;
-  if ((s = expert.size("ff", 1, 16000, &f.moe.ff))) return s;
+  if ((s = expert.size("ff", 1, pgk::kMoeMaxWidth, &f.moe.ff))) return s;
   if ((s = router.size("experts", 1, pgk::kMoeMaxExperts, &f.moe.experts))) return s;
   if ((s = router.size("top", 1, std::min(f.moe.experts, pgk::kMoeMaxTop), &f.moe.top))) return s;
   f.moe.ff_pad = up(f.moe.ff, 32);
@@ -759,6 +759,8 @@ pg_status stack_create(const std::string& config_path, const Json& config, const
     l.mix_pad = up(l.mix_cols, 32);
     if (l.mix_pad > kMaxWidth || (l.has_mlp && l.mlp.ff_pad > kMaxWidth))
       return n.bad("is too wide: heads * vdim of the mixers and ff may be up to " + std::to_string(kMaxWidth));
+    if (l.ffn.kind == PostFeedForward::kMoe && m->width_pad > pgk::kMoeMaxWidth)
+      return n.bad("needs a width of at most " + std::to_string(pgk::kMoeMaxWidth));
     m->max_in = std::max(m->max_in, l.n_in);
     m->max_mix = std::max(m->max_mix, l.mix_pad);
     m->max_ff = std::max(m->max_ff, l.has_mlp ? l.mlp.ff_pad : 0);
@@ -829,11 +831,12 @@ namespace {
     if (marks) PG_HIP(marks->mark(s, ProfileMarks::b)); \
   } while (0)
 
-// Experts of few rows read their weights pair by pair; beyond this many pairs they are sorted.
-constexpr long kMoeFewPairs = 64;
-bool moe_few(const pgk::Moe& m, int rows) { return (long)rows * m.top <= kMoeFewPairs; }
-// Slots to a tile of the sorted pairs.
-int moe_tile_rows(const pgk::Moe& m, int rows) { return m.w_bf16 && (long)rows * m.top >= 96L * m.experts ? 128 : 64; }
+// Slots to a tile of the sorted pairs: few rows stream the experts' weights, many fill tiles.
+int moe_tile_rows(const pgk::Moe& m, int rows) {
+  const long pairs = (long)rows * m.top;
+  if (pairs <= 32L * m.experts) return 32;
+  return m.w_bf16 && pairs >= 96L * m.experts ? 128 : 64;
+}
 
 // Working memory of a mixture of experts over `rows` rows, large enough for each layer added.
 struct MoeSizes {
@@ -842,7 +845,7 @@ struct MoeSizes {
     logits = std::max(logits, (size_t)rows * m.experts_pad);
     pairs = std::max(pairs, (size_t)rows * m.top);
     act = std::max(act, (size_t)rows * m.top * m.ff_pad);
-    if (moe_few(m, rows)) return;
+    if (rows == 1) return;
     const int tile = moe_tile_rows(m, rows);
     const size_t n = (size_t)pgk::moe_max_slots(m, rows, tile);
     experts = std::max(experts, (size_t)m.experts);
@@ -860,8 +863,11 @@ pg_status moe_rows(const pg_model* model, const StackLayer& l, const StackCache:
   const StackModel& m = *model->stack;
   const pgk::Moe& e = l.ffn.moe;
   const int Cp = m.width_pad;
-  if (moe_few(e, rows)) {
-    PG_HIP(pgk::launch_moe_few(e, x, b.logits, b.act, sub, rows, Cp, s));
+  if (rows == 1) {
+    pgk::MoeRow r{};
+    r.x = x; r.logits = b.logits; r.width = m.width; r.width_pad = Cp; r.eps = m.eps;
+    r.act = b.act; r.out = sub; r.expert = b.route.expert; r.weight = b.route.weight;
+    PG_HIP(pgk::launch_moe_row(e, r, s));
     PG_MARK(kMlpFc);
     PG_HIP(pgk::launch_add_norm_rows(x, sub, rows, m.width, Cp, l.norm2, m.eps, nullptr, nullptr, 0, s));
     return PG_OK;
@@ -1126,12 +1132,26 @@ pg_status post_norm_step(const pg_model* model, pg_kv_cache* c, ProfileMarks* ma
       PG_HIP(inner(st.act, f.ff_pad, f.down_w, f.down_b, st.sub, Cp, f.ff_pad, nullptr, 0, 0));
       PG_HIP(leave(l.norm2));
     } else if (f.kind == PostFeedForward::kMoe) {
-      PG_HIP(enter(f.router_w, nullptr, st.moe.logits, f.moe.experts_pad, false));
+      const bool fused = B == 1 && pgk::moe_router_fits(f.moe, Cp);
+      if (!fused) PG_HIP(enter(f.router_w, nullptr, st.moe.logits, f.moe.experts_pad, false));
       if (B > 1) {
         if (pg_status e = moe_rows(model, l, st.moe, x, st.sub, B, s, marks)) return e;
       } else {
+        pgk::MoeRow r{};
+        r.x = x; r.width = m.width; r.width_pad = Cp; r.eps = m.eps;
+        r.act = st.moe.act; r.out = st.sub; r.expert = st.moe.route.expert; r.weight = st.moe.route.weight;
+        if (fused) {
+          r.router = f.router_w;
+          r.add = st.sub; r.add_gain = pending; r.x_out = other;
+        } else {
+          r.logits = st.moe.logits;
+        }
         PG_MARK(kMlpFc);
-        PG_HIP(pgk::launch_moe_few(f.moe, x, st.moe.logits, st.moe.act, st.sub, 1, Cp, s));
+        PG_HIP(pgk::launch_moe_row(f.moe, r, s));
+        if (fused) {
+          std::swap(x, other);
+          pending = nullptr;
+        }
         PG_HIP(leave(l.norm2));
       }
     }
