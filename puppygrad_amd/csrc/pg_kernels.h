@@ -243,6 +243,13 @@ struct GemmArgs {
   // (GEMM_RESID_SCALED) != 0: ln_out receives row / sqrt(mean(row^2) + ln_eps) * ln_g[0] instead, the mean over the
   // first rms_cols columns (the others must hold zeros).
   int rms_cols = 0;
+  // (GEMM_BIAS) Optional: norm of the product added to the residual: post_x[M][N] += row / sqrt(mean(row^2)
+  // + ln_eps) * post_gain, the mean over the first post_n columns (the others hold zeros).  Fused into
+  // the split-K reduce where the chosen form has one (C is then working memory), a separate launch
+  // otherwise.  ldc == N.
+  float* post_x = nullptr;
+  const float* post_gain = nullptr;
+  int post_n = 0;
   // Packed form of an activation matrix of at most 32 rows (see packed32_index): which of
   // A, C and ln_out are held that way.  Only the 32-row decode kernel reads a packed A, so
   // launch_gemm refuses the flags for any other form (gemm_takes_rows32 tells beforehand).

@@ -40,8 +40,9 @@ __device__ __forceinline__ void turn(int pos, double freq, float* s, float* c) {
   a -= 6.283185307179586476925287 * rint(a * 0.15915494309189533577);
   sincosf((float)a, s, c);
 }
-__device__ __forceinline__ f4 load_w4(const void* w, int bf16, size_t at) {
-  if (bf16) {
+template <bool BF16>
+__device__ __forceinline__ f4 load_w4(const void* w, size_t at) {
+  if (BF16) {
     const uint2 u = *reinterpret_cast<const uint2*>(static_cast<const unsigned short*>(w) + at);
     return f4{__uint_as_float(u.x << 16), __uint_as_float(u.x & 0xffff0000u), __uint_as_float(u.y << 16),
               __uint_as_float(u.y & 0xffff0000u)};
@@ -75,65 +76,47 @@ __device__ void latent_row(const LatentAttn& a, const float* src, int pos, float
 
 // ---- one token per sequence ----
 // Queries in the latent space, times scale and log2(e): blocks (h < heads, part of 128 latent
-// columns) for NB sequences, which share what they read of W_uk; blocks (heads, 0) write the tokens'
-// rows of the caches.
-template <int NB>
+// columns); block (heads, 0) writes the token's row of the cache.
+template <bool BF16>
 __global__ __launch_bounds__(256) void k_latent_query(LatentDecode m, LatentAttn a) {
-  __shared__ float qs[NB][kMixMaxDim], red[4];
+  __shared__ float qs[kMixMaxDim], red[4];
   __shared__ __attribute__((aligned(16))) float sums[8][128];
   constexpr int PRE = 16;
-  const int tid = threadIdx.x, h = blockIdx.x, b0 = blockIdx.z * NB, nb = min(NB, m.nseq - b0), pos = *m.d_pos;
+  const int tid = threadIdx.x, h = blockIdx.x, b = blockIdx.z, pos = *m.d_pos;
   if (h == a.heads) {
     if (blockIdx.y == 0)
-      for (int b = b0; b < b0 + nb; ++b)
-        latent_row(a, m.y + (size_t)b * m.ld_y + a.c_col, pos, a.ring + (size_t)b * a.ring_seq + (size_t)(pos % a.window) * a.ld,
-                   red);
+      latent_row(a, m.y + (size_t)b * m.ld_y + a.c_col, pos, a.ring + (size_t)b * a.ring_seq + (size_t)(pos % a.window) * a.ld,
+                 red);
     return;
   }
-  const int dk = a.dim + a.rot_dim;
-  const float mul = a.scale * kLog2e;
+  const float* q = m.q + ((size_t)b * a.heads + h) * (a.dim + a.rot_dim);
+  float* qa = m.qa + ((size_t)b * a.heads + h) * a.ld;
+  const float mul = a.scale * kLog2e, mine = q[min(tid, a.dim - 1)];
   // 32 threads to the 128 columns, four each; eight groups take every eighth row of W_uk
   const int col = blockIdx.y * 128 + (tid & 31) * 4, grp = tid >> 5;
   const size_t w0 = (size_t)h * a.dim * a.kv_pad + min(col, a.kv_pad - 4);
   f4 w[PRE];
 #pragma unroll
-  for (int i = 0; i < PRE; ++i) w[i] = load_w4(a.up_w, a.w_bf16, w0 + (size_t)min(grp + 8 * i, a.dim - 1) * a.kv_pad);
-#pragma unroll
-  for (int b = 0; b < NB; ++b)
-    if (tid < a.dim) qs[b][tid] = m.q[((size_t)(b0 + min(b, nb - 1)) * a.heads + h) * dk + tid];
+  for (int i = 0; i < PRE; ++i) w[i] = load_w4<BF16>(a.up_w, w0 + (size_t)min(grp + 8 * i, a.dim - 1) * a.kv_pad);
+  if (tid < a.dim) qs[tid] = mine;
   __syncthreads();
-  f4 sum[NB];
-#pragma unroll
-  for (int b = 0; b < NB; ++b) sum[b] = f4{0.f, 0.f, 0.f, 0.f};
+  f4 sum = f4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
   for (int i = 0; i < PRE; ++i)
-#pragma unroll
-    for (int b = 0; b < NB; ++b)
-      if (grp + 8 * i < a.dim) sum[b] += w[i] * qs[b][grp + 8 * i];
+    if (grp + 8 * i < a.dim) sum += w[i] * qs[grp + 8 * i];
 #pragma unroll 8
-  for (int d = grp + 8 * PRE; d < a.dim; d += 8) {
-    const f4 x = load_w4(a.up_w, a.w_bf16, w0 + (size_t)d * a.kv_pad);
+  for (int d = grp + 8 * PRE; d < a.dim; d += 8) sum += load_w4<BF16>(a.up_w, w0 + (size_t)d * a.kv_pad) * qs[d];
+  *reinterpret_cast<f4*>(&sums[grp][(tid & 31) * 4]) = sum;
+  __syncthreads();
+  if (tid < 128 && blockIdx.y * 128 + tid < a.kv_pad) {
+    float s = 0.0f;
 #pragma unroll
-    for (int b = 0; b < NB; ++b) sum[b] += x * qs[b][d];
-  }
-#pragma unroll
-  for (int b = 0; b < NB; ++b) {
-    if (b) __syncthreads();
-    *reinterpret_cast<f4*>(&sums[grp][(tid & 31) * 4]) = sum[b];
-    __syncthreads();
-    if (b < nb && tid < 128 && blockIdx.y * 128 + tid < a.kv_pad) {
-      float s = 0.0f;
-#pragma unroll
-      for (int g = 0; g < 8; ++g) s += sums[g][tid];
-      m.qa[((size_t)(b0 + b) * a.heads + h) * a.ld + blockIdx.y * 128 + tid] = s * mul;
-    }
+    for (int g = 0; g < 8; ++g) s += sums[g][tid];
+    qa[blockIdx.y * 128 + tid] = s * mul;
   }
   if (blockIdx.y == 0) {
-    const int pairs = (a.ld - a.kv_pad) / 2;
-    for (int x = tid; x < nb * pairs; x += 256) {
-      const int b = x / pairs, i = x - b * pairs;
-      const float* rq = m.q + ((size_t)(b0 + b) * a.heads + h) * dk + a.dim;
-      float* qa = m.qa + ((size_t)(b0 + b) * a.heads + h) * a.ld + a.kv_pad;
+    const float* rq = q + a.dim;
+    for (int i = tid; i < (a.ld - a.kv_pad) / 2; i += 256) {
       float u = 2 * i < a.rot_dim ? rq[2 * i] : 0.0f, v = 2 * i + 1 < a.rot_dim ? rq[2 * i + 1] : 0.0f;
       if (i < a.half) {
         float s, c;
@@ -144,8 +127,8 @@ __global__ __launch_bounds__(256) void k_latent_query(LatentDecode m, LatentAttn
         u = u0 * c - v * s;
         v = v * c + u0 * s;
       }
-      qa[2 * i] = u * mul;
-      qa[2 * i + 1] = v * mul;
+      qa[a.kv_pad + 2 * i] = u * mul;
+      qa[a.kv_pad + 2 * i + 1] = v * mul;
     }
   }
 }
@@ -306,66 +289,69 @@ __global__ __launch_bounds__(256, 1) void k_latent_attn(LatentDecode m, LatentAt
   }
 }
 
-// The shares' sums brought together with the sink, and 32 rows of W_uv, for NB sequences.  Grid: x =
-// head, y = rows of W_uv, z = sequences.  NC: 256-column pieces of a latent.
+// The shares' sums brought together with the sink, and 32 rows of W_uv.  Grid: x = head, y = rows of
+// W_uv, z = sequence.  NC: 256-column pieces of a latent.
 constexpr int kMaxShares = 64;
-template <int NB, int NC>
+template <int NC, bool BF16>
 __global__ __launch_bounds__(256) void k_latent_out(LatentDecode m, LatentAttn a) {
-  __shared__ __attribute__((aligned(16))) float os[NB][256 * NC];
-  __shared__ float ws[NB][kMaxShares];
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, h = blockIdx.x;
-  const int b0 = blockIdx.z * NB, nb = min(NB, m.nseq - b0), e0 = blockIdx.y * 32 + wave;
-  const size_t ps = a.kv_pad + 2, seq = (size_t)a.heads * m.splits * ps;
-  const float* part = m.part + ((size_t)b0 * a.heads + h) * m.splits * ps;
-  // sequence `wave` (NB 1: every wavefront the same): a share per lane
-  if (wave < NB) {
-    const float* p = part + min(wave, nb - 1) * seq + min(lane, m.splits - 1) * ps + a.kv_pad;
-    const float sink = a.sink[h] * kLog2e;
-    const float mx = lane < m.splits ? p[0] : kNone, l = lane < m.splits ? p[1] : 0.0f;
-    float top = fmaxf(mx, sink);
+  __shared__ __attribute__((aligned(16))) float os[256 * NC];
+  __shared__ float ws[kMaxShares];
+  constexpr int PRE = 16;  // shares asked for before their weights are known
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, h = blockIdx.x, b = blockIdx.z;
+  const int e0 = blockIdx.y * 32 + wave, last = m.splits - 1;
+  const size_t ps = a.kv_pad + 2;
+  const float* part = m.part + ((size_t)b * a.heads + h) * m.splits * ps;
+  const float sink = a.sink[h] * kLog2e;
+  // a share per lane
+  const float* pl = part + min(lane, last) * ps + a.kv_pad;
+  const float mx = lane <= last ? pl[0] : kNone, l = lane <= last ? pl[1] : 0.0f;
+  float x[NC][PRE];
 #pragma unroll
-    for (int off = 32; off > 0; off >>= 1) top = fmaxf(top, __shfl_xor(top, off, 64));
-    const float f = l > 0.0f ? exp2f(mx - top) : 0.0f;
-    const float sum = wave_sum(l * f) + exp2f(sink - top);
-    ws[wave][lane] = f / sum;
-  }
+  for (int c = 0; c < NC; ++c)
+#pragma unroll
+    for (int s = 0; s < PRE; ++s) x[c][s] = part[min(s, last) * ps + min(tid + 256 * c, a.kv_pad - 1)];
   f4 w[8][NC];
 #pragma unroll
   for (int r = 0; r < 8; ++r)
 #pragma unroll
     for (int c = 0; c < NC; ++c)
-      w[r][c] = load_w4(a.up_w, a.w_bf16,
-                        ((size_t)a.v_row + h * a.vdim + min(e0 + 4 * r, a.vdim - 1)) * a.kv_pad + min(4 * lane + 256 * c, a.kv_pad - 4));
-  __syncthreads();
-  for (int i = tid; i < 256 * NC; i += 256) {
-    const int at = min(i, a.kv_pad - 1);
+      w[r][c] = load_w4<BF16>(a.up_w, ((size_t)a.v_row + h * a.vdim + min(e0 + 4 * r, a.vdim - 1)) * a.kv_pad + min(4 * lane + 256 * c, a.kv_pad - 4));
+  if (wave == 0) {
+    float top = fmaxf(mx, sink);
 #pragma unroll
-    for (int b = 0; b < NB; ++b) {
-      const float* p = part + min(b, nb - 1) * seq + at;
-      float o = 0.0f;
-#pragma unroll 8
-      for (int s = 0; s < m.splits; ++s) {
-        const float f = ws[b][s], x = p[s * ps];
-        o += f != 0.0f ? f * x : 0.0f;  // (a share without rows has left its sums unwritten)
-      }
-      os[b][i] = i < a.kv_pad ? o : 0.0f;
-    }
+    for (int off = 32; off > 0; off >>= 1) top = fmaxf(top, __shfl_xor(top, off, 64));
+    const float f = l > 0.0f ? exp2f(mx - top) : 0.0f;
+    const float sum = wave_sum(l * f) + exp2f(sink - top);
+    ws[lane] = f / sum;
   }
   __syncthreads();
 #pragma unroll
-  for (int b = 0; b < NB; ++b) {
-    if (b >= nb) break;
-    f4 o[NC];
+  for (int c = 0; c < NC; ++c) {
+    const int i = tid + 256 * c;
+    float o = 0.0f;
+    // (a share without rows has left its sums unwritten)
 #pragma unroll
-    for (int c = 0; c < NC; ++c) o[c] = *reinterpret_cast<const f4*>(&os[b][4 * lane + 256 * c]);
-#pragma unroll
-    for (int r = 0; r < 8; ++r) {
-      float s = 0.0f;
-#pragma unroll
-      for (int c = 0; c < NC; ++c) s += (w[r][c].x * o[c].x + w[r][c].y * o[c].y) + (w[r][c].z * o[c].z + w[r][c].w * o[c].w);
-      s = wave_sum(s);
-      if (lane == 0 && e0 + 4 * r < a.vdim) m.out[(size_t)(b0 + b) * m.ld_out + a.out_col + h * a.vdim + e0 + 4 * r] = s;
+    for (int s = 0; s < PRE; ++s)
+      if (s <= last && ws[s] != 0.0f) o += ws[s] * x[c][s];
+    const float* p = part + min(i, a.kv_pad - 1);
+#pragma unroll 8
+    for (int s = PRE; s <= last; ++s) {
+      const float f = ws[s], y = p[s * ps];
+      o += f != 0.0f ? f * y : 0.0f;
     }
+    os[i] = i < a.kv_pad ? o : 0.0f;
+  }
+  __syncthreads();
+  f4 o[NC];
+#pragma unroll
+  for (int c = 0; c < NC; ++c) o[c] = *reinterpret_cast<const f4*>(&os[4 * lane + 256 * c]);
+#pragma unroll
+  for (int r = 0; r < 8; ++r) {
+    float s = 0.0f;
+#pragma unroll
+    for (int c = 0; c < NC; ++c) s += (w[r][c].x * o[c].x + w[r][c].y * o[c].y) + (w[r][c].z * o[c].z + w[r][c].w * o[c].w);
+    s = wave_sum(s);
+    if (lane == 0 && e0 + 4 * r < a.vdim) m.out[(size_t)b * m.ld_out + a.out_col + h * a.vdim + e0 + 4 * r] = s;
   }
 }
 
@@ -632,10 +618,9 @@ hipError_t launch_latent_decode(const LatentDecode& m, const LatentAttn& a, hipS
   if (a.kv_pad > kLatentMaxRank || a.dim + a.rot_dim > kMixMaxDim || a.vdim > kMixMaxDim || a.kv_pad % 32 != 0 ||
       a.ld % 16 != 0 || a.ld > a.kv_pad + kMixMaxDim || m.splits != latent_decode_splits(a))
     return hipErrorInvalidValue;
-  const int groups = (m.nseq + 3) / 4;  // batches: four sequences share what a block reads of the weights
-  const dim3 qgrid(a.heads + 1, (a.kv_pad + 127) / 128, m.nseq == 1 ? 1 : groups);
-  if (m.nseq == 1) hipLaunchKernelGGL(k_latent_query<1>, qgrid, dim3(256), 0, s, m, a);
-  else hipLaunchKernelGGL(k_latent_query<4>, qgrid, dim3(256), 0, s, m, a);
+  const dim3 qgrid(a.heads + 1, (a.kv_pad + 127) / 128, m.nseq);
+  if (a.w_bf16) hipLaunchKernelGGL(k_latent_query<true>, qgrid, dim3(256), 0, s, m, a);
+  else hipLaunchKernelGGL(k_latent_query<false>, qgrid, dim3(256), 0, s, m, a);
   const dim3 grid(m.splits, (a.heads + 15) / 16, m.nseq);
   const size_t lds = 16 * (size_t)(a.ld + 4) * sizeof(float);
   const void* kernel = a.kv_pad <= 256   ? reinterpret_cast<const void*>(&k_latent_attn<4>)
@@ -648,10 +633,10 @@ hipError_t launch_latent_decode(const LatentDecode& m, const LatentAttn& a, hipS
   if (a.kv_pad <= 256) hipLaunchKernelGGL(k_latent_attn<4>, grid, dim3(256), lds, s, m, a);
   else if (a.kv_pad <= 512) hipLaunchKernelGGL(k_latent_attn<8>, grid, dim3(256), lds, s, m, a);
   else hipLaunchKernelGGL(k_latent_attn<16>, grid, dim3(256), lds, s, m, a);
-  const dim3 ogrid(a.heads, (a.vdim + 31) / 32, m.nseq == 1 ? 1 : groups);
-#define PG_OUT(C)                                                                              \
-  if (m.nseq == 1) hipLaunchKernelGGL((k_latent_out<1, C>), ogrid, dim3(256), 0, s, m, a);     \
-  else hipLaunchKernelGGL((k_latent_out<4, C>), ogrid, dim3(256), 0, s, m, a);
+  const dim3 ogrid(a.heads, (a.vdim + 31) / 32, m.nseq);
+#define PG_OUT(C)                                                                               \
+  if (a.w_bf16) hipLaunchKernelGGL((k_latent_out<C, true>), ogrid, dim3(256), 0, s, m, a);       \
+  else hipLaunchKernelGGL((k_latent_out<C, false>), ogrid, dim3(256), 0, s, m, a);
   if (a.kv_pad <= 256) {
     PG_OUT(1)
   } else if (a.kv_pad <= 512) {

@@ -8,6 +8,7 @@
 #include <math.h>
 
 #include <algorithm>
+#include <type_traits>
 
 namespace pgk {
 
@@ -277,38 +278,71 @@ __device__ __forceinline__ void conv_channels(const ShortConv& c, const float* y
     if (keep[n]) ring[(size_t)slot * c.channels + ch[n]] = cur[n];
 }
 
-// dst[i] = row row0 + i of a low-rank projection, i < n: eight lanes to a row, four rows at a time.
+// Rows row0 .. row0 + n - 1 of a low-rank projection, eight lanes to a row: the first 128 rows
+// and 128 columns of them are asked for by load() and used by store().  (The two kinds of
+// weights part ways around whole runs of loads: a branch per load would wait for each.)
 template <int NT>
-__device__ __forceinline__ void low_rank_rows(const LowRank& p, const float* y, int row0, int n, float* dst) {
-  constexpr int R = 4, STEP = NT / 8;
-  const int sub = threadIdx.x & 7;
-  const float* x = y + p.col;
-  for (int i0 = threadIdx.x >> 3; i0 - (int)(threadIdx.x >> 3) < n; i0 += R * STEP) {
-    float s[R];
-    size_t at[R];
+struct LowRankRows {
+  static constexpr int R = 1024 / NT, C = 4, STEP = NT / 8;
+  f4 w[R][C], x[C];  // (bf16 weights: in the first two words as they are)
+  static __device__ __forceinline__ f4 widened(const f4& raw, int bf16) {
+    const unsigned a = __float_as_uint(raw.x), b = __float_as_uint(raw.y);
+    return bf16 ? f4{__uint_as_float(a << 16), __uint_as_float(a & 0xffff0000u), __uint_as_float(b << 16),
+                     __uint_as_float(b & 0xffff0000u)}
+                : raw;
+  }
+  __device__ __forceinline__ void load(const LowRank& p, const float* y, int row0, int n) {
+    const int i0 = threadIdx.x >> 3, k0 = 4 * (threadIdx.x & 7);
 #pragma unroll
-    for (int q = 0; q < R; ++q) {
-      s[q] = 0.0f;
-      at[q] = (size_t)(row0 + min(i0 + q * STEP, n - 1)) * p.rank;
-    }
-#pragma unroll 4
-    for (int k = 4 * sub; k < p.rank; k += 32) {
-      const f4 v = *reinterpret_cast<const f4*>(x + k);
+    for (int c = 0; c < C; ++c) x[c] = *reinterpret_cast<const f4*>(y + p.col + min(k0 + 32 * c, p.rank - 4));
+    auto at = [&](int q, int c) __attribute__((always_inline)) {
+      return (size_t)(row0 + min(i0 + q * STEP, n - 1)) * p.rank + min(k0 + 32 * c, p.rank - 4);
+    };
+    if (p.w_bf16) {
 #pragma unroll
-      for (int q = 0; q < R; ++q) {
-        const f4 w = p.w_bf16 ? bf16x4(static_cast<const unsigned short*>(p.w) + at[q] + k)
-                              : *reinterpret_cast<const f4*>(static_cast<const float*>(p.w) + at[q] + k);
-        s[q] += (w.x * v.x + w.y * v.y) + (w.z * v.z + w.w * v.w);
-      }
-    }
+      for (int q = 0; q < R; ++q)
 #pragma unroll
-    for (int q = 0; q < R; ++q) {
+        for (int c = 0; c < C; ++c) {
+          const float2 v = *reinterpret_cast<const float2*>(static_cast<const unsigned short*>(p.w) + at(q, c));
+          w[q][c].x = v.x;
+          w[q][c].y = v.y;
+        }
+    } else {
 #pragma unroll
-      for (int off = 4; off > 0; off >>= 1) s[q] += __shfl_xor(s[q], off, 64);
-      if (sub == 0 && i0 + q * STEP < n) dst[i0 + q * STEP] = s[q];
+      for (int q = 0; q < R; ++q)
+#pragma unroll
+        for (int c = 0; c < C; ++c) w[q][c] = *reinterpret_cast<const f4*>(static_cast<const float*>(p.w) + at(q, c));
     }
   }
-}
+  // dst[i] = row row0 + i
+  __device__ __forceinline__ void store(const LowRank& p, const float* y, int row0, int n, float* dst) const {
+    const int i0 = threadIdx.x >> 3, sub = threadIdx.x & 7;
+    auto dot = [](const f4& a, const f4& b) { return (a.x * b.x + a.y * b.y) + (a.z * b.z + a.w * b.w); };
+    auto finish = [&](int i, float s) __attribute__((always_inline)) {
+#pragma unroll
+      for (int off = 4; off > 0; off >>= 1) s += __shfl_xor(s, off, 64);
+      if (sub == 0 && i < n) dst[i] = s;
+    };
+    auto rest = [&](int i, int k0, float s) __attribute__((always_inline)) {
+      const size_t at = (size_t)(row0 + min(i, n - 1)) * p.rank;
+      for (int k = k0 + 4 * sub; k < p.rank; k += 32) {
+        const f4 v = p.w_bf16 ? bf16x4(static_cast<const unsigned short*>(p.w) + at + k)
+                              : *reinterpret_cast<const f4*>(static_cast<const float*>(p.w) + at + k);
+        s += dot(v, *reinterpret_cast<const f4*>(y + p.col + k));
+      }
+      return s;
+    };
+#pragma unroll
+    for (int q = 0; q < R; ++q) {
+      float s = 0.0f;
+#pragma unroll
+      for (int c = 0; c < C; ++c)
+        if (32 * c < p.rank) s += dot(widened(w[q][c], p.w_bf16), x[c]);
+      finish(i0 + q * STEP, p.rank > 32 * C ? rest(i0 + q * STEP, 32 * C, s) : s);
+    }
+    for (int r0 = R * STEP; r0 < n; r0 += STEP) finish(r0 + i0, rest(r0 + i0, 0, 0.0f));
+  }
+};
 
 // One head of the recurrence.  A thread owns column v of the state and every `parts`-th of its
 // rows, RPT of them, in registers (parts * RPT <= kMixMaxDim; q and k are 0 past dim).
@@ -349,10 +383,11 @@ __device__ void recurrence_role(const MixDecode& m, int b, int h, float* lds) {
     float* ring = cv.ring + (size_t)b * cv.ring_seq;
     const bool first = h % (c.heads / c.kv_heads) == 0;
     const float yb = kSsd ? 0.0f : y[c.b_col + h], al0 = c.a_log[h];
-    const float ya = kChannel ? 0.0f : y[c.a_col + h], dt = kChannel ? 0.0f : c.dt_bias[h];
-    if (kChannel) {
-      low_rank_rows<NT>(c.low_a, y, h * dim, dim, al);
-      low_rank_rows<NT>(c.low_g, y, h * vdim, vdim, gs);
+    const float ya = kChannel ? 0.0f : y[c.a_col + h], dt = c.dt_bias[kChannel ? h * dim + min(tid, dim - 1) : h];
+    typename std::conditional<kChannel, LowRankRows<NT>, int>::type low_a, low_g;
+    if constexpr (kChannel) {
+      low_a.load(c.low_a, y, h * dim, dim);
+      low_g.load(c.low_g, y, h * vdim, vdim);
     }
     const int td = min(tid, dim - 1);
     const int ch[3] = {c.q_col - cv.col + kvh * dim + td, c.k_col - cv.col + kvh * dim + td,
@@ -360,6 +395,10 @@ __device__ void recurrence_role(const MixDecode& m, int b, int h, float* lds) {
     const bool keep[3] = {first && tid < dim, first && tid < dim, tid < vdim};
     float cq[3];
     conv_channels<3>(cv, y, ring, ch, keep, pos, cq);
+    if constexpr (kChannel) {
+      low_a.store(c.low_a, y, h * dim, dim, al);
+      low_g.store(c.low_g, y, h * vdim, vdim, gs);
+    }
     float qv = cq[0], kv = cq[1], x = cq[2];
     if (tid >= dim) qv = kv = 0.0f;
     if constexpr (kSsd) {
@@ -387,7 +426,7 @@ __device__ void recurrence_role(const MixDecode& m, int b, int h, float* lds) {
     }
     beta = sigmoid(yb);
     if constexpr (kChannel) {  // (al was written before the barrier above)
-      if (tid < dim) al[tid] = expf(delta_log_decay(al[tid], al0, c.dt_bias[h * dim + tid]));
+      if (tid < dim) al[tid] = expf(delta_log_decay(al[tid], al0, dt));
     } else {
       g = expf(delta_log_decay(ya, al0, dt));
     }

@@ -92,11 +92,13 @@ __device__ __forceinline__ float chunk_dot(const u4v& u, const float* x) {
 }
 
 constexpr int kRouterRows = 16;  // rows of a router that a wavefront multiplies at most
+constexpr int kRouterPre = 4;    // 64-chunk pieces of them asked for at the start
 
 // act[k][j] = silu(gate j . x) * (up j . x) of the row's k-th expert.  Every block brings x up to date
 // and routes the row for itself (a wavefront: every fourth row of the router); block (0, k) lists
-// the choice.  Grid: x = 4 RJ values of j, y = k.
-template <bool BF16, int RJ>
+// the choice.  Grid: x = 4 RJ values of j, y = k.  RR: rows of the router to a wavefront (0: the logits are
+// there).
+template <bool BF16, int RJ, int RR>
 __global__ __launch_bounds__(256) void k_moe_act(Moe m, MoeRow r) {
   extern __shared__ __attribute__((aligned(16))) float xs[];
   __shared__ float zs[4 * kRouterRows], red[4];
@@ -116,6 +118,14 @@ __global__ __launch_bounds__(256) void k_moe_act(Moe m, MoeRow r) {
         vg[p] = reinterpret_cast<const f4*>(r.add_gain)[i];
       }
     }
+  }
+  const u4v* rw = static_cast<const u4v*>(r.router);
+  u4v pre[RR > 0 ? RR : 1][kRouterPre];
+  if constexpr (RR > 0) {
+#pragma unroll
+    for (int e = 0; e < RR; ++e)
+#pragma unroll
+      for (int c = 0; c < kRouterPre; ++c) pre[e][c] = rw[(size_t)min(wave + 4 * e, m.experts - 1) * n + min(lane + 64 * c, n - 1)];
   }
   if (r.add) {
     float ss = 0.0f;
@@ -150,26 +160,19 @@ __global__ __launch_bounds__(256) void k_moe_act(Moe m, MoeRow r) {
   }
   __syncthreads();
   const float* z = r.logits;
-  if (r.router) {
-    const u4v* w = static_cast<const u4v*>(r.router);
-    float s[kRouterRows];
+  if constexpr (RR > 0) {
 #pragma unroll
-    for (int e = 0; e < kRouterRows; ++e) s[e] = 0.0f;
-    for (int j = lane; j < n; j += 64) {
-      u4v u[kRouterRows];
+    for (int e = 0; e < RR; ++e) {
+      if (wave + 4 * e >= m.experts) break;
+      float s = 0.0f;
 #pragma unroll
-      for (int e = 0; e < kRouterRows; ++e)
-        if (wave + 4 * e < m.experts) u[e] = w[(size_t)(wave + 4 * e) * n + j];
-#pragma unroll
-      for (int e = 0; e < kRouterRows; ++e)
-        if (wave + 4 * e < m.experts) s[e] += chunk_dot<BF16>(u[e], xs + PER * j);
+      for (int c = 0; c < kRouterPre; ++c)
+        if (lane + 64 * c < n) s += chunk_dot<BF16>(pre[e][c], xs + PER * (lane + 64 * c));
+#pragma unroll 4
+      for (int j = lane + 64 * kRouterPre; j < n; j += 64) s += chunk_dot<BF16>(rw[(size_t)(wave + 4 * e) * n + j], xs + PER * j);
+      s = wave_sum(s);
+      if (lane == 0) zs[wave + 4 * e] = s;
     }
-#pragma unroll
-    for (int e = 0; e < kRouterRows; ++e)
-      if (wave + 4 * e < m.experts) {
-        s[e] = wave_sum(s[e]);
-        if (lane == 0) zs[wave + 4 * e] = s[e];
-      }
     __syncthreads();
     z = zs;
   }
@@ -191,7 +194,7 @@ __global__ __launch_bounds__(256) void k_moe_act(Moe m, MoeRow r) {
   float s[2 * RJ];
 #pragma unroll
   for (int q = 0; q < 2 * RJ; ++q) s[q] = 0.0f;
-#pragma unroll 2
+#pragma unroll 4
   for (int i = lane; i < n; i += 64) {
     u4v u[2 * RJ];
 #pragma unroll
@@ -315,9 +318,10 @@ __global__ __launch_bounds__(256) void k_moe_place(Moe m, MoeRoute r, int pairs)
 }
 
 // All of it in one block, for a few rows.
-constexpr int kRouteSmallRows = 128;
+constexpr int kRouteSmallRows = 128, kRouteSmallPairs = 4096;
 __global__ __launch_bounds__(1024) void k_moe_route_small(Moe m, MoeRoute r, const float* logits, int rows) {
   __shared__ int count[kMoeMaxExperts], first[kMoeMaxExperts + 1];
+  __shared__ int pair[kRouteSmallPairs];  // expert and number within it
   const int tid = threadIdx.x, wave = tid >> 6;
   for (int i = tid; i < m.experts; i += 1024) count[i] = 0;
   for (int i = tid; i < r.max_slots; i += 1024) r.slot_row[i] = -1;
@@ -327,9 +331,8 @@ __global__ __launch_bounds__(1024) void k_moe_route_small(Moe m, MoeRoute r, con
     choose_any(logits + (size_t)row * m.experts_pad, m.experts, m.top, [&](int k, int e, float w) {
       if ((tid & 63) == 0) {
         const size_t p = (size_t)row * m.top + k;
-        r.expert[p] = e;
         r.weight[p] = w;
-        r.rank[p] = atomicAdd(&count[e], 1);
+        pair[p] = e << 16 | atomicAdd(&count[e], 1);
       }
     });
   __syncthreads();
@@ -338,7 +341,7 @@ __global__ __launch_bounds__(1024) void k_moe_route_small(Moe m, MoeRoute r, con
   for (int e = tid; e < m.experts; e += 1024)
     for (int t = first[e] / r.tile_rows; t < first[e + 1] / r.tile_rows; ++t) r.tile[t] = e;
   for (int p = tid; p < rows * m.top; p += 1024) {
-    const int s = first[r.expert[p]] + r.rank[p];
+    const int s = first[pair[p] >> 16] + (pair[p] & 0xffff);
     r.slot[p] = s;
     r.slot_row[s] = p / m.top;
   }
@@ -357,15 +360,28 @@ hipError_t launch_moe_row(const Moe& m, const MoeRow& r, hipStream_t s) {
   const dim3 up(m.ff_pad / (4 * rj), m.top), down((r.width_pad + 3) / 4);
   const int at_once = std::min(m.top, kMoeMaxWidth / m.ff_pad);
   const size_t xl = (size_t)r.width_pad * sizeof(float), al = (size_t)at_once * m.ff_pad * sizeof(float);
+  const int rr = !r.router ? 0 : m.experts <= 8 ? 2 : m.experts <= 16 ? 4 : kRouterRows;
+#define PG_ACT(B, J)                                                                                          \
+  if (rr == 0) hipLaunchKernelGGL((k_moe_act<B, J, 0>), up, dim3(256), xl, s, m, r);                           \
+  else if (rr == 2) hipLaunchKernelGGL((k_moe_act<B, J, 2>), up, dim3(256), xl, s, m, r);                      \
+  else if (rr == 4) hipLaunchKernelGGL((k_moe_act<B, J, 4>), up, dim3(256), xl, s, m, r);                      \
+  else hipLaunchKernelGGL((k_moe_act<B, J, kRouterRows>), up, dim3(256), xl, s, m, r);
   if (m.w_bf16) {
-    if (rj == 2) hipLaunchKernelGGL((k_moe_act<true, 2>), up, dim3(256), xl, s, m, r);
-    else hipLaunchKernelGGL((k_moe_act<true, 1>), up, dim3(256), xl, s, m, r);
+    if (rj == 2) {
+      PG_ACT(true, 2)
+    } else {
+      PG_ACT(true, 1)
+    }
     hipLaunchKernelGGL(k_moe_down<true>, down, dim3(256), al, s, m, r, at_once);
   } else {
-    if (rj == 2) hipLaunchKernelGGL((k_moe_act<false, 2>), up, dim3(256), xl, s, m, r);
-    else hipLaunchKernelGGL((k_moe_act<false, 1>), up, dim3(256), xl, s, m, r);
+    if (rj == 2) {
+      PG_ACT(false, 2)
+    } else {
+      PG_ACT(false, 1)
+    }
     hipLaunchKernelGGL(k_moe_down<false>, down, dim3(256), al, s, m, r, at_once);
   }
+#undef PG_ACT
   return hipGetLastError();
 }
 
@@ -379,7 +395,7 @@ hipError_t launch_moe_route(const Moe& m, const MoeRoute& r, const float* logits
   if (m.experts > kMoeMaxExperts || m.top > kMoeMaxTop || m.top > m.experts || r.max_slots != moe_max_slots(m, rows, r.tile_rows))
     return hipErrorInvalidValue;
   const int pairs = rows * m.top;
-  if (rows <= kRouteSmallRows) {
+  if (rows <= kRouteSmallRows && pairs <= kRouteSmallPairs) {
     hipLaunchKernelGGL(k_moe_route_small, dim3(1), dim3(1024), 0, s, m, r, logits, rows);
     return hipGetLastError();
   }

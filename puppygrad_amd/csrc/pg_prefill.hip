@@ -1082,6 +1082,52 @@ __global__ __launch_bounds__(256) void k_splitk_reduce_ln(GemmArgs a, int parts)
   }
 }
 
+// k_splitk_reduce for one whole row per block, whose norm is added to the residual (GemmArgs::post_x).
+// N <= 4096, a multiple of 4.
+template <bool EARLY>
+__global__ __launch_bounds__(256) void k_splitk_reduce_post(GemmArgs a, int parts) {
+  __shared__ float red[4];
+  const size_t m = blockIdx.x;
+  const int n4 = a.N / 4, tid = threadIdx.x;
+  const size_t stride = (size_t)a.M * a.N;
+  f4 c[4], v[EARLY ? 4 : 1][8], x[4], g[4];
+  auto request = [&](int q, f4 (&v)[8]) {
+    const size_t n = (size_t)min(tid + 256 * q, n4 - 1) * 4;
+#pragma unroll
+    for (int p = 0; p < 8; ++p)
+      v[p] = *reinterpret_cast<const f4*>(a.ws + (size_t)min(p, parts - 1) * stride + m * a.N + n);
+    x[q] = *reinterpret_cast<const f4*>(a.post_x + m * a.N + n);
+    g[q] = *reinterpret_cast<const f4*>(a.post_gain + n);
+  };
+  if (EARLY) {
+#pragma unroll
+    for (int q = 0; q < 4; ++q)
+      if (256 * q < n4) request(q, v[q]);  // (block-uniform)
+  }
+  float ss = 0.0f;
+#pragma unroll
+  for (int q = 0; q < 4; ++q) {
+    c[q] = f4{0.f, 0.f, 0.f, 0.f};
+    if (!EARLY && 256 * q < n4) request(q, v[0]);
+    if (tid + 256 * q < n4) {
+      c[q] = v[EARLY ? q : 0][0];
+#pragma unroll
+      for (int p = 1; p < 8; ++p)
+        if (p < parts) c[q] += v[EARLY ? q : 0][p];
+      if (a.bias) c[q] += *reinterpret_cast<const f4*>(a.bias + 4 * (tid + 256 * q));
+    }
+    ss += (c[q].x * c[q].x + c[q].y * c[q].y) + (c[q].z * c[q].z + c[q].w * c[q].w);
+  }
+#pragma unroll
+  for (int off = 32; off > 0; off >>= 1) ss += __shfl_xor(ss, off, 64);
+  if ((tid & 63) == 0) red[tid >> 6] = ss;
+  __syncthreads();
+  const float k = 1.0f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / (float)a.post_n + a.ln_eps);
+#pragma unroll
+  for (int q = 0; q < 4; ++q)
+    if (tid + 256 * q < n4) *reinterpret_cast<f4*>(a.post_x + m * a.N + 4 * (size_t)(tid + 256 * q)) = x[q] + c[q] * k * g[q];
+}
+
 // ---------------------------------------------------------------------------
 // A batch of at most MB rows against W (the projections of a batched decode step).  The
 // job is to stream W once at the speed of HBM, and tiles that stage W through LDS cut it
@@ -1985,6 +2031,12 @@ namespace {
 // Finishes a.ws[parts][M][N]: bias, epilogue and, where asked for and possible, the
 // LayerNorm of the result in the same launch (*ln_done tells).
 hipError_t launch_splitk_reduce(const GemmArgs& a, int epi, int parts, hipStream_t s, bool* ln_done) {
+  if (a.post_x && epi == GEMM_BIAS && a.N % 4 == 0 && a.N <= 4096) {
+    if (a.M <= 64) hipLaunchKernelGGL(k_splitk_reduce_post<true>, dim3(a.M), dim3(256), 0, s, a, parts);
+    else hipLaunchKernelGGL(k_splitk_reduce_post<false>, dim3(a.M), dim3(256), 0, s, a, parts);
+    *ln_done = true;
+    return hipGetLastError();
+  }
   if (a.ln_out && a.N % 4 == 0 && a.N <= 4096 && a.ldc == a.N) {
     const bool early = a.M <= 64;
     if (epi == GEMM_BIAS && early)
@@ -2330,8 +2382,11 @@ hipError_t launch_gemm(const GemmArgs& a, int epi, int num_cus, hipStream_t s) {
   if (a.ln_out && a.ldc != a.N) return hipErrorInvalidValue;
   if ((epi == GEMM_RESID_SCALED) != (a.col_scale != nullptr) || (a.rms_cols && epi != GEMM_RESID_SCALED))
     return hipErrorInvalidValue;
+  if (a.post_x && (epi != GEMM_BIAS || a.ln_out || a.ldc != a.N)) return hipErrorInvalidValue;
   bool ln_done = false;
   hipError_t e = launch_gemm_form(a, epi, num_cus, s, &ln_done);
+  if (e == hipSuccess && a.post_x && !ln_done)
+    return launch_add_norm_rows(a.post_x, a.C, a.M, a.post_n, a.N, a.post_gain, a.ln_eps, nullptr, nullptr, 0, s);
   if (e == hipSuccess && a.ln_out && !ln_done && a.rms_cols)
     return a.ln_packed ? hipErrorInvalidValue
                        : launch_rms_rows(a.C, a.ln_out, a.M, a.rms_cols, a.N, a.ln_g, a.ln_eps, 1.0f, nullptr, s);

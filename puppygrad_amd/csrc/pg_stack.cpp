@@ -1001,14 +1001,16 @@ struct Gemm {
     return pgk::launch_gemm(a, resid_scale ? pgk::GEMM_RESID_SCALED : pgk::GEMM_BIAS, m->num_cus, s);
   }
   // C[n_rows][N] = epilogue(A[n_rows][lda] . W[N][K]^T + bias)
+  // (post_x: the rows' norm is added to it instead, C is working memory)
   hipError_t product(int n_rows, const float* A, int lda, const void* W, float* C, int N, int K, const float* bias = nullptr,
-                     int epilogue = pgk::GEMM_BIAS) const {
+                     int epilogue = pgk::GEMM_BIAS, float* post_x = nullptr, const float* post_gain = nullptr) const {
     pgk::GemmArgs a{};
     a.A = A; a.w_bf16 = m->w_bf16; a.W = static_cast<const float*>(W); a.bias = bias; a.C = C;
     a.M = n_rows; a.N = N; a.K = K; a.lda = lda; a.ldc = N;
     a.ws = ws; a.ws_floats = ws_floats;
     a.split_items_per_cu = m->gemm_split_items;
     a.b9_min_rows = m->gemm_b9_min_rows;
+    a.post_x = post_x; a.post_gain = post_gain; a.post_n = m->stack->width; a.ln_eps = m->stack->eps;
     return pgk::launch_gemm(a, epilogue, m->num_cus, s);
   }
 };
@@ -1069,21 +1071,21 @@ pg_status post_norm_step(const pg_model* model, pg_kv_cache* c, ProfileMarks* ma
     pending = nullptr;
     return e;
   };
-  // y = W (norm of in) + bias; groups 0: no norm (batches norm their rows in place beforehand)
-  auto inner = [&](const float* in, int ld_in, const float* W, const float* bias, float* y, int nout, int K,
-                   const float* gain, int norm_n, int groups) -> hipError_t {
-    if (B > 1) return gemm.product(B, in, ld_in, W, y, nout, K, bias);
+  // y = W (norm of in) (one sequence; groups 0: no norm)
+  auto inner = [&](const float* in, const float* W, const float* bias, float* y, int nout, int K, const float* gain,
+                   int norm_n, int groups) -> hipError_t {
     pgk::GemvArgs a{};
     a.w_bf16 = model->w_bf16; a.W = W; a.bias = bias; a.x = in; a.y = y; a.K = K; a.nout = nout; a.eps = m.eps;
     if (groups == 0) return pgk::launch_gemv(a, pgk::PRO_NONE, pgk::EPI_BIAS, s);
     a.gain = gain; a.norm_n = norm_n; a.groups = groups;
     return pgk::launch_gemv(a, pgk::PRO_STACK, pgk::EPI_BIAS, s);
   };
-  // the sublayer's output is in st.sub
-  auto leave = [&](const float* gain) -> hipError_t {
-    if (B > 1) return pgk::launch_add_norm_rows(x, st.sub, B, m.width, Cp, gain, m.eps, nullptr, nullptr, 0, s);
-    pending = gain;
-    return hipSuccess;
+  // The end of a sublayer: W (norm of in) + bias, normed and added to x (batches norm `in` beforehand).
+  auto leave = [&](const float* in, const float* W, const float* bias, int K, const float* gain, int norm_n, int groups,
+                   const float* post) -> hipError_t {
+    if (B > 1) return gemm.product(B, in, K, W, st.sub, Cp, K, bias, pgk::GEMM_BIAS, x, post);
+    pending = post;
+    return inner(in, W, bias, st.sub, Cp, K, gain, norm_n, groups);
   };
   PG_HIP(pgk::launch_begin_step(x, m.embed, model->w_bf16, c->d_tok, B, Cp, st.words, s));
   PG_MARK(kNone);
@@ -1100,7 +1102,7 @@ pg_status post_norm_step(const pg_model* model, pg_kv_cache* c, ProfileMarks* ma
         PG_HIP(pgk::launch_group_rms_rows(st.y + a.q_col, l.n_in, st.cq, a.q_pad, B, a.q_rank, 1, a.q_norm, m.eps, nullptr, s));
         PG_HIP(gemm.product(B, st.cq, a.q_pad, l.uq_w, st.q, nq, a.q_pad));
       } else {
-        PG_HIP(inner(st.y + a.q_col, 0, l.uq_w, nullptr, st.q, nq, a.q_pad, a.q_norm, a.q_rank, 1));
+        PG_HIP(inner(st.y + a.q_col, l.uq_w, nullptr, st.q, nq, a.q_pad, a.q_norm, a.q_rank, 1));
       }
       pgk::LatentDecode d{};
       d.nseq = B; d.d_pos = &st.words->pos;
@@ -1122,15 +1124,13 @@ pg_status post_norm_step(const pg_model* model, pg_kv_cache* c, ProfileMarks* ma
                                           nullptr, s));
     }
     PG_MARK(kAttention);
-    PG_HIP(inner(st.mix, l.mix_pad, l.out_w, nullptr, st.sub, Cp, l.mix_pad, l.mix_norm, l.mix_cols, groups));
-    PG_HIP(leave(l.norm1));
+    PG_HIP(leave(st.mix, l.out_w, nullptr, l.mix_pad, l.mix_norm, l.mix_cols, groups, l.norm1));
     PG_MARK(kAttnProj);
     const PostFeedForward& f = l.ffn;
     if (f.kind == PostFeedForward::kDense) {
       PG_HIP(enter(f.up_w, f.up_b, st.act, f.ff_pad, true));
       PG_MARK(kMlpFc);
-      PG_HIP(inner(st.act, f.ff_pad, f.down_w, f.down_b, st.sub, Cp, f.ff_pad, nullptr, 0, 0));
-      PG_HIP(leave(l.norm2));
+      PG_HIP(leave(st.act, f.down_w, f.down_b, f.ff_pad, nullptr, 0, 0, l.norm2));
     } else if (f.kind == PostFeedForward::kMoe) {
       const bool fused = B == 1 && pgk::moe_router_fits(f.moe, Cp);
       if (!fused) PG_HIP(enter(f.router_w, nullptr, st.moe.logits, f.moe.experts_pad, false));
@@ -1148,11 +1148,8 @@ pg_status post_norm_step(const pg_model* model, pg_kv_cache* c, ProfileMarks* ma
         }
         PG_MARK(kMlpFc);
         PG_HIP(pgk::launch_moe_row(f.moe, r, s));
-        if (fused) {
-          std::swap(x, other);
-          pending = nullptr;
-        }
-        PG_HIP(leave(l.norm2));
+        if (fused) std::swap(x, other);
+        pending = l.norm2;
       }
     }
     PG_MARK(kMlpProj);
@@ -1392,15 +1389,13 @@ pg_status post_norm_rows(const pg_model* model, pg_kv_cache* c, const uint32_t* 
                                           nullptr, s));
     }
     PG_MARK(kAttention);
-    PG_HIP(gemm.product(R, mix, l.mix_pad, l.out_w, sub, (int)Cp, l.mix_pad));
-    PG_HIP(pgk::launch_add_norm_rows(x, sub, R, m.width, (int)Cp, l.norm1, m.eps, nullptr, nullptr, 0, s));
+    PG_HIP(gemm.product(R, mix, l.mix_pad, l.out_w, sub, (int)Cp, l.mix_pad, nullptr, pgk::GEMM_BIAS, x, l.norm1));
     PG_MARK(kAttnProj);
     const PostFeedForward& f = l.ffn;
     if (f.kind == PostFeedForward::kDense) {
       PG_HIP(gemm.product(R, x, (int)Cp, f.up_w, act, f.ff_pad, (int)Cp, f.up_b, pgk::GEMM_SQRELU));
       PG_MARK(kMlpFc);
-      PG_HIP(gemm.product(R, act, f.ff_pad, f.down_w, sub, (int)Cp, f.ff_pad, f.down_b));
-      PG_HIP(pgk::launch_add_norm_rows(x, sub, R, m.width, (int)Cp, l.norm2, m.eps, nullptr, nullptr, 0, s));
+      PG_HIP(gemm.product(R, act, f.ff_pad, f.down_w, sub, (int)Cp, f.ff_pad, f.down_b, pgk::GEMM_BIAS, x, l.norm2));
     } else if (f.kind == PostFeedForward::kMoe) {
       PG_HIP(gemm.product(R, x, (int)Cp, f.router_w, moe.logits, f.moe.experts_pad, (int)Cp));
       if (pg_status e = moe_rows(model, l, moe, x, sub, R, s, marks)) return e;
