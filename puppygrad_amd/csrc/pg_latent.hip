@@ -459,35 +459,60 @@ __global__ __launch_bounds__(256, 1) void k_latent_attn_rows(MixRows r, LatentAt
   float* ks = lds + kg * TILE;
   float* vs = ks + KT * LDK;
 
-  auto load4 = [&](const float* p, int d, int n) __attribute__((always_inline)) {
-    if (vec) return *reinterpret_cast<const f4*>(p + d);
-    f4 x;
-#pragma unroll
-    for (int e = 0; e < 4; ++e) x[e] = d + e < n ? p[d + e] : 0.0f;
-    return x;
-  };
+  // sixteen lanes (eight for narrow values) to 64 (32) columns of a row: column block c, row pass i
+  constexpr int VL = DV >= 64 ? 16 : 8;
+  constexpr int KC = DP / 64, KR = 32 * 16 / TH, VC = DV / (4 * VL), VR = 32 * VL / TH > 0 ? 32 * VL / TH : 1;
+  static_assert(KC * KR == NK && VC * VR == NV, "whole passes");
+  const int ki = st >> 4, kd = (st & 15) * 4, vi = st / VL, vd = (st % VL) * 4;
   f4 kreg[NK], vreg[NV];
   auto fetch = [&](int tile) __attribute__((always_inline)) {
+    const int j0 = jf + tile * KT;
+    if (vec) {
 #pragma unroll
-    for (int i = 0; i < NK; ++i) {
-      const int idx = st + TH * i, d = (idx % (DP / 4)) * 4;
-      const size_t j = min(jf + tile * KT + idx / (DP / 4), jl);
-      kreg[i] = f4{0.f, 0.f, 0.f, 0.f};
-      if (vec) {
-        if (d < dim) kreg[i] = *reinterpret_cast<const f4*>(kb + j * l.ld_kv + d);
-        else if (d < dk) kreg[i] = *reinterpret_cast<const f4*>(rb + j * a.ld + (d - dim));
-      } else {
+      for (int i = 0; i < KR; ++i) {
+        const int j = min(j0 + ki + TH / 16 * i, jl);
+        const float *k = kb + (size_t)j * l.ld_kv, *x = rb + (size_t)j * a.ld - dim;
 #pragma unroll
-        for (int e = 0; e < 4; ++e)
-          if (d + e < dk) kreg[i][e] = d + e < dim ? kb[j * l.ld_kv + d + e] : rb[j * a.ld + d + e - dim];
+        for (int c = 0; c < KC; ++c) {
+          const int d = kd + 64 * c;
+          kreg[i * KC + c] = f4{0.f, 0.f, 0.f, 0.f};
+          if (d < dk) kreg[i * KC + c] = *reinterpret_cast<const f4*>((d < dim ? k : x) + d);
+        }
       }
+#pragma unroll
+      for (int i = 0; i < VR; ++i) {
+        const float* v = vb + (size_t)min(j0 + vi + TH / VL * i, jl) * l.ld_kv;
+#pragma unroll
+        for (int c = 0; c < VC; ++c) {
+          const int d = vd + 4 * VL * c;
+          vreg[i * VC + c] = f4{0.f, 0.f, 0.f, 0.f};
+          if (d < vdim) vreg[i * VC + c] = *reinterpret_cast<const f4*>(v + d);
+        }
+      }
+      return;
     }
 #pragma unroll
-    for (int i = 0; i < NV; ++i) {
-      const int idx = st + TH * i, d = (idx % (DV / 4)) * 4;
-      const size_t j = min(jf + tile * KT + idx / (DV / 4), jl);
-      vreg[i] = f4{0.f, 0.f, 0.f, 0.f};
-      if (d < vdim) vreg[i] = load4(vb + j * l.ld_kv, d, vdim);
+    for (int i = 0; i < KR; ++i) {
+      const int j = min(j0 + ki + TH / 16 * i, jl);
+      const float *k = kb + (size_t)j * l.ld_kv, *x = rb + (size_t)j * a.ld - dim;
+#pragma unroll
+      for (int c = 0; c < KC; ++c)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const int d = kd + 64 * c + e;
+          kreg[i * KC + c][e] = d < dk ? (d < dim ? k : x)[d] : 0.0f;
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < VR; ++i) {
+      const float* v = vb + (size_t)min(j0 + vi + TH / VL * i, jl) * l.ld_kv;
+#pragma unroll
+      for (int c = 0; c < VC; ++c)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const int d = vd + 4 * VL * c + e;
+          vreg[i * VC + c][e] = d < vdim ? v[d] : 0.0f;
+        }
     }
   };
   fetch(min(kg, tiles - 1));
@@ -495,15 +520,13 @@ __global__ __launch_bounds__(256, 1) void k_latent_attn_rows(MixRows r, LatentAt
     const int tile = turn * KG + kg, k0 = jf + tile * KT;
     __syncthreads();  // (the previous tile has been read)
 #pragma unroll
-    for (int i = 0; i < NK; ++i) {
-      const int idx = st + TH * i;
-      *reinterpret_cast<f4*>(&ks[(idx / (DP / 4)) * LDK + (idx % (DP / 4)) * 4]) = kreg[i];
-    }
+    for (int i = 0; i < KR; ++i)
 #pragma unroll
-    for (int i = 0; i < NV; ++i) {
-      const int idx = st + TH * i;
-      *reinterpret_cast<f4*>(&vs[(idx / (DV / 4)) * LDV + (idx % (DV / 4)) * 4]) = vreg[i];
-    }
+      for (int c = 0; c < KC; ++c) *reinterpret_cast<f4*>(&ks[(ki + TH / 16 * i) * LDK + kd + 64 * c]) = kreg[i * KC + c];
+#pragma unroll
+    for (int i = 0; i < VR; ++i)
+#pragma unroll
+      for (int c = 0; c < VC; ++c) *reinterpret_cast<f4*>(&vs[(vi + TH / VL * i) * LDV + vd + 4 * VL * c]) = vreg[i * VC + c];
     __syncthreads();
     if (turn + 1 < turns) fetch(min(tile + KG, tiles - 1));
     // (wavefront-uniform: past the share's last tile, or no query of the group sees the tile)

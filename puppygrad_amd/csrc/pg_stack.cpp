@@ -835,7 +835,7 @@ namespace {
 int moe_tile_rows(const pgk::Moe& m, int rows) {
   const long pairs = (long)rows * m.top;
   if (pairs <= 32L * m.experts) return 32;
-  return m.w_bf16 && pairs >= 96L * m.experts ? 128 : 64;
+  return m.w_bf16 && pairs >= 512L * m.experts ? 128 : 64;
 }
 
 // Working memory of a mixture of experts over `rows` rows, large enough for each layer added.
