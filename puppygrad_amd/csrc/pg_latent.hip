@@ -143,17 +143,21 @@ __global__ __launch_bounds__(256) void k_latent_query(LatentDecode m, LatentAttn
 // Everything a tile needs is asked for before the first of it is used.  Which position a row of the
 // ring holds does not matter: the first min(position + 1, window) rows are the ones that the token
 // sees.  Grid: x = share, y = 16 heads, z = sequence.  NT: column tiles of a wavefront; a row has at most
-// 64 NT + 256 columns.
+// 64 NT + ROT columns.
 constexpr int kShareRows = 32;
-template <int NT>
-__global__ __launch_bounds__(256, 1) void k_latent_attn(LatentDecode m, LatentAttn a) {
-  constexpr int MAXLD = 64 * NT + kMixMaxDim, NS = MAXLD / 32, NQ = 16 * MAXLD / 1024;
-  extern __shared__ __attribute__((aligned(16))) float qs[];  // [16][ld + 4]
+constexpr int kLatentGroup = 6;  // steps taken together
+constexpr int latent_steps(int nt, int rot) { return ((64 * nt + rot) / 32 + kLatentGroup - 1) / kLatentGroup * kLatentGroup; }
+static_assert(32 * kLatentGroup <= kLatentTail, "what a group may read past a row");
+template <int NT, int ROT>
+__global__ __launch_bounds__(256, NT <= 8 && ROT <= 64 ? 2 : 1) void k_latent_attn(LatentDecode m, LatentAttn a) {
+  constexpr int NS = latent_steps(NT, ROT), G = kLatentGroup, LD = 32 * NS + 4;
+  extern __shared__ __attribute__((aligned(16))) float qs[];  // [16][LD], zeros past a row's columns
   __shared__ __attribute__((aligned(16))) float ps[2][16][36];
-  __shared__ float ms[16], ls[16], al[16];
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, quarter = lane >> 4, l16 = lane & 15;
+  __shared__ __attribute__((aligned(16))) float ms[16], ls[16], al[16];
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int quarter = lane >> 4, l16 = lane & 15;
   const int split = blockIdx.x, h0 = blockIdx.y * 16, b = blockIdx.z;
-  const int nh = min(16, a.heads - h0), ld = a.ld, LD = ld + 4;
+  const int nh = min(16, a.heads - h0), ld = a.ld;
   const int pos = *m.d_pos, n = min(pos + 1, a.window);
   const int per = ((a.window + m.splits - 1) / m.splits + kShareRows - 1) / kShareRows * kShareRows;
   const int j0 = split * per, j1 = min(n, j0 + per);
@@ -167,38 +171,40 @@ __global__ __launch_bounds__(256, 1) void k_latent_attn(LatentDecode m, LatentAt
     return;
   }
   const float* ring = a.ring + (size_t)b * a.ring_seq;
-  const int tiles = a.kv_pad / 16, steps = ld / 16, rows16 = 16 * (wave & 1), first = wave >> 1;
-  f4 qr[NQ];
+  const int tiles = a.kv_pad / 16, first = wave >> 1, rows16 = 16 * (wave & 1);
+  const int mine = (ld / 16 - first + 1) / 2;  // steps of this wavefront: 16 columns from 16 (first + 2 s) on
+  // sixteen threads to a head
+  f4 qr[NS / 2];
   {
-    const f4* q = reinterpret_cast<const f4*>(m.qa + ((size_t)b * a.heads + h0) * ld);  // (16 rows, dense)
+    const int h = tid >> 4;
+    const float* q = m.qa + ((size_t)b * a.heads + h0 + min(h, nh - 1)) * ld + 4 * (tid & 15);
 #pragma unroll
-    for (int i = 0; i < NQ; ++i) {
-      const int x = tid + 256 * i;
+    for (int i = 0; i < NS / 2; ++i) {
       qr[i] = f4{0.f, 0.f, 0.f, 0.f};
-      if (x < nh * (ld / 4)) qr[i] = q[x];
+      if (h < nh && 4 * (tid & 15) + 64 * i < ld) qr[i] = *reinterpret_cast<const f4*>(q + 64 * i);
     }
   }
   f4 kr[NS];
   float cr[NT][8];
   auto fetch = [&](int k0) __attribute__((always_inline)) {
-    const float* row = ring + (size_t)min(k0 + rows16 + l16, j1 - 1) * ld + 4 * quarter;
+    // (whole groups of steps: past the row's columns lies the next row, or what the ring ends with)
+    const float* row = ring + (size_t)min(k0 + rows16 + l16, j1 - 1) * ld + 16 * first + 4 * quarter;
 #pragma unroll
     for (int s = 0; s < NS; ++s)
-      if (first + 2 * s < steps) kr[s] = *reinterpret_cast<const f4*>(row + 16 * (first + 2 * s));
+      if (s / G * G < mine) kr[s] = *reinterpret_cast<const f4*>(row + 32 * s);
+    const float* col[8];
+#pragma unroll
+    for (int k = 0; k < 8; ++k) col[k] = ring + (size_t)min(k0 + 4 * k + quarter, j1 - 1) * ld + 16 * wave + l16;
 #pragma unroll
     for (int t = 0; t < NT; ++t)
       if (wave + 4 * t < tiles) {
 #pragma unroll
-        for (int k = 0; k < 8; ++k)
-          cr[t][k] = ring[(size_t)min(k0 + 4 * k + quarter, j1 - 1) * ld + 16 * (wave + 4 * t) + l16];
+        for (int k = 0; k < 8; ++k) cr[t][k] = col[k][64 * t];
       }
   };
   fetch(j0);
 #pragma unroll
-  for (int i = 0; i < NQ; ++i) {
-    const int x = tid + 256 * i, h = x / (ld / 4);
-    if (h < 16) *reinterpret_cast<f4*>(&qs[h * LD + (x - h * (ld / 4)) * 4]) = qr[i];
-  }
+  for (int i = 0; i < NS / 2; ++i) *reinterpret_cast<f4*>(&qs[(tid >> 4) * LD + 4 * (tid & 15) + 64 * i]) = qr[i];
   if (tid < 16) {
     ms[tid] = kNone;
     ls[tid] = 0.0f;
@@ -209,44 +215,42 @@ __global__ __launch_bounds__(256, 1) void k_latent_attn(LatentDecode m, LatentAt
   __syncthreads();
   for (int k0 = j0; k0 < j1; k0 += kShareRows) {
     {
-      const float* q = qs + l16 * LD + 4 * quarter;
+      const float* q = qs + l16 * LD + 16 * first + 4 * quarter;
       f4 s0 = f4{0.f, 0.f, 0.f, 0.f}, s1 = s0;
 #pragma unroll
-      for (int s = 0; s < NS; ++s)
-        if (first + 2 * s < steps) {
-          const f4 q4 = *reinterpret_cast<const f4*>(q + 16 * (first + 2 * s));
-          s0 = __builtin_amdgcn_mfma_f32_16x16x4f32(kr[s].x, q4.x, s0, 0, 0, 0);
-          s1 = __builtin_amdgcn_mfma_f32_16x16x4f32(kr[s].y, q4.y, s1, 0, 0, 0);
-          s0 = __builtin_amdgcn_mfma_f32_16x16x4f32(kr[s].z, q4.z, s0, 0, 0, 0);
-          s1 = __builtin_amdgcn_mfma_f32_16x16x4f32(kr[s].w, q4.w, s1, 0, 0, 0);
+      for (int g = 0; g < NS / G; ++g) {
+        if (g * G >= mine) break;
+        f4 q4[G];
+#pragma unroll
+        for (int s = 0; s < G; ++s) q4[s] = *reinterpret_cast<const f4*>(q + 32 * (g * G + s));
+#pragma unroll
+        for (int s = 0; s < G; ++s) {
+          const f4 k4 = kr[g * G + s];
+          s0 = __builtin_amdgcn_mfma_f32_16x16x4f32(k4.x, q4[s].x, s0, 0, 0, 0);
+          s1 = __builtin_amdgcn_mfma_f32_16x16x4f32(k4.y, q4[s].y, s1, 0, 0, 0);
+          s0 = __builtin_amdgcn_mfma_f32_16x16x4f32(k4.z, q4[s].z, s0, 0, 0, 0);
+          s1 = __builtin_amdgcn_mfma_f32_16x16x4f32(k4.w, q4[s].w, s1, 0, 0, 0);
         }
+      }
       *reinterpret_cast<f4*>(&ps[first][l16][rows16 + 4 * quarter]) = s0 + s1;
     }
     __syncthreads();
     {
       // sixteen lanes to a head, two rows each
       const int h = 4 * wave + quarter, key = 2 * l16;
-      float s[2], mx = -INFINITY;
-#pragma unroll
-      for (int v = 0; v < 2; ++v) {
-        s[v] = k0 + key + v < j1 ? ps[0][h][key + v] + ps[1][h][key + v] : -INFINITY;
-        mx = fmaxf(mx, s[v]);
-      }
+      const float2 p0 = *reinterpret_cast<const float2*>(&ps[0][h][key]), p1 = *reinterpret_cast<const float2*>(&ps[1][h][key]);
+      const float z0 = k0 + key < j1 ? p0.x + p1.x : -INFINITY, z1 = k0 + key + 1 < j1 ? p0.y + p1.y : -INFINITY;
+      float mx = fmaxf(z0, z1);
 #pragma unroll
       for (int off = 8; off > 0; off >>= 1) mx = fmaxf(mx, __shfl_xor(mx, off, 64));
       const float old = ms[h], now = fmaxf(old, mx);
-      float sum = 0.0f;
-#pragma unroll
-      for (int v = 0; v < 2; ++v) {
-        s[v] = exp2f(s[v] - now);
-        sum += s[v];
-      }
+      const float w0 = __builtin_amdgcn_exp2f(z0 - now), w1 = __builtin_amdgcn_exp2f(z1 - now);
+      float sum = w0 + w1;
 #pragma unroll
       for (int off = 8; off > 0; off >>= 1) sum += __shfl_xor(sum, off, 64);
-      ps[0][h][key] = s[0];
-      ps[0][h][key + 1] = s[1];
+      *reinterpret_cast<float2*>(&ps[0][h][key]) = float2{w0, w1};
       if (l16 == 0) {
-        const float f = exp2f(old - now);
+        const float f = __builtin_amdgcn_exp2f(old - now);
         al[h] = f;
         ms[h] = now;
         ls[h] = ls[h] * f + sum;
@@ -254,16 +258,17 @@ __global__ __launch_bounds__(256, 1) void k_latent_attn(LatentDecode m, LatentAt
     }
     __syncthreads();
     {
-      f4 f;
       float p[8];
 #pragma unroll
-      for (int v = 0; v < 4; ++v) f[v] = al[4 * quarter + v];
-#pragma unroll
       for (int k = 0; k < 8; ++k) p[k] = ps[0][l16][4 * k + quarter];
+      if (k0 > j0) {
+        const f4 f = *reinterpret_cast<const f4*>(&al[4 * quarter]);
+#pragma unroll
+        for (int t = 0; t < NT; ++t) o[t] *= f;
+      }
 #pragma unroll
       for (int t = 0; t < NT; ++t)
         if (wave + 4 * t < tiles) {
-          o[t] *= f;
 #pragma unroll
           for (int k = 0; k < 8; ++k) o[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(p[k], cr[t][k], o[t], 0, 0, 0);
         }
@@ -273,16 +278,16 @@ __global__ __launch_bounds__(256, 1) void k_latent_attn(LatentDecode m, LatentAt
       __syncthreads();
     }
   }
+  float* dst[4];
 #pragma unroll
-  for (int t = 0; t < NT; ++t) {
-    const int tile = wave + 4 * t;
-    if (tile >= tiles) break;
+  for (int v = 0; v < 4; ++v) dst[v] = part + (4 * quarter + v) * part_h + 16 * wave + l16;
 #pragma unroll
-    for (int v = 0; v < 4; ++v) {
-      const int h = 4 * quarter + v;
-      if (h < nh) part[h * part_h + 16 * tile + l16] = o[t][v];
+  for (int t = 0; t < NT; ++t)
+    if (wave + 4 * t < tiles) {
+#pragma unroll
+      for (int v = 0; v < 4; ++v)
+        if (4 * quarter + v < nh) dst[v][64 * t] = o[t][v];
     }
-  }
   if (tid < nh) {
     part[tid * part_h + a.kv_pad] = ms[tid];
     part[tid * part_h + a.kv_pad + 1] = ls[tid];
@@ -297,7 +302,7 @@ __global__ __launch_bounds__(256) void k_latent_out(LatentDecode m, LatentAttn a
   __shared__ __attribute__((aligned(16))) float os[256 * NC];
   __shared__ float ws[kMaxShares];
   constexpr int PRE = 16;  // shares asked for before their weights are known
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, h = blockIdx.x, b = blockIdx.z;
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), h = blockIdx.x, b = blockIdx.z;
   const int e0 = blockIdx.y * 32 + wave, last = m.splits - 1;
   const size_t ps = a.kv_pad + 2;
   const float* part = m.part + ((size_t)b * a.heads + h) * m.splits * ps;
@@ -420,7 +425,7 @@ __global__ __launch_bounds__(256, 1) void k_latent_attn_rows(MixRows r, LatentAt
   constexpr int NK = KT * DP / 4 / TH, NV = KT * DV / 4 / TH;
   constexpr int TILE = KT * (LDK + LDV);
   extern __shared__ __attribute__((aligned(16))) float lds[];  // [KG][K tile, V tile]
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int qg = wave % QG, kg = wave / QG, st = tid % TH;
   const int half = lane >> 5, l32 = lane & 31;
   const int h = blockIdx.x, b = blockIdx.z;
@@ -645,17 +650,25 @@ hipError_t launch_latent_decode(const LatentDecode& m, const LatentAttn& a, hipS
   if (a.w_bf16) hipLaunchKernelGGL(k_latent_query<true>, qgrid, dim3(256), 0, s, m, a);
   else hipLaunchKernelGGL(k_latent_query<false>, qgrid, dim3(256), 0, s, m, a);
   const dim3 grid(m.splits, (a.heads + 15) / 16, m.nseq);
-  const size_t lds = 16 * (size_t)(a.ld + 4) * sizeof(float);
-  const void* kernel = a.kv_pad <= 256   ? reinterpret_cast<const void*>(&k_latent_attn<4>)
-                       : a.kv_pad <= 512 ? reinterpret_cast<const void*>(&k_latent_attn<8>)
-                                         : reinterpret_cast<const void*>(&k_latent_attn<16>);
-  if (lds > 48 * 1024) {
-    hipError_t e = hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 96 * 1024);
-    if (e != hipSuccess) return e;
+#define PG_ATTN(T, R)                                                                                                  \
+  {                                                                                                                    \
+    constexpr int lds = 16 * (32 * latent_steps(T, R) + 4) * (int)sizeof(float);                                       \
+    if (lds > 48 * 1024) {                                                                                             \
+      hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&k_latent_attn<T, R>),                          \
+                                         hipFuncAttributeMaxDynamicSharedMemorySize, lds);                             \
+      if (e != hipSuccess) return e;                                                                                   \
+    }                                                                                                                  \
+    hipLaunchKernelGGL((k_latent_attn<T, R>), grid, dim3(256), lds, s, m, a);                                          \
   }
-  if (a.kv_pad <= 256) hipLaunchKernelGGL(k_latent_attn<4>, grid, dim3(256), lds, s, m, a);
-  else if (a.kv_pad <= 512) hipLaunchKernelGGL(k_latent_attn<8>, grid, dim3(256), lds, s, m, a);
-  else hipLaunchKernelGGL(k_latent_attn<16>, grid, dim3(256), lds, s, m, a);
+  const bool narrow = a.ld - a.kv_pad <= 64;
+  if (a.kv_pad <= 256) {
+    if (narrow) PG_ATTN(4, 64) else PG_ATTN(4, 256)
+  } else if (a.kv_pad <= 512) {
+    if (narrow) PG_ATTN(8, 64) else PG_ATTN(8, 256)
+  } else {
+    PG_ATTN(16, 256)
+  }
+#undef PG_ATTN
   const dim3 ogrid(a.heads, (a.vdim + 31) / 32, m.nseq);
 #define PG_OUT(C)                                                                               \
   if (a.w_bf16) hipLaunchKernelGGL((k_latent_out<C, true>), ogrid, dim3(256), 0, s, m, a);       \

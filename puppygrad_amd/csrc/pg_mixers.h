@@ -184,6 +184,7 @@ hipError_t launch_group_rms_rows(const float* src, int ld_src, float* dst, int l
 // Rotation: the pair (2 i, 2 i + 1) turns by position * freq[i], i < half, and grows by mag; the
 // values from 2 * half on pass unchanged.
 constexpr int kLatentMaxRank = 1024;
+constexpr int kLatentTail = 256;  // floats that the last ring is followed by (read, multiplied by zeros)
 struct LatentAttn {
   int heads, dim, rot_dim, vdim;
   int q_rank, q_pad;      // q_pad, kv_pad: multiples of 32

@@ -918,7 +918,7 @@ pg_status stack_cache_create(const pg_model* model, pg_kv_cache* c) {
       if (pgk::rec_has_conv(l.rec.kind) && (s = alloc(B * l.rec.conv.taps * l.rec.conv.channels, &k.conv))) return s;
       if ((s = alloc(B * l.rec.heads * l.rec.dim * l.rec.vdim, &k.state))) return s;
     }
-    if (l.has_latent && (s = alloc(B * l.latent.window * l.latent.ld, &k.latent))) return s;
+    if (l.has_latent && (s = alloc(B * l.latent.window * l.latent.ld + pgk::kLatentTail, &k.latent))) return s;
   }
   float* words = nullptr;
   if ((s = alloc(sizeof(pgk::StepWords) / sizeof(float), &words))) return s;
