@@ -49,7 +49,7 @@ struct GemvArgs {
   float eps;
   int norm_n;  // PRO_RMS, PRO_STACK
   // PRO_STACK: K a multiple of 4; add and gain may be null; all vectors hold at least K values from a
-  // multiple of 16 bytes on, those past norm_n (add_n) zeros
+  // multiple of 16 bytes on; past norm_n (add_n) the gains are zeros and x is finite
   const float *add = nullptr, *add_gain = nullptr, *gain = nullptr;
   float* x_out = nullptr;  // not x itself: other blocks still read it
   int add_n = 0, groups = 1;

@@ -217,7 +217,12 @@ __global__ __launch_bounds__(kBlock) void k_gemv(GemvArgs a) {
         }
       }
       if (a.gain && a.groups <= 4) {
-        // (values past norm_n are zeros)
+        // (x may hold anything past norm_n, where the gains are zeros)
+#pragma unroll
+        for (int p = 0; p < kIn; ++p)
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+            if (4 * (tid + kBlock * p) + e >= a.norm_n) (&vx[p].x)[e] = 0.0f;
         float inv[4] = {0.f, 0.f, 0.f, 0.f};
         const int n = a.norm_n / a.groups;
         if (a.groups == 1) {

@@ -50,7 +50,7 @@ def config(layers, width=48, vocab=61, eps=1e-5):
 
 
 MIXED = config([delta(mlp=moe()), latent(mlp=dense()), mamba(mlp=moe(5, 3, 20)), latent(3, 24, 6, 20, 33, 17, 19),
-                mamba(4, 16, 8, 4, 1, 2), delta(6, 3, 20, 16, 4, mlp=dense(33))])
+                mamba(4, 11, 8, 4, 1, 2), delta(6, 3, 20, 16, 4, mlp=dense(33))])
 
 
 def weights(cfg, seed, ranks=(5, 3), **fixed):
@@ -235,6 +235,14 @@ def test_layer_order_and_first_layers(tmp_path):
         cfg = config(layers)
         p = Pair(tmp_path / str(i), cfg, weights(cfg, 30 + i))
         all_ways(p, p.ids(45), ((11, 1),))
+
+
+def test_mixers_of_unequal_width(tmp_path):
+    """What a wide mixer leaves behind the columns of a narrow one is not part of the narrow one's norm."""
+    for i, groups in enumerate((1, 2, 3, 6)):
+        cfg = config([latent(4, 16, 8, 40), mamba(6, 7, 8, 2, groups), delta(4, 2, 8, 30), mamba(6, 5, 8, 2, groups, mlp=dense(7))])
+        p = Pair(tmp_path / str(i), cfg, weights(cfg, 35 + i))
+        all_ways(p, p.ids(40), ((11, 1),))
 
 
 def test_first_tokens(mixed):
