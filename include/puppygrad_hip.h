@@ -483,9 +483,9 @@ pg_status pg_gpt2_create_from_dir(const char* model_dir, const pg_hip_options* o
 /* The model of a directory (config.json + model.safetensors).  The architecture is the one
  * config.json names under `architecture`; a config.json without that key is a Hugging Face GPT-2's
  * (pg_gpt2_create_from_dir).  An unknown name is PG_INVALID_CONFIG.
- * "Tarepel" (a stack model): `layers` lists every layer with its mixers and their sizes; weights
- * are BF16 or F32 tensors, kept as weight_storage says (PG_STORE_F32 or PG_STORE_BF16; activations
- * and state are f32 either way).  A sequence's state has a fixed size, so its caches take
+ * "Tarepel" and "Movudra" (stack models): `layers` lists every layer with its mixers and their
+ * sizes; weights are BF16 or F32 tensors, kept as weight_storage says (PG_STORE_F32 or
+ * PG_STORE_BF16; activations and state are f32 either way).  A sequence's state has a fixed size, so its caches take
  * sequences of any length. */
 pg_status pg_model_create_from_dir(const char* model_dir, const pg_hip_options* options, pg_model** out);
 void pg_model_destroy(pg_model* model);
@@ -525,8 +525,8 @@ pg_status pg_model_stream_token_ids_with_stats(const pg_model* model, const uint
                                                uint64_t seed, pg_on_token on_token, void* user,
                                                uint32_t* out_ids, size_t* out_n, pg_generation_stats* stats);
 /* (Stack models: the input projections count as qkv_projection, the mixers as attention, the
- * products back to the residual as attention_projection and mlp_projection; the one-token step
- * has both of these in one launch, counted as mlp_projection.) */
+ * products back to the residual as attention_projection and mlp_projection; Tarepel's one-token
+ * step has both of these in one launch, counted as mlp_projection.) */
 pg_status pg_model_stream_token_ids_profiled(const pg_model* model, const uint32_t* ids, size_t n,
                                              uint32_t max_new, int64_t eos, const pg_sampling* sampling,
                                              uint64_t seed, pg_on_token on_token, void* user,

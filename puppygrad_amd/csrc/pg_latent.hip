@@ -85,8 +85,8 @@ __global__ __launch_bounds__(256) void k_latent_query(LatentDecode m, LatentAttn
   const int tid = threadIdx.x, h = blockIdx.x, b = blockIdx.z, pos = *m.d_pos;
   if (h == a.heads) {
     if (blockIdx.y == 0)
-      latent_row(a, m.y + (size_t)b * m.ld_y + a.c_col, pos, a.ring + (size_t)b * a.ring_seq + (size_t)(pos % a.window) * a.ld,
-                 red);
+      latent_row(a, m.y + (size_t)b * m.ld_y + a.c_col, pos,
+                 a.ring + (size_t)b * a.ring_seq + (size_t)(pos % a.window) * a.ld, red);
     return;
   }
   const float* q = m.q + ((size_t)b * a.heads + h) * (a.dim + a.rot_dim);
@@ -146,7 +146,9 @@ __global__ __launch_bounds__(256) void k_latent_query(LatentDecode m, LatentAttn
 // 64 NT + ROT columns.
 constexpr int kShareRows = 32;
 constexpr int kLatentGroup = 6;  // steps taken together
-constexpr int latent_steps(int nt, int rot) { return ((64 * nt + rot) / 32 + kLatentGroup - 1) / kLatentGroup * kLatentGroup; }
+constexpr int latent_steps(int nt, int rot) {
+  return ((64 * nt + rot) / 32 + kLatentGroup - 1) / kLatentGroup * kLatentGroup;
+}
 static_assert(32 * kLatentGroup <= kLatentTail, "what a group may read past a row");
 template <int NT, int ROT>
 __global__ __launch_bounds__(256, NT <= 8 && ROT <= 64 ? 2 : 1) void k_latent_attn(LatentDecode m, LatentAttn a) {
@@ -238,7 +240,8 @@ __global__ __launch_bounds__(256, NT <= 8 && ROT <= 64 ? 2 : 1) void k_latent_at
     {
       // sixteen lanes to a head, two rows each
       const int h = 4 * wave + quarter, key = 2 * l16;
-      const float2 p0 = *reinterpret_cast<const float2*>(&ps[0][h][key]), p1 = *reinterpret_cast<const float2*>(&ps[1][h][key]);
+      const float2 p0 = *reinterpret_cast<const float2*>(&ps[0][h][key]);
+      const float2 p1 = *reinterpret_cast<const float2*>(&ps[1][h][key]);
       const float z0 = k0 + key < j1 ? p0.x + p1.x : -INFINITY, z1 = k0 + key + 1 < j1 ? p0.y + p1.y : -INFINITY;
       float mx = fmaxf(z0, z1);
 #pragma unroll
@@ -302,7 +305,8 @@ __global__ __launch_bounds__(256) void k_latent_out(LatentDecode m, LatentAttn a
   __shared__ __attribute__((aligned(16))) float os[256 * NC];
   __shared__ float ws[kMaxShares];
   constexpr int PRE = 16;  // shares asked for before their weights are known
-  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), h = blockIdx.x, b = blockIdx.z;
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int h = blockIdx.x, b = blockIdx.z;
   const int e0 = blockIdx.y * 32 + wave, last = m.splits - 1;
   const size_t ps = a.kv_pad + 2;
   const float* part = m.part + ((size_t)b * a.heads + h) * m.splits * ps;
@@ -319,8 +323,10 @@ __global__ __launch_bounds__(256) void k_latent_out(LatentDecode m, LatentAttn a
 #pragma unroll
   for (int r = 0; r < 8; ++r)
 #pragma unroll
-    for (int c = 0; c < NC; ++c)
-      w[r][c] = load_w4<BF16>(a.up_w, ((size_t)a.v_row + h * a.vdim + min(e0 + 4 * r, a.vdim - 1)) * a.kv_pad + min(4 * lane + 256 * c, a.kv_pad - 4));
+    for (int c = 0; c < NC; ++c) {
+      const size_t row = (size_t)a.v_row + h * a.vdim + min(e0 + 4 * r, a.vdim - 1);
+      w[r][c] = load_w4<BF16>(a.up_w, row * a.kv_pad + min(4 * lane + 256 * c, a.kv_pad - 4));
+    }
   if (wave == 0) {
     float top = fmaxf(mx, sink);
 #pragma unroll
@@ -354,7 +360,8 @@ __global__ __launch_bounds__(256) void k_latent_out(LatentDecode m, LatentAttn a
   for (int r = 0; r < 8; ++r) {
     float s = 0.0f;
 #pragma unroll
-    for (int c = 0; c < NC; ++c) s += (w[r][c].x * o[c].x + w[r][c].y * o[c].y) + (w[r][c].z * o[c].z + w[r][c].w * o[c].w);
+    for (int c = 0; c < NC; ++c)
+      s += (w[r][c].x * o[c].x + w[r][c].y * o[c].y) + (w[r][c].z * o[c].z + w[r][c].w * o[c].w);
     s = wave_sum(s);
     if (lane == 0 && e0 + 4 * r < a.vdim) m.out[(size_t)b * m.ld_out + a.out_col + h * a.vdim + e0 + 4 * r] = s;
   }

@@ -1,5 +1,5 @@
 // gfx950 kernels of a mixture of experts (pg_mixers.h): routing, the sorting of (row, expert) pairs
-// for grouped products, and the experts of a few rows as matrix-vector products.
+// for grouped products, and the experts of one row as matrix-vector products.
 //
 // Shapes are checked on the host before any launch (pg_stack.cpp).
 #include "pg_mixers.h"

@@ -173,6 +173,15 @@ def test_experts_of_unequal_load(tmp_path):
     all_ways(p, p.ids(420), ((300, 33, 87),))
 
 
+@pytest.mark.parametrize("storage", [BF16, F32], ids=["bf16", "f32"])
+def test_experts_of_many_rows(tmp_path, storage):
+    """Enough rows for the largest tiles of an expert."""
+    cfg = config([mamba(1, 8, 8, 1, 1, 2, mlp=moe(2, 1, 70)), mamba(1, 8, 8, 1, 1, 2, mlp=moe(4, 3, 9))], width=100)
+    p = Pair(tmp_path, cfg, weights(cfg, 10), storage)
+    ids = p.ids(1100)
+    check(p.portions(ids, [1100]), p.ref.run(ids))
+
+
 def test_strong_decays(tmp_path):
     """Decays from none to a state that is wiped by a single token, side by side."""
     cfg = config([mamba(), delta(), delta(2, 2, 32, 16)])
