@@ -176,7 +176,7 @@ def test_experts_of_unequal_load(tmp_path):
 @pytest.mark.parametrize("storage", [BF16, F32], ids=["bf16", "f32"])
 def test_experts_of_many_rows(tmp_path, storage):
     """Enough rows for the largest tiles of an expert."""
-    cfg = config([mamba(1, 8, 8, 1, 1, 2, mlp=moe(2, 1, 70)), mamba(1, 8, 8, 1, 1, 2, mlp=moe(4, 3, 9))], width=100)
+    cfg = config([mamba(4, 16, 8, 1, 1, 2, mlp=moe(2, 1, 70)), mamba(4, 16, 8, 1, 1, 2, mlp=moe(4, 3, 9))], width=100)
     p = Pair(tmp_path, cfg, weights(cfg, 10), storage)
     ids = p.ids(1100)
     check(p.portions(ids, [1100]), p.ref.run(ids))
